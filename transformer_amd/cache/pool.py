@@ -71,14 +71,16 @@ RELEASED = -1      # stands in a slot's page list for a page that was given back
 
 
 class Slot:
-    __slots__ = ("index", "length", "pages", "released", "live")
+    __slots__ = ("index", "length", "pages", "kept", "released", "live")
 
     def __init__(self, index: int, num_groups: int):
         self.index = index
         self.length = 0
         # pages[g][i] holds positions [i * page_size, (i + 1) * page_size) in group g
         self.pages: List[List[int]] = [[] for _ in range(num_groups)]
-        self.released = [0] * num_groups      # leading entries of pages[g] that are RELEASED
+        # entries kept[g] .. released[g] - 1 of pages[g] are RELEASED; those before kept[g] stay held
+        self.kept = [0] * num_groups
+        self.released = [0] * num_groups
         self.live = False
 
 
@@ -135,9 +137,9 @@ class SlotPool:
 
     def _drop_pages(self, s: Slot) -> None:
         for g, pool in enumerate(self.pools):
-            pool.give(s.pages[g][s.released[g]:])
+            pool.give([p for p in s.pages[g] if p != RELEASED])
             s.pages[g] = []
-            s.released[g] = 0
+            s.kept[g] = s.released[g] = 0
 
     def reset(self, index: int) -> None:
         """The slot stays with its owner but forgets its tokens and gives its pages back."""
@@ -180,13 +182,18 @@ class SlotPool:
             raise CacheError(f"slot {index}: advancing by {tokens} tokens past its reserved pages")
         s.length += tokens
 
-    def release_before(self, index: int, group: int, position: int) -> int:
+    def release_before(self, index: int, group: int, position: int, keep_pages: int = 0) -> int:
         """Gives back the pages of one group that lie wholly before ``position``: a group
-        whose layers read a window of keys never looks at them again. Their places in the
+        whose layers read a window of keys never looks at them again, but for the sequence's first
+        ``keep_pages`` pages (the same number at every call). Their places in the
         slot's page list keep RELEASED, so that a position still finds its page by index.
         Returns the number of pages given back."""
         s = self._slot(index)
         upto = min(max(position, 0), s.length) // self.page_size
+        if s.released[group] == s.kept[group]:                  # nothing given back yet
+            s.kept[group] = s.released[group] = keep_pages
+        elif keep_pages != s.kept[group]:
+            raise CacheError(f"slot {index}: {keep_pages} pages are to be kept where {s.kept[group]} were")
         first = s.released[group]
         if upto <= first:
             return 0
@@ -219,11 +226,12 @@ class SlotPool:
         for g, pool in enumerate(self.pools):
             seen = set()
             for s in self.slots:
-                if any(p != RELEASED for p in s.pages[g][:s.released[g]]) or \
-                        any(p == RELEASED for p in s.pages[g][s.released[g]:]):
+                held = s.pages[g][:s.kept[g]] + s.pages[g][s.released[g]:]
+                if any(p != RELEASED for p in s.pages[g][s.kept[g]:s.released[g]]) or \
+                        any(p == RELEASED for p in held):
                     raise CacheError(f"slot {s.index}: released pages of group "
                                      f"{self.group_keys[g]!r} are out of place")
-                for p in s.pages[g][s.released[g]:]:
+                for p in held:
                     if p in seen:
                         raise CacheError(f"page {p} of group {self.group_keys[g]!r} is held twice")
                     seen.add(p)

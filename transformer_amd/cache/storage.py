@@ -30,15 +30,23 @@ from ..kernels import PAGE   # tokens per cache page: one constant, checked agai
 class KVNeed:
     """Keys and values of every position (or of a window of them). ``value_dim``: width of a
     value row where it differs from the key's (None: the same; 0: keys only, for a mixer that
-    keeps one row per token and derives both from it)."""
+    keeps one row per token and derives both from it). ``keep_first``: with a window, a sequence's
+    first tokens that stay readable besides it."""
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None     # None: every earlier position is read
     value_dim: Optional[int] = None
+    keep_first: int = 0
 
     def __post_init__(self):
         if self.value_dim is None:
             object.__setattr__(self, "value_dim", self.head_dim)
+        if self.window is None:                      # everything is kept anyway
+            object.__setattr__(self, "keep_first", 0)
+
+    @property
+    def keep_pages(self) -> int:
+        return -(-self.keep_first // PAGE)
 
 
 @dataclass(frozen=True)
@@ -106,9 +114,9 @@ class SequenceCache:
         if max_step_tokens is not None:
             for g, need in enumerate(self.kv_groups):
                 if need.window is not None:
-                    # a slot holds at most the pages that touch its window and its share of
-                    # the step: (window + n - 1) / PAGE + 2
-                    bound = max_slots * (need.window // PAGE + 3) + max_step_tokens // PAGE
+                    # a slot holds at most the pages of its kept first tokens and those that touch
+                    # its window and its share of the step: (window + n - 1) / PAGE + 2
+                    bound = max_slots * (need.keep_pages + need.window // PAGE + 3) + max_step_tokens // PAGE
                     self.group_pages[g] = max(1, min(self.num_pages, bound))
         self.pool = SlotPool(max_slots, PAGE, dict(enumerate(self.group_pages)))
         self.keys, self.values = [], []
@@ -153,11 +161,12 @@ class SequenceCache:
 
     def release_outside_windows(self, slot: int) -> None:
         """After a step: the next token of the slot sits at position ``length`` and a layer
-        with window w reads keys from ``length + 1 - w`` on; earlier pages go back."""
+        with window w reads keys from ``length + 1 - w`` on; earlier pages go back, but for those of
+        the first tokens that the layer keeps."""
         n = self.pool.length(slot)
         for g, need in enumerate(self.kv_groups):
             if need.window is not None:
-                self.pool.release_before(slot, g, n + 1 - need.window)
+                self.pool.release_before(slot, g, n + 1 - need.window, need.keep_pages)
 
     def bytes(self) -> int:
         n = sum(t.numel() * t.element_size() for t in self.keys + self.values + self.states)

@@ -80,12 +80,14 @@ class SwiGLUSpec:
 @dataclass(frozen=True)
 class BlockSpec:
     """x += mixer(norm1(x)); x += ffn(norm2(x))  (kind "prenorm"). ffn None (and norm2 None): the
-    block has the mixer only."""
+    block has the mixer only. side: a ``TokenSideSpec`` whose part then adds what it derives from
+    the stream and the step's tokens."""
     norm1: object
     mixer: object
     norm2: object = None
     ffn: object = None
     kind: str = "prenorm"
+    side: object = None
 
 
 @dataclass(frozen=True)
@@ -96,9 +98,12 @@ class RunSpec:
     cache_of: None = this run owns a cache layer of its own (if its mixer
     needs one); an int names an EARLIER schedule entry whose cache layer this
     run reads instead of writing one.
+    opening: None, or a row of the model's table of stream rows (``ModelSpec.stream_rows``) that is
+    added to the residual stream of every token right before this run.
     """
     block: int
     cache_of: Optional[int] = None
+    opening: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -117,6 +122,8 @@ class ModelSpec:
     # embedding, [wanted, vocab] for the logits). The Llama decoder has neither.
     after_embed: object = None
     on_logits: object = None
+    # rows of the learned table [stream_rows, hidden] that schedule entries name as their opening
+    stream_rows: int = 0
 
     def validate(self) -> None:
         if self.vocab <= 0 or self.hidden <= 0:
@@ -127,6 +134,9 @@ class ModelSpec:
             if not 0 <= run.block < len(self.blocks):
                 raise ConfigError(f"schedule[{i}] names block {run.block}, "
                                   f"model has {len(self.blocks)}")
+            if run.opening is not None and not 0 <= run.opening < self.stream_rows:
+                raise ConfigError(f"schedule[{i}].opening={run.opening}, the model has "
+                                  f"{self.stream_rows} stream rows")
             if run.cache_of is not None:
                 if not 0 <= run.cache_of < i:
                     raise ConfigError(f"schedule[{i}].cache_of={run.cache_of} must name an "
@@ -150,12 +160,16 @@ class ScalarNormSpec:
 
 @dataclass(frozen=True)
 class GLUSpec:
-    """down(act(gate(h)) * up(h)); activation "silu" or "gelu_tanh"."""
+    """down(act(gate(h)) * up(h)); activation "silu", "gelu_tanh", or "limited": g = min(gate(h),
+    limit), u = clamp(up(h), -limit, limit), down(g * sigmoid(gate_slope * g) * (u + up_shift))."""
     hidden: int
     intermediate: int
     activation: str = "silu"
     bias: bool = False
     kind: str = "glu"
+    limit: float = 0.0
+    gate_slope: float = 1.702
+    up_shift: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -342,13 +356,14 @@ class RoutedMLPSpec:
 class LatentAttentionSpec:
     """Softmax attention whose keys and values are linear maps of ONE cached latent per token.
 
-    Queries: cq = rms_norm(Dq h) (q_rank wide), q = Uq cq, per head [nope_dim unrotated |
+    Queries: cq = rms_norm(Dq h) (q_rank wide), q = Uq cq (q_rank None: q = Q h), per head [nope_dim unrotated |
     rope_dim rotated]. Keys/values: Dkv h = [kv_rank | rope_dim]; the first part, RMS-normed,
     is the latent c, the second, rotated, is a key part that all heads share; per head k =
     [Uk c | shared part], v = Uv c (value_dim). Rotation: the first rot_dims coordinates of a
     rotated part in pairs (2i, 2i + 1) by position * rot_base^(-2i/rot_dims). window: a query
     at p reads keys in (p - window, p]; None: all. gated: head h's result is multiplied by
-    sigmoid(g_h . h). own_kv False: no Dkv; the layer reads the rows that the layer whose cache
+    sigmoid(g_h . h). sink: a row's softmax denominator also holds exp(s_h), s_h a learned number per
+    head that is not scaled and has no value. own_kv False: no Dkv; the layer reads the rows that the layer whose cache
     it borrows stored (its schedule entry names it). cache_window: the window the cache layer
     is kept for (the widest of the layers that read it; None: everything)."""
     hidden: int
@@ -356,7 +371,7 @@ class LatentAttentionSpec:
     nope_dim: int
     rope_dim: int
     value_dim: int
-    q_rank: int
+    q_rank: Optional[int]
     kv_rank: int
     scale: float
     eps: float
@@ -367,6 +382,7 @@ class LatentAttentionSpec:
     gated: bool = True
     own_kv: bool = True
     kind: str = "latent_attention"
+    sink: bool = False
 
 
 @dataclass(frozen=True)
@@ -475,7 +491,12 @@ class SinkAttentionSpec:
     heads are multiplied by sigmoid(Wg h) before the output projection. own_kv False: no key and value
     projections; the layer reads what the layer whose cache it borrows stored (its schedule entry
     names it). cache_window: the window the cache layer is kept for (the widest of the layers that
-    read it; 0: everything; None: the layer's own window)."""
+    read it; 0: everything; None: the layer's own window).
+    keep_first: with a window, a query also reads the first keep_first keys of the sequence, wherever it
+    stands. unit_norm: every head of q and k is divided by its root mean square (eps) before the rotation.
+    values_from_keys: no value projection, a head's values are its keys as projected (before norm and
+    rotation; value_dim = key_dim). head_gate: every head's result is multiplied by the sigmoid of ONE
+    number, a projection of h."""
     hidden: int
     num_heads: int
     num_kv_heads: int
@@ -496,6 +517,11 @@ class SinkAttentionSpec:
     out_gate: bool = False
     own_kv: bool = True
     kind: str = "attention_sink"
+    keep_first: int = 0
+    unit_norm: bool = False
+    eps: float = 0.0
+    values_from_keys: bool = False
+    head_gate: bool = False
 
 
 @dataclass(frozen=True)
@@ -528,3 +554,37 @@ class BranchSumSpec:
     names: Tuple[str, ...]
     scales: Tuple[float, ...]
     kind: str = "branch_sum"
+
+
+# ---------------------------------------------------------------------------------------------
+# Parts that the Zirutar decoder added; as above, every size and constant is a field.
+
+@dataclass(frozen=True)
+class OffsetNormSpec:
+    """RMS norm whose weight is stored around zero: the gain of a coordinate is 1 + w."""
+    size: int
+    eps: float
+    kind: str = "rmsnorm_offset"
+
+
+@dataclass(frozen=True)
+class GatedDeltaSpec:
+    """Gated delta rule with a decay per head and key channel. q, k (num_kv_heads heads of key_dim) and v
+    (num_heads of value_dim) pass a causal convolution of ``taps`` per channel (no bias) and silu; q and k
+    become unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q is also scaled by key_dim^-1/2; head h reads
+    the q and k of group h // (num_heads / num_kv_heads). Per head a state S [key_dim, value_dim], float32,
+    zero at a sequence's start: S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, with beta =
+    sigmoid(Wb h) per head and g = exp(-exp(A_log_h) softplus(Wa2 (Wa1 h) + dt_bias)) per head and key
+    channel (Wa1 maps to decay_rank numbers). o is divided by its root mean square per head, times a weight
+    [value_dim] shared by the heads, times sigmoid(Wg2 (Wg1 h)) (Wg1 maps to gate_rank numbers), then
+    projected. State per sequence: S and the last taps - 1 rows of [q | k | v] as projected."""
+    hidden: int
+    num_heads: int
+    num_kv_heads: int
+    key_dim: int
+    value_dim: int
+    taps: int
+    decay_rank: int
+    gate_rank: int
+    eps: float
+    kind: str = "gated_delta"

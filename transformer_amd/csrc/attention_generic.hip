@@ -11,7 +11,8 @@
 //
 // Options (all off in the plain entry points): scores capped by cap * tanh(score / cap); one more
 // term in the softmax denominator that has no value (a "sink": exp(0), or exp of a learned number
-// per head); the result multiplied by the sigmoid of a gate row.
+// per head); the result multiplied by the sigmoid of a gate, element by element or one number per head;
+// a window that besides the last keys also shows a sequence's first `keep` keys.
 #include "common.h"
 
 #define ROWS 16
@@ -35,7 +36,7 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ pos0, int nh, int nkv, int dh, int dv, float scale, int window,
     float softcap, int sink_mode, const float* __restrict__ sink, const T* __restrict__ gate, int gate_stride,
-    int gate_dv) {
+    int gate_dv, int keep) {
   extern __shared__ float smem[];
   const int group = nh / nkv;
   const int b = blockIdx.z, kvh = blockIdx.y;
@@ -85,8 +86,15 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
   float m = -INFINITY, l = 0.f;
 
   const int* table = block_table + (size_t)b * max_blocks;
-  for (int c = tile_start / CHUNK; c * CHUNK < tile_end; ++c) {
+  // chunks of the kept first keys that the window has left behind, then the window's
+  const int win_chunk = tile_start / CHUNK;
+  int c = keep > 0 ? 0 : win_chunk;
+  for (; c * CHUNK < tile_end; ++c) {
     const int key0 = c * CHUNK;
+    if (c < win_chunk && key0 >= keep) {       // nothing between the kept keys and the window is read
+      c = win_chunk - 1;
+      continue;
+    }
     const size_t page = (size_t)table[key0 / TA_PAGE];
     const size_t base = ((page * nkv + kvh) * TA_PAGE + key0 % TA_PAGE) * (size_t)dh;
     const size_t vbase = (page * nkv + kvh) * (size_t)dv * TA_PAGE + key0 % TA_PAGE;
@@ -108,8 +116,8 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
       }
     }
     const int kk0 = key0 + lane, kk1 = kk0 + 16;
-    const bool v0 = row_ok && kk0 >= my_start && kk0 < my_end;
-    const bool v1 = row_ok && kk1 >= my_start && kk1 < my_end;
+    const bool v0 = row_ok && (kk0 >= my_start || kk0 < keep) && kk0 < my_end;
+    const bool v1 = row_ok && (kk1 >= my_start || kk1 < keep) && kk1 < my_end;
     s0 *= scale;
     s1 *= scale;
     if (softcap > 0.f) {              // capped scores: cap * tanh(score / cap)
@@ -161,10 +169,12 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
 #pragma unroll
       for (int i = 0; i < 16; ++i) acc[i] *= alpha;
     }
-    const float inv = l > 0.f ? 1.0f / l : 0.f;
+    float inv = l > 0.f ? 1.0f / l : 0.f;
+    if (gate && gate_dv == 0)          // one number per head
+      inv *= 1.0f / (1.0f + expf(-to_f32(gate[(size_t)(q0 + qi) * gate_stride + head])));
     T* o = out + (size_t)(q0 + qi) * out_stride + (size_t)head * dv + lane;
     // the gate's rows hold gate_dv columns per head (the values' own width where the cache pads them)
-    const T* gt = gate ? gate + (size_t)(q0 + qi) * gate_stride + (size_t)head * gate_dv + lane : nullptr;
+    const T* gt = gate && gate_dv > 0 ? gate + (size_t)(q0 + qi) * gate_stride + (size_t)head * gate_dv + lane : nullptr;
 #pragma unroll
     for (int i = 0; i < 16; ++i)
       if (i < nd && 16 * i + lane < dv) {
@@ -187,12 +197,13 @@ static int attention_generic_launch(hipStream_t stream, int dtype, const void* q
                                     const int* cu_q, const int* pos0, int batch, int max_qlen,
                                     int nh, int nkv, int dh, int dv, float scale, int window,
                                     float softcap = 0.f, int sink_mode = 0, const float* sink = nullptr,
-                                    const void* gate = nullptr, int gate_stride = 0, int gate_dv = 0) {
-  if (gate_dv <= 0) gate_dv = dv;
+                                    const void* gate = nullptr, int gate_stride = 0, int gate_dv = 0, int keep = 0) {
   TA_REQUIRE(batch >= 0 && max_qlen >= 0, "ta_attention_generic: bad batch=%d max_qlen=%d", batch, max_qlen);
   TA_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 2 || sink != nullptr) && softcap >= 0.f,
              "ta_attention_generic: sink mode %d, cap %f", sink_mode, softcap);
-  TA_REQUIRE(gate == nullptr || (gate_dv <= dv && gate_stride >= nh * gate_dv), "ta_attention_generic: gate rows of %d", gate_stride);
+  TA_REQUIRE(gate == nullptr || (gate_dv >= 0 && gate_dv <= dv && gate_stride >= nh * (gate_dv > 0 ? gate_dv : 1)),
+             "ta_attention_generic: gate rows of %d", gate_stride);
+  TA_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "ta_attention_generic: %d kept keys beside a window of %d", keep, window);
   TA_REQUIRE(nh > 0 && nkv > 0 && nh % nkv == 0, "ta_attention_generic: %d heads do not divide into %d kv heads", nh, nkv);
   TA_REQUIRE(dh >= 1 && dh <= 256 && dv >= 1 && dv <= 256,
              "ta_attention_generic: key width %d / value width %d outside [1, 256]", dh, dv);
@@ -207,12 +218,12 @@ static int attention_generic_launch(hipStream_t stream, int dtype, const void* q
     attn_generic_kernel<float><<<g, blk, lds, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)kcache,
         (const float*)vcache, block_table, max_blocks, cu_q, pos0, nh, nkv, dh, dv, scale, window,
-        softcap, sink_mode, sink, (const float*)gate, gate_stride, gate_dv);
+        softcap, sink_mode, sink, (const float*)gate, gate_stride, gate_dv, keep);
   else if (dtype == TA_BF16)
     attn_generic_kernel<bf16_t><<<g, blk, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache,
         (const bf16_t*)vcache, block_table, max_blocks, cu_q, pos0, nh, nkv, dh, dv, scale, window,
-        softcap, sink_mode, sink, (const bf16_t*)gate, gate_stride, gate_dv);
+        softcap, sink_mode, sink, (const bf16_t*)gate, gate_stride, gate_dv, keep);
   else
     return ta_fail("ta_attention_generic: unknown dtype %d", dtype);
   return ta_check_launch("ta_attention_generic");
@@ -240,15 +251,16 @@ extern "C" int ta_attention_generic_dv(hipStream_t stream, int dtype, const void
 // The same with the options of a capped, sunk and gated softmax: softcap > 0: score <- softcap *
 // tanh(score / softcap) after the scale; sink_mode 1: the denominator holds one more term exp(0);
 // 2: exp(sink[head]) (float32 [nh]); gate: rows [nt, >= nh*gate_dv] whose sigmoid multiplies the first gate_dv
-// columns of every head of the result (gate_dv <= dv; 0: dv).
+// columns of every head of the result (gate_dv <= dv; 0: rows [nt, >= nh] with one number per head). keep:
+// with a window, the first `keep` keys of a sequence are seen as well.
 extern "C" int ta_attention_generic_sink(hipStream_t stream, int dtype, const void* q, int q_stride,
                                          void* out, int out_stride, const void* kcache,
                                          const void* vcache, const int* block_table, int max_blocks,
                                          const int* cu_q, const int* pos0, int batch, int max_qlen,
                                          int nh, int nkv, int dh, int dv, float scale, int window,
                                          float softcap, int sink_mode, const float* sink, const void* gate,
-                                         int gate_stride, int gate_dv) {
+                                         int gate_stride, int gate_dv, int keep) {
   return attention_generic_launch(stream, dtype, q, q_stride, out, out_stride, kcache, vcache, block_table,
                                   max_blocks, cu_q, pos0, batch, max_qlen, nh, nkv, dh, dv, scale, window,
-                                  softcap, sink_mode, sink, gate, gate_stride, gate_dv);
+                                  softcap, sink_mode, sink, gate, gate_stride, gate_dv, keep);
 }

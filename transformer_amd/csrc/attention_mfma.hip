@@ -66,12 +66,14 @@ __device__ __forceinline__ uint32_t pack2(float a, float b) { return f32x2_to_bf
 //     float32 weight, so only keys and values are rounded to 16 bits
 //   sink_mode 1: the denominator holds one more term exp(0); 2: exp(sink[head])
 //   gate: rows [token][gate_stride] whose sigmoid multiplies the first gate_dv columns of every head
+//     (gate_dv 0: one number per head)
+//   keep: with a window, the sequence's first `keep` keys are seen as well
 struct AttnExtra {
   float cap_k, cap_r;
   int exact, sink_mode;
   const float* sink;
   const bf16_t* gate;
-  int gate_stride, gate_dv;
+  int gate_stride, gate_dv, keep;
 };
 
 __device__ __forceinline__ float capped_score(float s, float cap_k, float cap_r) {
@@ -85,9 +87,14 @@ __device__ __forceinline__ float sink_term(const AttnExtra& x, int head, float m
   return __builtin_amdgcn_exp2f(sv - m_use);
 }
 __device__ __forceinline__ float gate_factor(const AttnExtra& x, size_t token, int head, int d) {
-  if (x.gate == nullptr || d >= x.gate_dv) return 1.f;
+  if (x.gate == nullptr || d >= x.gate_dv) return 1.f;      // also with one number per head: head_gate
   const float g = to_f32(x.gate[token * x.gate_stride + (size_t)head * x.gate_dv + d]);
   return 1.0f / (1.0f + __expf(-g));
+}
+
+__device__ __forceinline__ float head_gate(const AttnExtra& x, size_t token, int head) {
+  if (x.gate == nullptr || x.gate_dv != 0) return 1.f;
+  return 1.0f / (1.0f + __expf(-to_f32(x.gate[token * x.gate_stride + head])));
 }
 
 // Maximum and sum over the lanes 16 or 32 apart, by the lane-swap instructions of gfx950 (one
@@ -188,7 +195,8 @@ __device__ __forceinline__ void wave_page(WaveState<DH>& w, const bf16_t* __rest
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
         const int key = key0 + sub * 32 + 8 * (r / 4) + 4 * h + (r % 4);
-        const float t = (key >= my_start && key < my_end) ? s[sub][r] : -INFINITY;
+        const bool in = XTRA ? (key >= my_start || key < x.keep) && key < my_end : key >= my_start && key < my_end;
+        const float t = in ? s[sub][r] : -INFINITY;
         s[sub][r] = t;
         mx = fmaxf(mx, t);
       }
@@ -300,7 +308,8 @@ __device__ __forceinline__ void rows_write(const WaveState<DH>& w, bf16_t* __res
                                            int h, const AttnExtra& x) {
   const float m_use = (w.m == -INFINITY) ? 0.f : w.m;
   const float l = XTRA ? w.l + sink_term(x, head, m_use) : w.l;
-  const float inv = l > 0.f ? 1.0f / l : 0.f;
+  float inv = l > 0.f ? 1.0f / l : 0.f;
+  if (XTRA) inv *= head_gate(x, token, head);
 #pragma unroll
   for (int mt = 0; mt < DH / 32; ++mt)
 #pragma unroll
@@ -309,7 +318,7 @@ __device__ __forceinline__ void rows_write(const WaveState<DH>& w, bf16_t* __res
       float r[4];
 #pragma unroll
       for (int e = 0; e < 4; ++e) r[e] = w.o[mt][4 * g4 + e] * inv;
-      if (XTRA && x.gate != nullptr) {
+      if (XTRA && x.gate != nullptr && x.gate_dv > 0) {
 #pragma unroll
         for (int e = 0; e < 4; ++e) r[e] *= gate_factor(x, token, head, d + e);
       }
@@ -364,12 +373,18 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(
   const bool all_rows = row0 + 32 <= nrows;
 
   const int* table = block_table + (size_t)b * max_blocks;
-  for (int pg = tile_start / TA_PAGE; pg * TA_PAGE < tile_end; ++pg) {
+  const int win_page = tile_start / TA_PAGE;
+  for (int pg = XTRA && x.keep > 0 ? 0 : win_page; pg * TA_PAGE < tile_end; ++pg) {
     const int key0 = pg * TA_PAGE;
+    if (XTRA && pg < win_page && key0 >= x.keep) {   // nothing between the kept keys and the window is read
+      pg = win_page - 1;
+      continue;
+    }
     const size_t page = (size_t)table[pg];
     const bf16_t* kp = kcache + (page * nkv + kvh) * (size_t)(TA_PAGE * DH);
     const bf16_t* vp = vcache + (page * nkv + kvh) * (size_t)(TA_PAGE * DH);
-    const bool all_visible = all_rows && key0 + TA_PAGE <= tile_min_end && key0 >= tile_max_start;
+    const bool all_visible = all_rows && key0 + TA_PAGE <= tile_min_end &&
+                             (key0 >= tile_max_start || (XTRA && key0 + TA_PAGE <= x.keep));
     wave_page<DH, DH, TA_PAGE, true, false, XTRA>(w, kp, vp, key0, my_start, my_end, kv_len, all_visible, scale_log2, j, h, x);
   }
   if (row_ok) rows_write<DH, XTRA>(w, out + (size_t)(q0 + qi) * out_stride + (size_t)head * DH, (size_t)(q0 + qi), head, h, x);
@@ -448,12 +463,22 @@ __global__ __launch_bounds__(256, 2) void attn_rows_lds_kernel(
   const bool all_rows = row0 + 32 <= nrows;
 
   const int* table = block_table + (size_t)b * max_blocks;
-  const int pg_first = wg_start / TA_PAGE;
-  const int pg_last = (wg_end - 1) / TA_PAGE;
+  // steps of the walk: pages [0, n_keep) with kept first keys that the window has left behind, then the
+  // window's from win_page on; `gap` pages lie between the two
+  const int win_page = wg_start / TA_PAGE;
+  int n_keep = 0;
+  if (XTRA) {
+    n_keep = (x.keep + TA_PAGE - 1) / TA_PAGE;
+    if (n_keep > win_page) n_keep = win_page;
+  }
+  const int gap = win_page - n_keep;
+  const int pg_first = 0;
+  const int pg_last = (wg_end - 1) / TA_PAGE - gap;
+#define WALK_PAGE(i_) ((i_) < n_keep ? (i_) : (i_) + gap)
   u32x4 kreg[PER], vreg[PER];
 #define FETCH_PAGE(pg_)                                                              \
   do {                                                                               \
-    const size_t page_ = (size_t)table[pg_];                                         \
+    const size_t page_ = (size_t)table[WALK_PAGE(pg_)];                              \
     const bf16_t* kp_ = kcache + (page_ * nkv + kvh) * (size_t)(TA_PAGE * DH);       \
     const bf16_t* vp_ = vcache + (page_ * nkv + kvh) * (size_t)(TA_PAGE * DH);       \
     _Pragma("unroll") for (int i = 0; i < PER; ++i) {                                \
@@ -465,7 +490,7 @@ __global__ __launch_bounds__(256, 2) void attn_rows_lds_kernel(
 
 #define STORE_PAGE(buf_, pg_)                                                        \
   do {                                                                               \
-    const int key0_ = (pg_) * TA_PAGE;                                               \
+    const int key0_ = WALK_PAGE(pg_) * TA_PAGE;                                      \
     _Pragma("unroll") for (int i = 0; i < PER; ++i) {                                \
       const int piece = threadIdx.x + i * 256;                                       \
       const int krow = piece / (DH / 8), kcol = (piece % (DH / 8)) * 8;              \
@@ -494,20 +519,22 @@ __global__ __launch_bounds__(256, 2) void attn_rows_lds_kernel(
   STORE_PAGE(pg_first & 1, pg_first);
   if (pg_first < pg_last) FETCH_PAGE(pg_first + 1);
   for (int pg = pg_first; pg <= pg_last; ++pg) {
-    const int key0 = pg * TA_PAGE;
+    const int key0 = WALK_PAGE(pg) * TA_PAGE;
     __syncthreads();
     if (pg < pg_last) {
       STORE_PAGE((pg + 1) & 1, pg + 1);
       if (pg + 1 < pg_last) FETCH_PAGE(pg + 2);
     }
-    if (key0 < tile_end && key0 + TA_PAGE > tile_start) {
-      const bool all_visible = all_rows && key0 + TA_PAGE <= tile_min_end && key0 >= tile_max_start;
+    if (key0 < tile_end && (key0 + TA_PAGE > tile_start || (XTRA && key0 < x.keep))) {
+      const bool all_visible = all_rows && key0 + TA_PAGE <= tile_min_end &&
+                               (key0 >= tile_max_start || (XTRA && key0 + TA_PAGE <= x.keep));
       wave_page<DH, KSTR, VSTR, false, false, XTRA>(w, Ks[pg & 1], Vs[pg & 1], key0, my_start, my_end, kv_len, all_visible,
                                        scale_log2, j, h, x);
     }
   }
 #undef STORE_PAGE
 #undef FETCH_PAGE
+#undef WALK_PAGE
   if (row_ok) rows_write<DH, XTRA>(w, out + (size_t)(q0 + qi) * out_stride + (size_t)head * DH, (size_t)(q0 + qi), head, h, x);
   }
 }
@@ -1088,16 +1115,20 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_keys_kernel(
   int pg_lo = unit_first;
   int pg_hi = unit_first + unit_count;
   if (pg_hi > n_pages) pg_hi = n_pages;
-  if (vis_start / TA_PAGE > pg_lo) pg_lo = vis_start / TA_PAGE;
+  const int win_page = vis_start / TA_PAGE;
+  const bool kept = XTRA && pg_lo < win_page && pg_lo * TA_PAGE < x.keep;     // the unit begins among the kept first keys
+  if (win_page > pg_lo && !kept) pg_lo = win_page;
   // keep every wave on its own residue so that a page is always taken by the same wave
   const int first = pg_lo + ((wave - pg_lo % WAVES) + WAVES) % WAVES;
   const int* table = block_table + (size_t)b * max_blocks;
   for (int pg = first; pg < pg_hi; pg += WAVES) {
     const int key0 = pg * TA_PAGE;
+    if (XTRA && pg < win_page && key0 >= x.keep) continue;    // between the kept keys and the window
     const size_t page = (size_t)table[pg];
     const bf16_t* kp = kcache + (page * nkv + kvh) * (size_t)(TA_PAGE * DH);
     const bf16_t* vp = vcache + (page * nkv + kvh) * (size_t)(TA_PAGE * DH);
-    const bool all_visible = key0 + TA_PAGE <= kv_len && key0 >= vis_start;   // rows beyond nrows are never written
+    const bool all_visible = key0 + TA_PAGE <= kv_len &&       // rows beyond nrows are never written
+                             (key0 >= vis_start || (XTRA && key0 + TA_PAGE <= x.keep));
     // (with the options the value operands are fetched where they are used: three pieces of weights
     // and the operands asked for ahead do not fit the registers together)
     wave_page<DH, DH, TA_PAGE, true, !XTRA, XTRA>(w, kp, vp, key0, my_start, my_end, kv_len, all_visible, scale_log2, j, h, x);
@@ -1135,7 +1166,7 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_keys_kernel(
     if (splits == 1) {
       if (XTRA) ll += sink_term(x, hd, m_use);
       const float inv = ll > 0.f ? 1.0f / ll : 0.f;
-      const float gf = XTRA ? gate_factor(x, (size_t)b, hd, d) : 1.f;
+      const float gf = XTRA ? gate_factor(x, (size_t)b, hd, d) * head_gate(x, (size_t)b, hd) : 1.f;
       out[(size_t)b * out_stride + (size_t)hd * DH + d] = from_f32<bf16_t>(XTRA ? acc * inv * gf : acc * inv);
     } else {
       float* pr = partial + ((size_t)blockIdx.y * nh + hd) * (DH + 2);
@@ -1847,7 +1878,7 @@ __global__ void attn_merge_kernel(const float* __restrict__ partial, bf16_t* __r
   }
   if (XTRA) ll += sink_term(x, hd, (mm == -INFINITY) ? 0.f : mm);
   const float inv = ll > 0.f ? 1.0f / ll : 0.f;
-  const float gf = XTRA ? gate_factor(x, (size_t)b, hd, d) : 1.f;
+  const float gf = XTRA ? gate_factor(x, (size_t)b, hd, d) * head_gate(x, (size_t)b, hd) : 1.f;
   out[(size_t)b * out_stride + (size_t)hd * DH + d] = from_f32<bf16_t>(XTRA ? acc * inv * gf : acc * inv);
 }
 
@@ -1882,11 +1913,13 @@ static const float LOG2E = 1.4426950408889634f;
 
 // Prompts (any mix of lengths, also single tokens). Same arguments as ta_attention_generic.
 static int make_extra(const char* what, AttnExtra* x, int nh, int dh, float scale, float softcap, int exact,
-                      int sink_mode, const float* sink, const void* gate, int gate_stride, int gate_dv) {
+                      int sink_mode, const float* sink, const void* gate, int gate_stride, int gate_dv, int window,
+                      int keep) {
   TA_REQUIRE(softcap >= 0.f && scale > 0.f, "%s: cap %f / scale %f", what, softcap, scale);
   TA_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 2 || sink != nullptr), "%s: sink mode %d", what, sink_mode);
-  TA_REQUIRE(gate == nullptr || (gate_dv >= 1 && gate_dv <= dh && gate_stride >= nh * gate_dv),
+  TA_REQUIRE(gate == nullptr || (gate_dv >= 0 && gate_dv <= dh && gate_stride >= nh * (gate_dv > 0 ? gate_dv : 1)),
              "%s: gate rows of %d for %d heads of %d", what, gate_stride, nh, gate_dv);
+  TA_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "%s: %d kept keys beside a window of %d", what, keep, window);
   x->cap_k = softcap > 0.f ? 2.0f * 1.4426950408889634f * scale / softcap : 0.f;
   x->cap_r = softcap > 0.f ? softcap / scale : 0.f;
   x->exact = exact ? 1 : 0;
@@ -1895,6 +1928,7 @@ static int make_extra(const char* what, AttnExtra* x, int nh, int dh, float scal
   x->gate = (const bf16_t*)gate;
   x->gate_stride = gate_stride;
   x->gate_dv = gate_dv;
+  x->keep = keep;
   return 0;
 }
 
@@ -1979,16 +2013,18 @@ extern "C" int ta_attention_rows_bf16(hipStream_t stream, const void* q, int q_s
 
 // The same with the options of a capped, sunk and gated softmax (see AttnExtra): softcap > 0 caps the
 // scaled scores; exact: 32-bit softmax weights in the second product; sink_mode / sink; gate rows
-// [tokens][gate_stride] with gate_dv columns per head. use_lds 0 or 1.
+// [tokens][gate_stride] with gate_dv columns per head (0: one number per head); keep: first keys that a
+// window shows as well. use_lds 0 or 1.
 extern "C" int ta_attention_rows_sink_bf16(hipStream_t stream, const void* q, int q_stride, void* out,
                                            int out_stride, const void* kcache, const void* vcache,
                                            const int* block_table, int max_blocks, const int* cu_q,
                                            const int* pos0, int batch, int max_qlen, int nh, int nkv,
                                            int dh, float scale, int window, int use_lds, float softcap, int exact,
                                            int sink_mode, const float* sink, const void* gate, int gate_stride,
-                                           int gate_dv) {
+                                           int gate_dv, int keep) {
   AttnExtra x;
-  if (make_extra("ta_attention_rows_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv))
+  if (make_extra("ta_attention_rows_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv, window,
+                 keep))
     return 1;
   TA_REQUIRE(use_lds == 0 || use_lds == 1, "ta_attention_rows_sink_bf16: kernels 0 and 1 take the options, not %d", use_lds);
   return attention_rows_launch(stream, q, q_stride, out, out_stride, kcache, vcache, block_table, max_blocks, cu_q,
@@ -2093,9 +2129,11 @@ extern "C" int ta_attention_keys_sink_bf16(hipStream_t stream, const void* q, in
                                            const int* pos0, int batch, int nh, int nkv, int dh, float scale,
                                            int window, const int* units, const int* seq_units, int n_units,
                                            int waves, float* scratch, float softcap, int exact, int sink_mode,
-                                           const float* sink, const void* gate, int gate_stride, int gate_dv) {
+                                           const float* sink, const void* gate, int gate_stride, int gate_dv,
+                                           int keep) {
   AttnExtra x;
-  if (make_extra("ta_attention_keys_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv))
+  if (make_extra("ta_attention_keys_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv, window,
+                 keep))
     return 1;
   return attention_keys_launch(stream, q, q_stride, nullptr, nullptr, 0, nullptr, out, out_stride, kcache, vcache,
                                block_table, max_blocks, pos0, batch, nh, nkv, dh, scale, window, units, seq_units,

@@ -5,6 +5,8 @@
 //   q <- rms_norm(q over all heads at once) * wq, k likewise with wk      (float32)
 //   the first `rot` coordinates of every head of q and k are rotated in pairs (i, i + rot/2)
 //   v <- (1 - lambda) v + lambda v_first      (where the layer mixes in the values of an earlier one)
+// The norm may also be one of every head on its own, with or without a weight, and the values may be
+// columns that another part of the row holds too (voff; a layer whose values are its keys before their norm).
 //   q is written back in place; k and v go to the paged cache (keys [pages][kv heads][PAGE][dk],
 //   values [pages][kv heads][dvs][PAGE], dvs >= dv, rows dv.. of a token zero).
 //
@@ -17,7 +19,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
     float eps, int normed, const float* __restrict__ angles, int rot,
     const float* __restrict__ lambda, const T* __restrict__ v_first, T* __restrict__ v_keep,
     const int* __restrict__ dest, T* __restrict__ kcache, T* __restrict__ vcache,
-    int nh, int nkv, int dk, int dv, int dvs, int k_inplace) {
+    int nh, int nkv, int dk, int dv, int dvs, int k_inplace, int voff) {
   extern __shared__ float buf[];          // [nh*dk + nkv*dk], then a factor per head [nh + nkv]
   __shared__ float red[8];
   const int t = blockIdx.x;
@@ -81,7 +83,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
     const int shift = turns ? (c < half ? half : -half) : 0;
     const float cs = ang ? ang[2 * pi] : 1.f, sn = ang ? ang[2 * pi + 1] : 0.f;
     float wv = 1.f, wo = 1.f;
-    if (normed) {                     // the same for every thread
+    if (normed && wq) {               // the same for every thread
       const int jw = normed == 2 ? c : j;
       wv = w[jw];
       wo = w[jw + shift];
@@ -105,7 +107,7 @@ __global__ __launch_bounds__(256) void qk_prepare_kernel(
   }
   const float lam = lambda ? lambda[0] : 0.f;
   for (int i = threadIdx.x; i < nv; i += 256) {
-    float v = to_f32(row[nq + nk + i]);
+    float v = to_f32(row[voff + i]);
     if (v_keep) v_keep[(size_t)t * nv + i] = from_f32<T>(v);
     if (v_first) v = (1.0f - lam) * v + lam * to_f32(v_first[(size_t)t * nv + i]);
     if (dest) {
@@ -163,7 +165,7 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
     float eps, int normed, const float* __restrict__ angles, int rot,
     const float* __restrict__ lambda, const T* __restrict__ v_first, T* __restrict__ v_keep,
     const int* __restrict__ dest, T* __restrict__ kcache, T* __restrict__ vcache,
-    int nh, int nkv, int dk, int dv, int dvs, int k_inplace) {
+    int nh, int nkv, int dk, int dv, int dvs, int k_inplace, int voff) {
   extern __shared__ float buf[];          // [nh*dk + nkv*dk], then a factor per head [nh + nkv]
   __shared__ float red[8];
   const int t = blockIdx.x;
@@ -221,7 +223,7 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
     float wv[8], wo[8], cs[8], sn[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) wv[e] = wo[e] = cs[e] = 1.f, sn[e] = 0.f;
-    if (normed) {
+    if (normed && wq) {
       const int jw = normed == 2 ? c : j;
       Eight<float>::load(w + jw, wv);
       Eight<float>::load(w + jw + shift, wo);
@@ -248,7 +250,7 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
   }
   const float lam = lambda ? lambda[0] : 0.f;
   for (int i = threadIdx.x; i < nv; i += 256) {
-    float v = to_f32(row[nq + nk + i]);
+    float v = to_f32(row[voff + i]);
     if (v_keep) v_keep[(size_t)t * nv + i] = from_f32<T>(v);
     if (v_first) v = (1.0f - lam) * v + lam * to_f32(v_first[(size_t)t * nv + i]);
     if (dest) {
@@ -266,7 +268,9 @@ __global__ __launch_bounds__(256) void qk_prepare_vec_kernel(
 }
 
 // qkv: [nt, stride] rows of [nh*dk | nkv*dk | nkv*dv]. normed 1: wq [nh*dk], wk [nkv*dk], one norm over
-// all heads of q and one over all of k; normed 2: wq, wk [dk], every head normed on its own; 0: no norm.
+// all heads of q and one over all of k; normed 2: wq, wk [dk] (or both null: no weights), every head
+// normed on its own; 0: no norm. voff: the column where a row's values start ((nh + nkv) * dk in a row of
+// three parts; nh * dk where the values are the keys as projected, which takes dest or no k_inplace).
 // k_inplace (no dest): the keys are written back into their rows as the queries are.
 // angles: [nt, rot/2, 2] (cos, sin) or null. lambda: one float on the device, v_first [nt, nkv*dv]
 // (both or neither). v_keep [nt, nkv*dv] or null: receives the unmixed values. dest [nt] or null:
@@ -275,14 +279,16 @@ extern "C" int ta_qk_prepare(hipStream_t stream, int dtype, void* qkv, int strid
                              const float* wk, float eps, int normed, const float* angles, int rot,
                              const float* lambda, const void* v_first, void* v_keep, const int* dest,
                              void* kcache, void* vcache, int nt, int nh, int nkv, int dk, int dv,
-                             int dvs, int k_inplace) {
+                             int dvs, int k_inplace, int voff) {
   TA_REQUIRE(nt >= 0 && nh > 0 && nkv > 0 && dk > 0 && dv > 0, "ta_qk_prepare: bad sizes");
   TA_REQUIRE(normed >= 0 && normed <= 2, "ta_qk_prepare: unknown norm mode %d", normed);
   TA_REQUIRE(!(k_inplace && dest), "ta_qk_prepare: keys go back in place or to the cache, not both");
-  TA_REQUIRE(stride >= (nh + nkv) * dk + nkv * dv, "ta_qk_prepare: row stride %d too small", stride);
+  TA_REQUIRE(stride >= (nh + nkv) * dk && voff >= nh * dk && stride >= voff + nkv * dv,
+             "ta_qk_prepare: row stride %d too small", stride);
+  TA_REQUIRE(voff >= (nh + nkv) * dk || !k_inplace, "ta_qk_prepare: keys written in place would be read as values");
   TA_REQUIRE(rot >= 0 && rot <= dk && rot % 2 == 0, "ta_qk_prepare: %d rotated coordinates of %d", rot, dk);
   TA_REQUIRE((lambda == nullptr) == (v_first == nullptr), "ta_qk_prepare: lambda and v_first go together");
-  TA_REQUIRE(!normed || (wq && wk), "ta_qk_prepare: norm weights missing");
+  TA_REQUIRE(!normed || (wq && wk) || (normed == 2 && !wq && !wk), "ta_qk_prepare: norm weights missing");
   TA_REQUIRE(!dest || (kcache && vcache), "ta_qk_prepare: cache layer missing");
   TA_REQUIRE(dvs >= dv, "ta_qk_prepare: cache rows of %d cannot hold values of %d", dvs, dv);
   const size_t lds = ((size_t)(nh + nkv) * dk + nh + nkv) * sizeof(float);
@@ -297,21 +303,21 @@ extern "C" int ta_qk_prepare(hipStream_t stream, int dtype, void* qkv, int strid
     if (dtype == TA_F32)
       qk_prepare_vec_kernel<float><<<nt, 256, lds, stream>>>(
           (float*)qkv, stride, wq, wk, eps, normed, angles, rot, lambda, (const float*)v_first, (float*)v_keep,
-          dest, (float*)kcache, (float*)vcache, nh, nkv, dk, dv, dvs, k_inplace);
+          dest, (float*)kcache, (float*)vcache, nh, nkv, dk, dv, dvs, k_inplace, voff);
     else
       qk_prepare_vec_kernel<bf16_t><<<nt, 256, lds, stream>>>(
           (bf16_t*)qkv, stride, wq, wk, eps, normed, angles, rot, lambda, (const bf16_t*)v_first, (bf16_t*)v_keep,
-          dest, (bf16_t*)kcache, (bf16_t*)vcache, nh, nkv, dk, dv, dvs, k_inplace);
+          dest, (bf16_t*)kcache, (bf16_t*)vcache, nh, nkv, dk, dv, dvs, k_inplace, voff);
     return ta_check_launch("ta_qk_prepare");
   }
   if (dtype == TA_F32)
     qk_prepare_kernel<float><<<nt, 256, lds, stream>>>(
         (float*)qkv, stride, wq, wk, eps, normed, angles, rot, lambda, (const float*)v_first, (float*)v_keep,
-        dest, (float*)kcache, (float*)vcache, nh, nkv, dk, dv, dvs, k_inplace);
+        dest, (float*)kcache, (float*)vcache, nh, nkv, dk, dv, dvs, k_inplace, voff);
   else if (dtype == TA_BF16)
     qk_prepare_kernel<bf16_t><<<nt, 256, lds, stream>>>(
         (bf16_t*)qkv, stride, wq, wk, eps, normed, angles, rot, lambda, (const bf16_t*)v_first, (bf16_t*)v_keep,
-        dest, (bf16_t*)kcache, (bf16_t*)vcache, nh, nkv, dk, dv, dvs, k_inplace);
+        dest, (bf16_t*)kcache, (bf16_t*)vcache, nh, nkv, dk, dv, dvs, k_inplace, voff);
   else
     return ta_fail("ta_qk_prepare: unknown dtype %d", dtype);
   return ta_check_launch("ta_qk_prepare");

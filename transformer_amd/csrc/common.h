@@ -45,6 +45,20 @@ template <> __device__ __forceinline__ bf16_t from_f32<bf16_t>(float f) {
   return r;
 }
 
+// How a product that owns a gate column and an up column joins them: silu(gate) * up, or, with a
+// limit, g * sigmoid(slope * g) * (u + shift) with g = min(gate, limit), u = clamp(up, -limit, limit).
+struct TaGlu {
+  float limit, slope, shift;      // limit 0: silu
+};
+__device__ __forceinline__ float ta_glu(const TaGlu& p, float g, float u) {
+  if (p.limit > 0.f) {
+    g = fminf(g, p.limit);
+    u = fminf(fmaxf(u, -p.limit), p.limit);
+    return g / (1.0f + expf(-p.slope * g)) * (u + p.shift);
+  }
+  return g / (1.0f + expf(-g)) * u;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = TA_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, TA_WAVE);

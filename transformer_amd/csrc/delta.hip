@@ -1,0 +1,532 @@
+// The gated delta rule: per head a matrix state S [dk][dv] that forgets per key channel and is
+// corrected, not just added to, by every token:
+//
+//     S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t
+//     g_t = exp(-exp(A_h) softplus(z_t + dt_bias)) per key channel,  beta_t = sigmoid(b_t),
+//     q_t, k_t of unit length (q_t times a constant besides); the heads of a group share q and k
+//
+//   delta_prepare   : unit q and k, their product k.q, decays and step sizes of all tokens at once
+//   delta_recurrent : walks a sequence's tokens in order with S in registers (prompts)
+//   delta_step      : a step of single tokens in one kernel: low-rank decay and gate, unit vectors,
+//                     the state's update, the readout's norm and gate
+//
+// The readout needs the updated state, but S_new^T q = (g S)^T q + u (k.q): both sums over key
+// channels are taken of the decayed state side by side, and the update is no part of the chain
+// that the readout waits for.
+//
+// State, decays, step sizes, unit vectors and sums are float32; tokens are walked in the same order
+// however a sequence was cut into steps.
+#include "common.h"
+
+__device__ __forceinline__ float dr_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float dr_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+
+#define DR_UNIT_EPS 1e-6f       // under the root of a vector's length
+
+// ------------------------------------------------------------------ what does not depend on the state
+// One workgroup per token; a wave takes units in turn: the G pairs (q, k), then the H decays.
+template <typename T>
+__global__ __launch_bounds__(256) void delta_prepare_kernel(
+    const T* __restrict__ qkv, int stride, const float* __restrict__ z, const float* __restrict__ dt_bias,
+    const float* __restrict__ a_log, const T* __restrict__ braw, int bstride, int G, int H, int dk, float qscale,
+    float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ decay, float* __restrict__ beta,
+    float* __restrict__ kq) {
+  const size_t t = blockIdx.x;
+  const int wave = threadIdx.x / TA_WAVE, lane = threadIdx.x % TA_WAVE;
+  for (int u = wave; u < G + H; u += 4) {
+    if (u < G) {
+      const T* q = qkv + t * stride + u * dk;
+      const T* k = q + G * dk;
+      float sq = 0.f, sk = 0.f, sx = 0.f;
+      for (int c = lane; c < dk; c += TA_WAVE) {
+        const float a = to_f32(q[c]), b = to_f32(k[c]);
+        sq = fmaf(a, a, sq);
+        sk = fmaf(b, b, sk);
+        sx = fmaf(a, b, sx);
+      }
+      sq = wave_sum(sq);
+      sk = wave_sum(sk);
+      sx = wave_sum(sx);
+      const float fq = qscale * rsqrtf(sq + DR_UNIT_EPS), fk = rsqrtf(sk + DR_UNIT_EPS);
+      for (int c = lane; c < dk; c += TA_WAVE) {
+        qn[(t * G + u) * dk + c] = to_f32(q[c]) * fq;
+        kn[(t * G + u) * dk + c] = to_f32(k[c]) * fk;
+      }
+      if (lane == 0) kq[t * G + u] = sx * fq * fk;
+    } else {
+      const int h = u - G;
+      const float rate = expf(a_log[h]);
+      for (int c = lane; c < dk; c += TA_WAVE) {
+        const size_t at = (t * H + h) * dk + c;
+        decay[at] = expf(-rate * dr_softplus(z[at] + dt_bias[h * dk + c]));
+      }
+      if (lane == 0) beta[t * H + h] = dr_sigmoid(to_f32(braw[t * bstride + h]));
+    }
+  }
+}
+
+// qkv: [nt, stride] rows of [q: G*dk | k: G*dk | ...] behind convolution and activation; z [nt, H*dk]
+// float32 decay inputs without their bias; braw: [nt] rows, bstride apart, of H step-size inputs.
+// qn, kn [nt, G, dk], decay [nt, H, dk], beta [nt, H], kq [nt, G]: float32.
+extern "C" int ta_delta_prepare(hipStream_t stream, int dtype, const void* qkv, int stride, const float* z,
+                                const float* dt_bias, const float* a_log, const void* braw, int bstride, int nt,
+                                int G, int H, int dk, float qscale, float* qn, float* kn, float* decay, float* beta,
+                                float* kq) {
+  TA_REQUIRE(nt >= 0 && G >= 1 && H >= 1 && H % G == 0 && dk >= 1, "ta_delta_prepare: bad sizes nt=%d heads=%d/%d width %d", nt, H, G, dk);
+  TA_REQUIRE(stride >= 2 * G * dk && bstride >= H, "ta_delta_prepare: rows of %d / %d are too short", stride, bstride);
+  if (nt == 0) return 0;
+  if (dtype == TA_F32)
+    delta_prepare_kernel<float><<<nt, 256, 0, stream>>>((const float*)qkv, stride, z, dt_bias, a_log, (const float*)braw,
+                                                        bstride, G, H, dk, qscale, qn, kn, decay, beta, kq);
+  else if (dtype == TA_BF16)
+    delta_prepare_kernel<bf16_t><<<nt, 256, 0, stream>>>((const bf16_t*)qkv, stride, z, dt_bias, a_log, (const bf16_t*)braw,
+                                                         bstride, G, H, dk, qscale, qn, kn, decay, beta, kq);
+  else return ta_fail("ta_delta_prepare: unknown dtype %d", dtype);
+  return ta_check_launch("ta_delta_prepare");
+}
+
+// ------------------------------------------------------------------ prompts
+// Sixteen lanes share a value column, each with R of its key channels (in runs of four: run i of lane l
+// holds channels 64 i + 4 l ..+3, so that a wave's operand reads from LDS meet every bank once); a wave
+// owns four columns. A token costs a wave some 5 R + 20 vector instructions and one exchange among 16
+// lanes for both sums. Operands of the next chunk of tokens are on their way to registers while this
+// chunk is worked on out of one of two LDS buffers, and the next token's leave LDS a token ahead.
+template <int CTRL>
+__device__ __forceinline__ float dr_dpp(float x) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
+}
+// the sum over 16 neighbouring lanes, the same bits in each: pairs, quads, halves of a row, rows
+__device__ __forceinline__ float dr_sum16(float x) {
+  x += dr_dpp<0xB1>(x);      // lanes 1 apart
+  x += dr_dpp<0x4E>(x);      // 2 apart
+  x += dr_dpp<0x141>(x);     // mirrored in eights
+  x += dr_dpp<0x140>(x);     // mirrored in sixteens
+  return x;
+}
+
+template <typename T, int R, int WAVES, bool VEC>
+__global__ __launch_bounds__(WAVES * 64) void delta_recurrent_kernel(
+    const float* __restrict__ qn, const float* __restrict__ kn, const float* __restrict__ decay,
+    const T* __restrict__ v, int v_stride, const float* __restrict__ beta, const float* __restrict__ kq,
+    float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ slots, int H, int G, int dk,
+    int dv, float* __restrict__ o_out) {
+  constexpr int TC = R <= 8 ? 16 : 8;              // tokens of a chunk (at most 16: see `kept`)
+  constexpr int DKP = 16 * R, COLS = 4 * WAVES, NT = 64 * WAVES;
+  constexpr int NF = (TC * DKP / 4 + NT - 1) / NT; // runs of four that a thread brings in of each operand
+  __shared__ __attribute__((aligned(16))) float sq[2][TC][DKP], sk[2][TC][DKP], sg[2][TC][DKP];
+  __shared__ float sv[2][TC][COLS], sb[2][TC], sx[2][TC];
+  const int h = blockIdx.x, col0 = blockIdx.y * COLS, b = blockIdx.z;
+  const int start = cu_q[b], end = cu_q[b + 1];
+  if (start >= end) return;
+  const int g = h / (H / G);
+  const int tid = threadIdx.x, lane = tid % 16, cl = tid / 16;
+  const int col = col0 + cl;
+  float* st = state + ((size_t)slots[b] * H + h) * dk * (size_t)dv;
+  float S[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = 64 * (i / 4) + 4 * lane + i % 4;
+    S[i] = (row < dk && col < dv) ? st[(size_t)row * dv + col] : 0.f;
+  }
+  struct Chunk {
+    float4 q[NF], k[NF], g[NF];
+    float v, b, x;
+  };
+  auto run4 = [&](const float* p, int c, float none) {      // four channels from c on; past dk: `none`
+    if (VEC) return c < dk ? *reinterpret_cast<const float4*>(p + c) : float4{none, none, none, none};
+    return float4{c < dk ? p[c] : none, c + 1 < dk ? p[c + 1] : none, c + 2 < dk ? p[c + 2] : none,
+                  c + 3 < dk ? p[c + 3] : none};
+  };
+  // a token past the sequence's end reads its last token's operands, which are then not used
+  auto fetch = [&](Chunk& f, int t0) {
+#pragma unroll
+    for (int e = 0; e < NF; ++e) {
+      const int idx = tid + NT * e;
+      const int tt = idx / (DKP / 4), c = (idx % (DKP / 4)) * 4;
+      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
+      f.q[e] = run4(qn + (t * G + g) * dk, c, 0.f);
+      f.k[e] = run4(kn + (t * G + g) * dk, c, 0.f);
+      f.g[e] = run4(decay + (t * H + h) * dk, c, 1.f);
+    }
+    {
+      const int tt = tid / COLS, c = col0 + tid % COLS;     // NT >= TC * COLS
+      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
+      f.v = (tt < TC && c < dv) ? to_f32(v[t * v_stride + (size_t)h * dv + c]) : 0.f;
+    }
+    {
+      const size_t t = t0 + tid % TC < end ? t0 + tid % TC : end - 1;
+      f.b = beta[t * H + h];
+      f.x = kq[t * G + g];
+    }
+  };
+  auto stash = [&](const Chunk& f, int buf) {
+#pragma unroll
+    for (int e = 0; e < NF; ++e) {
+      const int idx = tid + NT * e;
+      if (TC * DKP / 4 % NT == 0 || idx < TC * DKP / 4) {
+        reinterpret_cast<float4*>(&sq[buf][0][0])[idx] = f.q[e];
+        reinterpret_cast<float4*>(&sk[buf][0][0])[idx] = f.k[e];
+        reinterpret_cast<float4*>(&sg[buf][0][0])[idx] = f.g[e];
+      }
+    }
+    if (tid < TC * COLS) (&sv[buf][0][0])[tid] = f.v;
+    if (tid < TC) {
+      sb[buf][tid] = f.b;
+      sx[buf][tid] = f.x;
+    }
+  };
+  struct Token {
+    float4 q[R / 4], k[R / 4], g[R / 4];
+    float v, b, x;
+  };
+  auto take = [&](Token& o, int buf, int tt) {
+    if (tt > TC - 1) tt = TC - 1;                           // past the chunk: not used
+#pragma unroll
+    for (int i = 0; i < R / 4; ++i) {
+      o.q[i] = *reinterpret_cast<const float4*>(&sq[buf][tt][64 * i + 4 * lane]);
+      o.k[i] = *reinterpret_cast<const float4*>(&sk[buf][tt][64 * i + 4 * lane]);
+      o.g[i] = *reinterpret_cast<const float4*>(&sg[buf][tt][64 * i + 4 * lane]);
+    }
+    o.v = sv[buf][tt][cl];
+    o.b = sb[buf][tt];
+    o.x = sx[buf][tt];
+  };
+  float kept = 0.f;                     // lane l keeps the readout of the chunk's token l
+  auto token = [&](const Token& o, int tt) {
+    float w[4] = {0.f, 0.f, 0.f, 0.f}, r[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < R / 4; ++i) {
+      const float gs[4] = {o.g[i].x, o.g[i].y, o.g[i].z, o.g[i].w};
+      const float ks[4] = {o.k[i].x, o.k[i].y, o.k[i].z, o.k[i].w};
+      const float qs[4] = {o.q[i].x, o.q[i].y, o.q[i].z, o.q[i].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[4 * i + e] *= gs[e];
+        w[e] = fmaf(S[4 * i + e], ks[e], w[e]);
+        r[e] = fmaf(S[4 * i + e], qs[e], r[e]);
+      }
+    }
+    const float ws = dr_sum16((w[0] + w[1]) + (w[2] + w[3]));
+    const float rs = dr_sum16((r[0] + r[1]) + (r[2] + r[3]));
+    const float u = o.b * (o.v - ws);
+#pragma unroll
+    for (int i = 0; i < R / 4; ++i) {
+      S[4 * i + 0] = fmaf(o.k[i].x, u, S[4 * i + 0]);
+      S[4 * i + 1] = fmaf(o.k[i].y, u, S[4 * i + 1]);
+      S[4 * i + 2] = fmaf(o.k[i].z, u, S[4 * i + 2]);
+      S[4 * i + 3] = fmaf(o.k[i].w, u, S[4 * i + 3]);
+    }
+    const float out = fmaf(u, o.x, rs);
+    kept = lane == tt ? out : kept;
+  };
+  {
+    Chunk f;
+    fetch(f, start);
+    stash(f, 0);
+  }
+  __syncthreads();
+  int buf = 0;
+  for (int t0 = start; t0 < end; t0 += TC, buf ^= 1) {
+    const int n = end - t0 < TC ? end - t0 : TC;
+    const bool more = t0 + TC < end;
+    Chunk f;
+    if (more) fetch(f, t0 + TC);
+    Token a, c;
+    take(a, buf, 0);
+    for (int tt = 0; tt < n; tt += 2) {
+      take(c, buf, tt + 1);
+      token(a, tt);
+      take(a, buf, tt + 2);
+      if (tt + 1 < n) token(c, tt + 1);
+    }
+    if (lane < n && col < dv) o_out[((size_t)(t0 + lane) * H + h) * dv + col] = kept;
+    // the other buffer's readers are behind the barrier at the end of the turn before
+    if (more) stash(f, buf ^ 1);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = 64 * (i / 4) + 4 * lane + i % 4;
+    if (row < dk && col < dv) st[(size_t)row * dv + col] = S[i];
+  }
+}
+
+// qn, kn, decay, beta, kq: what ta_delta_prepare left. v: [nt] rows, v_stride apart, of H*dv values in
+// the engine's type. state [slots, H, dk, dv] float32; o_out [nt, H, dv] float32. waves per workgroup
+// (2 or 4; 0: chosen by the number of heads and sequences): four value columns each.
+extern "C" int ta_delta_recurrent(hipStream_t stream, int dtype, const float* qn, const float* kn, const float* decay,
+                                  const void* v, int v_stride, const float* beta, const float* kq, float* state,
+                                  const int* cu_q, const int* slots, int batch, int nt, int H, int G, int dk, int dv,
+                                  int waves, float* o_out) {
+  TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch, "ta_delta_recurrent: bad batch %d / tokens %d", batch, nt);
+  TA_REQUIRE(G >= 1 && H >= 1 && H % G == 0 && dk >= 1 && dk <= 256 && dv >= 1 && v_stride >= H * dv,
+             "ta_delta_recurrent: %d heads in %d groups of %d / %d", H, G, dk, dv);
+  TA_REQUIRE(waves == 0 || waves == 2 || waves == 4, "ta_delta_recurrent: %d waves", waves);
+  TA_REQUIRE(dtype == TA_F32 || dtype == TA_BF16, "ta_delta_recurrent: unknown dtype %d", dtype);
+  if (waves == 0) waves = (long long)batch * H * ((dv + 15) / 16) >= 512 ? 4 : 2;
+  const int cols = 4 * waves;
+  TA_REQUIRE((dv + cols - 1) / cols <= 65535, "ta_delta_recurrent: values of %d", dv);
+  dim3 g(H, (dv + cols - 1) / cols, batch);
+  const bool vec = dk % 4 == 0 && (((uintptr_t)qn | (uintptr_t)kn | (uintptr_t)decay) & 15) == 0;
+#define DR_RUN(T, RR, W, VE)                                                                                  \
+  delta_recurrent_kernel<T, RR, W, VE><<<g, W * 64, 0, stream>>>(qn, kn, decay, (const T*)v, v_stride, beta, kq, \
+                                                                 state, cu_q, slots, H, G, dk, dv, o_out)
+#define DR_BY_VEC(T, RR, W) \
+  if (vec) DR_RUN(T, RR, W, true); else DR_RUN(T, RR, W, false)
+#define DR_BY_WIDTH(T, W)                                 \
+  if (dk <= 64) { DR_BY_VEC(T, 4, W); }                   \
+  else if (dk <= 128) { DR_BY_VEC(T, 8, W); }             \
+  else if (dk <= 192) { DR_BY_VEC(T, 12, W); }            \
+  else { DR_BY_VEC(T, 16, W); }
+  if (dtype == TA_F32) {
+    if (waves == 4) { DR_BY_WIDTH(float, 4) } else { DR_BY_WIDTH(float, 2) }
+  } else {
+    if (waves == 4) { DR_BY_WIDTH(bf16_t, 4) } else { DR_BY_WIDTH(bf16_t, 2) }
+  }
+#undef DR_BY_WIDTH
+#undef DR_BY_VEC
+#undef DR_RUN
+  return ta_check_launch("ta_delta_recurrent");
+}
+
+// ------------------------------------------------------------------ steps of single tokens
+// One workgroup of DS_NT threads per (head, sequence). A thread keeps VW neighbouring value columns of
+// every RG-th key channel in registers; the state is asked for first, and everything else (unit vectors,
+// low-rank products) is formed while it is on its way.
+#define DS_NT 512
+
+template <typename T>
+__device__ __forceinline__ void ds_load8(const T* p, float* o);
+template <>
+__device__ __forceinline__ void ds_load8<float>(const float* p, float* o) {
+  const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+  o[0] = a.x; o[1] = a.y; o[2] = a.z; o[3] = a.w; o[4] = b.x; o[5] = b.y; o[6] = b.z; o[7] = b.w;
+}
+template <>
+__device__ __forceinline__ void ds_load8<bf16_t>(const bf16_t* p, float* o) {
+  const uint4 r = *reinterpret_cast<const uint4*>(p);
+  const uint32_t w[4] = {r.x, r.y, r.z, r.w};
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    o[2 * i] = __uint_as_float(w[i] << 16);
+    o[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
+  }
+}
+
+// The product of a weight row with a low-rank input in LDS, four lanes a row (all four get the sum).
+template <typename TW>
+__device__ __forceinline__ float ds_row_dot(const TW* __restrict__ w, const float* low, int rank, int part, bool vec) {
+  float s = 0.f;
+  if (vec) {
+    for (int r = 8 * part; r < rank; r += 32) {
+      float a[8];
+      ds_load8<TW>(w + r, a);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) s = fmaf(a[e], low[r + e], s);
+    }
+  } else {
+    for (int r = part; r < rank; r += 4) s = fmaf(to_f32(w[r]), low[r], s);
+  }
+  s += __shfl_xor(s, 1, TA_WAVE);
+  s += __shfl_xor(s, 2, TA_WAVE);
+  return s;
+}
+
+template <typename T, typename TW, int VW, int ROWS>
+__global__ __launch_bounds__(DS_NT) void delta_step_kernel(
+    const T* __restrict__ qkv, int stride, const T* __restrict__ proj, int pstride, int aoff, int ra, int goff, int rg,
+    int boff, const TW* __restrict__ a2, const TW* __restrict__ g2, const float* __restrict__ dt_bias,
+    const float* __restrict__ a_log, float* __restrict__ state, const int* __restrict__ slots, int H, int G, int dk,
+    int dv, float qscale, const float* __restrict__ norm_w, float eps, int a_vec, int g_vec, T* __restrict__ out) {
+  extern __shared__ float lds[];
+  const int CV = dv / VW, RG = DS_NT / CV;           // column groups; row groups
+  float* qs = lds;                                   // [dk]
+  float* ks = qs + dk;                               // [dk]
+  float* gs = ks + dk;                               // [dk]
+  float* gate = gs + dk;                             // [dv]
+  float* us = gate + dv;                             // [dv]
+  float* la = us + dv;                               // [ra]
+  float* lg = la + ra;                               // [rg]
+  float* pw = lg + rg;                               // [RG][dv]
+  float* pr = pw + RG * dv;                          // [RG][dv]
+  __shared__ float red[DS_NT / TA_WAVE];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const int kvh = h / (H / G);
+  float* st = state + ((size_t)slots[b] * H + h) * dk * (size_t)dv;
+  const int r0 = tid / CV, c0 = (tid % CV) * VW;
+  const bool on = r0 < RG;
+  float S[ROWS][VW];
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int row = r0 + RG * i;
+    const bool ok = on && row < dk;
+    const float* p = st + (size_t)(ok ? row : 0) * dv + c0;
+    if (VW == 4) {
+      const float4 a = *reinterpret_cast<const float4*>(p);
+      S[i][0] = ok ? a.x : 0.f;
+      S[i][VW > 1 ? 1 : 0] = VW > 1 ? (ok ? a.y : 0.f) : S[i][0];
+      S[i][VW > 2 ? 2 : 0] = VW > 2 ? (ok ? a.z : 0.f) : S[i][0];
+      S[i][VW > 3 ? 3 : 0] = VW > 3 ? (ok ? a.w : 0.f) : S[i][0];
+    } else {
+      const float a = p[0];
+      S[i][0] = ok ? a : 0.f;
+    }
+  }
+  // ---- operands to LDS
+  const T* row = qkv + (size_t)b * stride;
+  for (int c = tid; c < dk; c += DS_NT) {
+    qs[c] = to_f32(row[kvh * dk + c]);
+    ks[c] = to_f32(row[(G + kvh) * dk + c]);
+  }
+  const T* prow = proj + (size_t)b * pstride;
+  for (int c = tid; c < ra; c += DS_NT) la[c] = to_f32(prow[aoff + c]);
+  for (int c = tid; c < rg; c += DS_NT) lg[c] = to_f32(prow[goff + c]);
+  const float beta = dr_sigmoid(to_f32(prow[boff + h]));
+  const float rate = expf(a_log[h]);
+  __syncthreads();
+  // ---- factors of the unit vectors (every wave for itself), decays, output gates
+  float sq = 0.f, sk = 0.f, sx = 0.f;
+  for (int c = tid % TA_WAVE; c < dk; c += TA_WAVE) {
+    const float a = qs[c], k = ks[c];
+    sq = fmaf(a, a, sq);
+    sk = fmaf(k, k, sk);
+    sx = fmaf(a, k, sx);
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  sx = wave_sum(sx);
+  const float fq = qscale * rsqrtf(sq + DR_UNIT_EPS), fk = rsqrtf(sk + DR_UNIT_EPS);
+  const float kq = sx * fq * fk;
+  // (whole groups of four lanes take a row; the loop's bound is the same for the four)
+  for (int i = tid / 4; i < dk + dv; i += DS_NT / 4) {
+    const bool dec = i < dk;
+    const int j = dec ? i : i - dk;
+    const float s = dec ? ds_row_dot<TW>(a2 + ((size_t)h * dk + j) * ra, la, ra, tid % 4, a_vec)
+                        : ds_row_dot<TW>(g2 + ((size_t)h * dv + j) * rg, lg, rg, tid % 4, g_vec);
+    if (tid % 4 == 0) {
+      if (dec) gs[j] = expf(-rate * dr_softplus(s + dt_bias[h * dk + j]));
+      else gate[j] = dr_sigmoid(s);
+    }
+  }
+  __syncthreads();
+  // ---- the decayed state and its products with k and q
+  float w[VW], r[VW];
+#pragma unroll
+  for (int e = 0; e < VW; ++e) w[e] = r[e] = 0.f;
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int rw = r0 + RG * i;
+    const bool ok = on && rw < dk;
+    const float g = gs[ok ? rw : 0], k = ks[ok ? rw : 0] * fk, q = qs[ok ? rw : 0] * fq;
+#pragma unroll
+    for (int e = 0; e < VW; ++e) {
+      S[i][e] *= g;
+      w[e] = fmaf(S[i][e], k, w[e]);
+      r[e] = fmaf(S[i][e], q, r[e]);
+    }
+  }
+  if (on) {
+#pragma unroll
+    for (int e = 0; e < VW; ++e) {
+      pw[r0 * dv + c0 + e] = w[e];
+      pr[r0 * dv + c0 + e] = r[e];
+    }
+  }
+  __syncthreads();
+  float ss = 0.f;
+  const T* vrow = row + 2 * G * dk + (size_t)h * dv;
+  for (int j = tid; j < dv; j += DS_NT) {            // row groups in order
+    float ws = 0.f, rs = 0.f;
+    for (int i = 0; i < RG; ++i) {
+      ws += pw[i * dv + j];
+      rs += pr[i * dv + j];
+    }
+    const float u = beta * (to_f32(vrow[j]) - ws);
+    const float o = fmaf(u, kq, rs);
+    us[j] = u;
+    pr[j] = o;                                       // column j of row group 0 is this thread's alone now
+    ss = fmaf(o, o, ss);
+  }
+  ss = wave_sum(ss);
+  if (tid % TA_WAVE == 0) red[tid / TA_WAVE] = ss;
+  __syncthreads();
+  // ---- the update
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int rw = r0 + RG * i;
+    if (on && rw < dk) {
+      const float k = ks[rw] * fk;
+      float n[VW];
+#pragma unroll
+      for (int e = 0; e < VW; ++e) n[e] = fmaf(k, us[c0 + e], S[i][e]);
+      float* p = st + (size_t)rw * dv + c0;
+      if (VW == 4) *reinterpret_cast<float4*>(p) = float4{n[0], n[VW > 1 ? 1 : 0], n[VW > 2 ? 2 : 0], n[VW > 3 ? 3 : 0]};
+      else p[0] = n[0];
+    }
+  }
+  // ---- the readout's norm and gate
+  float tot = 0.f;
+#pragma unroll
+  for (int i = 0; i < DS_NT / TA_WAVE; ++i) tot += red[i];
+  const float f = rsqrtf(tot / (float)dv + eps);
+  for (int j = tid; j < dv; j += DS_NT)
+    out[(size_t)b * H * dv + (size_t)h * dv + j] = from_f32<T>(pr[j] * f * norm_w[j] * gate[j]);
+}
+
+static int delta_step_rows(int dk, int dv) {          // key channels a thread keeps; 0: not taken
+  const int cv = dv % 4 == 0 ? dv / 4 : dv;
+  if (cv < 1 || cv > DS_NT) return 0;
+  const int rg = DS_NT / cv;
+  const int rows = (dk + rg - 1) / rg;
+  return rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : rows <= 32 ? 32 : 0;
+}
+static size_t delta_step_lds(int dk, int dv, int ra, int rg) {
+  const int cv = dv % 4 == 0 ? dv / 4 : dv;
+  return ((size_t)3 * dk + 2 * dv + ra + rg + (size_t)2 * (DS_NT / cv) * dv) * sizeof(float);
+}
+
+// Whether ta_delta_step takes heads of dk x dv with low-rank inputs of ra and rg.
+extern "C" int ta_delta_step_fits(int dk, int dv, int ra, int rg) {
+  return dk >= 1 && ra >= 1 && rg >= 1 && delta_step_rows(dk, dv) > 0 && delta_step_lds(dk, dv, ra, rg) <= 60000;
+}
+
+// qkv: [batch] rows, stride apart, of [q: G*dk | k: G*dk | v: H*dv] behind convolution and activation;
+// proj: [batch] rows, pstride apart, holding the decay's low-rank input (ra) at aoff, the gate's (rg) at
+// goff and the step sizes' (H) at boff; a2 [H*dk, ra], g2 [H*dv, rg]; state [slots, H, dk, dv] float32;
+// norm_w [dv]; out [batch, H*dv] = the readout over its root mean square per head, times norm_w, gated.
+extern "C" int ta_delta_step(hipStream_t stream, int dtype, int wdtype, const void* qkv, int stride, const void* proj,
+                             int pstride, int aoff, int ra, int goff, int rg, int boff, const void* a2, const void* g2,
+                             const float* dt_bias, const float* a_log, float* state, const int* slots, int batch, int H,
+                             int G, int dk, int dv, float qscale, const float* norm_w, float eps, void* out) {
+  TA_REQUIRE(batch > 0 && batch <= 65535 && G >= 1 && H >= 1 && H % G == 0, "ta_delta_step: batch %d, %d heads in %d groups", batch, H, G);
+  TA_REQUIRE(ta_delta_step_fits(dk, dv, ra, rg), "ta_delta_step: heads of %d x %d, ranks %d / %d", dk, dv, ra, rg);
+  TA_REQUIRE(stride >= 2 * G * dk + H * dv && aoff >= 0 && goff >= 0 && boff >= 0 && pstride >= aoff + ra &&
+             pstride >= goff + rg && pstride >= boff + H, "ta_delta_step: rows of %d / %d are too short", stride, pstride);
+  const int rows = delta_step_rows(dk, dv);
+  const size_t lds = delta_step_lds(dk, dv, ra, rg);
+  const int a_vec = ra % 8 == 0 && (uintptr_t)a2 % 16 == 0, g_vec = rg % 8 == 0 && (uintptr_t)g2 % 16 == 0;
+  const bool wide = dv % 4 == 0 && (uintptr_t)state % 16 == 0;
+  TA_REQUIRE(wide || dv % 4 != 0, "ta_delta_step: the state must be 16-byte aligned");
+  dim3 g(H, batch);
+#define DS_RUN(T, TW, VWV, RW)                                                                                       \
+  delta_step_kernel<T, TW, VWV, RW><<<g, DS_NT, lds, stream>>>(                                                      \
+      (const T*)qkv, stride, (const T*)proj, pstride, aoff, ra, goff, rg, boff, (const TW*)a2, (const TW*)g2, dt_bias, \
+      a_log, state, slots, H, G, dk, dv, qscale, norm_w, eps, a_vec, g_vec, (T*)out)
+#define DS_BY_ROWS(T, TW, VWV)                 \
+  switch (rows) {                              \
+    case 4: DS_RUN(T, TW, VWV, 4); break;      \
+    case 8: DS_RUN(T, TW, VWV, 8); break;      \
+    case 16: DS_RUN(T, TW, VWV, 16); break;    \
+    default: DS_RUN(T, TW, VWV, 32); break;    \
+  }
+#define DS_BY_COLS(T, TW) \
+  if (wide) { DS_BY_ROWS(T, TW, 4) } else { DS_BY_ROWS(T, TW, 1) }
+  if (dtype == TA_F32 && wdtype == TA_F32) { DS_BY_COLS(float, float) }
+  else if (dtype == TA_BF16 && wdtype == TA_BF16) { DS_BY_COLS(bf16_t, bf16_t) }
+  else if (dtype == TA_BF16 && wdtype == TA_F32) { DS_BY_COLS(bf16_t, float) }
+  else return ta_fail("ta_delta_step: unsupported dtypes %d / %d", dtype, wdtype);
+#undef DS_BY_COLS
+#undef DS_BY_ROWS
+#undef DS_RUN
+  return ta_check_launch("ta_delta_step");
+}

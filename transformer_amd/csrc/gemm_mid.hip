@@ -25,7 +25,8 @@
 // `splits` workgroups; each writes its partial result to its own [M, N] float32 plane and
 // the reader adds the planes in order (the residual add of the next norm does).
 //
-// SWIGLU: W holds gate rows then up rows (N = 2*di) and the kernel writes silu(gate) * up.
+// SWIGLU: W holds gate rows then up rows (N = 2*di) and the kernel writes silu(gate) * up, or the
+// limited form of ``TaGlu``.
 // Up to 48 rows a workgroup owns 32 columns: waves 0, 1 of a half take their gate tiles, waves
 // 2, 3 the up tiles, which they hand over through LDS at the end. At 49 to 64 rows a wave takes
 // the gate tile and the up tile of its 16 columns (two tiles per wave: it reads each piece of
@@ -71,7 +72,7 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(const bf16_t* __restrict_
                                                        const float* __restrict__ bias,
                                                        TC* __restrict__ C, int ldc, size_t c_plane,
                                                        int M, int n_out, int K, int chunks_per_split,
-                                                       int vec_ok) {
+                                                       int vec_ok, TaGlu glu) {
   static_assert(NTW == 1 || SWIGLU, "two tiles per wave are the gate and the up tile of its columns");
   static_assert(KW == 2 || (KW == 4 && !SWIGLU), "the range of K is halved, or quartered for a plain product");
   constexpr int CW = 8 / KW;                     // waves side by side along the columns
@@ -266,7 +267,7 @@ __global__ __launch_bounds__(512) void gemm_mid_kernel(const bf16_t* __restrict_
           g += bias[n + i];
           u += bias[n_out + n + i];
         }
-        o[i] = g / (1.0f + expf(-g)) * u;
+        o[i] = ta_glu(glu, g, u);
       }
     } else {
       floatx4 vs = acc[0][j];                              // the parts are added in their order
@@ -310,10 +311,13 @@ extern "C" int ta_gemm_mid_splits(int n_out, int K) {
 // out_dtype TA_BF16 or TA_F32. swiglu != 0: W is [2*n_out, K] (gate rows, then up rows), C is
 // [M, n_out], bias has 2*n_out entries, splits must be 1. Otherwise W is [n_out, K] and, with
 // splits > 1, C holds `splits` planes of c_plane elements each (float32), whose sum is the
-// product (the bias is in plane 0).
+// product (the bias is in plane 0). limit > 0 (with swiglu): the limited form of the activation.
 extern "C" int ta_gemm_mid_bf16(hipStream_t stream, int out_dtype, int swiglu, const void* A, int lda,
                                 const void* W, int ldw, const float* bias, void* C, int ldc,
-                                long long c_plane, int M, int n_out, int K, int splits) {
+                                long long c_plane, int M, int n_out, int K, int splits, float limit,
+                                float slope, float shift) {
+  TA_REQUIRE(limit >= 0.f && (limit == 0.f || swiglu), "ta_gemm_mid_bf16: limit %g", (double)limit);
+  const TaGlu glu = {limit, slope, shift};
   TA_REQUIRE(M >= 0 && M <= 64, "ta_gemm_mid_bf16: M=%d outside [0, 64]", M);
   TA_REQUIRE(n_out > 0 && K > 0, "ta_gemm_mid_bf16: bad sizes N=%d K=%d", n_out, K);
   TA_REQUIRE(K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0 && lda >= K && ldw >= K && ldc >= n_out,
@@ -344,7 +348,7 @@ extern "C" int ta_gemm_mid_bf16(hipStream_t stream, int out_dtype, int swiglu, c
   const int vec_ok = ((uintptr_t)C % (4 * esz)) == 0 && ldc % 4 == 0 && (splits == 1 || c_plane % 4 == 0);
 #define LAUNCH_K(MRV, SW, TL, TC, KWV)                                                                     \
   gemm_mid_kernel<MRV, (SW && MRV == 4 ? 2 : 1), SW, TL, TC, KWV><<<g, b, 0, stream>>>(                     \
-      (const bf16_t*)A, lda, (const bf16_t*)W, ldw, bias, (TC*)C, ldc, (size_t)c_plane, M, n_out, K, per, vec_ok)
+      (const bf16_t*)A, lda, (const bf16_t*)W, ldw, bias, (TC*)C, ldc, (size_t)c_plane, M, n_out, K, per, vec_ok, glu)
 #define LAUNCH_T(MRV, SW, TL, TC) \
   if (!SW && kw == 4) LAUNCH_K(MRV, SW, TL, TC, (SW ? 2 : 4)); else LAUNCH_K(MRV, SW, TL, TC, 2)
 #define LAUNCH_TL(MRV, SW, TC) \

@@ -17,8 +17,8 @@
 // permuted by the row number on the way in, so the operand reads meet no bank twice.
 //
 // SWIGLU: W holds gate rows then up rows (N = 2*di); the workgroup computes both
-// tiles for its 16 columns and writes silu(gate) * up, so the [M, 2*di] product never
-// reaches memory.
+// tiles for its 16 columns and writes silu(gate) * up (or the limited form of ``TaGlu``), so the
+// [M, 2*di] product never reaches memory.
 //
 // A product may also take over the RMS norm that stands between two products, so that a
 // single-token step needs no kernel of its own for it. The product in front of the norm
@@ -39,6 +39,7 @@ struct SkinnyNorm {
   bf16_t* H;                  // [M][ldh] (X + product) * norm_w
   int ldh;
   float* out_parts;           // [tiles][16]
+  TaGlu glu;                  // SWIGLU: how gate and up are joined
 };
 
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;
@@ -217,7 +218,7 @@ __global__ __launch_bounds__(WAVES * 64) void gemm_skinny_kernel(const bf16_t* _
     if (bias && col_ok) v[nt] += bias[nt * n_out + n];
   }
   float o = v[0];
-  if (SWIGLU) o = v[0] / (1.0f + expf(-v[0])) * v[NT - 1];
+  if (SWIGLU) o = ta_glu(nm.glu, v[0], v[NT - 1]);
   if (FOLD) {
     float xn = 0.f;
     if (col_ok) {
@@ -359,7 +360,7 @@ __global__ __launch_bounds__(1024) void gemm_skinny_hold_kernel(const bf16_t* __
           if (sizeof(TC) == 2) sum = to_f32(from_f32<bf16_t>(sum));
           if (bias) sum += bias[(i & 1) * n_out + n];
           if (i & 1)
-            C[(size_t)m * ldc + n] = from_f32<TC>(gate / (1.0f + expf(-gate)) * sum);
+            C[(size_t)m * ldc + n] = from_f32<TC>(ta_glu(nm.glu, gate, sum));
           else
             gate = sum;
         } else {
@@ -398,18 +399,20 @@ extern "C" int ta_gemm_skinny_bf16(hipStream_t stream, int out_dtype, int swiglu
   return skinny_launch(stream, out_dtype, swiglu, A, lda, W, ldw, bias, C, ldc, M, n_out, K, waves, nm);
 }
 
-// The same product around an RMS norm (see the head of this file). scale_parts != null:
+// The product around an RMS norm (see the head of this file). scale_parts != null:
 // A holds rows that are not yet scaled; [n_parts][16] sums of squares, `size` the norm's
 // width. X != null (not with swiglu): the product (+ bias) is added to X [M][ldx] in place,
 // H [M][ldh] gets the new rows times norm_w [n_out], out_parts [ceil(n_out/16)][16] their
-// sums of squares; C is not written.
+// sums of squares; C is not written. limit > 0 (with swiglu): the limited form of the activation.
 extern "C" int ta_gemm_skinny_norm_bf16(hipStream_t stream, int out_dtype, int swiglu, const void* A,
                                         int lda, const void* W, int ldw, const float* bias, void* C,
                                         int ldc, int M, int n_out, int K, int waves,
                                         const float* scale_parts, int n_parts, float eps, int size,
                                         float* X, int ldx, const float* norm_w, void* H, int ldh,
-                                        float* out_parts) {
+                                        float* out_parts, float limit, float slope, float shift) {
+  TA_REQUIRE(limit >= 0.f && (limit == 0.f || swiglu), "ta_gemm_skinny_norm_bf16: limit %g", (double)limit);
   SkinnyNorm nm = {};
+  nm.glu = TaGlu{limit, slope, shift};
   if (scale_parts) {
     TA_REQUIRE(n_parts > 0 && size > 0, "ta_gemm_skinny_norm_bf16: %d partial sums over a width of %d", n_parts, size);
     nm.scale_parts = scale_parts; nm.n_parts = n_parts; nm.eps = eps; nm.inv_size = 1.0f / (float)size;

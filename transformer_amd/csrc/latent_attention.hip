@@ -15,7 +15,8 @@
 //   latent_query_rot : the rotated part of every head's query, rotated, into the last `rot`
 //                      coordinates of the wide query rows
 //   latent_attention : causal (windowed) softmax attention of the wide queries over the
-//                      cached rows with an output gate per (token, head): float32 on the
+//                      cached rows, with an output gate per (token, head) and one more term
+//                      exp(sink[head]) of the denominator where they are given: float32 on the
 //                      vector ALU; for bfloat16 rows on the matrix cores, with a workgroup's
 //                      waves sharing their chunks of keys in steps of many rows and a row's
 //                      keys dealt to several waves in steps of few
@@ -110,7 +111,7 @@ extern "C" int ta_latent_prepare(hipStream_t stream, int dtype, const void* proj
 
 // ------------------------------------------------------------------ rotated query parts
 template <typename T>
-__global__ __launch_bounds__(256) void latent_query_rot_kernel(const T* __restrict__ q, int H, int dn, int rot,
+__global__ __launch_bounds__(256) void latent_query_rot_kernel(const T* __restrict__ q, int q_stride, int H, int dn, int rot,
                                                                int rot_dims, const float* __restrict__ angles,
                                                                T* __restrict__ qa, int rank, int dc) {
   const size_t t = blockIdx.x;
@@ -122,7 +123,7 @@ __global__ __launch_bounds__(256) void latent_query_rot_kernel(const T* __restri
   const int pairs = (rot + 1) / 2;
   for (int idx = threadIdx.x; idx < H * pairs; idx += 256) {
     const int h = idx / pairs, i = idx % pairs;
-    const T* src = q + (t * H + h) * (size_t)(dn + rot) + dn;
+    const T* src = q + t * q_stride + h * (dn + rot) + dn;
     T* dst = qa + (t * H + h) * (size_t)dc + rank;
     const float u = to_f32(src[2 * i]);
     if (2 * i + 1 >= rot) { dst[2 * i] = from_f32<T>(u); continue; }
@@ -138,18 +139,18 @@ __global__ __launch_bounds__(256) void latent_query_rot_kernel(const T* __restri
   }
 }
 
-// q: [nt, H, dn + rot] (each head: unrotated part, then the part to rotate); qa: [nt, H, dc], dc >=
+// q: [nt] rows, q_stride elements apart, of [H, dn + rot] (each head: unrotated part, then the part to rotate); qa: [nt, H, dc], dc >=
 // rank + rot, whose coordinates from ``rank`` on are written (the rotated part, then zeros).
-extern "C" int ta_latent_query_rot(hipStream_t stream, int dtype, const void* q, int H, int dn, int rot,
+extern "C" int ta_latent_query_rot(hipStream_t stream, int dtype, const void* q, int q_stride, int H, int dn, int rot,
                                    int rot_dims, const float* angles, void* qa, int rank, int dc, int nt) {
   TA_REQUIRE(nt >= 0 && H >= 1 && dn >= 0 && rot >= 0 && rank >= 1 && rot_dims >= 0 && rot_dims <= rot && rot_dims % 2 == 0,
              "ta_latent_query_rot: bad sizes");
-  TA_REQUIRE(dc >= rank + rot, "ta_latent_query_rot: rows of %d for %d + %d", dc, rank, rot);
+  TA_REQUIRE(dc >= rank + rot && q_stride >= H * (dn + rot), "ta_latent_query_rot: rows of %d for %d + %d", dc, rank, rot);
   if (nt == 0 || dc == rank) return 0;
   if (dtype == TA_F32)
-    latent_query_rot_kernel<float><<<nt, 256, 0, stream>>>((const float*)q, H, dn, rot, rot_dims, angles, (float*)qa, rank, dc);
+    latent_query_rot_kernel<float><<<nt, 256, 0, stream>>>((const float*)q, q_stride, H, dn, rot, rot_dims, angles, (float*)qa, rank, dc);
   else if (dtype == TA_BF16)
-    latent_query_rot_kernel<bf16_t><<<nt, 256, 0, stream>>>((const bf16_t*)q, H, dn, rot, rot_dims, angles, (bf16_t*)qa, rank, dc);
+    latent_query_rot_kernel<bf16_t><<<nt, 256, 0, stream>>>((const bf16_t*)q, q_stride, H, dn, rot, rot_dims, angles, (bf16_t*)qa, rank, dc);
   else
     return ta_fail("ta_latent_query_rot: unknown dtype %d", dtype);
   return ta_check_launch("ta_latent_query_rot");
@@ -178,7 +179,7 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     const T* __restrict__ qa, T* __restrict__ out, const T* __restrict__ kcache,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ pos0, int H, int rank, int rot, float scale, int window,
-    const T* __restrict__ gate, int gate_stride, int dc) {
+    const T* __restrict__ gate, int gate_stride, int dc, const float* __restrict__ sink) {
   extern __shared__ float smem[];
   const int D = rank + rot, DP = D + 1;
   const int b = blockIdx.y;
@@ -271,6 +272,12 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     }
   }
   if (row_ok) {
+    if (sink) {                              // one more term of the denominator, with no value
+      const float sv = sink[head], m_new = fmaxf(m, sv), alpha = expf(m - m_new);
+      l = l * alpha + expf(sv - m_new);
+#pragma unroll
+      for (int i = 0; i < NACC; ++i) acc[i] *= alpha;
+    }
     float f = l > 0.f ? 1.0f / l : 0.f;
     if (gate) {
       const float g = to_f32(gate[(size_t)(q0 + qi) * gate_stride + head]);
@@ -287,7 +294,7 @@ template <typename T, int NACC>
 static int latent_attention_run(hipStream_t stream, dim3 g, size_t lds, const void* qa, void* out,
                                 const void* kcache, const int* block_table, int max_blocks, const int* cu_q,
                                 const int* pos0, int H, int rank, int rot, float scale, int window,
-                                const void* gate, int gate_stride, int dc) {
+                                const void* gate, int gate_stride, int dc, const float* sink) {
   auto kern = latent_attention_kernel<T, NACC>;
   static size_t allowed = 64 * 1024;                    // per instantiation: asked for once, not at every launch
   if (lds > allowed) {
@@ -297,7 +304,7 @@ static int latent_attention_run(hipStream_t stream, dim3 g, size_t lds, const vo
     allowed = lds;
   }
   kern<<<g, 256, lds, stream>>>((const T*)qa, (T*)out, (const T*)kcache, block_table, max_blocks, cu_q, pos0, H,
-                                rank, rot, scale, window, (const T*)gate, gate_stride, dc);
+                                rank, rot, scale, window, (const T*)gate, gate_stride, dc, sink);
   return 0;
 }
 
@@ -315,6 +322,12 @@ static int latent_attention_run(hipStream_t stream, dim3 g, size_t lds, const vo
 // and long key ranges.
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 la_bf16x8;
 typedef __attribute__((__vector_size__(4 * sizeof(float)))) float la_floatx4;
+// 1 / (sum of weights + the sink's term) of a row whose weights are relative to m (log2 domain)
+__device__ __forceinline__ float la_inverse(float l, float m, const float* __restrict__ sink, int head) {
+  if (sink) l += __builtin_amdgcn_exp2f(sink[head] * 1.4426950408889634f - (m == -INFINITY ? 0.f : m));
+  return l > 0.f ? 1.0f / l : 0.f;
+}
+
 union LaFrag {
   la_bf16x8 v;
   uint4 q;
@@ -425,7 +438,8 @@ __global__ __launch_bounds__(256, ((KS <= 6 && RT == 1) ? 2 : 1)) void latent_at
     const bf16_t* __restrict__ qa, bf16_t* __restrict__ out, const bf16_t* __restrict__ kcache,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ pos0, int H, int rank, int dc, float scale_log2, int window,
-    const bf16_t* __restrict__ gate, int gate_stride, int splits, int tiles_max, float* __restrict__ partial) {
+    const bf16_t* __restrict__ gate, int gate_stride, int splits, int tiles_max, float* __restrict__ partial,
+    const float* __restrict__ sink) {
   extern __shared__ __attribute__((aligned(16))) unsigned char la_lds[];
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const int c = lane % 16, g = lane / 16;
@@ -556,7 +570,7 @@ __global__ __launch_bounds__(256, ((KS <= 6 && RT == 1) ? 2 : 1)) void latent_at
       if (g == 0 && half == 0) { dst[rank] = m[rt]; dst[rank + 1] = l[rt]; }
       continue;
     }
-    float f = l[rt] > 0.f ? 1.0f / l[rt] : 0.f;
+    float f = la_inverse(l[rt], m[rt], sink, row % H);
     if (gate) {
       const float gv = to_f32(gate[(size_t)(q0 + row / H) * gate_stride + row % H]);
       f *= 1.0f / (1.0f + expf(-gv));
@@ -584,7 +598,7 @@ __global__ __launch_bounds__(256, (KS <= 10 ? 2 : 1)) void latent_attention_mfma
     const bf16_t* __restrict__ qa, bf16_t* __restrict__ out, const bf16_t* __restrict__ kcache,
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ pos0, int H, int rank, int dc, float scale_log2, int window,
-    const bf16_t* __restrict__ gate, int gate_stride) {
+    const bf16_t* __restrict__ gate, int gate_stride, const float* __restrict__ sink) {
   extern __shared__ __attribute__((aligned(16))) unsigned char la_lds[];
   constexpr int NBUF = 3;
   const int tid = threadIdx.x, wave = tid / 64, lane = tid % 64;
@@ -696,7 +710,7 @@ __global__ __launch_bounds__(256, (KS <= 10 ? 2 : 1)) void latent_attention_mfma
   }
   if (!active || !ok[0]) return;
   const int row = row0 + c;
-  float f = l[0] > 0.f ? 1.0f / l[0] : 0.f;
+  float f = la_inverse(l[0], m[0], sink, row % H);
   if (gate) {
     const float gv = to_f32(gate[(size_t)(q0 + row / H) * gate_stride + row % H]);
     f *= 1.0f / (1.0f + expf(-gv));
@@ -714,7 +728,8 @@ __global__ __launch_bounds__(256, (KS <= 10 ? 2 : 1)) void latent_attention_mfma
 template <int KS, int CT>
 static int latent_mfma_wg_run(hipStream_t stream, dim3 g, size_t lds, const void* qa, void* out, const void* kcache,
                               const int* block_table, int max_blocks, const int* cu_q, const int* pos0, int H,
-                              int rank, int dc, float scale_log2, int window, const void* gate, int gate_stride) {
+                              int rank, int dc, float scale_log2, int window, const void* gate, int gate_stride,
+                              const float* sink) {
   auto kern = latent_attention_mfma_wg_kernel<KS, CT>;
   static size_t allowed = 64 * 1024;                    // per instantiation: asked for once, not at every launch
   if (lds > allowed) {
@@ -724,7 +739,7 @@ static int latent_mfma_wg_run(hipStream_t stream, dim3 g, size_t lds, const void
     allowed = lds;
   }
   kern<<<g, 256, lds, stream>>>((const bf16_t*)qa, (bf16_t*)out, (const bf16_t*)kcache, block_table, max_blocks,
-                                cu_q, pos0, H, rank, dc, scale_log2, window, (const bf16_t*)gate, gate_stride);
+                                cu_q, pos0, H, rank, dc, scale_log2, window, (const bf16_t*)gate, gate_stride, sink);
   return 0;
 }
 
@@ -732,7 +747,8 @@ static int latent_mfma_wg_run(hipStream_t stream, dim3 g, size_t lds, const void
 __global__ __launch_bounds__(64) void latent_merge_kernel(const float* __restrict__ partial, bf16_t* __restrict__ out,
                                                           const int* __restrict__ cu_q, int H, int rank, int splits,
                                                           int tiles_max, int rows_per_tile,
-                                                          const bf16_t* __restrict__ gate, int gate_stride) {
+                                                          const bf16_t* __restrict__ gate, int gate_stride,
+                                                          const float* __restrict__ sink) {
   const int b = blockIdx.y, row = blockIdx.x;
   const int q0 = cu_q[b], qlen = cu_q[b + 1] - q0;
   if (row >= qlen * H) return;
@@ -752,7 +768,7 @@ __global__ __launch_bounds__(64) void latent_merge_kernel(const float* __restric
   }
   L = wave_sum(L);
   __syncthreads();
-  float f = L > 0.f ? 1.0f / L : 0.f;
+  float f = la_inverse(L, M, sink, row % H);
   if (gate) {
     const float gv = to_f32(gate[(size_t)(q0 + row / H) * gate_stride + row % H]);
     f *= 1.0f / (1.0f + expf(-gv));
@@ -770,7 +786,7 @@ template <int KS, int CT, int RT>
 static int latent_mfma_run(hipStream_t stream, dim3 g, size_t lds, const void* qa, void* out, const void* kcache,
                            const int* block_table, int max_blocks, const int* cu_q, const int* pos0, int H,
                            int rank, int dc, float scale_log2, int window, const void* gate, int gate_stride,
-                           int splits, int tiles_max, float* partial) {
+                           int splits, int tiles_max, float* partial, const float* sink) {
   auto kern = latent_attention_mfma_kernel<KS, CT, RT>;
   static size_t allowed = 64 * 1024;                    // per instantiation: asked for once, not at every launch
   if (lds > allowed) {
@@ -781,7 +797,7 @@ static int latent_mfma_run(hipStream_t stream, dim3 g, size_t lds, const void* q
   }
   kern<<<g, 256, lds, stream>>>((const bf16_t*)qa, (bf16_t*)out, (const bf16_t*)kcache, block_table, max_blocks,
                                 cu_q, pos0, H, rank, dc, scale_log2, window, (const bf16_t*)gate, gate_stride, splits,
-                                tiles_max, partial);
+                                tiles_max, partial, sink);
   return 0;
 }
 
@@ -801,14 +817,16 @@ extern "C" long long ta_latent_mfma_scratch(int batch, int max_qlen, int H, int 
 
 // qa: [nt, H, dc] wide queries (dc >= rank + rot, the rest zero). out: [nt, H, rank]. kcache: one
 // layer, [pages][1][TA_PAGE][dc]. gate (or null): pre-activation of a sigmoid gate per
-// (token, head), element h of a row of gate_stride elements. window <= 0: all earlier keys.
+// (token, head), element h of a row of gate_stride elements. sink (or null): [H] float32, a row's
+// denominator also holds exp(sink[head]). window <= 0: all earlier keys.
 // bfloat16 with rows of whole 16-byte pieces runs on the matrix cores; `splits` > 1 deals a
 // row's keys to that many waves (scratch: ta_latent_mfma_scratch floats). float32, and rows
 // that are no multiple of 8 wide, run on the vector ALU (splits is ignored).
 extern "C" int ta_latent_attention(hipStream_t stream, int dtype, const void* qa, void* out, const void* kcache,
                                    const int* block_table, int max_blocks, const int* cu_q, const int* pos0,
                                    int batch, int max_qlen, int H, int rank, int rot, int dc, float scale, int window,
-                                   const void* gate, int gate_stride, int splits, float* scratch) {
+                                   const void* gate, int gate_stride, int splits, float* scratch,
+                                   const float* sink) {
   TA_REQUIRE(batch >= 0 && batch <= 65535 && max_qlen >= 0 && H >= 1, "ta_latent_attention: bad batch=%d max_qlen=%d heads=%d", batch, max_qlen, H);
   TA_REQUIRE(rank >= 1 && rank <= 512 && rot >= 0 && rot <= 512, "ta_latent_attention: latent of %d / rotated part of %d outside [1, 512] / [0, 512]", rank, rot);
   TA_REQUIRE(dc >= rank + rot, "ta_latent_attention: rows of %d for %d + %d", dc, rank, rot);
@@ -826,7 +844,7 @@ extern "C" int ta_latent_attention(hipStream_t stream, int dtype, const void* qa
       const size_t ldw = (size_t)3 * 32 * (dc + 8) * sizeof(bf16_t);
       const float sl2w = scale * 1.4426950408889634f;
       int rcw;
-#define LA_WG(KS, CT) latent_mfma_wg_run<KS, CT>(stream, gw, ldw, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, dc, sl2w, window, gate, gate_stride)
+#define LA_WG(KS, CT) latent_mfma_wg_run<KS, CT>(stream, gw, ldw, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, dc, sl2w, window, gate, gate_stride, sink)
       if (dc <= 192 && rank <= 128) rcw = LA_WG(6, 8);
       else if (dc <= 320 && rank <= 256) rcw = LA_WG(10, 16);
       else rcw = LA_WG(18, 32);
@@ -841,7 +859,7 @@ extern "C" int ta_latent_attention(hipStream_t stream, int dtype, const void* qa
     const size_t lds = (size_t)4 * 32 * (dc + 8) * sizeof(bf16_t);
     const float sl2 = scale * 1.4426950408889634f;
     int rc;
-#define LA_MFMA(KS, CT, RT) latent_mfma_run<KS, CT, RT>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, dc, sl2, window, gate, gate_stride, splits, (int)tiles, scratch)
+#define LA_MFMA(KS, CT, RT) latent_mfma_run<KS, CT, RT>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, dc, sl2, window, gate, gate_stride, splits, (int)tiles, scratch, sink)
     if (dc <= 192 && rank <= 128) rc = rows == 32 ? LA_MFMA(6, 8, 2) : LA_MFMA(6, 8, 1);
     else if (dc <= 320 && rank <= 256) rc = LA_MFMA(10, 16, 1);
     else rc = LA_MFMA(18, 32, 1);
@@ -850,7 +868,7 @@ extern "C" int ta_latent_attention(hipStream_t stream, int dtype, const void* qa
     if (splits > 1) {
       dim3 gm((unsigned)(max_qlen * H), batch);
       latent_merge_kernel<<<gm, 64, (size_t)splits * sizeof(float), stream>>>(scratch, (bf16_t*)out, cu_q, H, rank, splits, (int)tiles, rows,
-                                                 (const bf16_t*)gate, gate_stride);
+                                                 (const bf16_t*)gate, gate_stride, sink);
     }
     return ta_check_launch("ta_latent_attention");
   }
@@ -862,9 +880,9 @@ extern "C" int ta_latent_attention(hipStream_t stream, int dtype, const void* qa
   TA_REQUIRE(lds <= 160 * 1024, "ta_latent_attention: rows of %d do not fit the LDS", D);
   int rc;
 #define LA_RUN(T)                                                                                              \
-  (rank <= 128 ? latent_attention_run<T, 8>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc)   \
-   : rank <= 256 ? latent_attention_run<T, 16>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc) \
-                 : latent_attention_run<T, 32>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc))
+  (rank <= 128 ? latent_attention_run<T, 8>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc, sink)   \
+   : rank <= 256 ? latent_attention_run<T, 16>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc, sink) \
+                 : latent_attention_run<T, 32>(stream, g, lds, qa, out, kcache, block_table, max_blocks, cu_q, pos0, H, rank, rot, scale, window, gate, gate_stride, dc, sink))
   if (dtype == TA_F32) rc = LA_RUN(float);
   else if (dtype == TA_BF16) rc = LA_RUN(bf16_t);
   else return ta_fail("ta_latent_attention: unknown dtype %d", dtype);

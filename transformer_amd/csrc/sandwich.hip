@@ -5,6 +5,8 @@
 //                      layer scale), optionally followed in the same pass by a copy of the
 //                      new row in the engine's type and by the NEXT norm of the stream,
 //                      out = rms_norm(x) * w_next, so that a row is read and written once
+//   stream_add       : x += delta (+ a row), with a copy of the new rows in the engine's type: where
+//                      something reads the stream itself before its next norm
 //   activation       : out = act(in) (* rows of a float32 side table), act one of gelu (erf),
 //                      gelu (tanh), relu squared, silu
 //
@@ -142,6 +144,58 @@ extern "C" int ta_postnorm_add(hipStream_t stream, int out_dtype, float* x, cons
   }
 #undef PN_RUN
   return ta_check_launch("ta_postnorm_add");
+}
+
+// ------------------------------------------------------------------ an add without a norm
+template <typename TO, int VW>
+__global__ __launch_bounds__(256) void stream_add_kernel(float* __restrict__ x, const float* __restrict__ delta,
+                                                         int planes, size_t plane, const float* __restrict__ bias,
+                                                         TO* __restrict__ xcast, int d, size_t total) {
+  for (size_t i = ((size_t)blockIdx.x * 256 + threadIdx.x) * VW; i < total; i += (size_t)gridDim.x * 256 * VW) {
+    if (VW == 4) {
+      float4 v = *reinterpret_cast<const float4*>(x + i);
+      if (delta)
+        for (int p = 0; p < planes; ++p) {
+          const float4 a = *reinterpret_cast<const float4*>(delta + p * plane + i);
+          v.x += a.x; v.y += a.y; v.z += a.z; v.w += a.w;
+        }
+      if (bias) {
+        const float4 a = *reinterpret_cast<const float4*>(bias + i % d);
+        v.x += a.x; v.y += a.y; v.z += a.z; v.w += a.w;
+      }
+      if (delta || bias) *reinterpret_cast<float4*>(x + i) = v;
+      if (xcast) store4<TO>(xcast + i, v.x, v.y, v.z, v.w);
+    } else {
+      float v = x[i];
+      if (delta)
+        for (int p = 0; p < planes; ++p) v += delta[p * plane + i];
+      if (bias) v += bias[i % d];
+      if (delta || bias) x[i] = v;
+      if (xcast) xcast[i] = from_f32<TO>(v);
+    }
+  }
+}
+
+// x [nt, d] += sum of the planes of delta [planes, nt, d] (or null) + bias [d] (or null), float32, in
+// place; xcast (or null) [nt, d] receives the new rows.
+extern "C" int ta_stream_add(hipStream_t stream, int cast_dtype, float* x, const float* delta, int planes,
+                             long long plane, const float* bias, void* xcast, int nt, int d) {
+  TA_REQUIRE(nt >= 0 && d > 0 && planes >= 1 && planes <= TA_MAX_PLANES, "ta_stream_add: bad sizes nt=%d d=%d planes=%d", nt, d, planes);
+  if (nt == 0) return 0;
+  const size_t total = (size_t)nt * d;
+  const bool vec = d % 4 == 0 && plane % 4 == 0 && (((uintptr_t)x | (uintptr_t)delta | (uintptr_t)bias | (uintptr_t)xcast) & 15) == 0;
+  const size_t work = vec ? total / 4 : total;
+  const unsigned blocks = (unsigned)((work + 255) / 256 < 4096 ? (work + 255) / 256 : 4096);
+#define SA_RUN(T, V) stream_add_kernel<T, V><<<blocks, 256, 0, stream>>>(x, delta, planes, (size_t)plane, bias, (T*)xcast, d, total)
+  if (cast_dtype == TA_F32) {
+    if (vec) SA_RUN(float, 4); else SA_RUN(float, 1);
+  } else if (cast_dtype == TA_BF16) {
+    if (vec) SA_RUN(bf16_t, 4); else SA_RUN(bf16_t, 1);
+  } else {
+    return ta_fail("ta_stream_add: unknown dtype %d", cast_dtype);
+  }
+#undef SA_RUN
+  return ta_check_launch("ta_stream_add");
 }
 
 // ------------------------------------------------------------------ activations

@@ -124,6 +124,8 @@ class DecoderModel:
         out.update(self.final_norm.all_params("final_norm."))
         for n, p in self._extras().items():
             out.update(p.all_params(n + "."))
+        if s.stream_rows:
+            out["stream_rows"] = Param((s.stream_rows, s.hidden), "vector")
         out["head.weight"] = Param((s.vocab, s.hidden), "matrix")
         return out
 
@@ -142,6 +144,11 @@ class DecoderModel:
                 raise ValueError(f"parameter {n} has shape {tuple(tensors[n].shape)}, "
                                  f"expected {tuple(want[n].shape)}")
         self.w = {"embed": tensors["embed.weight"], "head": tensors["head.weight"]}
+        if self.spec.stream_rows:
+            if tuple(tensors["stream_rows"].shape) != tuple(want["stream_rows"].shape):
+                raise ValueError(f"parameter stream_rows has shape {tuple(tensors['stream_rows'].shape)}, "
+                                 f"expected {tuple(want['stream_rows'].shape)}")
+            self.w["stream_rows"] = tensors["stream_rows"]
         self.tensors = {n: tensors[n] for n in want}     # every parameter by its declared name
 
     def weight_bytes(self) -> int:
@@ -196,7 +203,10 @@ class DecoderModel:
             # a part may hand intermediates of its own to the dump: ``ctx.dump(name, tensor)``
             ctx.dump = None if self.dump is None else (lambda n, t, i=i: self.dump(f"run.{i}.{n}", t))
             kw = {}
-            if getattr(block, "folds_norms", False) and i + 1 < len(s.schedule):
+            if run.opening is not None:
+                pending = self._open(x, pending, self.w["stream_rows"][run.opening])
+            # the block in front may prepare the next block's norm, unless something is added in between
+            if getattr(block, "folds_norms", False) and i + 1 < len(s.schedule) and s.schedule[i + 1].opening is None:
                 kw["after"] = self.blocks[s.schedule[i + 1].block]    # it may prepare that block's norm
             pending = block.run(x, pending, ctx, cache, self.cache_layer[i],
                                 writes_cache=run.cache_of is None, **kw)
@@ -216,6 +226,14 @@ class DecoderModel:
         if self.dump is not None:
             self.dump("logits", logits)
         return logits
+
+    @staticmethod
+    def _open(x, pending, row):
+        """A row for every token of the stream: it joins what the next norm adds anyway."""
+        if isinstance(pending, tuple) and pending[1] is None and not isinstance(pending[0], kernels.GatedDelta):
+            return pending[0], row
+        kernels.stream_add(x, bias=row)
+        return pending
 
     def _run_extra(self, name, t, ctx, cache):
         part = getattr(self, name)

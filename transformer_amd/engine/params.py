@@ -21,5 +21,7 @@ def declared_params(spec: ModelSpec) -> Dict[str, Param]:
     for name in ("after_embed", "on_logits"):
         if getattr(spec, name, None) is not None:
             out.update(build_part(getattr(spec, name), torch.float32, "cpu").all_params(name + "."))
+    if spec.stream_rows:
+        out["stream_rows"] = Param((spec.stream_rows, spec.hidden), "vector")
     out["head.weight"] = Param((spec.vocab, spec.hidden), "matrix")
     return out

@@ -359,7 +359,19 @@ def key_unit_count(batch: int, num_kv_heads: int) -> int:
 UNIT_INTS = 8      # int32 values in a unit's record, fixed in csrc/common.h (TA_UNIT_INTS)
 
 
-def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tables=None):
+def seen_pages(length: int, window: Optional[int], keep_first: int = 0):
+    """Page ranges [(first, pages), ...] that a single token at position ``length`` - 1 reads: the pages of
+    its window behind those of the sequence's kept first keys (one range where the two meet)."""
+    n = max(1, -(-int(length) // PAGE))
+    first = max(0, int(length) - window) // PAGE if window else 0
+    kept = min(-(-int(keep_first) // PAGE), first)
+    if kept == first:
+        return [(0, n)]
+    return ([(0, kept)] if kept else []) + [(first, n - first)]
+
+
+def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tables=None,
+                   window: Optional[int] = None, keep_first: int = 0):
     """Cuts sequences of ``kv_lens`` tokens (this step's token included) into at most
     ``n_units`` runs of pages of about equal length, none shorter than ``min_pages`` unless
     it is a whole sequence: a CU can ask only so much of the memory in a given time, so the
@@ -367,18 +379,22 @@ def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tab
     first page, pages, the sequence's length, page numbers of the unit's first two pages (from
     ``tables[b]``, the sequence's row of the block table; 0 without), units of the sequence,
     0), spare units holding 0 pages, and seq_units [batch, 2] = (first unit, units); a
-    sequence's units follow one another and cover its pages in order. Pure host."""
+    sequence's units follow one another and cover its pages in order. With a window only the pages
+    that the token sees are dealt out (``seen_pages``), unless there are too few units. Pure host."""
     import heapq
     import numpy as np
     min_pages = min_pages or _KEYS_MIN_PER
     B = len(kv_lens)
     if n_units < B:
         raise KernelError(f"{n_units} units of work cannot hold {B} sequences")
-    pages = [max(1, -(-int(n) // PAGE)) for n in kv_lens]
-    count = [1] * B
-    heap = [(-pages[b], b) for b in range(B)]
+    ranges = [(b, first, n) for b in range(B) for first, n in seen_pages(kv_lens[b], window, keep_first)]
+    if n_units < len(ranges):
+        ranges = [(b, first, n) for b in range(B) for first, n in seen_pages(kv_lens[b], None)]
+    pages = [r[2] for r in ranges]
+    count = [1] * len(ranges)
+    heap = [(-pages[b], b) for b in range(len(ranges))]
     heapq.heapify(heap)
-    spare = n_units - B
+    spare = n_units - len(ranges)
     while spare > 0 and heap:
         _, b = heapq.heappop(heap)
         if pages[b] < min_pages * (count[b] + 1):      # another cut would make its runs too short
@@ -389,10 +405,13 @@ def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tab
     cuts = []
     # sequences with the longest runs first: workgroups start in the order of their units, so
     # where there are more units than the CUs hold at once the short ones fill the end
-    for b in sorted(range(B), key=lambda b: (-(pages[b] / count[b]), b)):
-        base, extra = divmod(pages[b], count[b])
-        first = 0
-        for i in range(count[b]):
+    longest = [0.0] * B
+    for r, (b, _, n) in enumerate(ranges):
+        longest[b] = max(longest[b], n / count[r])
+    for r in sorted(range(len(ranges)), key=lambda r: (-longest[ranges[r][0]], r)):
+        b, first, pages_r = ranges[r]
+        base, extra = divmod(pages_r, count[r])
+        for i in range(count[r]):
             n = base + (1 if i < extra else 0)
             cuts.append((b, first, n))
             first += n
@@ -577,10 +596,12 @@ class NormFold:
 
 def gemm_skinny(a: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor], swiglu: bool = False,
                 bias: Optional[torch.Tensor] = None, waves: int = 0,
-                scale: Optional[RowScale] = None, fold: Optional[NormFold] = None):
+                scale: Optional[RowScale] = None, fold: Optional[NormFold] = None,
+                limits: Optional[Sequence[float]] = None):
     """out = a @ w.T for at most 16 rows of bfloat16 ``a`` (decode steps), float32
     accumulation, out bfloat16 or float32. swiglu: w is [2*n, k] (gate rows, up rows)
-    and out [m, n] = silu(a @ gate.T) * (a @ up.T). waves: 4, 8 or 16 waves of a
+    and out [m, n] = silu(a @ gate.T) * (a @ up.T); limits = (limit, slope, shift): joined as
+    ``glu_limit`` does instead. waves: 4, 8 or 16 waves of a
     workgroup split k; 0 lets the library choose by the weight's shape.
 
     scale: the rows of ``a`` still lack their norm's factor, which is applied to the
@@ -604,7 +625,9 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor], s
         _dev(bias, "bias", torch.float32)
         if bias.numel() != N:
             raise KernelError("gemm_skinny: bias must hold one entry per row of w")
-    if scale is None and fold is None:
+    if limits is not None and not (swiglu and limits[0] > 0):
+        raise KernelError(f"gemm_skinny: limits {tuple(limits)} belong to a gated activation")
+    if scale is None and fold is None and limits is None:
         _check(library().ta_gemm_skinny_bf16(_stream(), c_int(out_code), c_int(int(swiglu)),
                                              _ptr(a), c_int(lda), _ptr(w), c_int(ldw), _ptr(bias),
                                              _ptr(out), c_int(ldc), c_int(M), c_int(n_out), c_int(K),
@@ -635,7 +658,7 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, out: Optional[torch.Tensor], s
         _stream(), c_int(out_code), c_int(int(swiglu)), _ptr(a), c_int(lda), _ptr(w), c_int(ldw),
         _ptr(bias), _ptr(out) if fold is None else None, c_int(ldc), c_int(M), c_int(n_out), c_int(K),
         c_int(waves), _ptr(sp), c_int(n_parts), c_float(eps), c_int(size), _ptr(x), c_int(ldx),
-        _ptr(nw), _ptr(h), c_int(ldh), _ptr(op)))
+        _ptr(nw), _ptr(h), c_int(ldh), _ptr(op), *[c_float(v) for v in (limits or (0.0, 0.0, 0.0))]))
     return out
 
 
@@ -650,12 +673,15 @@ def mid_splits(w: torch.Tensor) -> int:
 
 
 def gemm_mid(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, swiglu: bool = False,
-             bias: Optional[torch.Tensor] = None):
+             bias: Optional[torch.Tensor] = None, limits: Optional[Sequence[float]] = None):
     """out = a @ w.T for at most 64 rows of bfloat16 ``a``, float32 accumulation. out is
     [m, n] (bfloat16 or float32) or, float32 only, [planes, m, n] whose planes add up to the
     product (``mid_splits`` planes at most; the bias is in plane 0). swiglu: w is [2*n, k]
-    (gate rows, up rows) and out [m, n] = silu(a @ gate.T) * (a @ up.T)."""
+    (gate rows, up rows) and out [m, n] = silu(a @ gate.T) * (a @ up.T); limits as in
+    ``gemm_skinny``."""
     _dev(a, "a", torch.bfloat16, contiguous=False); _dev(w, "w", torch.bfloat16, contiguous=False)
+    if limits is not None and not (swiglu and limits[0] > 0):
+        raise KernelError(f"gemm_mid: limits {tuple(limits)} belong to a gated activation")
     M, lda = _rows2d(a, "a"); N, ldw = _rows2d(w, "w")
     K = a.shape[1]
     n_out = N // 2 if swiglu else N
@@ -678,7 +704,8 @@ def gemm_mid(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, swiglu: bool =
             raise KernelError("gemm_mid: bias must hold one entry per row of w")
     _check(library().ta_gemm_mid_bf16(_stream(), c_int(_code(out.dtype)), c_int(int(swiglu)), _ptr(a),
                                       c_int(lda), _ptr(w), c_int(ldw), _ptr(bias), _ptr(out), c_int(ldc),
-                                      c_longlong(plane), c_int(M), c_int(n_out), c_int(K), c_int(planes)))
+                                      c_longlong(plane), c_int(M), c_int(n_out), c_int(K), c_int(planes),
+                                      *[c_float(v) for v in (limits or (0.0, 0.0, 0.0))]))
     return out
 
 
@@ -979,7 +1006,7 @@ def qk_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_dim: in
                v_first: Optional[torch.Tensor] = None, v_keep: Optional[torch.Tensor] = None,
                dest: Optional[torch.Tensor] = None, kcache: Optional[torch.Tensor] = None,
                vcache: Optional[torch.Tensor] = None, per_head: bool = False,
-               k_inplace: bool = False) -> torch.Tensor:
+               k_inplace: bool = False, unit_norm: bool = False, values_from_keys: bool = False) -> torch.Tensor:
     """On rows [q | k | v] of ``qkv`` (nh*dk, nkv*dk, nkv*dv columns): RMS norm of q and of k
     over all their heads at once (weights given: else none; ``per_head``: every head on its own,
     the weights then have the head's width and serve all heads), rotation of the first ``rot``
@@ -987,14 +1014,21 @@ def qk_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_dim: in
     q written back in place, k and v stored at ``dest`` into the cache layer. ``v_keep``
     receives the values before mixing. The cache's value rows may be wider than the values
     (vcache [pages, nkv, dvs, PAGE], dvs >= value_dim): the rest of a token's column is zeroed.
-    ``k_inplace`` (no ``dest``): the keys are written back into their rows as the queries are."""
+    ``k_inplace`` (no ``dest``): the keys are written back into their rows as the queries are.
+    ``unit_norm``: every head of q and k is divided by its root mean square, without weights.
+    ``values_from_keys``: rows are [q | k] and a head's values are its keys as projected."""
     _dev(qkv, "qkv", contiguous=False)
     nt, stride = _rows2d(qkv, "qkv")
     nq, nk, nv = num_heads * key_dim, num_kv_heads * key_dim, num_kv_heads * value_dim
-    if qkv.shape[1] != nq + nk + nv:
-        raise KernelError(f"qk_prepare: rows of {qkv.shape[1]}, expected {nq + nk + nv}")
-    normed = q_weight is not None
-    if normed:
+    cols = nq + nk if values_from_keys else nq + nk + nv
+    if qkv.shape[1] != cols:
+        raise KernelError(f"qk_prepare: rows of {qkv.shape[1]}, expected {cols}")
+    if values_from_keys and (value_dim != key_dim or k_inplace):
+        raise KernelError(f"qk_prepare: keys of {key_dim} do not serve as values of {value_dim}, or go back in place")
+    if unit_norm and q_weight is not None:
+        raise KernelError("qk_prepare: a norm has weights or none")
+    normed = q_weight is not None or unit_norm
+    if q_weight is not None:
         _dev(q_weight, "q_weight", torch.float32); _dev(k_weight, "k_weight", torch.float32)
         want = ((key_dim,), (key_dim,)) if per_head else ((nq,), (nk,))
         if (tuple(q_weight.shape), tuple(k_weight.shape)) != want:
@@ -1028,10 +1062,12 @@ def qk_prepare(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_dim: in
             raise KernelError("qk_prepare: dest must hold one entry per token")
     _check(library().ta_qk_prepare(
         _stream(), c_int(_code(qkv.dtype)), _ptr(qkv), c_int(stride), _ptr(q_weight), _ptr(k_weight),
-        c_float(eps), c_int(2 if normed and per_head else int(normed)), _ptr(angles), c_int(rot), _ptr(mix), _ptr(v_first), _ptr(v_keep),
+        c_float(eps), c_int(2 if normed and (per_head or unit_norm) else int(normed)), _ptr(angles), c_int(rot), _ptr(mix),
+        _ptr(v_first), _ptr(v_keep),
         _ptr(dest), _ptr(kcache if dest is not None else None), _ptr(vcache if dest is not None else None),
         c_int(nt), c_int(num_heads), c_int(num_kv_heads), c_int(key_dim), c_int(value_dim),
-        c_int(store_dim if dest is not None else value_dim), c_int(int(k_inplace))))
+        c_int(store_dim if dest is not None else value_dim), c_int(int(k_inplace)),
+        c_int(nq if values_from_keys else nq + nk)))
     return qkv
 
 
@@ -1246,6 +1282,32 @@ def postnorm_add(x: torch.Tensor, delta: torch.Tensor, weight: torch.Tensor, eps
     _check(library().ta_postnorm_add(_stream(), c_int(F32 if code is None else code), _ptr(x), _ptr(delta),
                                      c_int(planes), c_longlong(plane), _ptr(weight), c_float(eps), _ptr(xcast),
                                      _ptr(next_weight), c_float(next_eps), _ptr(out), c_int(nt), c_int(d)))
+    return x
+
+
+def stream_add(x: torch.Tensor, delta: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None,
+               xcast: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """x += delta + bias, float32 and in place; ``xcast`` receives the new rows in its own type. delta
+    [nt, d] or [planes, nt, d] float32 (planes added in order), bias float32 [d]."""
+    _dev(x, "x", torch.float32)
+    nt, d = x.shape
+    planes, plane = 1, 0
+    if delta is not None:
+        _dev(delta, "delta", torch.float32)
+        if delta.dim() == 3 and delta.shape[1:] == x.shape:
+            planes, plane = delta.shape[0], nt * d
+        elif delta.shape != x.shape:
+            raise KernelError(f"stream_add: delta is {tuple(delta.shape)}, x is {tuple(x.shape)}")
+    if bias is not None:
+        _dev(bias, "bias", torch.float32)
+        if bias.shape != (d,):
+            raise KernelError(f"stream_add: bias is {tuple(bias.shape)}, expected {(d,)}")
+    if xcast is not None:
+        _dev(xcast, "xcast")
+        if xcast.shape != x.shape:
+            raise KernelError(f"stream_add: xcast is {tuple(xcast.shape)}, x is {tuple(x.shape)}")
+    _check(library().ta_stream_add(_stream(), c_int(F32 if xcast is None else _code(xcast.dtype)), _ptr(x), _ptr(delta),
+                                   c_int(planes), c_longlong(plane), _ptr(bias), _ptr(xcast), c_int(nt), c_int(d)))
     return x
 
 
@@ -1468,16 +1530,16 @@ def latent_prepare(proj: torch.Tensor, q_rank: int, q_weight, cq, kv_offset: int
 def latent_query_rot(q: torch.Tensor, heads: int, nope: int, rot: int, rot_dims: int, angles, qa: torch.Tensor,
                      rank: int) -> torch.Tensor:
     """qa[t, h, rank:] = the last ``rot`` coordinates of head h of q[t], the first rot_dims of
-    them rotated, then zeros up to the rows' width. q [nt, H*(nope + rot)], qa [nt, H, >= rank + rot]."""
-    _dev(q, "q"); _dev(qa, "qa", q.dtype)
-    nt = q.shape[0]
+    them rotated, then zeros up to the rows' width. q [nt, H*(nope + rot)] (contiguous rows), qa [nt, H, >= rank + rot]."""
+    _dev(q, "q", contiguous=False); _dev(qa, "qa", q.dtype)
+    nt, qs = _rows2d(q, "q")
     if q.shape != (nt, heads * (nope + rot)) or qa.dim() != 3 or qa.shape[:2] != (nt, heads) or qa.shape[2] < rank + rot:
         raise KernelError(f"latent_query_rot: q {tuple(q.shape)} qa {tuple(qa.shape)}")
     if rot_dims:
         _dev(angles, "angles", torch.float32)
         if tuple(angles.shape) != (nt, rot_dims // 2, 2):
             raise KernelError(f"latent_query_rot: angles are {tuple(angles.shape)}")
-    _check(library().ta_latent_query_rot(_stream(), c_int(_code(q.dtype)), _ptr(q), c_int(heads), c_int(nope),
+    _check(library().ta_latent_query_rot(_stream(), c_int(_code(q.dtype)), _ptr(q), c_int(qs), c_int(heads), c_int(nope),
                                          c_int(rot), c_int(rot_dims), _ptr(angles if rot_dims else None), _ptr(qa),
                                          c_int(rank), c_int(qa.shape[2]), c_int(nt)))
     return qa
@@ -1511,11 +1573,11 @@ def latent_key_shares(batch: int, max_qlen: int, heads: int, rank: int, width: i
 
 def latent_attention(qa: torch.Tensor, out: torch.Tensor, kcache: torch.Tensor, block_table, cu_q, pos0,
                      max_qlen: int, rank: int, rot: int, scale: float, window=None, gate=None,
-                     shares: int = 1) -> torch.Tensor:
+                     shares: int = 1, sink: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Causal softmax attention of wide queries qa [nt, H, width] over cached rows kcache
     [pages, 1, PAGE, width] (width >= rank + rot, the rest zero); out [nt, H, rank] = weighted
     sums of the rows' first ``rank`` coordinates, times sigmoid(gate[t, h]) (gate [nt, >= H],
-    contiguous rows). bfloat16 rows of whole 16-byte pieces run on the matrix cores, where
+    contiguous rows). sink (float32 [H]): a row's denominator also holds exp(sink[h]). bfloat16 rows of whole 16-byte pieces run on the matrix cores, where
     ``shares`` waves divide a row's keys (``latent_key_shares``); all else on the vector ALU."""
     _dev(qa, "qa"); _dev(out, "out", qa.dtype); _dev(kcache, "kcache", qa.dtype)
     nt, H = qa.shape[0], qa.shape[1]
@@ -1533,6 +1595,10 @@ def latent_attention(qa: torch.Tensor, out: torch.Tensor, kcache: torch.Tensor, 
         ng, gs = _rows2d(gate, "gate")
         if ng != nt or gate.shape[1] < H:
             raise KernelError(f"latent_attention: gate is {tuple(gate.shape)}")
+    if sink is not None:
+        _dev(sink, "sink", torch.float32)
+        if sink.shape != (H,):
+            raise KernelError(f"latent_attention: sink is {tuple(sink.shape)}, expected {(H,)}")
     scratch = None
     if shares > 1:
         need = library().ta_latent_mfma_scratch
@@ -1546,7 +1612,7 @@ def latent_attention(qa: torch.Tensor, out: torch.Tensor, kcache: torch.Tensor, 
         _stream(), c_int(_code(qa.dtype)), _ptr(qa), _ptr(out), _ptr(kcache), _ptr(block_table),
         c_int(block_table.shape[1]), _ptr(cu_q), _ptr(pos0), c_int(B), c_int(max_qlen), c_int(H), c_int(rank),
         c_int(rot), c_int(width), c_float(scale), c_int(window or 0), _ptr(gate), c_int(gs), c_int(shares),
-        _ptr(scratch)))
+        _ptr(scratch), _ptr(sink)))
     return out
 
 
@@ -1728,13 +1794,14 @@ def qk_rotate_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_di
 
 def attention_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, num_heads, num_kv_heads, key_dim,
                    value_dim, scale, window=None, softcap: Optional[float] = None, sink=None,
-                   gate: Optional[torch.Tensor] = None, gate_dim: Optional[int] = None):
+                   gate: Optional[torch.Tensor] = None, gate_dim: Optional[int] = None, keep_first: int = 0):
     """``attention_generic_dv`` with the options of a capped, sunk and gated softmax. softcap: score <-
     softcap * tanh(score / softcap) after the scale. sink: None; "unit": the denominator holds one more
     term exp(0) = 1; a float32 tensor [heads]: one more term exp(sink[head]). gate: rows [nt, >= heads *
     value_dim] of q's type whose sigmoid multiplies the result element by element. gate_dim: columns per
     head of the gate's rows where that is less than value_dim (a cache whose value rows are padded): the
-    result's columns beyond it are not gated."""
+    result's columns beyond it are not gated; 0: the gate's rows [nt, >= heads] hold one number per head.
+    keep_first: with a window, that many first keys of a sequence are seen as well."""
     _dev(q, "q", contiguous=False); _dev(out, "out", q.dtype, contiguous=False)
     nt, qs = _rows2d(q, "q")
     nto, os_ = _rows2d(out, "out")
@@ -1749,16 +1816,23 @@ def attention_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, nu
     if cu_q.numel() != B + 1 or block_table.dim() != 2 or block_table.shape[0] != B:
         raise KernelError("attention: cu_q / pos0 / block_table disagree about the batch size")
     gd = value_dim if gate_dim is None else int(gate_dim)
-    if not 1 <= gd <= value_dim:
-        raise KernelError(f"attention: gate columns per head {gd} outside [1, {value_dim}]")
+    if not 0 <= gd <= value_dim:
+        raise KernelError(f"attention: gate columns per head {gd} outside [0, {value_dim}]")
     cap, mode, sink_t, gate, gs = _sink_args("attention", q, num_heads, gd, softcap, sink, gate)
     _check(library().ta_attention_generic_sink(
         _stream(), c_int(_code(q.dtype)), _ptr(q), c_int(qs), _ptr(out), c_int(os_), _ptr(kcache),
         _ptr(vcache), _ptr(block_table), c_int(block_table.shape[1]), _ptr(cu_q), _ptr(pos0),
         c_int(B), c_int(max_qlen), c_int(num_heads), c_int(num_kv_heads), c_int(key_dim),
         c_int(value_dim), c_float(scale), c_int(window or 0), c_float(cap), c_int(mode),
-        _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd)))
+        _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window))))
     return out
+
+
+def _kept(keep_first, window) -> int:
+    """First keys that a window shows besides its own: without a window every key is seen anyway."""
+    if keep_first < 0:
+        raise KernelError(f"attention: {keep_first} kept first keys")
+    return int(keep_first) if window else 0
 
 
 def _sink_args(what, q, num_heads, value_dim, softcap, sink, gate):
@@ -1777,7 +1851,7 @@ def _sink_args(what, q, num_heads, value_dim, softcap, sink, gate):
     if gate is not None:
         _dev(gate, "gate", q.dtype, contiguous=False)
         ng, gs = _rows2d(gate, "gate")
-        if ng != q.shape[0] or gate.shape[1] < num_heads * value_dim:
+        if ng != q.shape[0] or gate.shape[1] < num_heads * max(value_dim, 1):
             raise KernelError(f"{what}: gate rows are {tuple(gate.shape)}")
     if softcap is not None and not softcap > 0:
         raise KernelError(f"{what}: a cap must be positive, got {softcap}")
@@ -1786,10 +1860,10 @@ def _sink_args(what, q, num_heads, value_dim, softcap, sink, gate):
 
 def attention_rows_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, num_heads, num_kv_heads,
                         head_dim, scale, window=None, softcap=None, sink=None, gate=None, gate_dim=None,
-                        exact=True, through_lds=None):
+                        exact=True, through_lds=None, keep_first=0):
     """``attention_rows`` (matrix cores, bfloat16, values as wide as the keys) with the options of
     ``attention_sink``. gate_dim: columns per head of the gate's rows (the values' own width where the
-    cache pads them to the keys'); out's columns beyond it are not gated. exact: the softmax weights
+    cache pads them to the keys'; 0: one number per head); out's columns beyond it are not gated. exact: the softmax weights
     enter the second product as three bfloat16 pieces, so they keep 32 bits. through_lds 0 or 1 (None:
     1 from 256 rows on)."""
     if through_lds is None:
@@ -1803,13 +1877,13 @@ def attention_rows_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qle
         _ptr(block_table), c_int(block_table.shape[1]), _ptr(cu_q), _ptr(pos0), c_int(B),
         c_int(max_qlen), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_float(scale),
         c_int(window or 0), c_int(int(through_lds)), c_float(cap), c_int(int(exact)), c_int(mode), _ptr(sink_t),
-        _ptr(gate), c_int(gs), c_int(gd)))
+        _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window))))
     return out
 
 
 def attention_keys_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_kv_len, num_heads, num_kv_heads,
                         head_dim, scale, window=None, softcap=None, sink=None, gate=None, gate_dim=None,
-                        exact=True, units=None, seq_units=None):
+                        exact=True, units=None, seq_units=None, keep_first=0):
     """``attention_keys`` (single tokens on the matrix cores; q holds rotated heads, the cache the step's
     keys and values) with the options of ``attention_rows_sink``: the kernel whose four waves take a
     unit's pages in turn, and the merge, which adds the sink's share and applies the gate."""
@@ -1837,7 +1911,8 @@ def attention_keys_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_kv_
         _stream(), _ptr(q), c_int(qs), _ptr(out), c_int(os_), _ptr(kcache), _ptr(vcache), _ptr(block_table),
         c_int(block_table.shape[1]), _ptr(pos0), c_int(B), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim),
         c_float(scale), c_int(window or 0), _ptr(units), _ptr(seq_units), c_int(n_units), c_int(4), _ptr(scratch),
-        c_float(cap), c_int(int(exact)), c_int(mode), _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd)))
+        c_float(cap), c_int(int(exact)), c_int(mode), _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd),
+        c_int(_kept(keep_first, window))))
     return out
 
 
@@ -1996,4 +2071,98 @@ def weighted_sum(deltas: Sequence[torch.Tensor], scales: Sequence[float], out: t
     dp = (c_void_p * n)(*[t.data_ptr() for t in deltas])
     _check(library().ta_weighted_sum(_stream(), c_int(n), dp, (c_int * n)(*planes), (c_longlong * n)(*plane),
                                      (c_float * n)(*[float(v) for v in scales]), _ptr(out), c_int(nt), c_int(d)))
+    return out
+
+
+# ------------------------------------------------------------------ gated delta rule
+DELTA_MAX_KEY_DIM = 256
+
+
+def delta_prepare(qkv: torch.Tensor, z: torch.Tensor, dt_bias, a_log, b_raw: torch.Tensor, groups: int, heads: int,
+                  key_dim: int, q_scale: float, qn, kn, decay, beta, kq) -> None:
+    """What the delta rule needs of every token, float32: from rows [q | k | ...] of ``qkv`` (groups x
+    key_dim each, behind convolution and activation) unit vectors per group, qn = q_scale * q / |q| and
+    kn = k / |k| ([nt, groups, key_dim]; |x|^2 = sum of squares + 1e-6), and kq = kn . qn [nt, groups];
+    decay [nt, heads, key_dim] = exp(-exp(a_log[h]) * softplus(z + dt_bias)), z [nt, heads * key_dim];
+    beta [nt, heads] = sigmoid(b_raw)."""
+    _dev(qkv, "qkv", contiguous=False); _dev(z, "z", torch.float32); _dev(b_raw, "b_raw", qkv.dtype, contiguous=False)
+    nt, stride = _rows2d(qkv, "qkv")
+    nb, bs = _rows2d(b_raw, "b_raw")
+    G, H, dk = groups, heads, key_dim
+    for t, n, shape in ((dt_bias, "dt_bias", (H * dk,)), (a_log, "a_log", (H,)), (z, "z", (nt, H * dk)),
+                        (qn, "qn", (nt, G, dk)), (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H, dk)),
+                        (beta, "beta", (nt, H)), (kq, "kq", (nt, G))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"delta_prepare: {n} is {tuple(t.shape)}, expected {shape}")
+    if nb != nt or b_raw.shape[1] != H or qkv.shape[1] < 2 * G * dk or G < 1 or H % G:
+        raise KernelError(f"delta_prepare: qkv {tuple(qkv.shape)} / b_raw {tuple(b_raw.shape)} for {H} heads in {G} groups of {dk}")
+    _check(library().ta_delta_prepare(
+        _stream(), c_int(_code(qkv.dtype)), _ptr(qkv), c_int(stride), _ptr(z), _ptr(dt_bias), _ptr(a_log), _ptr(b_raw),
+        c_int(bs), c_int(nt), c_int(G), c_int(H), c_int(dk), c_float(q_scale), _ptr(qn), _ptr(kn), _ptr(decay),
+        _ptr(beta), _ptr(kq)))
+
+
+def delta_recurrent(qn: torch.Tensor, kn: torch.Tensor, decay: torch.Tensor, v: torch.Tensor, beta: torch.Tensor,
+                    kq: torch.Tensor, state: torch.Tensor, cu_q, slots, o_out: torch.Tensor, waves: int = 0) -> torch.Tensor:
+    """The delta rule along every sequence: S <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o =
+    S^T q, head h with the q and k of group h // (heads / groups). qn, kn [nt, G, dk], decay [nt, H, dk],
+    beta [nt, H], kq [nt, G] (k . q) float32; v [nt, H * dv] rows in the engine's type; ``state`` [slots, H,
+    dk, dv] float32; o_out [nt, H, dv] float32. waves of a workgroup: 2 or 4 (0: chosen by the shape)."""
+    nt, G, dk = qn.shape
+    H = decay.shape[1]
+    _dev(v, "v", contiguous=False); _dev(state, "state", torch.float32)
+    nv, vs = _rows2d(v, "v")
+    batch = _step_tables(cu_q, slots, nt, "delta_recurrent")
+    dv = state.shape[3] if state.dim() == 4 else -1
+    for t, n, shape in ((qn, "qn", (nt, G, dk)), (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H, dk)),
+                        (beta, "beta", (nt, H)), (kq, "kq", (nt, G)), (o_out, "o_out", (nt, H, dv))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"delta_recurrent: {n} is {tuple(t.shape)}, expected {shape}")
+    if nv != nt or v.shape[1] != H * dv or tuple(state.shape[1:3]) != (H, dk) or H % G:
+        raise KernelError(f"delta_recurrent: v {tuple(v.shape)} / state {tuple(state.shape)} for {H} heads in {G} groups")
+    if dk > DELTA_MAX_KEY_DIM:
+        raise KernelError(f"delta_recurrent: key widths up to {DELTA_MAX_KEY_DIM}, not {dk}")
+    _check(library().ta_delta_recurrent(
+        _stream(), c_int(_code(v.dtype)), _ptr(qn), _ptr(kn), _ptr(decay), _ptr(v), c_int(vs), _ptr(beta), _ptr(kq),
+        _ptr(state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(H), c_int(G), c_int(dk), c_int(dv),
+        c_int(waves), _ptr(o_out)))
+    return o_out
+
+
+def delta_step_fits(key_dim: int, value_dim: int, decay_rank: int, gate_rank: int) -> bool:
+    """Whether ``delta_step`` takes heads of this size."""
+    return bool(library().ta_delta_step_fits(c_int(key_dim), c_int(value_dim), c_int(decay_rank), c_int(gate_rank)))
+
+
+def delta_step(qkv: torch.Tensor, proj: torch.Tensor, a_off: int, g_off: int, b_off: int, decay_w, gate_w, dt_bias, a_log,
+               state: torch.Tensor, slots, heads: int, groups: int, q_scale: float, norm_w, eps: float,
+               out: torch.Tensor) -> torch.Tensor:
+    """A step of single tokens of the delta rule in one kernel (row b belongs to sequence b): qkv rows
+    [q | k | v] behind convolution and activation; the rows of ``proj`` hold the decay's low-rank input at
+    column a_off, the output gate's at g_off and the step sizes' at b_off; decay_w [H*dk, ra], gate_w
+    [H*dv, rg]. out [batch, H*dv] = o / rms(o per head) * norm_w * sigmoid(gate)."""
+    _dev(qkv, "qkv", contiguous=False); _dev(proj, "proj", qkv.dtype, contiguous=False); _dev(out, "out", qkv.dtype)
+    B, stride = _rows2d(qkv, "qkv")
+    Bp, ps = _rows2d(proj, "proj")
+    _dev(state, "state", torch.float32); _dev(slots, "slots", torch.int32); _dev(decay_w, "decay_w"); _dev(gate_w, "gate_w")
+    if state.dim() != 4 or state.shape[1] != heads or decay_w.dtype != gate_w.dtype:
+        raise KernelError(f"delta_step: state {tuple(state.shape)} for {heads} heads, weights {decay_w.dtype} / {gate_w.dtype}")
+    dk, dv, H, G = state.shape[2], state.shape[3], heads, groups
+    ra, rg = decay_w.shape[1], gate_w.shape[1]
+    for t, n, shape in ((dt_bias, "dt_bias", (H * dk,)), (a_log, "a_log", (H,)), (norm_w, "norm_w", (dv,))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"delta_step: {n} is {tuple(t.shape)}, expected {shape}")
+    if Bp != B or slots.numel() != B or qkv.shape[1] != 2 * G * dk + H * dv or decay_w.shape[0] != H * dk or \
+            gate_w.shape[0] != H * dv or out.shape != (B, H * dv) or H % G or min(a_off, g_off, b_off) < 0 or \
+            max(a_off + ra, g_off + rg, b_off + H) > proj.shape[1]:
+        raise KernelError(f"delta_step: qkv {tuple(qkv.shape)} proj {tuple(proj.shape)} out {tuple(out.shape)} for {H} "
+                          f"heads in {G} groups of {dk} / {dv}, ranks {ra} / {rg}")
+    _check(library().ta_delta_step(
+        _stream(), c_int(_code(qkv.dtype)), c_int(_wcode(decay_w, qkv.dtype, "delta_step")), _ptr(qkv), c_int(stride),
+        _ptr(proj), c_int(ps), c_int(a_off), c_int(ra), c_int(g_off), c_int(rg), c_int(b_off), _ptr(decay_w), _ptr(gate_w),
+        _ptr(dt_bias), _ptr(a_log), _ptr(state), _ptr(slots), c_int(B), c_int(H), c_int(G), c_int(dk), c_int(dv),
+        c_float(q_scale), _ptr(norm_w), c_float(eps), _ptr(out)))
     return out

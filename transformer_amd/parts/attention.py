@@ -20,22 +20,26 @@ from .. import kernels
 from ..cache.storage import KVNeed
 from ..weights.loader import Param
 from .base import Part, PartError, build_part, register_part
-from .linear import adds_in_place, linear, linear_delta
+from .linear import adds_in_place, aligned_rows, finish, linear, linear_delta
 
 
 @dataclass(frozen=True)
 class KeyUnitPlanner:
     """The work plan of the single-token attention kernels, made on the host with every step's
     tables: the sequences of the step cut into units of work of about equal length
-    (``kernels.plan_key_units``). Mixers with the same number of kv heads share one plan."""
+    (``kernels.plan_key_units``). Mixers with the same number of kv heads (and, where the plan leaves
+    out pages that no token of the step sees, the same window and kept first keys) share one plan."""
     num_kv_heads: int
+    window: int = 0
+    keep_first: int = 0
 
     def ints(self, batch: int) -> int:
         return kernels.UNIT_INTS * kernels.key_unit_count(batch, self.num_kv_heads) + 2 * batch
 
     def tables(self, kv_lens, block_table):
         units, seq_units = kernels.plan_key_units(
-            kv_lens, kernels.key_unit_count(len(kv_lens), self.num_kv_heads), tables=block_table)
+            kv_lens, kernels.key_unit_count(len(kv_lens), self.num_kv_heads), tables=block_table,
+            window=self.window or None, keep_first=self.keep_first)
         return {"units": units, "seq_units": seq_units}
 
 
@@ -251,12 +255,14 @@ class SinkAttention(Part):
     more term in the softmax denominator (``SinkAttentionSpec``).
 
     One merged product gives [q | k | v | gate] (k and v only where the layer has keys and values of
-    its own, the gate only where the heads are gated). Where the spec names a convolution, q, k and
+    its own, v only where it is not the key as projected, the gate only where the heads are gated,
+    element by element or with one number each). Where the spec names a convolution, q, k and
     v pass it channel by channel (``kernels.causal_conv``, which keeps a sequence's last projected
     rows between steps). ``kernels.qk_rotate_store`` adds the biases where there is no convolution to
     take them, turns q and k and writes k and v to the paged cache; ``kernels.attention_sink`` reads
     the cache with scores, cap, sink, softmax and sums in float32 and applies the heads' gate; the
-    output projection follows. A layer that borrows reads the lender's cache layer through its
+    output projection follows. Where the heads of q and k are normed or the values are the keys,
+    ``kernels.qk_prepare`` does norm, rotation and cache write instead. A layer that borrows reads the lender's cache layer through its
     schedule entry and declares the same need."""
     graph_safe = True
 
@@ -264,7 +270,8 @@ class SinkAttention(Part):
         s = spec
         if s.num_heads % s.num_kv_heads:
             raise PartError(f"{s.num_heads} heads do not divide into {s.num_kv_heads} kv heads")
-        if not (2 <= s.key_dim <= 256 and s.key_dim % 2 == 0 and 1 <= s.value_dim <= 256):
+        odd_ok = s.unit_norm or s.values_from_keys
+        if not (1 <= s.key_dim <= 256 and (odd_ok or s.key_dim % 2 == 0) and 1 <= s.value_dim <= 256):
             raise PartError(f"attention takes even key widths and value widths in [1, 256], not {s.key_dim} / {s.value_dim}")
         if s.rot_dims % 2 or not 0 <= s.rot_dims <= s.key_dim or s.rot_style not in ("half", "interleaved"):
             raise PartError(f"{s.rot_dims} rotated coordinates ({s.rot_style!r}) do not fit heads of {s.key_dim}")
@@ -279,10 +286,24 @@ class SinkAttention(Part):
             raise PartError(f"a score cap must be positive, got {s.softcap}")
         if s.conv_taps < 0 or (s.conv_taps and not s.own_kv):
             raise PartError("a convolution on q, k and v needs keys and values of the layer's own")
+        if s.keep_first < 0 or (s.keep_first and s.window is None):
+            raise PartError(f"{s.keep_first} kept first keys need a window beside them")
+        # q and k normed per head, or values that are the keys: the kernel that prepares such rows
+        self.prepared = s.unit_norm or s.values_from_keys
+        if self.prepared and (not s.own_kv or s.qkv_bias or s.conv_taps or
+                              (s.rot_dims and s.rot_style != "half")):
+            raise PartError("normed heads, or values that are keys, go without biases, convolutions, borrowed keys, "
+                            "and with a rotation in halves at most")
+        if s.values_from_keys and s.value_dim != s.key_dim:
+            raise PartError(f"keys of {s.key_dim} do not serve as values of {s.value_dim}")
+        if s.out_gate and s.head_gate:
+            raise PartError("the heads are gated element by element or with one number each, not both")
         self.spec, self.dtype = s, dtype
         self.nq, self.nkv, self.dk, self.dv = s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim
-        self.qkv_width = self.nq * self.dk + (self.nkv * (self.dk + self.dv) if s.own_kv else 0)
-        self.width = self.qkv_width + (self.nq * self.dv if s.out_gate else 0)
+        own = self.nkv * (self.dk + (0 if s.values_from_keys else self.dv)) if s.own_kv else 0
+        self.qkv_width = self.nq * self.dk + own
+        self.gate_dim = self.dv if s.out_gate else 0                # gate columns per head (0: one number)
+        self.width = self.qkv_width + (self.nq * self.dv if s.out_gate else self.nq if s.head_gate else 0)
         self.rotary = None
         if s.rot_dims:
             from ..config.spec import PositionSpec
@@ -311,13 +332,14 @@ class SinkAttention(Part):
         return self.dtype == torch.bfloat16 and self.dk % 32 == 0 and 32 <= self.dk <= 256 and self.dv <= self.dk
 
     def _on_matrix_cores(self) -> bool:
-        # ... and rows of q that start on 16 bytes; a layer whose rows do not reads the padded cache
-        # through the vector-ALU kernel
-        return self._pads_values() and self.width % 8 == 0 and self.qkv_width % 8 == 0
+        # ... and rows of q that start on 16 bytes (the projection's rows do, whatever their width; those
+        # of a convolution's result have the width of q, k and v); a layer whose rows do not reads the
+        # padded cache through the vector-ALU kernel
+        return self._pads_values() and (self.spec.conv_taps == 0 or self.qkv_width % 8 == 0)
 
     def step_planner(self):
         if self._on_matrix_cores() and kernels.keys_sink_fits(self.nq, self.nkv, self.dk):
-            return KeyUnitPlanner(self.nkv)
+            return KeyUnitPlanner(self.nkv, self._cache_window() or 0, self.spec.keep_first)
         return None
 
     def bind(self, tensors):
@@ -329,11 +351,14 @@ class SinkAttention(Part):
             wide[:, :, :self.dv] = w.view(w.shape[0], self.nq, self.dv)
             self.out_wide = wide.view(w.shape[0], self.nq * self.dk)
 
+    def _cache_window(self):
+        # cache_window None: the layer's own window; 0: every token is kept; else that many
+        s = self.spec
+        return s.window if s.cache_window is None else (s.cache_window or None)
+
     def cache_need(self):
         s = self.spec
-        # cache_window None: the layer's own window; 0: every token is kept; else that many
-        window = s.window if s.cache_window is None else (s.cache_window or None)
-        kv = KVNeed(self.nkv, self.dk, window, self.dk if self._pads_values() else self.dv)
+        kv = KVNeed(self.nkv, self.dk, self._cache_window(), self.dk if self._pads_values() else self.dv, s.keep_first)
         if s.conv_taps > 1:
             from ..cache.storage import StateNeed
             return [kv, StateNeed((s.conv_taps - 1, self.qkv_width), torch.float32)]
@@ -344,11 +369,19 @@ class SinkAttention(Part):
         w = self.out_wide if getattr(self, "out_wide", None) is not None else self.w["out.weight"]
         return adds_in_place(nt, w)
 
-    def run(self, h, ctx, cache, layer, writes_cache=True, into=None):
+    # single-token steps: the norm in front and the norm behind ride on the products (``PreNormBlock``)
+    def takes_scaled(self, nt: int) -> bool:
+        return kernels.skinny_takes(nt, self.w["in.weight"])
+
+    def can_fold(self, nt: int) -> bool:
+        w = self.out_wide if getattr(self, "out_wide", None) is not None else self.w["out.weight"]
+        return kernels.skinny_folds(nt, w)
+
+    def run(self, h, ctx, cache, layer, writes_cache=True, scale=None, fold=None, into=None):
         s, nt = self.spec, h.shape[0]
         if not s.own_kv and writes_cache:
             raise PartError("a layer without keys and values of its own runs on another layer's cache")
-        proj = linear(h, self.w["in.weight"], ctx.ws.take("attention.in", (nt, self.width), self.dtype))
+        proj = linear(h, self.w["in.weight"], aligned_rows(ctx.ws, "attention.in", nt, self.width, self.dtype), scale=scale)
         kv_layer = layer[0] if isinstance(layer, (list, tuple)) else layer
         kc, vc, group = cache.layer_kv(kv_layer)
         meta = ctx.kv[group]
@@ -362,17 +395,23 @@ class SinkAttention(Part):
         else:
             qkv = proj[:, :self.qkv_width]
         angles = self.rotary.angles(ctx) if self.rotary is not None else None
-        kernels.qk_rotate_store(qkv, self.nq, self.nkv, self.dk, self.dv, s.own_kv, bias, angles, s.rot_dims,
-                                s.rot_style, meta.dest if (writes_cache and s.own_kv) else None, kc, vc)
+        if self.prepared:
+            kernels.qk_prepare(qkv, self.nq, self.nkv, self.dk, self.dv, float(s.eps), None, None, angles, s.rot_dims,
+                               dest=meta.dest if writes_cache else None, kcache=kc, vcache=vc, unit_norm=s.unit_norm,
+                               values_from_keys=s.values_from_keys)
+        else:
+            kernels.qk_rotate_store(qkv, self.nq, self.nkv, self.dk, self.dv, s.own_kv, bias, angles, s.rot_dims,
+                                    s.rot_style, meta.dest if (writes_cache and s.own_kv) else None, kc, vc)
         sink = self.w["sink"] if s.sink == "learned" else s.sink
-        gate = proj[:, self.qkv_width:] if s.out_gate else None
+        gate = proj[:, self.qkv_width:] if s.out_gate or s.head_gate else None
         w = self.out_wide if self.out_wide is not None else self.w["out.weight"]
         if not self._on_matrix_cores():
             vd = self.dk if self._pads_values() else self.dv          # the width of the cache's value rows
             o = ctx.ws.take("attention.o", (nt, self.nq * vd), self.dtype)
             kernels.attention_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_qlen, self.nq,
-                                   self.nkv, self.dk, vd, float(s.scale), s.window, s.softcap, sink, gate, self.dv)
-            return linear_delta(o, w, ctx.ws, "attention.delta", into=into), None
+                                   self.nkv, self.dk, vd, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
+                                   keep_first=s.keep_first)
+            return finish(o, w, ctx.ws, "attention.delta", fold, into)
         # matrix cores: scores and sums in float32, the softmax weights kept at 32 bits by three pieces
         o = ctx.ws.take("attention.o", (nt, self.nq * self.dk), self.dtype)
         planner = self.step_planner()
@@ -381,12 +420,13 @@ class SinkAttention(Part):
         plan = meta.plans.get(planner) if planner is not None else None
         if ctx.all_single and plan:
             kernels.attention_keys_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_kv_len, self.nq,
-                                        self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.dv,
-                                        units=plan.get("units"), seq_units=plan.get("seq_units"))
+                                        self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
+                                        keep_first=s.keep_first, units=plan.get("units"), seq_units=plan.get("seq_units"))
         else:
             kernels.attention_rows_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_qlen, self.nq,
-                                        self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.dv)
-        return linear_delta(o, w, ctx.ws, "attention.delta", into=into), None
+                                        self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
+                                        keep_first=s.keep_first)
+        return finish(o, w, ctx.ws, "attention.delta", fold, into)
 
 
 register_part("attention_sink", SinkAttention)

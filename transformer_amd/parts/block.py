@@ -3,7 +3,9 @@
 "prenorm": x += mixer(norm1(x)); x += ffn(norm2(x)), the reference's block
 (models/llama/common/src/compute.rs:204-292). The adds are
 carried as a pending (delta, bias) pair and folded into the next norm, so the
-float32 residual stream is read and written once per norm.
+float32 residual stream is read and written once per norm. A block may end in a part
+that reads the stream itself (``BlockSpec.side``): the last add then happens in
+front of it, and the part's own last kernel applies the next block's norm.
 """
 from __future__ import annotations
 
@@ -21,11 +23,15 @@ class PreNormBlock(Part):
         # a block without a feed-forward has the mixer's sublayer only
         self.ffn = build_part(spec.ffn, dtype, device) if spec.ffn is not None else None
         self.norm2 = build_part(spec.norm2, dtype, device) if spec.ffn is not None else None
+        self.side = build_part(spec.side, dtype, device) if getattr(spec, "side", None) is not None else None
+        self._ones = None
 
     def children(self):
         c = {"norm1": self.norm1, "mixer": self.mixer}
         if self.ffn is not None:
             c.update(norm2=self.norm2, ffn=self.ffn)
+        if self.side is not None:
+            c["side"] = self.side
         return c
 
     def cache_need(self):
@@ -63,21 +69,51 @@ class PreNormBlock(Part):
             return None
         return self.norm1.fold(x, ctx.ws.take("block.h", x.shape, self.dtype), ctx)
 
+    def entry_norm(self):
+        """The norm that reads the stream first, for a block in front that applies it in its last
+        add; None where it is of another kind."""
+        return self.norm1 if hasattr(self.norm1, "gain") and hasattr(self.norm1, "eps") else None
+
+    def _cast_fold(self, x, xcast, ctx):
+        """For the product in front of the side part: it adds itself to the stream and leaves the new
+        rows, unweighted, in the engine's type (a norm's fold with a weight of ones)."""
+        if self._ones is None:
+            self._ones = torch.ones(x.shape[1], dtype=torch.float32, device=x.device)
+        parts = ctx.ws.take("block.castparts", kernels.NormFold.parts_shape(x.shape[1]), torch.float32)
+        return kernels.NormFold(x, self._ones, 0.0, xcast, parts)
+
+    def _run_side(self, x, xcast, ctx, after, h):
+        follow = getattr(after, "entry_norm", None)
+        follow = follow() if follow is not None else None
+        with span(ctx, "side"):
+            self.side.run(x, xcast, ctx, next_norm=follow, out=None if follow is None else h)
+        return "normed" if follow is not None else (None, None)
+
     def run(self, x, pending, ctx, cache, layer, writes_cache=True, after=None):
         """x: float32 residual stream [nt, hidden]; pending: (delta, bias) not yet added to
-        x, (None, None), or the ``RowScale`` of an ``entry_fold`` that the block in front has
-        served. after: the block that runs next, if any. Returns the new pending."""
+        x, (None, None), the ``RowScale`` of an ``entry_fold`` that the block in front has
+        served, or "normed" (it has left norm1's rows in the shared buffer). after: the block that
+        runs next, if any. Returns the new pending."""
         nt = x.shape[0]
         h = ctx.ws.take("block.h", x.shape, self.dtype)
         kw = {}
         if isinstance(pending, kernels.RowScale):
             kw["scale"] = pending                  # h already holds the rows, not yet scaled
-        else:
+        elif not (isinstance(pending, str) and pending == "normed"):
             with span(ctx, "norm"):
                 self.norm1.run(x, h, pending[0], pending[1])
+        # the rows that the side part reads: the stream itself where the engine computes in float32
+        xcast = None
+        if self.side is not None:
+            xcast = x if self.dtype == torch.float32 else ctx.ws.take("block.xcast", x.shape, self.dtype)
         if self.ffn is None:
             with span(ctx, "mixer"):
-                return self.mixer.run(h, ctx, cache, layer, writes_cache, **kw)
+                pending = self.mixer.run(h, ctx, cache, layer, writes_cache, **kw)
+            if self.side is None:
+                return pending
+            with span(ctx, "norm"):
+                kernels.stream_add(x, pending[0], pending[1], None if xcast is x else xcast)
+            return self._run_side(x, xcast, ctx, after, h)
         fusable = self._fusable(nt)
         if (fusable and hasattr(self.norm2, "fold") and self._offers(self.mixer, "can_fold", nt)
                 and self._offers(self.ffn, "takes_scaled", nt)):
@@ -94,6 +130,18 @@ class PreNormBlock(Part):
         else:
             with span(ctx, "norm"):
                 self.norm2.run(x, h, pending[0], pending[1])
+        if self.side is not None:
+            if fusable and self._offers(self.ffn, "can_fold", nt):
+                with span(ctx, "ffn"):
+                    self.ffn.run(h, ctx, fold=self._cast_fold(x, xcast, ctx), **kw2)
+            else:
+                if self._offers(self.ffn, "can_add", nt):
+                    kw2["into"] = x
+                with span(ctx, "ffn"):
+                    pending = self.ffn.run(h, ctx, **kw2)
+                with span(ctx, "norm"):
+                    kernels.stream_add(x, pending[0], pending[1], None if xcast is x else xcast)
+            return self._run_side(x, xcast, ctx, after, h)
         handover = None
         if fusable and after is not None and self._offers(self.ffn, "can_fold", nt):
             entry = getattr(after, "entry_fold", None)

@@ -17,6 +17,7 @@ from .linear import adds_in_place, linear, linear_delta
 
 class SwiGLU(Part):
     graph_safe = True
+    limits = None           # (limit, slope, shift) of the limited activation; None: silu(gate) * up
 
     def __init__(self, spec, dtype, device):
         self.spec, self.dtype = spec, dtype
@@ -49,15 +50,19 @@ class SwiGLU(Part):
         if scale is not None or kernels.skinny_wins(h, self.w["gate_up.weight"]):
             # few rows: the product applies the activation itself and [nt, 2*di] is never stored
             kernels.gemm_skinny(h, self.w["gate_up.weight"], act, swiglu=True,
-                                bias=self.w.get("gate_up.bias"), scale=scale)
+                                bias=self.w.get("gate_up.bias"), scale=scale, limits=self.limits)
         elif h.dtype == torch.bfloat16 and kernels.mid_takes(nt, self.w["gate_up.weight"]):
             # up to 64 rows the product of our own applies the activation itself: 44 to 54 us on
             # the 8B shape where the vendor library's product and the activation's kernel take 55
-            kernels.gemm_mid(h, self.w["gate_up.weight"], act, swiglu=True, bias=self.w.get("gate_up.bias"))
+            kernels.gemm_mid(h, self.w["gate_up.weight"], act, swiglu=True, bias=self.w.get("gate_up.bias"),
+                             limits=self.limits)
         else:
             gu = linear(h, self.w["gate_up.weight"],
                         ctx.ws.take("swiglu.gate_up", (nt, 2 * s.intermediate), self.dtype))
-            kernels.swiglu(gu, act, self.w.get("gate_up.bias"))
+            if self.limits is None:
+                kernels.swiglu(gu, act, self.w.get("gate_up.bias"))
+            else:
+                kernels.glu_limit(gu, act, *self.limits)
         if fold is not None:
             kernels.gemm_skinny(act, self.w["down.weight"], None, bias=self.w.get("down.bias"), fold=fold)
             return None
@@ -66,21 +71,27 @@ class SwiGLU(Part):
 
 
 class GLU(SwiGLU):
-    """The same feed-forward with the activation as a parameter of the spec ("silu",
-    "gelu_tanh"). Silu takes every path of ``SwiGLU`` (the products that apply it themselves
-    included); another activation runs the product and then the activation's kernel."""
+    """The same feed-forward with the activation as a parameter of the spec ("silu", "gelu_tanh",
+    "limited"). Silu and the limited form take every path of ``SwiGLU`` (the products that apply it
+    themselves included); another activation runs the product and then the activation's kernel."""
 
     def __init__(self, spec, dtype, device):
         super().__init__(spec, dtype, device)
-        if spec.activation not in ("silu", "gelu_tanh"):
+        if spec.activation not in ("silu", "gelu_tanh", "limited"):
             raise PartError(f"unknown feed-forward activation {spec.activation!r}")
         self.activation = spec.activation
+        if spec.activation == "limited":
+            if not spec.limit > 0:
+                raise PartError(f"a limited feed-forward needs a positive limit, got {spec.limit}")
+            if spec.bias:
+                raise PartError("a limited feed-forward has no biases")
+            self.limits = (float(spec.limit), float(spec.gate_slope), float(spec.up_shift))
 
     def takes_scaled(self, nt: int) -> bool:
-        return self.activation == "silu" and super().takes_scaled(nt)
+        return self.activation in ("silu", "limited") and super().takes_scaled(nt)
 
     def run(self, h, ctx, scale=None, fold=None, into=None):
-        if self.activation == "silu":
+        if self.activation in ("silu", "limited"):
             return super().run(h, ctx, scale=scale, fold=fold, into=into)
         s, nt = self.spec, h.shape[0]
         gu = linear(h, self.w["gate_up.weight"],

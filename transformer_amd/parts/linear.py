@@ -137,3 +137,19 @@ def linear_delta(x: torch.Tensor, weight: torch.Tensor, ws: Workspace, name: str
                   out_dtype=torch.float32, out=out)
         return out
     return linear(x, weight, ws.take(name, (nt, n), torch.float32))
+
+
+def finish(x: torch.Tensor, weight: torch.Tensor, ws: Workspace, name: str, fold=None,
+           into: Optional[torch.Tensor] = None):
+    """A mixer's last product: what its ``run`` returns, (delta, None); None with ``fold``, which has
+    then taken the result; (None, None) with ``into``, the residual stream it has then joined."""
+    if fold is not None:
+        kernels.gemm_skinny(x, weight, None, fold=fold)
+        return None
+    return linear_delta(x, weight, ws, name, into=into), None
+
+
+def aligned_rows(ws: Workspace, name: str, rows: int, width: int, dtype: torch.dtype) -> torch.Tensor:
+    """[rows, width] whose rows start on 16 bytes whatever the width."""
+    piece = 16 // torch.empty((), dtype=dtype).element_size()
+    return ws.take(name, (rows, -(-width // piece) * piece), dtype)[:, :width]

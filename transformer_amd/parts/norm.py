@@ -67,5 +67,21 @@ class ScalarRMSNorm(RMSNorm):
         return self._gain
 
 
+class OffsetRMSNorm(RMSNorm):
+    """The same norm with a weight stored around zero: the gain is 1 + w, formed in float32 once, when
+    the weights are bound."""
+
+    def params(self):
+        return {"weight": Param((self.size,), "vector")}
+
+    def bind(self, tensors):
+        super().bind(tensors)
+        self._gain = (tensors["weight"].to(torch.float32) + 1.0).contiguous()
+
+    def gain(self):
+        return self._gain
+
+
+register_part("rmsnorm_offset", OffsetRMSNorm)
 register_part("rmsnorm", RMSNorm)
 register_part("rmsnorm_scalar", ScalarRMSNorm)

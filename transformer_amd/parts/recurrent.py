@@ -15,7 +15,7 @@ from .. import kernels
 from ..cache.storage import StateNeed
 from ..weights.loader import Param
 from .base import Part, PartError, register_part
-from .linear import linear, linear_delta
+from .linear import adds_in_place, aligned_rows, finish, linear, linear_delta
 
 
 class DiagonalRecurrence(Part):
@@ -301,6 +301,99 @@ class StateSpace(Part):
         return linear_delta(y, self.w["out.weight"], ctx.ws, "state_space.delta"), None
 
 
+class GatedDelta(Part):
+    """The gated delta rule with a decay per head and key channel (``GatedDeltaSpec``).
+
+    One product gives [q | k | v | decay input | gate input | step sizes]; ``kernels.causal_conv`` runs the
+    convolution with silu over [q | k | v] (its memory is the second piece of state). A step of single
+    tokens then takes ONE kernel to the normed and gated readout (``kernels.delta_step``); longer steps
+    form the two low-rank products, ``kernels.delta_prepare`` makes unit vectors, decays and step sizes of
+    all tokens, ``kernels.delta_recurrent`` walks them, and the head norm with its gate follows. State,
+    decays, step sizes, unit vectors and readout stay float32."""
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        s = spec
+        if min(s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim, s.taps, s.decay_rank, s.gate_rank) < 1 \
+                or s.num_heads % s.num_kv_heads:
+            raise PartError(f"delta rule: {s.num_heads} heads of {s.key_dim} / {s.value_dim} in {s.num_kv_heads} groups, "
+                            f"{s.taps} taps, ranks {s.decay_rank} / {s.gate_rank}")
+        if s.key_dim > kernels.DELTA_MAX_KEY_DIM:
+            raise PartError(f"delta rule: key widths up to {kernels.DELTA_MAX_KEY_DIM}, not {s.key_dim}")
+        self.spec, self.dtype = s, dtype
+        self.nk, self.nv = s.num_kv_heads * s.key_dim, s.num_heads * s.value_dim
+        self.conv_width = 2 * self.nk + self.nv
+        self.a_off = self.conv_width
+        self.g_off = self.a_off + s.decay_rank
+        self.b_off = self.g_off + s.gate_rank
+        self.width = self.b_off + s.num_heads
+
+    def params(self):
+        s = self.spec
+        H = s.num_heads
+        return {"in.weight": Param((self.width, s.hidden), "matrix"),     # q, k, v, decay input, gate input, step sizes
+                "conv.weight": Param((self.conv_width, s.taps), "vector"),
+                "decay.weight": Param((H * s.key_dim, s.decay_rank), "matrix"),
+                "gate.weight": Param((self.nv, s.gate_rank), "matrix"),
+                "dt_bias": Param((H * s.key_dim,), "vector", init="zero"),
+                "A_log": Param((H,), "vector", init="zero"),
+                "norm.weight": Param((s.value_dim,), "vector", init="around_one"),
+                "out.weight": Param((s.hidden, self.nv), "matrix")}
+
+    def cache_need(self):
+        s = self.spec
+        need = [StateNeed((s.num_heads, s.key_dim, s.value_dim), torch.float32)]
+        if s.taps > 1:
+            need.append(StateNeed((s.taps - 1, self.conv_width), torch.float32))
+        return need
+
+    # with many rows the output projection can add itself to the residual stream (``into``); in
+    # single-token steps the norms around the mixer ride on its products (``PreNormBlock``)
+    def can_add(self, nt: int) -> bool:
+        return adds_in_place(nt, self.w["out.weight"])
+
+    def takes_scaled(self, nt: int) -> bool:
+        return kernels.skinny_takes(nt, self.w["in.weight"])
+
+    def can_fold(self, nt: int) -> bool:
+        return kernels.skinny_folds(nt, self.w["out.weight"])
+
+    def _low_rank(self, x, weight, out):
+        # rows that do not start and end on 16 bytes go to the framework's own product
+        if x.dtype == torch.bfloat16 and (x.data_ptr() % 16 or x.stride(0) % 8 or x.shape[1] % 8):
+            return kernels.gemm_simple(x, weight, out)
+        return linear(x, weight, out)
+
+    def run(self, h, ctx, cache, layer, writes_cache=True, scale=None, fold=None, into=None):
+        s, nt = self.spec, h.shape[0]
+        H, G, dk, dv = s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim
+        take, f32 = ctx.ws.take, torch.float32
+        state = cache.layer_state(layer[0])
+        proj = linear(h, self.w["in.weight"], aligned_rows(ctx.ws, "delta.in", nt, self.width, self.dtype), scale=scale)
+        qkv = take("delta.qkv", (nt, self.conv_width), self.dtype)
+        kernels.causal_conv(proj, 0, self.conv_width, self.w["conv.weight"], qkv,
+                            cache.layer_state(layer[1]) if s.taps > 1 else None, ctx.cu_q, ctx.slots, ctx.max_qlen,
+                            activation="silu")
+        y = take("delta.y", (nt, self.nv), self.dtype)
+        q_scale = float(dk) ** -0.5
+        if ctx.all_single and kernels.delta_step_fits(dk, dv, s.decay_rank, s.gate_rank):
+            kernels.delta_step(qkv, proj, self.a_off, self.g_off, self.b_off, self.w["decay.weight"], self.w["gate.weight"],
+                               self.w["dt_bias"], self.w["A_log"], state, ctx.slots, H, G, q_scale, self.w["norm.weight"],
+                               float(s.eps), y)
+            return finish(y, self.w["out.weight"], ctx.ws, "delta.delta", fold, into)
+        z = self._low_rank(proj[:, self.a_off:self.g_off], self.w["decay.weight"], take("delta.z", (nt, H * dk), f32))
+        gate = self._low_rank(proj[:, self.g_off:self.b_off], self.w["gate.weight"], take("delta.gate", (nt, self.nv), self.dtype))
+        qn, kn = take("delta.qn", (nt, G, dk), f32), take("delta.kn", (nt, G, dk), f32)
+        decay, beta, kq = take("delta.decay", (nt, H, dk), f32), take("delta.beta", (nt, H), f32), take("delta.kq", (nt, G), f32)
+        kernels.delta_prepare(qkv, z, self.w["dt_bias"], self.w["A_log"], proj[:, self.b_off:self.width], G, H, dk, q_scale,
+                              qn, kn, decay, beta, kq)
+        o = kernels.delta_recurrent(qn, kn, decay, qkv[:, 2 * self.nk:], beta, kq, state, ctx.cu_q, ctx.slots,
+                                    take("delta.o", (nt, H, dv), f32))
+        kernels.head_norm_gate(o.unsqueeze(0), gate, H, dv, self.w["norm.weight"], float(s.eps), y, "sigmoid")
+        return finish(y, self.w["out.weight"], ctx.ws, "delta.delta", fold, into)
+
+
+register_part("gated_delta", GatedDelta)
 register_part("state_space", StateSpace)
 register_part("diagonal_recurrence", DiagonalRecurrence)
 register_part("decay_linear_attention", DecayLinearAttention)
