@@ -304,6 +304,50 @@ def saredra_shapes():
             "w4096": shape(4096, 32, 8, 128, 64, 6, 1408, 14336, 32000)}
 
 
+def zirutar_shapes():
+    """Layer sizes that resemble real models' (random weights): Zirutar models whose layers are all
+    attention, all latent attention or all delta rule (each with the limited feed-forward and the
+    token input), the mixed order, and the closest layers of the other decoders at the same width and
+    heads: the Saredra decoder's windowed attention, the Kunitar decoder's latent attention, the Vametar
+    decoder's gated linear attention, and the Llama layer."""
+    def shape(width, heads, kv, q_rank, rank, window, keep, low, ff, vocab):
+        mlp = {"kind": "dense", "ff": ff, "limit": 7.0}
+        dense = {"kind": "dense", "ff": ff}
+        att = {"type": "attention", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 2.0,
+                                                          "mask": {"size": window, "keep_first": keep}}}
+        latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": rank, "scale": 192 ** -0.5,
+                  "rot": {"base": 500000.0, "dims": 64}}
+        lat = {"type": "latent_attention", "mixer": latent, "mlp": mlp}
+        delta = {"type": "channel_delta", "mlp": mlp, "mixer": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4,
+                                                               "decay_rank": low, "gate_rank": low}}
+        base = {"architecture": "Zirutar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "embedding": {"scale": 2.0},
+                "logit_scale": 0.5, "token_side": {"dim": 64}}
+        kinds = {"attention": [att] * 4, "latent": [lat] * 4, "delta": [delta] * 4, "mixed": [att, delta, lat, att]}
+        near = {
+            "saredra_attention": ("Saredra", {"architecture": "Saredra", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+                                              "layers": [{"type": "attention", "mlp": dense, "mixer": {
+                                                  "heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+                                                  "mask": {"size": window}, "rot": {"base": 500000.0, "dims": 64}}}] * 4}),
+            "kunitar_latent": ("Kunitar", {"architecture": "Kunitar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+                                           "embedding": {"scale": 2.0}, "token_side": {"dim": 64},
+                                           "layers": [{"type": "latent_attention", "mixer": {**latent, "q_rank": q_rank},
+                                                       "mlp": dense}] * 4}),
+            "vametar_gla": ("Vametar", {"architecture": "Vametar", "vocab": vocab, "width": width, "norm": {"eps": 1e-5},
+                                        "residual_mult": 0.7, "logit_scale": 2.0,
+                                        "embedding": {"bigram": {"buckets": 65521, "mul_prev": 31, "mul_cur": 7}},
+                                        "layers": [{"type": "gla", "mlp": dense, "mixer": {
+                                            "heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "rank": low}}] * 4}),
+            "llama": ("llama", {"architectures": ["LlamaForCausalLM"], "model_type": "llama", "hidden_size": width,
+                                "num_attention_heads": heads, "num_key_value_heads": kv, "head_dim": 128,
+                                "intermediate_size": ff, "vocab_size": vocab, "rope_theta": 500000.0, "rms_norm_eps": 1e-5,
+                                "tie_word_embeddings": False, "max_position_embeddings": 1 << 20, "rope_scaling": None,
+                                "num_hidden_layers": 4}),
+        }
+        return base, kinds, near
+    return {"w2048": shape(2048, 16, 4, 768, 256, 1024, 64, 64, 8192, 32000),
+            "w4096": shape(4096, 32, 8, 1536, 512, 1024, 128, 128, 14336, 32000)}
+
+
 def _routed_parts(model):
     return [b.ffn for b in model.blocks if getattr(getattr(b, "ffn", None), "spec", None) is not None
             and getattr(b.ffn.spec, "kind", "") == "routed_mlp"]
@@ -348,7 +392,7 @@ def generic_step_bytes(model, contexts):
     windowed = 0
     for need in model.cache_needs:       # a window bounds what a layer reads of a sequence
         if isinstance(need, KVNeed) and need.window is not None:
-            windowed += sum(max(0, c - need.window) for c in contexts) * need.num_kv_heads * \
+            windowed += sum(max(0, c - need.window - need.keep_first) for c in contexts) * need.num_kv_heads * \
                 (need.head_dim + need.value_dim) * item
     return w + sum(contexts) * per_token - windowed + len(contexts) * per_seq
 
@@ -436,61 +480,26 @@ def bench_kunitar(a):
     return 0
 
 
-def bench_luduvik(a):
-    """Prefill and decode throughput of Luduvik models whose layers are all lightning, all
-    parallel, and the mixed order, beside the closest layers of the other decoders at the same
-    width. One JSON line of its own; the default workload is untouched."""
+def bench_beside(a, design, architecture, shapes):
+    """Prefill and decode throughput of a design's models, each of layers of one kind and of the mixed
+    order (``shapes``: {size: (base configuration, {kind: layers}, {name: (architecture,
+    configuration)} of the closest layers of the other decoders at the same width)}). One JSON line
+    of its own; the default workload is untouched."""
     import torch
     import transformer_amd as ta
     dkey = "bf16" if a.dtype == "bfloat16" else "fp32"
     layers = a.layers or 4
-    out = {"design": "luduvik", "dtype": dkey, "layers": layers, "batch": a.batch,
+    out = {"design": design, "dtype": dkey, "layers": layers, "batch": a.batch,
            "prefill_tokens": a.prefill_tokens, "data": "synthetic", "sizes": {}}
 
     def fit(lay):
         return (list(lay) * (-(-layers // len(lay))))[:layers]
 
-    for size, (base, kinds, near) in luduvik_shapes().items():
+    for size, (base, kinds, near) in shapes.items():
         if a.design_size and size not in a.design_size.split(","):
             continue
         cases = [(n, arch, c) for n, (arch, c) in near.items()] + \
-                [(n, "Luduvik", {**base, "layers": lay}) for n, lay in kinds.items()]
-        if a.design_case:
-            cases = [c for c in cases if c[0] in a.design_case.split(",")]
-        rows = {}
-        for name, arch, cfg in cases:
-            if arch == "llama":
-                model = ta.random_model(ta.LlamaConfig.from_dict({**cfg, "num_hidden_layers": layers}), seed=0, dtype=a.dtype)
-            else:
-                model = ta.random_model({**cfg, "layers": fit(cfg["layers"])}, seed=0, dtype=a.dtype, architecture=arch)
-            rows[name] = _design_row(model, a, dkey)
-            del model
-            torch.cuda.empty_cache()
-            print(f"[bench] {size} {name}: {rows[name]}", file=sys.stderr, flush=True)
-        out["sizes"][size] = rows
-    print(json.dumps(out))
-    return 0
-
-
-def bench_saredra(a):
-    """Prefill and decode throughput of Saredra models whose layers are all attention, all
-    parallel, and the mixed order, beside the closest layers of the other decoders at the same
-    width. One JSON line of its own; the default workload is untouched."""
-    import torch
-    import transformer_amd as ta
-    dkey = "bf16" if a.dtype == "bfloat16" else "fp32"
-    layers = a.layers or 4
-    out = {"design": "saredra", "dtype": dkey, "layers": layers, "batch": a.batch,
-           "prefill_tokens": a.prefill_tokens, "data": "synthetic", "sizes": {}}
-
-    def fit(lay):
-        return (list(lay) * (-(-layers // len(lay))))[:layers]
-
-    for size, (base, kinds, near) in saredra_shapes().items():
-        if a.design_size and size not in a.design_size.split(","):
-            continue
-        cases = [(n, arch, c) for n, (arch, c) in near.items()] + \
-                [(n, "Saredra", {**base, "layers": lay}) for n, lay in kinds.items()]
+                [(n, architecture, {**base, "layers": lay}) for n, lay in kinds.items()]
         if a.design_case:
             cases = [c for c in cases if c[0] in a.design_case.split(",")]
         rows = {}
@@ -591,18 +600,20 @@ def main():
                     help="tokens of the prompt whose step is timed (the line's \"prefill\")")
     ap.add_argument("--prefill-only", action="store_true",
                     help="run only the 2,048-token prefill (for profiling); prints its own line")
-    ap.add_argument("--design", default=None, choices=["vametar", "kunitar", "luduvik", "saredra"],
+    ap.add_argument("--design", default=None, choices=["vametar", "kunitar", "luduvik", "saredra", "zirutar"],
                     help="instead of the default workload: prefill and decode of this design at a few "
                          "layer sizes, beside the Llama decoder at the same sizes (a line of its own)")
     ap.add_argument("--design-size", default=None, help="with --design: only these sizes (w2048,w4096)")
-    ap.add_argument("--design-case", default=None, help="with --design kunitar, luduvik or saredra: only these rows (llama,latent,...)")
+    ap.add_argument("--design-case", default=None, help="with --design kunitar, luduvik, saredra or zirutar: only these rows (llama,latent,...)")
     a = ap.parse_args()
     if a.design == "kunitar" and a.gpus == 1:
         return bench_kunitar(a)
     if a.design == "luduvik" and a.gpus == 1:
-        return bench_luduvik(a)
+        return bench_beside(a, "luduvik", "Luduvik", luduvik_shapes())
     if a.design == "saredra" and a.gpus == 1:
-        return bench_saredra(a)
+        return bench_beside(a, "saredra", "Saredra", saredra_shapes())
+    if a.design == "zirutar" and a.gpus == 1:
+        return bench_beside(a, "zirutar", "Zirutar", zirutar_shapes())
     if a.design and a.gpus == 1:
         return bench_design(a)
     if a.gpus != 1:

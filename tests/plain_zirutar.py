@@ -298,7 +298,8 @@ def tensor_shapes(c, ranks=(3, 5)):
 def random_weights(c, seed, edit=None):
     """float64 weights, already rounded to bfloat16 values so that a bfloat16 file holds them
     exactly. Matrices ~ N(0, 1/sqrt(in)), the feed-forward's gate and up matrices larger so that
-    their limits are met; stored-around-zero gains near 0, the others near 1; decays between about
+    their limits are met, the token input's gate smaller (far down gelu's tail all its numbers are near
+    zero, and the norm behind them would blow up their rounding); stored-around-zero gains near 0, the others near 1; decays between about
     0.3 and 0.999 a token, so that a state forgets and also remembers."""
     rng = np.random.default_rng(seed)
     w = {}
@@ -320,6 +321,8 @@ def random_weights(c, seed, edit=None):
             a = rng.standard_normal(shape) * (0.3 if name == "embed" else 1.0)
         elif name == "loop.step":
             a = 0.7 * rng.standard_normal(shape)
+        elif name.endswith("side.gate"):
+            a = 0.3 * rng.standard_normal(shape) / np.sqrt(shape[-1])
         elif ".mlp." in name and last in ("gate", "up"):
             a = 1.5 * rng.standard_normal(shape) / np.sqrt(shape[-1])
         else:

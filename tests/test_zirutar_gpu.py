@@ -1,0 +1,741 @@
+"""The Zirutar decoder on the GPU against the plain implementation in ``plain_zirutar``.
+
+Each mechanism alone (its kernels against the plain function, with cache and state carried over
+cuts), then the engine: layers, whole prompts, portions, token-by-token decoding, unequal
+batches, slots and pages used again, recorded steps, far keys and keys at the borders of pages,
+windows and kept first tokens, long decoding, greedy generation, the replayer and the command line."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+import plain_zirutar as P
+import zirutar_util as U
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda:0"
+DTYPES = ["float32", "bfloat16"]
+TD = {"float32": torch.float32, "bfloat16": torch.bfloat16}
+
+
+def _t(a, dtype=torch.float32):
+    return torch.tensor(np.asarray(a), dtype=dtype, device=DEV)
+
+
+def _bf(a, dtype="bfloat16"):
+    from plain_llama import round_bf16
+    a = np.asarray(a, dtype=np.float64)
+    return round_bf16(a) if dtype == "bfloat16" else a.astype(np.float32).astype(np.float64)
+
+
+def _np(t):
+    return t.detach().float().cpu().numpy().astype(np.float64)
+
+
+def _close(got, want, dtype, what="", scale=1.0):
+    tol = (3e-5 if dtype == "float32" else 2.5e-2) * scale
+    assert np.abs(got - want).max() <= tol * max(1.0, np.abs(want).max()), what
+
+
+# ----------------------------------------------------------------------------- mechanisms alone
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("d", [72, 90, 1024])
+def test_offset_norm_and_the_add_in_front_of_a_reader(d, dtype):
+    from transformer_amd import kernels as K
+    from transformer_amd.config.spec import OffsetNormSpec
+    from transformer_amd.parts.base import build_part
+    rng = np.random.default_rng(d)
+    w = _bf(0.3 * rng.standard_normal(d))
+    norm = build_part(OffsetNormSpec(size=d, eps=1e-4), TD[dtype], DEV)
+    norm.bind({"weight": _t(w)})
+    for nt in (1, 7, 130):
+        x0, row = rng.standard_normal((nt, d)).astype(np.float32), rng.standard_normal(d).astype(np.float32)
+        delta = rng.standard_normal((3, nt, d)).astype(np.float32)
+        x, out = _t(x0), torch.empty(nt, d, dtype=TD[dtype], device=DEV)
+        norm.run(x, out, None, _t(row))                          # nothing pending but a row for every token
+        np.testing.assert_allclose(_np(x), x0 + row, atol=1e-6)
+        _close(_np(out), P.offset_norm(x0.astype(np.float64) + row, w, 1e-4), dtype)
+        for planes, bias, cast in ((3, None, True), (1, row, True), (0, row, False), (0, None, True)):
+            x, xc = _t(x0), torch.empty(nt, d, dtype=TD[dtype], device=DEV)
+            K.stream_add(x, None if planes == 0 else _t(delta[:planes] if planes > 1 else delta[0]),
+                         None if bias is None else _t(bias), xc if cast else None)
+            want = x0 + delta[:planes].sum(0) + (0.0 if bias is None else bias)
+            np.testing.assert_allclose(_np(x), want, atol=1e-5)
+            if cast:
+                assert torch.equal(xc, x.to(TD[dtype]))
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("geom", [(64, 40, 0.7), (72, 33, 2.0), (1024, 704, 1.3), (2048, 5632, 0.5)])
+def test_limited_feed_forward_in_every_product(geom, dtype):
+    """The few-rows, the 17-to-64-rows and the library's product (which differ in who applies the
+    activation), with gate and up numbers on both sides of the limits."""
+    from transformer_amd.config.spec import GLUSpec
+    from transformer_amd.parts.base import build_part
+    from transformer_amd.parts.linear import Workspace
+    d, ff, limit = geom
+    if dtype == "float32" and d > 1024:
+        pytest.skip("the float32 engine has one product for every number of rows")
+    rng = np.random.default_rng(d)
+    w = {n: _bf(1.5 * rng.standard_normal(s) / np.sqrt(s[-1])) for n, s in
+         {"gate": (ff, d), "up": (ff, d), "down": (d, ff)}.items()}
+    part = build_part(GLUSpec(hidden=d, intermediate=ff, activation="limited", limit=limit), TD[dtype], DEV)
+    part.bind({"gate_up.weight": _t(np.concatenate([w["gate"], w["up"]]), TD[dtype]), "down.weight": _t(w["down"], TD[dtype])})
+
+    class Ctx:
+        ws = Workspace(DEV)
+    for nt in (1, 5, 16, 33, 64, 100):
+        h = _bf(rng.standard_normal((nt, d)))
+        g, u = h @ w["gate"].T, h @ w["up"].T
+        assert (g > limit).any() and (u > limit).any() and (u < -limit).any() and (np.abs(u) < limit).any()
+        delta, bias = part.run(_t(h, TD[dtype]), Ctx)
+        assert bias is None
+        got = _np(delta)
+        _close(got.sum(0) if got.ndim == 3 else got, P.limited_glu(h, w, "", limit), dtype, f"{nt} rows")
+
+
+def _attention_case(H, G, dh, T, rng, dtype):
+    """Rows [q | k | gate] with keys of very different lengths (the values are not the normed keys)."""
+    rows = rng.standard_normal((T, (H + G) * dh + H))
+    rows[:, H * dh:(H + G) * dh] *= rng.uniform(0.2, 4.0, (T, 1))
+    return _bf(rows, dtype)
+
+
+def _plain_attention(rows, H, G, dh, scale, size, keep, eps, round_keys=None):
+    T = len(rows)
+    q = P.unit_rms(rows[:, :H * dh].reshape(T, H, dh), eps)
+    k = rows[:, H * dh:(H + G) * dh].reshape(T, G, dh)
+    kn = P.unit_rms(k, eps)
+    if round_keys is not None:
+        q, kn = round_keys(q), round_keys(kn)
+    see, out = P.visible(T, size, keep), np.zeros((T, H, dh))
+    for a in range(H):
+        out[:, a] = P.softmax_rows(q[:, a] @ kn[:, a // (H // G)].T * scale, see) @ k[:, a // (H // G)]
+    return (out * P.sigmoid(rows[:, (H + G) * dh:])[:, :, None]).reshape(T, H * dh)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("geom", [(6, 2, 20, 37, 5), (4, 4, 16, None, 0), (1, 1, 33, 64, 0), (5, 5, 7, 65, 64), (2, 1, 34, 1, 3),
+                                  (4, 1, 40, 100, 130), (8, 2, 96, 72, 20), (3, 1, 256, 90, 65), (6, 6, 12, 3, 1)])
+def test_window_with_kept_tokens_on_the_vector_kernel(dtype, geom):
+    """Norm of the heads without a weight, values that are the keys as projected, the window and the
+    kept first tokens, one gate number per head; keys and values into shuffled pages that held NaN; a
+    prompt in two portions, single tokens and portions of two."""
+    from transformer_amd import kernels as K
+    from transformer_amd.kernels import PAGE
+    H, G, dh, size, keep = geom
+    rng = np.random.default_rng(H * 7 + dh)
+    T, scale, eps = 330, 1.7, 1e-5
+    rows = _attention_case(H, G, dh, T, rng, dtype)
+    want = _plain_attention(rows, H, G, dh, scale, size, keep, eps, lambda a: _bf(a, dtype))
+    kc = torch.full((9, G, PAGE, dh), float("nan"), dtype=TD[dtype], device=DEV)
+    vc = torch.full((9, G, dh, PAGE), float("nan"), dtype=TD[dtype], device=DEV)
+    pages = np.array([7, 2, 5, 0, 8, 3])
+    got, at = [], 0
+    for n in (70, 120, 1, 2, 1, 2, 134):
+        p = np.arange(at, at + n)
+        proj = _t(rows[p], TD[dtype])
+        dest = _t(pages[p // PAGE] * PAGE + p % PAGE, torch.int32)
+        K.qk_prepare(proj[:, :(H + G) * dh], H, G, dh, dh, eps, None, None, None, 0, dest=dest, kcache=kc, vcache=vc,
+                     unit_norm=True, values_from_keys=True)
+        o = torch.empty(n, H * dh, dtype=TD[dtype], device=DEV)
+        K.attention_sink(proj[:, :(H + G) * dh], o, kc, vc, _t([pages], torch.int32), _t([0, n], torch.int32),
+                         _t([at], torch.int32), n, H, G, dh, dh, scale, size, None, None, proj[:, (H + G) * dh:], 0,
+                         keep_first=keep)
+        got.append(_np(o))
+        at += n
+    _close(np.concatenate(got), want, dtype, scale=1.5)
+
+
+@pytest.mark.parametrize("geom", [(8, 2, 128, 100, 20), (4, 4, 32, None, 0), (16, 4, 64, 129, 70), (2, 1, 96, 64, 64),
+                                  (6, 1, 160, 1, 3), (64, 2, 64, 200, 129), (5, 5, 32, 65, 1), (8, 1, 256, 150, 200)])
+def test_window_with_kept_tokens_on_matrix_cores(geom):
+    """The same on the matrix-core kernels (bfloat16): prompts through the kernel that reads pages
+    directly and the one that shares them through LDS, single tokens through the kernel of four waves
+    and the merge, planned with and without the window."""
+    from transformer_amd import kernels as K
+    from transformer_amd.kernels import PAGE
+    H, G, dh, size, keep = geom
+    dtype = "bfloat16"
+    rng = np.random.default_rng(H * 7 + dh)
+    T, scale, eps = 700, 1.7, 1e-5
+    rows = _attention_case(H, G, dh, T, rng, dtype)
+    want = _plain_attention(rows, H, G, dh, scale, size, keep, eps, _bf)
+    kc = torch.full((12, G, PAGE, dh), float("nan"), dtype=TD[dtype], device=DEV)
+    vc = torch.full((12, G, dh, PAGE), float("nan"), dtype=TD[dtype], device=DEV)
+    pages = np.array([7, 2, 5, 11, 0, 9, 4, 1, 3, 10, 8, 0])
+    width = -(-rows.shape[1] // 8) * 8
+    got, at = [], 0
+    for n, how in ((70, 0), (300, 1), (1, "planned"), (1, None), (28, 0), (1, "planned"), (199, 1), (99, 1), (1, "planned")):
+        p = np.arange(at, at + n)
+        proj = torch.zeros(n, width, dtype=TD[dtype], device=DEV)[:, :rows.shape[1]]
+        proj.copy_(_t(rows[p], TD[dtype]))
+        qk, gate = proj[:, :(H + G) * dh], proj[:, (H + G) * dh:]
+        dest = _t(pages[p // PAGE] * PAGE + p % PAGE, torch.int32)
+        K.qk_prepare(qk, H, G, dh, dh, eps, None, None, None, 0, dest=dest, kcache=kc, vcache=vc,
+                     unit_norm=True, values_from_keys=True)
+        o = torch.empty(n, H * dh, dtype=TD[dtype], device=DEV)
+        args = (qk, o, kc, vc, _t([pages], torch.int32), _t([0, n], torch.int32), _t([at], torch.int32))
+        opts = dict(window=size, gate=gate, gate_dim=0, keep_first=keep)
+        if how in (0, 1):
+            K.attention_rows_sink(*args, n, H, G, dh, scale, through_lds=how if dh <= 192 else 0, **opts)
+        elif not K.keys_sink_fits(H, G, dh):
+            K.attention_rows_sink(*args, n, H, G, dh, scale, **opts)
+        else:
+            plan = {}
+            if how == "planned":
+                u, s = K.plan_key_units([at + 1], 7, tables=[pages], window=size, keep_first=keep)
+                plan = dict(units=_t(u, torch.int32), seq_units=_t(s, torch.int32))
+            K.attention_keys_sink(*args, at + 1, H, G, dh, scale, **opts, **plan)
+        got.append(_np(o))
+        at += n
+    _close(np.concatenate(got), want, dtype, scale=1.5)
+
+
+EDGES = [(0, None, 0), (63, None, 0), (64, None, 0), (298, None, 0), (200, 100, 0), (199, 100, 0), (236, 64, 10), (235, 64, 10),
+         (171, 129, 5), (170, 129, 5), (299, 1, 2), (298, 1, 2), (0, 50, 1), (1, 50, 1), (19, 72, 20), (20, 72, 20), (63, 30, 64),
+         (64, 30, 64), (129, 90, 130), (130, 90, 130), (128, 65, 128)]
+
+
+@pytest.mark.parametrize("kernel", ["vector32", "vector16", "matrix"])
+@pytest.mark.parametrize("where", ["prompt", "decode"])
+@pytest.mark.parametrize("mark,window,keep", EDGES)
+def test_one_key_stands_out(where, kernel, mark, window, keep):
+    """The last query points at ONE earlier key (the first, the last of the kept ones and the next, the
+    last and the first of a page, the first inside a window and the last outside): its score stands
+    out, so the result is that key's value where the mask shows it, and something else where not."""
+    from transformer_amd import kernels as K
+    from transformer_amd.kernels import PAGE
+    dtype = "float32" if kernel == "vector32" else "bfloat16"
+    H, G, dh, T = 4, 2, 32, 300
+    rng = np.random.default_rng(mark)
+    q, k = 0.05 * rng.standard_normal((T, H * dh)), rng.standard_normal((T, G * dh))
+    k[:, 0::dh] *= 0.1
+    k.reshape(T, G, dh)[mark] = 0.01 * rng.standard_normal((G, dh))
+    k.reshape(T, G, dh)[mark, :, 0] = 2.0
+    q.reshape(T, H, dh)[T - 1, :, 0] = 3.0
+    rows = _bf(np.concatenate([q, k, np.full((T, H), 30.0)], 1), dtype)        # gates of 1
+    pages = np.array([4, 1, 3, 0, 5])
+    kc = torch.full((6, G, PAGE, dh), float("nan"), dtype=TD[dtype], device=DEV)
+    vc = torch.full((6, G, dh, PAGE), float("nan"), dtype=TD[dtype], device=DEV)
+    nq = 1 if where == "decode" else 70
+    for p in (np.arange(0, T - nq), np.arange(T - nq, T)):
+        proj = torch.zeros(len(p), 200, dtype=TD[dtype], device=DEV)[:, :rows.shape[1]]
+        proj.copy_(_t(rows[p], TD[dtype]))
+        dest = _t(pages[p // PAGE] * PAGE + p % PAGE, torch.int32)
+        K.qk_prepare(proj[:, :(H + G) * dh], H, G, dh, dh, 1e-5, None, None, None, 0, dest=dest, kcache=kc, vcache=vc,
+                     unit_norm=True, values_from_keys=True)
+    o = torch.empty(nq, H * dh, dtype=TD[dtype], device=DEV)
+    qk, gate = proj[:, :(H + G) * dh], proj[:, (H + G) * dh:]
+    args = (qk, o, kc, vc, _t([pages], torch.int32), _t([0, nq], torch.int32), _t([T - nq], torch.int32))
+    if kernel != "matrix":
+        K.attention_sink(*args, nq, H, G, dh, dh, 2.0, window, None, None, gate, 0, keep_first=keep)
+    elif where == "decode":
+        K.attention_keys_sink(*args, T, H, G, dh, 2.0, window, gate=gate, gate_dim=0, keep_first=keep)
+    else:
+        K.attention_rows_sink(*args, nq, H, G, dh, 2.0, window, gate=gate, gate_dim=0, keep_first=keep)
+    marked = np.repeat(rows[mark, H * dh:(H + G) * dh].reshape(G, dh), H // G, axis=0).reshape(-1)
+    err = np.abs(_np(o[-1]) - marked).max()
+    if bool(P.visible(T, window, keep)[T - 1, mark]):
+        assert err < (1e-3 if dtype == "float32" else 2e-2)
+    else:
+        assert err > 0.5
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("geom", [(5, 12, 6, 9, 20), (1, 16, 2, 16, 8), (3, 5, 4, 11, 13), (8, 64, 32, 64, 128), (6, 32, 16, 32, 300),
+                                  (16, 16, 64, 24, 512), (2, 8, 0, 8, 24)])
+def test_latent_attention_part_with_a_sink(dtype, geom):
+    """The part as the block runs it (direct queries, the norm of the latent, rotation, scores with a
+    learned extra term of the denominator, both kernels' ways of dealing out keys): one sequence in a
+    prompt, a portion of two and single tokens, beside another sequence."""
+    from transformer_amd.cache.storage import SequenceCache
+    from transformer_amd.config.spec import LatentAttentionSpec
+    from transformer_amd.engine.batch import Entry, Uploader, plan_step
+    from transformer_amd.parts.base import build_part
+    from transformer_amd.parts.linear import Workspace
+    H, dn, dr, dv, r = geom
+    d, T = 48, 150
+    rng = np.random.default_rng(H + r)
+    m = {"heads": H, "dim": dn, "rot_dim": dr, "vdim": dv, "kv_rank": r, "scale": 0.5, "rot": {"base": 200.0, "dims": dr}}
+    shapes = {"q": (H * (dn + dr), d), "dkv": (r + dr, d), "uk": (H * dn, r), "uv": (H * dv, r), "o": (d, H * dv)}
+    w = {n: _bf((3.0 if n == "q" else 1.0) * rng.standard_normal(s) / np.sqrt(s[-1])) for n, s in shapes.items()}
+    w["dkv.norm"], w["sink"] = 1.0 + 0.2 * rng.standard_normal(r).astype(np.float32), (2.0 * rng.standard_normal(H)).astype(np.float32)
+    w["sink"][0] = 4.0
+    spec = LatentAttentionSpec(hidden=d, num_heads=H, nope_dim=dn, rope_dim=dr, value_dim=dv, q_rank=None, kv_rank=r, scale=0.5,
+                               eps=1e-5, rot_dims=dr, rot_base=200.0, gated=False, sink=True)
+    part = build_part(spec, TD[dtype], DEV)
+    mat = lambda a: _t(a, TD[dtype])
+    part.bind({"in.weight": mat(np.concatenate([w["q"], w["dkv"]])), "uk.weight": mat(w["uk"]), "uv.weight": mat(w["uv"]),
+               "out.weight": mat(w["o"]), "kv_norm.weight": _t(w["dkv.norm"]), "sink": _t(w["sink"])})
+    hs = [_bf(rng.standard_normal((T, d))), _bf(rng.standard_normal((T, d)))]
+    cache = SequenceCache([part.cache_need()], 1024, 3, TD[dtype], DEV)
+    for t in cache.keys:
+        t.fill_(float("nan"))
+    slots = [cache.alloc_slot(), cache.alloc_slot()]
+    ws, up = Workspace(DEV), Uploader(DEV)
+    got, at = [[], []], [0, 0]
+    for n0, n1 in ((70, 3), (2, 64), (1, 1), (1, 1), (1, 1), (75, 0)):
+        take = [(i, n) for i, n in ((0, n0), (1, n1)) if n]
+        ctx = plan_step([Entry(slots[i], [0] * n) for i, n in take], cache, 10, up, ws)
+        h = np.concatenate([hs[i][at[i]:at[i] + n] for i, n in take])
+        delta, bias = part.run(mat(h), ctx, cache, 0)
+        out, o = _np(delta), 0
+        out = out.sum(0) if out.ndim == 3 else out
+        for i, n in take:
+            got[i].append(out[o:o + n])
+            o += n
+            at[i] += n
+            cache.pool.advance(slots[i], n)
+    for i in range(2):
+        want = P.latent_attention(hs[i][:at[i]], w, "", m, 1e-5)
+        none = P.latent_attention(hs[i][:at[i]], {**w, "sink": np.full(H, -1e3)}, "", m, 1e-5)
+        _close(np.concatenate(got[i]), want, dtype, f"sequence {i}", scale=1.5)
+        assert np.abs(want - none).max() > 0.1                                 # the extra term matters
+
+
+def _delta_case(geom, rng, dtype, lens):
+    H, G, dk, dv, taps, ra, rg = geom
+    d = 40
+    shapes = {"q": (G * dk, d), "k": (G * dk, d), "v": (H * dv, d), "b": (H, d), "a1": (ra, d), "a2": (H * dk, ra), "g1": (rg, d),
+              "g2": (H * dv, rg), "o": (d, H * dv)}
+    w = {n: _bf(rng.standard_normal(s) / np.sqrt(s[-1])) for n, s in shapes.items()}
+    for n in "qkv":
+        w[n + ".conv"] = _bf(rng.standard_normal((shapes[n][0], taps)))
+    f = lambda a: np.asarray(a, dtype=np.float32).astype(np.float64)
+    w["A_log"], w["dt_bias"], w["norm"] = f(rng.uniform(-1, 1, H)), f(rng.uniform(-5, 0, H * dk)), f(1 + 0.2 * rng.standard_normal(dv))
+    m = {"heads": H, "kv_heads": G, "dim": dk, "vdim": dv, "conv": taps}
+    return w, m, [_bf(rng.standard_normal((L, d))) for L in lens]
+
+
+def _delta_part(w, geom, dtype):
+    from transformer_amd.config.spec import GatedDeltaSpec
+    from transformer_amd.parts.base import build_part
+    H, G, dk, dv, taps, ra, rg = geom
+    part = build_part(GatedDeltaSpec(hidden=40, num_heads=H, num_kv_heads=G, key_dim=dk, value_dim=dv, taps=taps,
+                                     decay_rank=ra, gate_rank=rg, eps=1e-5), TD[dtype], DEV)
+    mat = lambda a: _t(a, TD[dtype])
+    part.bind({"in.weight": mat(np.concatenate([w[n] for n in ("q", "k", "v", "a1", "g1", "b")])),
+               "conv.weight": _t(np.concatenate([w[n + ".conv"] for n in "qkv"])), "decay.weight": mat(w["a2"]),
+               "gate.weight": mat(w["g2"]), "dt_bias": _t(w["dt_bias"]), "A_log": _t(w["A_log"]), "norm.weight": _t(w["norm"]),
+               "out.weight": mat(w["o"])})
+    return part
+
+
+DELTA_GEOMS = [(2, 2, 32, 64, 3, 24, 24), (6, 3, 24, 12, 4, 8, 5), (1, 1, 64, 8, 1, 1, 2), (3, 1, 33, 7, 9, 5, 3), (2, 1, 6, 66, 2, 9, 16),
+               (4, 2, 128, 128, 4, 16, 32), (2, 1, 160, 40, 2, 8, 8), (2, 2, 250, 20, 3, 4, 4), (1, 1, 200, 256, 4, 16, 16),
+               (3, 3, 16, 100, 4, 8, 8)]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("geom", DELTA_GEOMS)
+def test_delta_rule_part_over_cuts(dtype, geom):
+    """The whole mixer over three sequences of unequal lengths in slots that held something else, in cuts
+    of many, one, two and two tokens: convolution, unit vectors, decays, the state and the readout's norm
+    and gate, prompts through the walking kernel and single tokens through the fused one."""
+    from transformer_amd.cache.storage import SequenceCache
+    from transformer_amd.engine.batch import Entry, Uploader, plan_step
+    from transformer_amd.parts.linear import Workspace
+    rng = np.random.default_rng(geom[2] * 10 + geom[3])
+    lens = [61, 8, 40]
+    w, m, hs = _delta_case(geom, rng, dtype, lens)
+    part = _delta_part(w, geom, dtype)
+    cache = SequenceCache(part.cache_need(), 1024, 5, TD[dtype], DEV)
+    layers = tuple(range(len(part.cache_need())))
+    for t in cache.states:
+        t.fill_(3.0)
+    slots = [cache.alloc_slot() for _ in range(5)][1:4]
+    ws, up = Workspace(DEV), Uploader(DEV)
+    got, at = [[] for _ in lens], [0] * len(lens)
+    for cut in ((37, 1, 18), (1, 1, 1), (2, 2, 2), (2, 2, 2), (1, 1, 1), (18, 1, 16)):
+        ctx = plan_step([Entry(s, [0] * n) for s, n in zip(slots, cut)], cache, 10, up, ws)
+        h = np.concatenate([x[a:a + n] for x, a, n in zip(hs, at, cut)])
+        delta, _ = part.run(_t(h, TD[dtype]), ctx, cache, layers)
+        out, o = _np(delta), 0
+        out = out.sum(0) if out.ndim == 3 else out
+        for i, n in enumerate(cut):
+            got[i].append(out[o:o + n])
+            o += n
+            at[i] += n
+            cache.pool.advance(slots[i], n)
+    for i, L in enumerate(lens):
+        _close(np.concatenate(got[i]), P.channel_delta(hs[i], w, "", m, 1e-5), dtype, f"sequence {i}", scale=3.0)
+    for t in cache.states:
+        assert float(t[:, 0].abs().max()) == 0.0 and float(t[:, 5].min()) == 3.0     # slots of others stay as they are
+
+
+@pytest.mark.parametrize("waves", [2, 4])
+@pytest.mark.parametrize("geom", [(3, 3, 32, 16), (4, 2, 128, 40), (2, 1, 47, 5), (2, 2, 192, 33), (1, 1, 256, 70), (16, 4, 64, 64)])
+def test_delta_recurrence_alone(geom, waves):
+    """The recurrence's kernel on operands of its own (decays down to 0 and up to 1, steps of 0 and 1,
+    keys that are no unit vectors), sequences that end inside and at the edge of a chunk."""
+    from transformer_amd import kernels as K
+    H, G, dk, dv = geom
+    rng = np.random.default_rng(dk)
+    lens = [1, 16, 17, 50]
+    nt = sum(lens)
+    q, k = 0.3 * rng.standard_normal((nt, G, dk)), rng.standard_normal((nt, G, dk)) / np.sqrt(dk)
+    g, b = rng.uniform(0.5, 1.0, (nt, H, dk)), rng.uniform(0, 1, (nt, H))
+    g[:, 0, ::3], g[::5] = 1.0, 0.0
+    b[::7], b[1::7] = 0.0, 1.0
+    v = rng.standard_normal((nt, H, dv))
+    S0 = rng.standard_normal((len(lens), H, dk, dv))
+    state = torch.zeros((6, H, dk, dv), device=DEV)
+    slots = [4, 0, 5, 2]
+    for s, a in zip(slots, S0):
+        state[s] = _t(a)
+    cu = np.concatenate([[0], np.cumsum(lens)])
+    o = torch.full((nt, H, dv), float("nan"), device=DEV)
+    f = lambda a: _t(np.asarray(a, dtype=np.float32))
+    K.delta_recurrent(f(q), f(k), f(g), f(v.reshape(nt, -1)), f(b), f((q * k).sum(-1)), state, _t(cu, torch.int32),
+                      _t(slots, torch.int32), o, waves=waves)
+    rep = lambda a: np.repeat(a, H // G, axis=1)
+    for i, n in enumerate(lens):
+        r = slice(cu[i], cu[i + 1])
+        want, S = P.delta_rule(rep(q[r]), rep(k[r]), v[r], g[r], b[r], S0[i])
+        np.testing.assert_allclose(_np(o[r]), want, atol=3e-4)
+        np.testing.assert_allclose(_np(state[slots[i]]), S, atol=3e-4)
+    assert float(state[1].abs().max()) == 0.0 and float(state[3].abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("where", ["prompt", "decode"])
+def test_a_far_token_in_the_state(where):
+    """A token 497 steps back wrote its value under a key that nobody touched since: head 0, whose decay
+    is 1 to float32, gives it back as on the first day, head 1 has forgotten it at once, and in head 2 it
+    has faded."""
+    H, dk, dv, T, far = 3, 8, 5, 500, 2
+    geom = (H, 1, dk, dv, 1, 1, 1)
+    rng = np.random.default_rng(5)
+    w, m, _ = _delta_case(geom, rng, "float32", [1])
+    d = 40
+    h = np.zeros((T, d))
+    for n, c in (("q", 0), ("k", dk)):                            # q and k read coordinates of h, v others
+        w[n] = np.zeros((dk, d)); w[n][:, c:c + dk] = np.eye(dk)
+        w[n + ".conv"] = np.ones((dk, 1))
+    w["v"] = np.zeros((H * dv, d)); w["v"][:, 2 * dk:2 * dk + H * dv] = np.eye(H * dv)
+    w["v.conv"] = np.ones((H * dv, 1))
+    w["b"], w["a1"], w["g1"] = np.zeros((H, d)), np.zeros((1, d)), np.zeros((1, d))
+    w["b"][:, 2 * dk + H * dv] = 5.0                              # h's next coordinate is 1: steps near 1
+    w["norm"], w["o"] = np.ones(dv), np.eye(d, H * dv)
+    w["A_log"], w["dt_bias"] = np.array([-40.0, 5.0, np.log(0.01)]), np.zeros(H * dk)
+    h[:, 2 * dk + H * dv] = 1.0
+    h[:, dk + 1], h[:, 1] = 9.0, 9.0                              # everyone's key but one
+    h[far, dk + 1], h[far, dk] = -30.0, 9.0
+    h[T - 1, 1], h[T - 1, 0] = -30.0, 9.0
+    h[:, 2 * dk:2 * dk + H * dv] = 0.01 * rng.standard_normal((T, H * dv))
+    h[far, 2 * dk:2 * dk + H * dv] = 4.0
+    part = _delta_part(w, geom, "float32")
+    from transformer_amd.cache.storage import SequenceCache
+    from transformer_amd.engine.batch import Entry, Uploader, plan_step
+    from transformer_amd.parts.linear import Workspace
+    cache = SequenceCache(part.cache_need(), 1024, 1, torch.float32, DEV)
+    slot, ws, up = cache.alloc_slot(), Workspace(DEV), Uploader(DEV)
+    nq = 1 if where == "decode" else 33
+    for lo, hi in ((0, T - nq), (T - nq, T)):
+        ctx = plan_step([Entry(slot, [0] * (hi - lo))], cache, 10, up, ws)
+        delta, _ = part.run(_t(h[lo:hi]), ctx, cache, (0,))
+        cache.pool.advance(slot, hi - lo)
+    want = P.channel_delta(h, w, "", m, 1e-5)
+    np.testing.assert_allclose(_np(delta[-1]), want[-1], atol=2e-3)
+    S = _np(cache.layer_state(0)[slot])
+    assert np.abs(S[0, 0] - P.silu(4.0)).max() < 0.1              # kept
+    assert np.abs(S[1, 0]).max() < 0.01 and 0 < np.abs(S[2, 0]).max() < 0.1 * P.silu(4.0)    # 0.99^(0.69 * 497)
+
+
+# ----------------------------------------------------------------------------- the engine
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["A", "B", "C", "D"])
+def test_layers_and_whole_prompt(name, dtype):
+    from transformer_amd import Entry
+    model, toks = U.engine(name, dtype), U.tokens(name, 140, 1)
+    dumps = {}
+    model.dump = lambda n, t: dumps.__setitem__(n, t.detach().float().cpu().numpy().copy())
+    try:
+        cache = model.new_cache(256)
+        got = model.step(cache, [Entry(cache.alloc_slot(), toks, list(range(len(toks))))]).cpu().numpy()
+    finally:
+        model.dump = None
+    layers = []
+    want = U.plain(name, dtype).forward(toks, layers)
+    tol = 1e-4 if dtype == "float32" else 0.15
+    opens = {i for i, r in enumerate(model.spec.schedule) if r.opening is not None}
+    assert len(layers) == len(model.spec.schedule)
+    for i, l in enumerate(layers):
+        assert np.abs(dumps[f"run.{i}"] - l).max() < tol * max(1.0, np.abs(l).max()), f"layer run {i} (passes open at {opens})"
+    assert U.row_error(got, want).max() < U.TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name,edit", [("A", None), ("B", None), ("D", None), ("A", "sharp"), ("D", "sharp")])
+def test_cuts_agree_with_plain(name, edit, dtype):
+    """Whole, portions down to two tokens, and every token alone: all against the plain model."""
+    model, toks = U.engine(name, dtype, edit), U.tokens(name, 150, 2)
+    cache = model.new_cache(512, max_slots=3)
+    for cuts in ([150], [2, 2, 61, 3, 64, 17], [130], []):
+        slot = cache.alloc_slot()
+        got = U.run_cuts(model, cache, slot, toks, cuts)
+        cache.free_slot(slot)                      # the next cut takes the same slot and pages
+        U.check_against_plain(name, dtype, edit, toks, got, f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_prompt_in_portions_over_pages_windows_and_kept_tokens(dtype):
+    """400 tokens with peaked softmax: portions end at and around the borders of pages, of the windows, of
+    the kept first tokens and of the recurrence's chunks; pages that leave every window are given back
+    meanwhile, those of the kept tokens are not."""
+    name, edit = "A", "sharp"
+    model, toks = U.engine(name, dtype, edit), U.tokens(name, 400, 7)
+    cache = model.new_cache(512, max_slots=1)
+    for cuts in ([400], [257, 63, 65, 15], [64, 256, 33, 31, 16], [255, 129, 8, 7, 1], [7, 50, 13, 70, 20, 70], [6, 64, 2, 2]):
+        slot = cache.alloc_slot()
+        got = U.run_cuts(model, cache, slot, toks, cuts)
+        held = [cache.pool.pages(slot, g) for g in range(len(cache.kv_groups))]
+        for need, pages in zip(cache.kv_groups, held):
+            gone = [p < 0 for p in pages]
+            assert gone[:need.keep_pages] == [False] * need.keep_pages
+            assert any(gone) == (need.window is not None)
+        cache.free_slot(slot)
+        U.check_against_plain(name, dtype, edit, toks, got, f"cuts {cuts}")
+        cache.pool.check()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_unequal_batch_then_decoding_in_used_slots(dtype):
+    """The second batch lives in slots and pages that a first one left dirty; a sequence leaves early and
+    its slot is taken again; another joins while the rest decode."""
+    from transformer_amd import Entry
+    name = "A"
+    model = U.engine(name, dtype)
+    cache = model.new_cache(1024, max_slots=4)
+    old = [cache.alloc_slot() for _ in range(4)]
+    model.step(cache, [Entry(s, U.tokens(name, 100 + 7 * s, 50 + s), [0]) for s in old])
+    for s in old:
+        cache.free_slot(s)
+    lens = [1, 70, 131, 2]
+    seqs = [U.tokens(name, n + 45, 10 + i) for i, n in enumerate(lens)]
+    slots = [cache.alloc_slot() for _ in seqs]
+    got = [[] for _ in seqs]
+    lg = model.step(cache, [Entry(sl, s[:n], list(range(n))) for sl, s, n in zip(slots, seqs, lens)]).cpu().numpy()
+    at = 0
+    for i, n in enumerate(lens):
+        got[i].append(lg[at:at + n].copy())
+        at += n
+    live = list(range(len(seqs)))
+    for step in range(40):
+        if step == 25:
+            cache.free_slot(slots[1])
+            live.remove(1)
+            slots[1] = cache.alloc_slot()
+        lg = model.step(cache, [Entry(slots[i], [seqs[i][lens[i] + step]], [0]) for i in live]).cpu().numpy()
+        for j, i in enumerate(live):
+            got[i].append(lg[j:j + 1].copy())
+    late = U.tokens(name, 33, 99)                      # the slot that came back: a prompt beside single tokens
+    lg = model.step(cache, [Entry(slots[0], [seqs[0][lens[0] + 40]], [0]), Entry(slots[1], late[:31], list(range(31))),
+                            Entry(slots[2], seqs[2][lens[2] + 40:lens[2] + 42], [0, 1])]).cpu().numpy()
+    got[0].append(lg[:1].copy())
+    got[2].append(lg[32:34].copy())
+    tail = model.step(cache, [Entry(slots[1], late[31:], [0, 1])]).cpu().numpy()
+    U.check_against_plain(name, dtype, None, late, np.concatenate([lg[1:32], tail]), "the late sequence")
+    for i in range(len(seqs)):
+        U.check_against_plain(name, dtype, None, seqs[i], np.concatenate(got[i]), f"sequence {i}")
+    cache.pool.check()
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("name", ["A", "B", "D"])
+def test_recorded_steps_match_eager_steps(name, dtype):
+    from transformer_amd import Entry
+    model = U.engine(name, dtype)
+    seqs = [U.tokens(name, 60, 20 + i) for i in range(3)]
+    outs = []
+    for graphs in (True, False):
+        model.use_graphs = graphs
+        try:
+            cache = model.new_cache(512, max_slots=4)
+            slots = [cache.alloc_slot() for _ in seqs]
+            rows = []
+            for t in range(60):
+                lg = model.step(cache, [Entry(sl, [s[t]], [0]) for sl, s in zip(slots, seqs)])
+                rows.append(lg.cpu().numpy().copy())
+            outs.append(np.stack(rows))
+            assert bool(cache.graphs) == graphs and not cache.graphs_failed
+        finally:
+            model.use_graphs = True
+    assert np.abs(outs[0] - outs[1]).max() < (1e-5 if dtype == "float32" else 3e-2) * np.abs(outs[1]).max()
+    want = np.stack([U.plain_logits(name, dtype, None, tuple(s)) for s in seqs], 1)
+    assert U.row_error(outs[0], want).max() < U.TOL[dtype]
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_wide_model_in_three_cuts(dtype):
+    """Width 512: heads of 128 on the matrix cores, delta heads of 64 x 96, products of 17 to 64 rows,
+    prompts through the library and single tokens through the few-rows products; 330 tokens pass the
+    borders of pages, of both windows and of the kept first tokens."""
+    name = "C"
+    model, toks = U.engine(name, dtype), U.tokens(name, 330, 3)
+    cache = model.new_cache(512, max_slots=2)
+    for cuts in ([330], [100, 40, 70, 20, 9], [310]):
+        slot = cache.alloc_slot()
+        got = U.run_cuts(model, cache, slot, toks, cuts)
+        cache.free_slot(slot)
+        U.check_against_plain(name, dtype, None, toks, got, f"cuts {cuts}")
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_decoding_over_page_and_window_borders(dtype):
+    name, edit = "A", "sharp"
+    model, toks = U.engine(name, dtype, edit), U.tokens(name, 330, 4)
+    cache = model.new_cache(512, max_slots=1)
+    got = U.run_cuts(model, cache, cache.alloc_slot(), toks, [5])     # 325 single tokens over 5 borders, from inside the kept ones on
+    U.check_against_plain(name, dtype, edit, toks, got)
+
+
+def test_greedy_generation_through_the_entry_point():
+    import transformer_amd as ta
+    from transformer_amd.engine.generate import generate
+    name, dtype = "A", "float32"
+    model, plain = U.engine(name, dtype), U.plain(name, dtype)
+    prompts = [U.tokens(name, n, 30 + n) for n in (5, 1, 23)]
+    res = generate(model, prompts, max_new_tokens=12, sample_args=ta.SampleArgs(), stop_ids=())
+    for p, out in zip(prompts, res.tokens):
+        assert len(out) == 12
+        seq = list(p)
+        for t in out:                         # the engine's choice is the plain model's best, or ties with it
+            lg = plain.forward(seq)[-1]
+            assert lg.max() - lg[t] < 1e-3
+            seq.append(t)
+    again = generate(model, prompts, max_new_tokens=12, sample_args=ta.SampleArgs(), stop_ids=())
+    assert again.tokens == res.tokens
+
+
+def test_replayer_and_command_line():
+    name, dtype = "D", "float32"
+    folder = U.folder(name, dtype)
+    toks = U.tokens(name, 40, 5)
+    want = U.plain_logits(name, dtype, None, tuple(toks))
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    import tempfile
+    with tempfile.TemporaryDirectory() as out:
+        lines = [{"step": 0, "entries": [{"id": "a", "tokens": toks[:30], "want": [0, 29]},
+                                         {"id": "b", "tokens": toks[:1], "want": [0]}], "end": ["b"]}]
+        lines += [{"step": 1 + i, "entries": [{"id": "a", "tokens": [toks[30 + i]], "want": [0]}],
+                   "end": ["a"] if i == 9 else []} for i in range(10)]
+        r = subprocess.run([sys.executable, os.path.join(root, "bin", "trace_run"), "--model", folder, "--dtype",
+                            dtype, "--out", out, "--max-tokens", "128"],
+                           input="\n".join(json.dumps(l) for l in lines) + "\n", capture_output=True, text=True,
+                           timeout=600)
+        assert r.returncode == 0, r.stderr[-2000:]
+        assert [l for l in r.stdout.splitlines() if l.startswith("done")] == [f"done {i}" for i in range(11)]
+        first = np.fromfile(os.path.join(out, "0.f32"), dtype="<f4").reshape(3, -1)
+        assert U.row_error(first, want[[0, 29, 0]]).max() < U.TOL[dtype]
+        last = np.fromfile(os.path.join(out, "10.f32"), dtype="<f4").reshape(1, -1)
+        assert U.row_error(last, want[39:40]).max() < U.TOL[dtype]
+    r = subprocess.run([sys.executable, "-m", "transformer_amd", "generate", "--model", folder, "--dtype", dtype,
+                        "--prompt", ",".join(map(str, toks[:6])), "--max-steps", "5"],
+                       capture_output=True, text=True, timeout=600, cwd=root)
+    assert r.returncode == 0, r.stderr[-2000:]
+
+
+def test_random_weights_and_save_round_trip():
+    import copy
+    import tempfile
+    import transformer_amd as ta
+    from transformer_amd import Entry
+    cfg = copy.deepcopy(U.CFG_A)
+    for l in cfg["layers"]:
+        if "ranks" in l["mixer"]:
+            l["mixer"]["decay_rank"], l["mixer"]["gate_rank"] = l["mixer"].pop("ranks")
+    model = ta.random_model(cfg, seed=3, dtype="float32", architecture="Zirutar")
+    toks = U.tokens("A", 60, 6)
+    cache = model.new_cache(128)
+    a = model.step(cache, [Entry(cache.alloc_slot(), toks, [59])]).cpu().numpy().copy()
+    with tempfile.TemporaryDirectory() as d:
+        ta.save_model(model, d)
+        want = P.PlainZirutar(d).forward(toks)[-1:]
+        again = ta.load_model(d, "float32")
+        cache = again.new_cache(128)
+        b = again.step(cache, [Entry(cache.alloc_slot(), toks, [59])]).cpu().numpy()
+    assert np.abs(a - b).max() < 1e-6 * max(1.0, np.abs(a).max())
+    assert U.row_error(a, want).max() < U.TOL["float32"]
+
+
+def _draw_config(case):
+    """A random Zirutar configuration: any order of the three layer types, every option present or
+    absent, sizes that are odd, equal to one another, or 1, loops anywhere."""
+    r = np.random.default_rng(case)
+    pick = lambda *a: a[int(r.integers(0, len(a)))]
+    layers = []
+    for _ in range(int(r.integers(1, 6))):
+        kind = int(r.integers(0, 3))
+        mlp = U._dense(int(pick(8, 20, 33, 64)), float(pick(0.4, 1.0, 3.0))) if r.integers(0, 4) else None
+        if kind == 0:
+            G = int(pick(1, 2, 3))
+            dh = int(pick(4, 9, 16, 32, 64))
+            layers.append(U._att(G * int(pick(1, 2, 4)), G, dh, float(pick(3.0, 8.0, 14.0)) / dh,
+                                 pick(None, 1, 5, 63, 64, 65, 100), pick(None, 0, 1, 8, 64, 65, 90), mlp))
+        elif kind == 1:
+            dr = int(pick(2, 4, 8, 16))
+            layers.append(U._lat(int(pick(1, 2, 3, 8)), int(pick(1, 8, 16, 30)), dr, int(pick(3, 8, 16, 32)),
+                                 int(pick(4, 9, 32, 130)), float(pick(0.2, 0.5)), float(pick(50.0, 1e4, 1e6)), mlp))
+        else:
+            G = int(pick(1, 2, 3))
+            layers.append(U._delta(G * int(pick(1, 2, 3)), G, int(pick(4, 9, 16, 32, 70)), int(pick(2, 6, 16, 33, 64)), int(pick(1, 2, 3, 4)),
+                                   (int(pick(1, 3, 8, 16)), int(pick(1, 5, 8, 24))), mlp))
+    n = len(layers)
+    cfg = {"architecture": "Zirutar", "vocab": int(pick(5, 97, 300, 1001)), "width": int(pick(40, 64, 66, 100, 136, 33, 257)),
+           "norm": {"eps": float(pick(1e-6, 1e-5, 1e-3))}, "layers": layers}
+    if r.integers(0, 2):
+        cfg["embedding"] = {"scale": float(pick(1.0, 4.0))}
+    if r.integers(0, 2):
+        cfg["logit_scale"] = float(pick(0.5, 1.0, 2.0))
+    if r.integers(0, 3):
+        cfg["token_side"] = {"dim": int(pick(1, 5, 16, 40))}
+    if r.integers(0, 3):
+        a = int(r.integers(0, n))
+        cfg["loop"] = {"start": a, "stop": int(r.integers(a + 1, n + 1)), "times": int(pick(1, 2, 3))}
+    lens = [int(x) for x in r.integers(1, 150, size=int(r.integers(1, 5)))]
+    return cfg, lens, r
+
+
+@pytest.mark.parametrize("first", [9000, 9006, 9012, 9018])
+def test_random_configurations_against_the_plain_model(first):
+    """A batch of unequal prompts in one step into poisoned pages, then eight single tokens each
+    (recorded steps), every row, in float32 and in bfloat16."""
+    import tempfile
+    import transformer_amd as ta
+    from gpu_util import poison
+    for case in range(first, first + 6):
+        cfg, lens, r = _draw_config(case)
+        toks = [[int(t) for t in r.integers(0, cfg["vocab"], size=n + 8)] for n in lens]
+        for dtype in DTYPES:
+            with tempfile.TemporaryDirectory(prefix="zi_rand_") as d:
+                P.make_model_folder(d, cfg, case, storage=U.STORAGE[dtype])
+                ref = P.PlainZirutar(d)
+                model = ta.load_model(d, dtype, "cuda:0")
+            want = [ref.forward(t) for t in toks]
+            cache = model.new_cache(64 * sum(-(-(n + 8) // 64) for n in lens), max_slots=len(lens))
+            poison(cache)
+            slots = [cache.alloc_slot() for _ in lens]
+            what = f"case {case} {dtype} {json.dumps(cfg)} prompts {lens}"
+            got = model.step(cache, [ta.Entry(s, t[:n], list(range(n))) for s, t, n in zip(slots, toks, lens)]).cpu().numpy()
+            errs, at = [], 0
+            for i, n in enumerate(lens):
+                errs += list(U.row_error(got[at:at + n], want[i][:n]))
+                at += n
+            for j in range(8):
+                got = model.step(cache, [ta.Entry(s, [t[n + j]], [0]) for s, t, n in zip(slots, toks, lens)]).cpu().numpy()
+                errs += [U.row_error(got[i], want[i][n + j]) for i, n in enumerate(lens)]
+            errs = np.asarray(errs)
+            assert np.isfinite(errs).all(), what
+            if dtype == "float32":
+                assert errs.max() < U.TOL[dtype], (what, errs.max())
+            else:
+                # (a row now and then is badly conditioned: a norm of numbers near zero)
+                assert np.median(errs) < 0.5 * U.TOL[dtype] and np.quantile(errs, 0.9) < 1.5 * U.TOL[dtype], (what, np.quantile(errs, [0.5, 0.9]))
+            for s in slots:
+                cache.free_slot(s)
+            cache.pool.check()

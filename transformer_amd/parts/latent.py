@@ -80,10 +80,13 @@ class LatentAttention(Part):
         s = self.spec
         # per head: Uk^T and Uv as right operands. The framework's own product reads [N, K], the library's
         # (bfloat16) a contiguous [K, N]
+        def packed(t):                      # contiguous strides also where an axis has one entry
+            return torch.empty(t.shape, dtype=t.dtype, device=t.device).copy_(t)
+
         uk = tensors["uk.weight"].view(self.H, self.dn, s.kv_rank) if self.dn else None     # [K, N] of Uk^T
         uv = tensors["uv.weight"].view(self.H, self.dv, s.kv_rank)                          # [N, K]
-        self.uk_op = None if uk is None else uk if self._by_library(uk) else uk.transpose(1, 2).contiguous()
-        self.uv_op = uv.transpose(1, 2).contiguous() if self._by_library(uv) else uv
+        self.uk_op = None if uk is None else uk if self._by_library(uk) else packed(uk.transpose(1, 2))
+        self.uv_op = packed(uv.transpose(1, 2)) if self._by_library(uv) else uv
 
     def _by_library(self, w) -> bool:
         return self.dtype == torch.bfloat16 and w.dtype == torch.bfloat16
