@@ -368,9 +368,9 @@ def test_delta_rule_part_over_cuts(dtype, geom):
         assert float(t[:, 0].abs().max()) == 0.0 and float(t[:, 5].min()) == 3.0     # slots of others stay as they are
 
 
-@pytest.mark.parametrize("waves", [2, 4])
+@pytest.mark.parametrize("lanes", [0, 16, 32])
 @pytest.mark.parametrize("geom", [(3, 3, 32, 16), (4, 2, 128, 40), (2, 1, 47, 5), (2, 2, 192, 33), (1, 1, 256, 70), (16, 4, 64, 64)])
-def test_delta_recurrence_alone(geom, waves):
+def test_delta_recurrence_alone(geom, lanes):
     """The recurrence's kernel on operands of its own (decays down to 0 and up to 1, steps of 0 and 1,
     keys that are no unit vectors), sequences that end inside and at the edge of a chunk."""
     from transformer_amd import kernels as K
@@ -392,7 +392,7 @@ def test_delta_recurrence_alone(geom, waves):
     o = torch.full((nt, H, dv), float("nan"), device=DEV)
     f = lambda a: _t(np.asarray(a, dtype=np.float32))
     K.delta_recurrent(f(q), f(k), f(g), f(v.reshape(nt, -1)), f(b), f((q * k).sum(-1)), state, _t(cu, torch.int32),
-                      _t(slots, torch.int32), o, waves=waves)
+                      _t(slots, torch.int32), o, lanes=lanes)
     rep = lambda a: np.repeat(a, H // G, axis=1)
     for i, n in enumerate(lens):
         r = slice(cu[i], cu[i + 1])

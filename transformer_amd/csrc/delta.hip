@@ -86,11 +86,15 @@ extern "C" int ta_delta_prepare(hipStream_t stream, int dtype, const void* qkv, 
 }
 
 // ------------------------------------------------------------------ prompts
-// Sixteen lanes share a value column, each with R of its key channels (in runs of four: run i of lane l
-// holds channels 64 i + 4 l ..+3, so that a wave's operand reads from LDS meet every bank once); a wave
-// owns four columns. A token costs a wave some 5 R + 20 vector instructions and one exchange among 16
-// lanes for both sums. Operands of the next chunk of tokens are on their way to registers while this
-// chunk is worked on out of one of two LDS buffers, and the next token's leave LDS a token ahead.
+// LANES (16 or 32) lanes share a value column, each with R of its key channels (in runs of four: run i of
+// lane l holds channels 4 LANES i + 4 l ..+3, so that a wave's operand reads from LDS meet every bank once);
+// a wave owns 64 / LANES columns. A token costs a wave some 5 R + 20 vector instructions, and a wave alone on
+// its SIMD issues one every five cycles or so: with few heads and sequences 32 lanes share a column, which
+// shortens the walk; with many, 16 lanes waste less on the exchange. Operands of the next chunk of tokens
+// are on their way to registers while this chunk is worked on out of one of two LDS buffers, and the next
+// token's leave LDS a token ahead.
+#define DR_FEW_COLUMNS 3072
+
 template <int CTRL>
 __device__ __forceinline__ float dr_dpp(float x) {
   return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
@@ -104,92 +108,117 @@ __device__ __forceinline__ float dr_sum16(float x) {
   return x;
 }
 
-template <typename T, int R, int WAVES, bool VEC>
-__global__ __launch_bounds__(WAVES * 64) void delta_recurrent_kernel(
+// both sums over the lanes of a column, the same bits in each of them
+template <int LANES>
+__device__ __forceinline__ void dr_sums(float& w, float& r) {
+  if (LANES == 16) {
+    w = dr_sum16(w);
+    r = dr_sum16(r);
+    return;
+  }
+  // rows of 16 lanes trade places: the even ones are left with what both rows have of w, the odd ones with
+  // theirs of r, one exchange sums either, and a second trade hands both to all lanes
+  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(w), __float_as_uint(r), false, false);
+  const float t = dr_sum16(__uint_as_float(a[0]) + __uint_as_float(a[1]));
+  const auto c = __builtin_amdgcn_permlane16_swap(__float_as_uint(t), __float_as_uint(t), false, false);
+  w = __uint_as_float(c[0]);
+  r = __uint_as_float(c[1]);
+}
+
+template <typename T, int LANES, int R, bool VEC>
+__global__ __launch_bounds__(256) void delta_recurrent_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn, const float* __restrict__ decay,
     const T* __restrict__ v, int v_stride, const float* __restrict__ beta, const float* __restrict__ kq,
     float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ slots, int H, int G, int dk,
     int dv, float* __restrict__ o_out) {
-  constexpr int TC = R <= 8 ? 16 : 8;              // tokens of a chunk (at most 16: see `kept`)
-  constexpr int DKP = 16 * R, COLS = 4 * WAVES, NT = 64 * WAVES;
+  constexpr int DKP = LANES * R, NT = 256, COLS = NT / LANES;
+  constexpr int TC = DKP <= 128 ? 16 : 8;          // tokens of a chunk (at most LANES: see `kept`)
   constexpr int NF = (TC * DKP / 4 + NT - 1) / NT; // runs of four that a thread brings in of each operand
   __shared__ __attribute__((aligned(16))) float sq[2][TC][DKP], sk[2][TC][DKP], sg[2][TC][DKP];
-  __shared__ float sv[2][TC][COLS], sb[2][TC], sx[2][TC];
+  __shared__ float sv[2][NT / COLS][COLS];         // TC rows are used
+  __shared__ float2 sbx[2][TC];                    // step size, k . q
   const int h = blockIdx.x, col0 = blockIdx.y * COLS, b = blockIdx.z;
   const int start = cu_q[b], end = cu_q[b + 1];
   if (start >= end) return;
   const int g = h / (H / G);
-  const int tid = threadIdx.x, lane = tid % 16, cl = tid / 16;
+  const int tid = threadIdx.x, lane = tid % LANES, cl = tid / LANES;
   const int col = col0 + cl;
   float* st = state + ((size_t)slots[b] * H + h) * dk * (size_t)dv;
   float S[R];
 #pragma unroll
   for (int i = 0; i < R; ++i) {
-    const int row = 64 * (i / 4) + 4 * lane + i % 4;
+    const int row = 4 * LANES * (i / 4) + 4 * lane + i % 4;
     S[i] = (row < dk && col < dv) ? st[(size_t)row * dv + col] : 0.f;
   }
   struct Chunk {
     float4 q[NF], k[NF], g[NF];
-    float v, b, x;
+    T v;
+    float b, x;
   };
-  auto run4 = [&](const float* p, int c, float none) {      // four channels from c on; past dk: `none`
-    if (VEC) return c < dk ? *reinterpret_cast<const float4*>(p + c) : float4{none, none, none, none};
-    return float4{c < dk ? p[c] : none, c + 1 < dk ? p[c + 1] : none, c + 2 < dk ? p[c + 2] : none,
-                  c + 3 < dk ? p[c + 3] : none};
+  // Every load is issued without a condition (a channel past dk, a column past dv, a token past the
+  // sequence's end read what is there and are replaced or not used), so that none is waited for before
+  // its chunk goes to LDS. Offsets fit 32 bits (checked on the host).
+  auto run4 = [&](const float* p, uint32_t at, int c) {
+    if (VEC) return *reinterpret_cast<const float4*>(p + at + (c < dk ? c : 0));
+    return float4{p[at + (c < dk ? c : 0)], p[at + (c + 1 < dk ? c + 1 : 0)], p[at + (c + 2 < dk ? c + 2 : 0)],
+                  p[at + (c + 3 < dk ? c + 3 : 0)]};
   };
-  // a token past the sequence's end reads its last token's operands, which are then not used
+  const uint32_t qstep = (uint32_t)(G * dk), gstep = (uint32_t)(H * dk);
   auto fetch = [&](Chunk& f, int t0) {
 #pragma unroll
     for (int e = 0; e < NF; ++e) {
       const int idx = tid + NT * e;
       const int tt = idx / (DKP / 4), c = (idx % (DKP / 4)) * 4;
-      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
-      f.q[e] = run4(qn + (t * G + g) * dk, c, 0.f);
-      f.k[e] = run4(kn + (t * G + g) * dk, c, 0.f);
-      f.g[e] = run4(decay + (t * H + h) * dk, c, 1.f);
+      const uint32_t t = t0 + tt < end ? t0 + tt : end - 1;
+      f.q[e] = run4(qn, t * qstep + g * dk, c);
+      f.k[e] = run4(kn, t * qstep + g * dk, c);
+      f.g[e] = run4(decay, t * gstep + h * dk, c);
     }
     {
-      const int tt = tid / COLS, c = col0 + tid % COLS;     // NT >= TC * COLS
-      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
-      f.v = (tt < TC && c < dv) ? to_f32(v[t * v_stride + (size_t)h * dv + c]) : 0.f;
+      const int c = col0 + tid % COLS;
+      const uint32_t t = t0 + tid / COLS < end ? t0 + tid / COLS : end - 1;
+      f.v = v[t * (size_t)v_stride + h * dv + (c < dv ? c : 0)];
     }
-    {
-      const size_t t = t0 + tid % TC < end ? t0 + tid % TC : end - 1;
-      f.b = beta[t * H + h];
-      f.x = kq[t * G + g];
-    }
+    const uint32_t t = t0 + tid % TC < end ? t0 + tid % TC : end - 1;
+    f.b = beta[t * (uint32_t)H + h];
+    f.x = kq[t * (uint32_t)G + g];
   };
   auto stash = [&](const Chunk& f, int buf) {
 #pragma unroll
     for (int e = 0; e < NF; ++e) {
-      const int idx = tid + NT * e;
+      const int idx = tid + NT * e, c = (idx % (DKP / 4)) * 4;
       if (TC * DKP / 4 % NT == 0 || idx < TC * DKP / 4) {
-        reinterpret_cast<float4*>(&sq[buf][0][0])[idx] = f.q[e];
-        reinterpret_cast<float4*>(&sk[buf][0][0])[idx] = f.k[e];
-        reinterpret_cast<float4*>(&sg[buf][0][0])[idx] = f.g[e];
+        float4 q = f.q[e], k = f.k[e], w = f.g[e];
+        if (c + 4 > dk) {                                     // channels past dk: nothing to read or write, no decay
+          if (c + 0 >= dk) { q.x = k.x = 0.f; w.x = 1.f; }
+          if (c + 1 >= dk) { q.y = k.y = 0.f; w.y = 1.f; }
+          if (c + 2 >= dk) { q.z = k.z = 0.f; w.z = 1.f; }
+          q.w = k.w = 0.f;
+          w.w = 1.f;
+        }
+        reinterpret_cast<float4*>(&sq[buf][0][0])[idx] = q;
+        reinterpret_cast<float4*>(&sk[buf][0][0])[idx] = k;
+        reinterpret_cast<float4*>(&sg[buf][0][0])[idx] = w;
       }
     }
-    if (tid < TC * COLS) (&sv[buf][0][0])[tid] = f.v;
-    if (tid < TC) {
-      sb[buf][tid] = f.b;
-      sx[buf][tid] = f.x;
-    }
+    (&sv[buf][0][0])[tid] = to_f32(f.v);
+    sbx[buf][tid % TC] = float2{f.b, f.x};                    // (several threads write the same)
   };
   struct Token {
     float4 q[R / 4], k[R / 4], g[R / 4];
-    float v, b, x;
+    float v;
+    float2 bx;
   };
   auto take = [&](Token& o, int buf, int tt) {
     if (tt > TC - 1) tt = TC - 1;                           // past the chunk: not used
 #pragma unroll
     for (int i = 0; i < R / 4; ++i) {
-      o.q[i] = *reinterpret_cast<const float4*>(&sq[buf][tt][64 * i + 4 * lane]);
-      o.k[i] = *reinterpret_cast<const float4*>(&sk[buf][tt][64 * i + 4 * lane]);
-      o.g[i] = *reinterpret_cast<const float4*>(&sg[buf][tt][64 * i + 4 * lane]);
+      o.g[i] = *reinterpret_cast<const float4*>(&sg[buf][tt][4 * LANES * i + 4 * lane]);
+      o.k[i] = *reinterpret_cast<const float4*>(&sk[buf][tt][4 * LANES * i + 4 * lane]);
+      o.q[i] = *reinterpret_cast<const float4*>(&sq[buf][tt][4 * LANES * i + 4 * lane]);
     }
     o.v = sv[buf][tt][cl];
-    o.b = sb[buf][tt];
-    o.x = sx[buf][tt];
+    o.bx = sbx[buf][tt];
   };
   float kept = 0.f;                     // lane l keeps the readout of the chunk's token l
   auto token = [&](const Token& o, int tt) {
@@ -206,9 +235,9 @@ __global__ __launch_bounds__(WAVES * 64) void delta_recurrent_kernel(
         r[e] = fmaf(S[4 * i + e], qs[e], r[e]);
       }
     }
-    const float ws = dr_sum16((w[0] + w[1]) + (w[2] + w[3]));
-    const float rs = dr_sum16((r[0] + r[1]) + (r[2] + r[3]));
-    const float u = o.b * (o.v - ws);
+    float ws = (w[0] + w[1]) + (w[2] + w[3]), rs = (r[0] + r[1]) + (r[2] + r[3]);
+    dr_sums<LANES>(ws, rs);
+    const float u = o.bx.x * (o.v - ws);
 #pragma unroll
     for (int i = 0; i < R / 4; ++i) {
       S[4 * i + 0] = fmaf(o.k[i].x, u, S[4 * i + 0]);
@@ -216,7 +245,7 @@ __global__ __launch_bounds__(WAVES * 64) void delta_recurrent_kernel(
       S[4 * i + 2] = fmaf(o.k[i].z, u, S[4 * i + 2]);
       S[4 * i + 3] = fmaf(o.k[i].w, u, S[4 * i + 3]);
     }
-    const float out = fmaf(u, o.x, rs);
+    const float out = fmaf(u, o.bx.y, rs);
     kept = lane == tt ? out : kept;
   };
   {
@@ -228,61 +257,75 @@ __global__ __launch_bounds__(WAVES * 64) void delta_recurrent_kernel(
   int buf = 0;
   for (int t0 = start; t0 < end; t0 += TC, buf ^= 1) {
     const int n = end - t0 < TC ? end - t0 : TC;
-    const bool more = t0 + TC < end;
     Chunk f;
-    if (more) fetch(f, t0 + TC);
+    fetch(f, t0 + TC);                  // behind the last chunk: its last token again, for nothing
     Token a, c;
+    // the next token's operands are asked for in front of this token's arithmetic, and stay there
+    __builtin_amdgcn_sched_barrier(0);
     take(a, buf, 0);
-    for (int tt = 0; tt < n; tt += 2) {
-      take(c, buf, tt + 1);
-      token(a, tt);
-      take(a, buf, tt + 2);
-      if (tt + 1 < n) token(c, tt + 1);
+    if (n == TC) {
+#pragma unroll
+      for (int tt = 0; tt < TC; tt += 2) {
+        take(c, buf, tt + 1);
+        __builtin_amdgcn_sched_barrier(0);
+        token(a, tt);
+        __builtin_amdgcn_sched_barrier(0);
+        if (tt + 2 < TC) take(a, buf, tt + 2);
+        __builtin_amdgcn_sched_barrier(0);
+        token(c, tt + 1);
+        __builtin_amdgcn_sched_barrier(0);
+      }
+    } else {
+      for (int tt = 0; tt < n; ++tt) {
+        token(a, tt);
+        take(a, buf, tt + 1);
+      }
     }
     if (lane < n && col < dv) o_out[((size_t)(t0 + lane) * H + h) * dv + col] = kept;
     // the other buffer's readers are behind the barrier at the end of the turn before
-    if (more) stash(f, buf ^ 1);
+    stash(f, buf ^ 1);
     __syncthreads();
   }
 #pragma unroll
   for (int i = 0; i < R; ++i) {
-    const int row = 64 * (i / 4) + 4 * lane + i % 4;
+    const int row = 4 * LANES * (i / 4) + 4 * lane + i % 4;
     if (row < dk && col < dv) st[(size_t)row * dv + col] = S[i];
   }
 }
 
 // qn, kn, decay, beta, kq: what ta_delta_prepare left. v: [nt] rows, v_stride apart, of H*dv values in
-// the engine's type. state [slots, H, dk, dv] float32; o_out [nt, H, dv] float32. waves per workgroup
-// (2 or 4; 0: chosen by the number of heads and sequences): four value columns each.
+// the engine's type. state [slots, H, dk, dv] float32; o_out [nt, H, dv] float32. lanes that share a value
+// column (16 or 32; 0: chosen by the number of heads and sequences).
 extern "C" int ta_delta_recurrent(hipStream_t stream, int dtype, const float* qn, const float* kn, const float* decay,
                                   const void* v, int v_stride, const float* beta, const float* kq, float* state,
                                   const int* cu_q, const int* slots, int batch, int nt, int H, int G, int dk, int dv,
-                                  int waves, float* o_out) {
+                                  int lanes, float* o_out) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch, "ta_delta_recurrent: bad batch %d / tokens %d", batch, nt);
   TA_REQUIRE(G >= 1 && H >= 1 && H % G == 0 && dk >= 1 && dk <= 256 && dv >= 1 && v_stride >= H * dv,
              "ta_delta_recurrent: %d heads in %d groups of %d / %d", H, G, dk, dv);
-  TA_REQUIRE(waves == 0 || waves == 2 || waves == 4, "ta_delta_recurrent: %d waves", waves);
+  TA_REQUIRE(lanes == 0 || lanes == 16 || lanes == 32, "ta_delta_recurrent: %d lanes", lanes);
+  TA_REQUIRE((long long)nt * H * dk < (1ll << 31), "ta_delta_recurrent: %d tokens of %d heads of %d in one step", nt, H, dk);
   TA_REQUIRE(dtype == TA_F32 || dtype == TA_BF16, "ta_delta_recurrent: unknown dtype %d", dtype);
-  if (waves == 0) waves = (long long)batch * H * ((dv + 15) / 16) >= 512 ? 4 : 2;
-  const int cols = 4 * waves;
+  // 32 lanes a column while that leaves a SIMD no more than about two waves
+  if (lanes == 0) lanes = (long long)batch * H * dv > DR_FEW_COLUMNS ? 16 : 32;
+  if (dk <= 64) lanes = 16;
+  const int cols = 256 / lanes;
   TA_REQUIRE((dv + cols - 1) / cols <= 65535, "ta_delta_recurrent: values of %d", dv);
   dim3 g(H, (dv + cols - 1) / cols, batch);
   const bool vec = dk % 4 == 0 && (((uintptr_t)qn | (uintptr_t)kn | (uintptr_t)decay) & 15) == 0;
-#define DR_RUN(T, RR, W, VE)                                                                                  \
-  delta_recurrent_kernel<T, RR, W, VE><<<g, W * 64, 0, stream>>>(qn, kn, decay, (const T*)v, v_stride, beta, kq, \
-                                                                 state, cu_q, slots, H, G, dk, dv, o_out)
-#define DR_BY_VEC(T, RR, W) \
-  if (vec) DR_RUN(T, RR, W, true); else DR_RUN(T, RR, W, false)
-#define DR_BY_WIDTH(T, W)                                 \
-  if (dk <= 64) { DR_BY_VEC(T, 4, W); }                   \
-  else if (dk <= 128) { DR_BY_VEC(T, 8, W); }             \
-  else if (dk <= 192) { DR_BY_VEC(T, 12, W); }            \
-  else { DR_BY_VEC(T, 16, W); }
-  if (dtype == TA_F32) {
-    if (waves == 4) { DR_BY_WIDTH(float, 4) } else { DR_BY_WIDTH(float, 2) }
-  } else {
-    if (waves == 4) { DR_BY_WIDTH(bf16_t, 4) } else { DR_BY_WIDTH(bf16_t, 2) }
+#define DR_RUN(T, L, RR, VE)                                                                              \
+  delta_recurrent_kernel<T, L, RR, VE><<<g, 256, 0, stream>>>(qn, kn, decay, (const T*)v, v_stride, beta, kq, \
+                                                              state, cu_q, slots, H, G, dk, dv, o_out)
+#define DR_BY_VEC(T, L, RR) \
+  if (vec) DR_RUN(T, L, RR, true); else DR_RUN(T, L, RR, false)
+#define DR_BY_WIDTH(T)                                                  \
+  if (dk <= 64) { DR_BY_VEC(T, 16, 4); }                                \
+  else if (dk <= 128) {                                                 \
+    if (lanes == 32) { DR_BY_VEC(T, 32, 4); } else { DR_BY_VEC(T, 16, 8); } \
+  } else {                                                              \
+    if (lanes == 32) { DR_BY_VEC(T, 32, 8); } else { DR_BY_VEC(T, 16, 16); } \
   }
+  if (dtype == TA_F32) { DR_BY_WIDTH(float) } else { DR_BY_WIDTH(bf16_t) }
 #undef DR_BY_WIDTH
 #undef DR_BY_VEC
 #undef DR_RUN

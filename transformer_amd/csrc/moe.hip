@@ -733,11 +733,24 @@ __global__ __launch_bounds__(256) void glu_limit_kernel(const T* __restrict__ gu
   const size_t t = blockIdx.y;
   const T* g = gu + t * (size_t)ld;
   T* o = out + t * (size_t)di;
-  for (int i = blockIdx.x * 256 + threadIdx.x; i < di; i += gridDim.x * 256) {
-    const float a = fminf(to_f32(g[i]), limit);
-    const float u = fminf(fmaxf(to_f32(g[di + i]), -limit), limit);
-    o[i] = from_f32<T>(a / (1.0f + expf(-slope * a)) * (u + shift));
+  auto unit = [&](T gate, T up) {
+    const float a = fminf(to_f32(gate), limit);
+    const float u = fminf(fmaxf(to_f32(up), -limit), limit);
+    return from_f32<T>(a / (1.0f + expf(-slope * a)) * (u + shift));
+  };
+  constexpr int V = 16 / sizeof(T);     // values of a 16-byte piece
+  struct alignas(16) Piece { T x[V]; };
+  if (di % V == 0 && ld % V == 0 && ((uintptr_t)gu | (uintptr_t)out) % 16 == 0) {
+    for (int i = V * (blockIdx.x * 256 + threadIdx.x); i < di; i += V * gridDim.x * 256) {
+      const Piece a = *reinterpret_cast<const Piece*>(g + i), u = *reinterpret_cast<const Piece*>(g + di + i);
+      Piece r;
+#pragma unroll
+      for (int e = 0; e < V; ++e) r.x[e] = unit(a.x[e], u.x[e]);
+      *reinterpret_cast<Piece*>(o + i) = r;
+    }
+    return;
   }
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < di; i += gridDim.x * 256) o[i] = unit(g[i], g[di + i]);
 }
 
 extern "C" int ta_glu_limit(hipStream_t stream, int dtype, const void* gate_up, int ld, void* out, int nt, int di,

@@ -2104,11 +2104,11 @@ def delta_prepare(qkv: torch.Tensor, z: torch.Tensor, dt_bias, a_log, b_raw: tor
 
 
 def delta_recurrent(qn: torch.Tensor, kn: torch.Tensor, decay: torch.Tensor, v: torch.Tensor, beta: torch.Tensor,
-                    kq: torch.Tensor, state: torch.Tensor, cu_q, slots, o_out: torch.Tensor, waves: int = 0) -> torch.Tensor:
+                    kq: torch.Tensor, state: torch.Tensor, cu_q, slots, o_out: torch.Tensor, lanes: int = 0) -> torch.Tensor:
     """The delta rule along every sequence: S <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o =
     S^T q, head h with the q and k of group h // (heads / groups). qn, kn [nt, G, dk], decay [nt, H, dk],
     beta [nt, H], kq [nt, G] (k . q) float32; v [nt, H * dv] rows in the engine's type; ``state`` [slots, H,
-    dk, dv] float32; o_out [nt, H, dv] float32. waves of a workgroup: 2 or 4 (0: chosen by the shape)."""
+    dk, dv] float32; o_out [nt, H, dv] float32. lanes that share a column: 16 or 32 (0: chosen by the shape)."""
     nt, G, dk = qn.shape
     H = decay.shape[1]
     _dev(v, "v", contiguous=False); _dev(state, "state", torch.float32)
@@ -2127,7 +2127,7 @@ def delta_recurrent(qn: torch.Tensor, kn: torch.Tensor, decay: torch.Tensor, v: 
     _check(library().ta_delta_recurrent(
         _stream(), c_int(_code(v.dtype)), _ptr(qn), _ptr(kn), _ptr(decay), _ptr(v), c_int(vs), _ptr(beta), _ptr(kq),
         _ptr(state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(H), c_int(G), c_int(dk), c_int(dv),
-        c_int(waves), _ptr(o_out)))
+        c_int(lanes), _ptr(o_out)))
     return o_out
 
 
