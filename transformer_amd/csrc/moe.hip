@@ -738,9 +738,9 @@ __global__ __launch_bounds__(256) void glu_limit_kernel(const T* __restrict__ gu
     const float u = fminf(fmaxf(to_f32(up), -limit), limit);
     return from_f32<T>(a / (1.0f + expf(-slope * a)) * (u + shift));
   };
-  constexpr int V = 16 / sizeof(T);     // values of a 16-byte piece
-  struct alignas(16) Piece { T x[V]; };
-  if (di % V == 0 && ld % V == 0 && ((uintptr_t)gu | (uintptr_t)out) % 16 == 0) {
+  constexpr int V = 4;
+  struct alignas(V * sizeof(T)) Piece { T x[V]; };
+  if (di % V == 0 && ld % V == 0 && ((uintptr_t)gu | (uintptr_t)out) % sizeof(Piece) == 0) {
     for (int i = V * (blockIdx.x * 256 + threadIdx.x); i < di; i += V * gridDim.x * 256) {
       const Piece a = *reinterpret_cast<const Piece*>(g + i), u = *reinterpret_cast<const Piece*>(g + di + i);
       Piece r;
