@@ -8,9 +8,9 @@ sequence's first tokens stay visible, a gate per head), "latent_attention" (a ca
 a rotated key part that the heads share, a learned extra term of the softmax denominator per head)
 and "channel_delta" (a delta rule on a matrix state with a decay per head and key channel, behind short
 convolutions). The feed-forward is a gated unit with limits. The stream's norms have gains stored
-around zero; a range of layers may run several times in a row with the same weights, every pass with
-a cache and state of its own and a learned row added to the stream before it; the embedding is scaled
-and doubles as the output matrix, whose logits are scaled.
+around zero; a span of layers can be walked more than once, each repeat with cache layers and state rows
+of its own and a learned row added to the stream in front of it; the embedding is scaled and
+doubles as the output matrix, whose logits are scaled.
 
 Keys: ``architecture``, ``vocab``, ``width``, ``norm.eps``, ``embedding.scale``, ``logit_scale``,
 ``token_side.dim``, ``loop.{start, stop, times}``, ``layers[i].{type, mixer, mlp}``. ``mixer`` by type:
