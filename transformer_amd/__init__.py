@@ -1,4 +1,4 @@
-"""A small decoder engine for one MI355X (Llama, Vametar, Kunitar, Luduvik, Saredra, Zirutar): typed configuration, weights by name,
+"""A small decoder engine for one MI355X (Llama, Vametar, Kunitar, Luduvik, Saredra, Zirutar, Linonex): typed configuration, weights by name,
 blocks assembled from parts, a paged per-sequence cache, one batched step
 function, a generation loop, sampling and trace replay, on hand-written HIP
 kernels for gfx950."""
@@ -8,6 +8,7 @@ from .engine.batch import Entry  # noqa: F401
 from .config.llama import LlamaConfig  # noqa: F401
 from .config.vametar import VametarConfig  # noqa: F401
 from .config.kunitar import KunitarConfig  # noqa: F401
+from .config.linonex import LinonexConfig  # noqa: F401
 from .config.luduvik import LuduvikConfig  # noqa: F401
 from .config.saredra import SaredraConfig  # noqa: F401
 from .config.zirutar import ZirutarConfig  # noqa: F401

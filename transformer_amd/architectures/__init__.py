@@ -1,2 +1,2 @@
 """Registry entries. Importing the package registers them."""
-from . import kunitar, llama, luduvik, saredra, vametar, zirutar  # noqa: F401
+from . import kunitar, linonex, llama, luduvik, saredra, vametar, zirutar  # noqa: F401

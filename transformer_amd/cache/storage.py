@@ -23,7 +23,7 @@ import torch
 
 from .pool import CacheError, CacheFull, SlotPool
 
-from ..kernels import PAGE   # tokens per cache page: one constant, checked against the kernel library
+from ..kernels import PAGE, first_key   # tokens per cache page: one constant, checked against the kernel library
 
 
 @dataclass(frozen=True)
@@ -31,14 +31,18 @@ class KVNeed:
     """Keys and values of every position (or of a window of them). ``value_dim``: width of a
     value row where it differs from the key's (None: the same; 0: keys only, for a mixer that
     keeps one row per token and derives both from it). ``keep_first``: with a window, a sequence's
-    first tokens that stay readable besides it."""
+    first tokens that stay readable besides it. ``chunk``: instead of a window, a position reads the
+    keys of its own chunk of that many tokens, counted from position 0."""
     num_kv_heads: int
     head_dim: int
     window: Optional[int] = None     # None: every earlier position is read
     value_dim: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
 
     def __post_init__(self):
+        if self.chunk is not None and (self.chunk < 1 or self.window is not None):
+            raise CacheError(f"chunks of {self.chunk} tokens beside a window of {self.window}")
         if self.value_dim is None:
             object.__setattr__(self, "value_dim", self.head_dim)
         if self.window is None:                      # everything is kept anyway
@@ -47,6 +51,15 @@ class KVNeed:
     @property
     def keep_pages(self) -> int:
         return -(-self.keep_first // PAGE)
+
+    @property
+    def span(self) -> Optional[int]:
+        """The most tokens behind a position that it reads; None: all."""
+        return self.window if self.chunk is None else self.chunk
+
+    def first_key(self, length: int) -> int:
+        """The first key (besides the kept first tokens) that the token at position ``length`` reads."""
+        return first_key(length + 1, self.window, self.chunk)
 
 
 @dataclass(frozen=True)
@@ -113,10 +126,10 @@ class SequenceCache:
         self.group_pages = [self.num_pages] * len(self.kv_groups)
         if max_step_tokens is not None:
             for g, need in enumerate(self.kv_groups):
-                if need.window is not None:
+                if need.span is not None:
                     # a slot holds at most the pages of its kept first tokens and those that touch
-                    # its window and its share of the step: (window + n - 1) / PAGE + 2
-                    bound = max_slots * (need.keep_pages + need.window // PAGE + 3) + max_step_tokens // PAGE
+                    # its window (or chunk) and its share of the step: (window + n - 1) / PAGE + 2
+                    bound = max_slots * (need.keep_pages + need.span // PAGE + 3) + max_step_tokens // PAGE
                     self.group_pages[g] = max(1, min(self.num_pages, bound))
         self.pool = SlotPool(max_slots, PAGE, dict(enumerate(self.group_pages)))
         self.keys, self.values = [], []
@@ -161,12 +174,12 @@ class SequenceCache:
 
     def release_outside_windows(self, slot: int) -> None:
         """After a step: the next token of the slot sits at position ``length`` and a layer
-        with window w reads keys from ``length + 1 - w`` on; earlier pages go back, but for those of
-        the first tokens that the layer keeps."""
+        with window w reads keys from ``length + 1 - w`` on, one with chunks those of its own chunk; earlier
+        pages go back, but for those of the first tokens that the layer keeps."""
         n = self.pool.length(slot)
         for g, need in enumerate(self.kv_groups):
-            if need.window is not None:
-                self.pool.release_before(slot, g, n + 1 - need.window, need.keep_pages)
+            if need.span is not None:
+                self.pool.release_before(slot, g, need.first_key(n), need.keep_pages)
 
     def bytes(self) -> int:
         n = sum(t.numel() * t.element_size() for t in self.keys + self.values + self.states)

@@ -100,10 +100,13 @@ class RunSpec:
     run reads instead of writing one.
     opening: None, or a row of the model's table of stream rows (``ModelSpec.stream_rows``) that is
     added to the residual stream of every token right before this run.
+    reenter: what the embedding (with ``ModelSpec.after_embed``) gave is added to the stream once more
+    right before this run.
     """
     block: int
     cache_of: Optional[int] = None
     opening: Optional[int] = None
+    reenter: bool = False
 
 
 @dataclass(frozen=True)
@@ -350,6 +353,12 @@ class RoutedMLPSpec:
     up_shift: float = 1.0
     groups: int = 1
     keep_groups: int = 1
+    # identity: behind the experts the router has that many outputs more; an identity expert hands back
+    # its input and has no matrices. correction: a learned number per router output is added to the scores
+    # for the choice alone. factor: the weights (behind ``renormalize``) are multiplied by it.
+    identity: int = 0
+    correction: bool = False
+    factor: float = 1.0
 
 
 @dataclass(frozen=True)
@@ -522,6 +531,8 @@ class SinkAttentionSpec:
     eps: float = 0.0
     values_from_keys: bool = False
     head_gate: bool = False
+    # chunk: instead of a window, a query at position p reads the keys of its own chunk, [p // chunk * chunk, p]
+    chunk: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -569,14 +580,15 @@ class OffsetNormSpec:
 
 @dataclass(frozen=True)
 class GatedDeltaSpec:
-    """Gated delta rule with a decay per head and key channel. q, k (num_kv_heads heads of key_dim) and v
+    """Gated delta rule with a decay per head and key channel, or per head. q, k (num_kv_heads heads of key_dim) and v
     (num_heads of value_dim) pass a causal convolution of ``taps`` per channel (no bias) and silu; q and k
     become unit vectors per head (x / sqrt(sum x^2 + 1e-6)), q is also scaled by key_dim^-1/2; head h reads
     the q and k of group h // (num_heads / num_kv_heads). Per head a state S [key_dim, value_dim], float32,
     zero at a sequence's start: S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q, with beta =
     sigmoid(Wb h) per head and g = exp(-exp(A_log_h) softplus(Wa2 (Wa1 h) + dt_bias)) per head and key
-    channel (Wa1 maps to decay_rank numbers). o is divided by its root mean square per head, times a weight
-    [value_dim] shared by the heads, times sigmoid(Wg2 (Wg1 h)) (Wg1 maps to gate_rank numbers), then
+    channel (Wa1 maps to decay_rank numbers; decay_rank None: one number per head, softplus(Wa h + dt_bias)). o
+    is divided by its root mean square per head, times a weight [value_dim] shared by the heads, times
+    act(Wg2 (Wg1 h)) (Wg1 maps to gate_rank numbers; gate_rank None: act(Wg h)), act = gate_activation, then
     projected. State per sequence: S and the last taps - 1 rows of [q | k | v] as projected."""
     hidden: int
     num_heads: int
@@ -584,7 +596,37 @@ class GatedDeltaSpec:
     key_dim: int
     value_dim: int
     taps: int
-    decay_rank: int
-    gate_rank: int
+    decay_rank: Optional[int]
+    gate_rank: Optional[int]
     eps: float
     kind: str = "gated_delta"
+    gate_activation: str = "sigmoid"
+
+
+# ---------------------------------------------------------------------------------------------
+# Parts that the Linonex decoder added; as above, every size and constant is a field.
+
+@dataclass(frozen=True)
+class LearnedPositionSpec:
+    """An ``after_embed`` part: row p of a learned table [positions, hidden] is added to the token at
+    position p."""
+    hidden: int
+    positions: int
+    kind: str = "learned_positions"
+
+
+@dataclass(frozen=True)
+class MatrixMemorySpec:
+    """The matrix memory of xLSTM (mLSTM). Per head a state S [key_dim, value_dim], a normaliser n [key_dim]
+    and a running maximum m, all float32 and zero at a sequence's start. With q = Wq h * key_dim^-1/2, k = Wk h,
+    v = Wv h and the logarithms of the gates i = cap tanh((Wi h + bi) / cap), f = log sigmoid(cap tanh((Wf h +
+    bf) / cap)) (one per head, cap = gate_cap): m' = max(f + m, i), a = exp(f + m - m'), b = exp(i - m'), S <- a S
+    + b k v^T, n <- a n + b k, o = S^T q / (max(|n . q|, exp(-m')) + 1e-6). o is divided by its root mean square
+    per head, times a weight over all heads' channels, times sigmoid(Wg h), then projected."""
+    hidden: int
+    num_heads: int
+    key_dim: int
+    value_dim: int
+    gate_cap: float
+    eps: float
+    kind: str = "matrix_memory"

@@ -36,7 +36,7 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
     const int* __restrict__ block_table, int max_blocks, const int* __restrict__ cu_q,
     const int* __restrict__ pos0, int nh, int nkv, int dh, int dv, float scale, int window,
     float softcap, int sink_mode, const float* __restrict__ sink, const T* __restrict__ gate, int gate_stride,
-    int gate_dv, int keep) {
+    int gate_dv, int keep, int chunk) {
   extern __shared__ float smem[];
   const int group = nh / nkv;
   const int b = blockIdx.z, kvh = blockIdx.y;
@@ -67,17 +67,9 @@ __global__ __launch_bounds__(256) void attn_generic_kernel(
   const int qi_min = row0 / group;
   const int last_row = (row0 + ROWS - 1 < nrows - 1) ? row0 + ROWS - 1 : nrows - 1;
   const int tile_end = p0 + last_row / group + 1;                       // exclusive
-  int tile_start = 0;
-  if (window > 0) {
-    tile_start = p0 + qi_min + 1 - window;
-    if (tile_start < 0) tile_start = 0;
-  }
+  const int tile_start = ta_first_key(p0 + qi_min + 1, window, chunk);
   const int my_end = p0 + qi + 1;
-  int my_start = 0;
-  if (window > 0) {
-    my_start = my_end - window;
-    if (my_start < 0) my_start = 0;
-  }
+  const int my_start = ta_first_key(my_end, window, chunk);
 
   const int nd = (dv + 15) / 16;          // output columns lane, lane + 16, ... of this lane
   float acc[16];
@@ -197,13 +189,15 @@ static int attention_generic_launch(hipStream_t stream, int dtype, const void* q
                                     const int* cu_q, const int* pos0, int batch, int max_qlen,
                                     int nh, int nkv, int dh, int dv, float scale, int window,
                                     float softcap = 0.f, int sink_mode = 0, const float* sink = nullptr,
-                                    const void* gate = nullptr, int gate_stride = 0, int gate_dv = 0, int keep = 0) {
+                                    const void* gate = nullptr, int gate_stride = 0, int gate_dv = 0, int keep = 0,
+                                    int chunk = 0) {
   TA_REQUIRE(batch >= 0 && max_qlen >= 0, "ta_attention_generic: bad batch=%d max_qlen=%d", batch, max_qlen);
   TA_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 2 || sink != nullptr) && softcap >= 0.f,
              "ta_attention_generic: sink mode %d, cap %f", sink_mode, softcap);
   TA_REQUIRE(gate == nullptr || (gate_dv >= 0 && gate_dv <= dv && gate_stride >= nh * (gate_dv > 0 ? gate_dv : 1)),
              "ta_attention_generic: gate rows of %d", gate_stride);
   TA_REQUIRE(keep >= 0 && (keep == 0 || window > 0), "ta_attention_generic: %d kept keys beside a window of %d", keep, window);
+  TA_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "ta_attention_generic: chunks of %d beside a window of %d", chunk, window);
   TA_REQUIRE(nh > 0 && nkv > 0 && nh % nkv == 0, "ta_attention_generic: %d heads do not divide into %d kv heads", nh, nkv);
   TA_REQUIRE(dh >= 1 && dh <= 256 && dv >= 1 && dv <= 256,
              "ta_attention_generic: key width %d / value width %d outside [1, 256]", dh, dv);
@@ -218,12 +212,12 @@ static int attention_generic_launch(hipStream_t stream, int dtype, const void* q
     attn_generic_kernel<float><<<g, blk, lds, stream>>>(
         (const float*)q, q_stride, (float*)out, out_stride, (const float*)kcache,
         (const float*)vcache, block_table, max_blocks, cu_q, pos0, nh, nkv, dh, dv, scale, window,
-        softcap, sink_mode, sink, (const float*)gate, gate_stride, gate_dv, keep);
+        softcap, sink_mode, sink, (const float*)gate, gate_stride, gate_dv, keep, chunk);
   else if (dtype == TA_BF16)
     attn_generic_kernel<bf16_t><<<g, blk, lds, stream>>>(
         (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)kcache,
         (const bf16_t*)vcache, block_table, max_blocks, cu_q, pos0, nh, nkv, dh, dv, scale, window,
-        softcap, sink_mode, sink, (const bf16_t*)gate, gate_stride, gate_dv, keep);
+        softcap, sink_mode, sink, (const bf16_t*)gate, gate_stride, gate_dv, keep, chunk);
   else
     return ta_fail("ta_attention_generic: unknown dtype %d", dtype);
   return ta_check_launch("ta_attention_generic");
@@ -252,15 +246,16 @@ extern "C" int ta_attention_generic_dv(hipStream_t stream, int dtype, const void
 // tanh(score / softcap) after the scale; sink_mode 1: the denominator holds one more term exp(0);
 // 2: exp(sink[head]) (float32 [nh]); gate: rows [nt, >= nh*gate_dv] whose sigmoid multiplies the first gate_dv
 // columns of every head of the result (gate_dv <= dv; 0: rows [nt, >= nh] with one number per head). keep:
-// with a window, the first `keep` keys of a sequence are seen as well.
+// with a window, the first `keep` keys of a sequence are seen as well. chunk > 0 (without a window): a query
+// at position p sees the keys from (p / chunk) * chunk on.
 extern "C" int ta_attention_generic_sink(hipStream_t stream, int dtype, const void* q, int q_stride,
                                          void* out, int out_stride, const void* kcache,
                                          const void* vcache, const int* block_table, int max_blocks,
                                          const int* cu_q, const int* pos0, int batch, int max_qlen,
                                          int nh, int nkv, int dh, int dv, float scale, int window,
                                          float softcap, int sink_mode, const float* sink, const void* gate,
-                                         int gate_stride, int gate_dv, int keep) {
+                                         int gate_stride, int gate_dv, int keep, int chunk) {
   return attention_generic_launch(stream, dtype, q, q_stride, out, out_stride, kcache, vcache, block_table,
                                   max_blocks, cu_q, pos0, batch, max_qlen, nh, nkv, dh, dv, scale, window,
-                                  softcap, sink_mode, sink, gate, gate_stride, gate_dv, keep);
+                                  softcap, sink_mode, sink, gate, gate_stride, gate_dv, keep, chunk);
 }

@@ -68,12 +68,13 @@ __device__ __forceinline__ uint32_t pack2(float a, float b) { return f32x2_to_bf
 //   gate: rows [token][gate_stride] whose sigmoid multiplies the first gate_dv columns of every head
 //     (gate_dv 0: one number per head)
 //   keep: with a window, the sequence's first `keep` keys are seen as well
+//   chunk: instead of a window, a query at position p sees the keys from (p / chunk) * chunk on (0: not)
 struct AttnExtra {
   float cap_k, cap_r;
   int exact, sink_mode;
   const float* sink;
   const bf16_t* gate;
-  int gate_stride, gate_dv, keep;
+  int gate_stride, gate_dv, keep, chunk;
 };
 
 __device__ __forceinline__ float capped_score(float s, float cap_k, float cap_r) {
@@ -357,19 +358,10 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(
   const int last_row = (row0 + 31 < nrows - 1) ? row0 + 31 : nrows - 1;
   const int tile_end = p0 + last_row / group + 1;          // largest my_end of the tile
   const int tile_min_end = p0 + row0 / group + 1;          // smallest my_end of the tile
-  int tile_start = 0, tile_max_start = 0;
-  if (window > 0) {
-    tile_start = tile_min_end - window;
-    if (tile_start < 0) tile_start = 0;
-    tile_max_start = tile_end - window;
-    if (tile_max_start < 0) tile_max_start = 0;
-  }
-  int my_end = row_ok ? p0 + qi + 1 : 0;
-  int my_start = 0;
-  if (window > 0 && row_ok) {
-    my_start = my_end - window;
-    if (my_start < 0) my_start = 0;
-  }
+  const int chunk = XTRA ? x.chunk : 0;
+  const int tile_start = ta_first_key(tile_min_end, window, chunk), tile_max_start = ta_first_key(tile_end, window, chunk);
+  const int my_end = row_ok ? p0 + qi + 1 : 0;
+  const int my_start = row_ok ? ta_first_key(my_end, window, chunk) : 0;
   const bool all_rows = row0 + 32 <= nrows;
 
   const int* table = block_table + (size_t)b * max_blocks;
@@ -439,27 +431,15 @@ __global__ __launch_bounds__(256, 2) void attn_rows_lds_kernel(
   // key ranges: of the workgroup (what is loaded) and of this wave (what it multiplies)
   const int wg_last = (wg_row0 + 127 < nrows - 1) ? wg_row0 + 127 : nrows - 1;
   const int wg_end = p0 + wg_last / group + 1;
-  int wg_start = 0;
-  if (window > 0) {
-    wg_start = p0 + wg_row0 / group + 1 - window;
-    if (wg_start < 0) wg_start = 0;
-  }
+  const int chunk = XTRA ? x.chunk : 0;
+  const int wg_start = ta_first_key(p0 + wg_row0 / group + 1, window, chunk);
   const int last_row = (row0 + 31 < nrows - 1) ? row0 + 31 : nrows - 1;
   const int tile_end = wave_ok ? p0 + last_row / group + 1 : 0;
   const int tile_min_end = p0 + row0 / group + 1;
-  int tile_start = 0, tile_max_start = 0;
-  if (window > 0 && wave_ok) {
-    tile_start = tile_min_end - window;
-    if (tile_start < 0) tile_start = 0;
-    tile_max_start = tile_end - window;
-    if (tile_max_start < 0) tile_max_start = 0;
-  }
+  const int tile_start = wave_ok ? ta_first_key(tile_min_end, window, chunk) : 0;
+  const int tile_max_start = wave_ok ? ta_first_key(tile_end, window, chunk) : 0;
   const int my_end = row_ok ? p0 + qi + 1 : 0;
-  int my_start = 0;
-  if (window > 0 && row_ok) {
-    my_start = my_end - window;
-    if (my_start < 0) my_start = 0;
-  }
+  const int my_start = row_ok ? ta_first_key(my_end, window, chunk) : 0;
   const bool all_rows = row0 + 32 <= nrows;
 
   const int* table = block_table + (size_t)b * max_blocks;
@@ -1104,13 +1084,9 @@ __global__ __launch_bounds__(WAVES * 64, 2) void attn_keys_kernel(
     }
   }
 
+  const int vis_start = ta_first_key(kv_len, window, XTRA ? x.chunk : 0);
   const int my_end = row_ok ? kv_len : 0;
-  int my_start = 0;
-  if (window > 0 && row_ok) {
-    my_start = my_end - window;
-    if (my_start < 0) my_start = 0;
-  }
-  const int vis_start = (window > 0 && kv_len > window) ? kv_len - window : 0;
+  const int my_start = row_ok ? vis_start : 0;
   const int n_pages = (kv_len + TA_PAGE - 1) / TA_PAGE;
   int pg_lo = unit_first;
   int pg_hi = unit_first + unit_count;
@@ -1914,7 +1890,7 @@ static const float LOG2E = 1.4426950408889634f;
 // Prompts (any mix of lengths, also single tokens). Same arguments as ta_attention_generic.
 static int make_extra(const char* what, AttnExtra* x, int nh, int dh, float scale, float softcap, int exact,
                       int sink_mode, const float* sink, const void* gate, int gate_stride, int gate_dv, int window,
-                      int keep) {
+                      int keep, int chunk) {
   TA_REQUIRE(softcap >= 0.f && scale > 0.f, "%s: cap %f / scale %f", what, softcap, scale);
   TA_REQUIRE(sink_mode >= 0 && sink_mode <= 2 && (sink_mode != 2 || sink != nullptr), "%s: sink mode %d", what, sink_mode);
   TA_REQUIRE(gate == nullptr || (gate_dv >= 0 && gate_dv <= dh && gate_stride >= nh * (gate_dv > 0 ? gate_dv : 1)),
@@ -1928,7 +1904,9 @@ static int make_extra(const char* what, AttnExtra* x, int nh, int dh, float scal
   x->gate = (const bf16_t*)gate;
   x->gate_stride = gate_stride;
   x->gate_dv = gate_dv;
+  TA_REQUIRE(chunk >= 0 && (chunk == 0 || window <= 0), "%s: chunks of %d beside a window of %d", what, chunk, window);
   x->keep = keep;
+  x->chunk = chunk;
   return 0;
 }
 
@@ -2014,17 +1992,17 @@ extern "C" int ta_attention_rows_bf16(hipStream_t stream, const void* q, int q_s
 // The same with the options of a capped, sunk and gated softmax (see AttnExtra): softcap > 0 caps the
 // scaled scores; exact: 32-bit softmax weights in the second product; sink_mode / sink; gate rows
 // [tokens][gate_stride] with gate_dv columns per head (0: one number per head); keep: first keys that a
-// window shows as well. use_lds 0 or 1.
+// window shows as well; chunk > 0: keys of the query's own chunk instead of a window. use_lds 0 or 1.
 extern "C" int ta_attention_rows_sink_bf16(hipStream_t stream, const void* q, int q_stride, void* out,
                                            int out_stride, const void* kcache, const void* vcache,
                                            const int* block_table, int max_blocks, const int* cu_q,
                                            const int* pos0, int batch, int max_qlen, int nh, int nkv,
                                            int dh, float scale, int window, int use_lds, float softcap, int exact,
                                            int sink_mode, const float* sink, const void* gate, int gate_stride,
-                                           int gate_dv, int keep) {
+                                           int gate_dv, int keep, int chunk) {
   AttnExtra x;
   if (make_extra("ta_attention_rows_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv, window,
-                 keep))
+                 keep, chunk))
     return 1;
   TA_REQUIRE(use_lds == 0 || use_lds == 1, "ta_attention_rows_sink_bf16: kernels 0 and 1 take the options, not %d", use_lds);
   return attention_rows_launch(stream, q, q_stride, out, out_stride, kcache, vcache, block_table, max_blocks, cu_q,
@@ -2130,10 +2108,10 @@ extern "C" int ta_attention_keys_sink_bf16(hipStream_t stream, const void* q, in
                                            int window, const int* units, const int* seq_units, int n_units,
                                            int waves, float* scratch, float softcap, int exact, int sink_mode,
                                            const float* sink, const void* gate, int gate_stride, int gate_dv,
-                                           int keep) {
+                                           int keep, int chunk) {
   AttnExtra x;
   if (make_extra("ta_attention_keys_sink_bf16", &x, nh, dh, scale, softcap, exact, sink_mode, sink, gate, gate_stride, gate_dv, window,
-                 keep))
+                 keep, chunk))
     return 1;
   return attention_keys_launch(stream, q, q_stride, nullptr, nullptr, 0, nullptr, out, out_stride, kcache, vcache,
                                block_table, max_blocks, pos0, batch, nh, nkv, dh, scale, window, units, seq_units,

@@ -338,9 +338,17 @@ __global__ __launch_bounds__(256) void qk_rotate_store_kernel(
   const int t = blockIdx.x;
   T* row = qkv + (size_t)t * stride;
   const int nq = nh * dk, nk = nkv_own * dk, nv = nkv_own * dv;
-  const int half = rot / 2, hd2 = dk / 2;              // dk is even
+  const int half = rot / 2, hd2 = dk / 2;              // dk is even where something is added or turned
   const float2* ang = cs ? cs + (size_t)t * half : nullptr;
   const int page = dest ? dest[t] / TA_PAGE : 0, off = dest ? dest[t] % TA_PAGE : 0;
+  // nothing to add or to turn: q stays as it is, the keys are copied
+  if (ang == nullptr && bias == nullptr) {
+    if (dest)
+      for (int i = threadIdx.x; i < nk; i += 256) {
+        const int g = i / dk, c = i - g * dk;
+        kcache[(((size_t)page * nkv + g) * TA_PAGE + off) * dk + c] = row[nq + i];
+      }
+  } else
   for (int i = threadIdx.x; i < (nq + nk) / 2; i += 256) {
     const int head = i / hd2, p = i - head * hd2;      // pair p of head (q heads first, then k heads)
     int c0, c1;
@@ -387,8 +395,8 @@ extern "C" int ta_qk_rotate_store(hipStream_t stream, int dtype, void* qkv, int 
                                   const float* cs, int rot, int style, const int* dest, void* kcache, void* vcache,
                                   int nt, int nh, int nkv, int nkv_own, int dk, int dv, int dvs) {
   TA_REQUIRE(dvs >= dv, "ta_qk_rotate_store: value rows of %d do not hold values of %d", dvs, dv);
-  TA_REQUIRE(nt >= 0 && nh >= 1 && nkv >= 1 && (nkv_own == 0 || nkv_own == nkv) && dk >= 2 && dk % 2 == 0 && dv >= 1,
-             "ta_qk_rotate_store: bad sizes nt=%d heads=%d/%d (%d own) widths %d/%d", nt, nh, nkv, nkv_own, dk, dv);
+  TA_REQUIRE(nt >= 0 && nh >= 1 && nkv >= 1 && (nkv_own == 0 || nkv_own == nkv) && dk >= 1 && dv >= 1 &&
+             (dk % 2 == 0 || (rot == 0 && bias == nullptr)), "ta_qk_rotate_store: bad sizes nt=%d heads=%d/%d (%d own) widths %d/%d", nt, nh, nkv, nkv_own, dk, dv);
   TA_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dk && (rot == 0 || cs != nullptr) && (style == 0 || style == 1),
              "ta_qk_rotate_store: %d rotated coordinates of %d, style %d", rot, dk, style);
   TA_REQUIRE(stride >= nh * dk + nkv_own * (dk + dv), "ta_qk_rotate_store: rows of %d are too short", stride);

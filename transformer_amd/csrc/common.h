@@ -59,6 +59,13 @@ __device__ __forceinline__ float ta_glu(const TaGlu& p, float g, float u) {
   return g / (1.0f + expf(-g)) * u;
 }
 
+// The first key that a query sees whose own key is the last before `end`: a window shows the last
+// `window` keys, chunks those from its chunk's start on (chunk counted from position 0); both 0: all.
+__device__ __forceinline__ int ta_first_key(int end, int window, int chunk) {
+  if (chunk > 0) return end > 0 ? (int)((unsigned)(end - 1) / (unsigned)chunk * (unsigned)chunk) : 0;
+  return (window > 0 && end > window) ? end - window : 0;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = TA_WAVE / 2; o > 0; o >>= 1) v += __shfl_xor(v, o, TA_WAVE);

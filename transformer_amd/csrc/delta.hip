@@ -2,13 +2,14 @@
 // corrected, not just added to, by every token:
 //
 //     S <- diag(g_t) S,   u_t = beta_t (v_t - S^T k_t),   S <- S + k_t u_t^T,   o_t = S^T q_t
-//     g_t = exp(-exp(A_h) softplus(z_t + dt_bias)) per key channel,  beta_t = sigmoid(b_t),
+//     g_t = exp(-exp(A_h) softplus(z_t + dt_bias)) per key channel, or one for the whole head,
+//     beta_t = sigmoid(b_t),
 //     q_t, k_t of unit length (q_t times a constant besides); the heads of a group share q and k
 //
 //   delta_prepare   : unit q and k, their product k.q, decays and step sizes of all tokens at once
 //   delta_recurrent : walks a sequence's tokens in order with S in registers (prompts)
-//   delta_step      : a step of single tokens in one kernel: low-rank decay and gate, unit vectors,
-//                     the state's update, the readout's norm and gate
+//   delta_step      : a step of single tokens in one kernel: decay and gate (low-rank products, or
+//                     projections of their own), unit vectors, the state's update, the readout's norm and gate
 //
 // The readout needs the updated state, but S_new^T q = (g S)^T q + u (k.q): both sums over key
 // channels are taken of the decayed state side by side, and the update is no part of the chain
@@ -24,16 +25,17 @@ __device__ __forceinline__ float dr_softplus(float z) { return fmaxf(z, 0.f) + l
 #define DR_UNIT_EPS 1e-6f       // under the root of a vector's length
 
 // ------------------------------------------------------------------ what does not depend on the state
-// One workgroup per token; a wave takes units in turn: the G pairs (q, k), then the H decays.
-template <typename T>
+// One workgroup per token; a wave takes units in turn: the G pairs (q, k), then the H decays (HEAD: z
+// holds one number per head, in the engine's type, and all heads' decays are one unit).
+template <typename T, typename TZ, bool HEAD>
 __global__ __launch_bounds__(256) void delta_prepare_kernel(
-    const T* __restrict__ qkv, int stride, const float* __restrict__ z, const float* __restrict__ dt_bias,
+    const T* __restrict__ qkv, int stride, const TZ* __restrict__ z, int zstride, const float* __restrict__ dt_bias,
     const float* __restrict__ a_log, const T* __restrict__ braw, int bstride, int G, int H, int dk, float qscale,
     float* __restrict__ qn, float* __restrict__ kn, float* __restrict__ decay, float* __restrict__ beta,
     float* __restrict__ kq) {
   const size_t t = blockIdx.x;
   const int wave = threadIdx.x / TA_WAVE, lane = threadIdx.x % TA_WAVE;
-  for (int u = wave; u < G + H; u += 4) {
+  for (int u = wave; u < G + (HEAD ? 1 : H); u += 4) {
     if (u < G) {
       const T* q = qkv + t * stride + u * dk;
       const T* k = q + G * dk;
@@ -53,35 +55,44 @@ __global__ __launch_bounds__(256) void delta_prepare_kernel(
         kn[(t * G + u) * dk + c] = to_f32(k[c]) * fk;
       }
       if (lane == 0) kq[t * G + u] = sx * fq * fk;
+    } else if (HEAD) {
+      for (int h = lane; h < H; h += TA_WAVE) {
+        decay[t * H + h] = expf(-expf(a_log[h]) * dr_softplus(to_f32(z[t * zstride + h]) + dt_bias[h]));
+        beta[t * H + h] = dr_sigmoid(to_f32(braw[t * bstride + h]));
+      }
     } else {
       const int h = u - G;
       const float rate = expf(a_log[h]);
       for (int c = lane; c < dk; c += TA_WAVE) {
         const size_t at = (t * H + h) * dk + c;
-        decay[at] = expf(-rate * dr_softplus(z[at] + dt_bias[h * dk + c]));
+        decay[at] = expf(-rate * dr_softplus(to_f32(z[t * zstride + h * dk + c]) + dt_bias[h * dk + c]));
       }
       if (lane == 0) beta[t * H + h] = dr_sigmoid(to_f32(braw[t * bstride + h]));
     }
   }
 }
 
-// qkv: [nt, stride] rows of [q: G*dk | k: G*dk | ...] behind convolution and activation; z [nt, H*dk]
-// float32 decay inputs without their bias; braw: [nt] rows, bstride apart, of H step-size inputs.
+// qkv: [nt, stride] rows of [q: G*dk | k: G*dk | ...] behind convolution and activation; z: decay inputs
+// without their bias, [nt, H*dk] float32, or with per_head rows, zstride apart, of H numbers in the engine's
+// type (dt_bias then holds H, decay is [nt, H]); braw: [nt] rows, bstride apart, of H step-size inputs.
 // qn, kn [nt, G, dk], decay [nt, H, dk], beta [nt, H], kq [nt, G]: float32.
-extern "C" int ta_delta_prepare(hipStream_t stream, int dtype, const void* qkv, int stride, const float* z,
-                                const float* dt_bias, const float* a_log, const void* braw, int bstride, int nt,
+extern "C" int ta_delta_prepare(hipStream_t stream, int dtype, const void* qkv, int stride, const void* z,
+                                int zstride, int per_head, const float* dt_bias, const float* a_log, const void* braw, int bstride, int nt,
                                 int G, int H, int dk, float qscale, float* qn, float* kn, float* decay, float* beta,
                                 float* kq) {
   TA_REQUIRE(nt >= 0 && G >= 1 && H >= 1 && H % G == 0 && dk >= 1, "ta_delta_prepare: bad sizes nt=%d heads=%d/%d width %d", nt, H, G, dk);
-  TA_REQUIRE(stride >= 2 * G * dk && bstride >= H, "ta_delta_prepare: rows of %d / %d are too short", stride, bstride);
+  TA_REQUIRE(stride >= 2 * G * dk && bstride >= H && zstride >= (per_head ? H : H * dk), "ta_delta_prepare: rows of %d / %d are too short", stride, bstride);
   if (nt == 0) return 0;
-  if (dtype == TA_F32)
-    delta_prepare_kernel<float><<<nt, 256, 0, stream>>>((const float*)qkv, stride, z, dt_bias, a_log, (const float*)braw,
-                                                        bstride, G, H, dk, qscale, qn, kn, decay, beta, kq);
-  else if (dtype == TA_BF16)
-    delta_prepare_kernel<bf16_t><<<nt, 256, 0, stream>>>((const bf16_t*)qkv, stride, z, dt_bias, a_log, (const bf16_t*)braw,
-                                                         bstride, G, H, dk, qscale, qn, kn, decay, beta, kq);
-  else return ta_fail("ta_delta_prepare: unknown dtype %d", dtype);
+#define DP_RUN(T, TZ, HD)                                                                                           \
+  delta_prepare_kernel<T, TZ, HD><<<nt, 256, 0, stream>>>((const T*)qkv, stride, (const TZ*)z, zstride, dt_bias, a_log, \
+                                                          (const T*)braw, bstride, G, H, dk, qscale, qn, kn, decay,    \
+                                                          beta, kq)
+  if (dtype == TA_F32) {
+    if (per_head) DP_RUN(float, float, true); else DP_RUN(float, float, false);
+  } else if (dtype == TA_BF16) {
+    if (per_head) DP_RUN(bf16_t, bf16_t, true); else DP_RUN(bf16_t, float, false);
+  } else return ta_fail("ta_delta_prepare: unknown dtype %d", dtype);
+#undef DP_RUN
   return ta_check_launch("ta_delta_prepare");
 }
 
@@ -125,7 +136,8 @@ __device__ __forceinline__ void dr_sums(float& w, float& r) {
   r = __uint_as_float(c[1]);
 }
 
-template <typename T, int LANES, int R, bool VEC>
+// HEAD: one decay per token and head, [nt, H]; it travels with the step size.
+template <typename T, int LANES, int R, bool VEC, bool HEAD>
 __global__ __launch_bounds__(256) void delta_recurrent_kernel(
     const float* __restrict__ qn, const float* __restrict__ kn, const float* __restrict__ decay,
     const T* __restrict__ v, int v_stride, const float* __restrict__ beta, const float* __restrict__ kq,
@@ -134,9 +146,10 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
   constexpr int DKP = LANES * R, NT = 256, COLS = NT / LANES;
   constexpr int TC = DKP <= 128 ? 16 : 8;          // tokens of a chunk (at most LANES: see `kept`)
   constexpr int NF = (TC * DKP / 4 + NT - 1) / NT; // runs of four that a thread brings in of each operand
-  __shared__ __attribute__((aligned(16))) float sq[2][TC][DKP], sk[2][TC][DKP], sg[2][TC][DKP];
+  __shared__ __attribute__((aligned(16))) float sq[2][TC][DKP], sk[2][TC][DKP], sg[2][HEAD ? 1 : TC][DKP];
   __shared__ float sv[2][NT / COLS][COLS];         // TC rows are used
   __shared__ float2 sbx[2][TC];                    // step size, k . q
+  __shared__ float sgh[2][TC];                     // the head's decay (HEAD)
   const int h = blockIdx.x, col0 = blockIdx.y * COLS, b = blockIdx.z;
   const int start = cu_q[b], end = cu_q[b + 1];
   if (start >= end) return;
@@ -151,9 +164,9 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
     S[i] = (row < dk && col < dv) ? st[(size_t)row * dv + col] : 0.f;
   }
   struct Chunk {
-    float4 q[NF], k[NF], g[NF];
+    float4 q[NF], k[NF], g[HEAD ? 1 : NF];
     T v;
-    float b, x;
+    float b, x, gh;
   };
   // Every load is issued without a condition (a channel past dk, a column past dv, a token past the
   // sequence's end read what is there and are replaced or not used), so that none is waited for before
@@ -172,7 +185,7 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
       const uint32_t t = t0 + tt < end ? t0 + tt : end - 1;
       f.q[e] = run4(qn, t * qstep + g * dk, c);
       f.k[e] = run4(kn, t * qstep + g * dk, c);
-      f.g[e] = run4(decay, t * gstep + h * dk, c);
+      if (!HEAD) f.g[e] = run4(decay, t * gstep + h * dk, c);
     }
     {
       const int c = col0 + tid % COLS;
@@ -182,13 +195,14 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
     const uint32_t t = t0 + tid % TC < end ? t0 + tid % TC : end - 1;
     f.b = beta[t * (uint32_t)H + h];
     f.x = kq[t * (uint32_t)G + g];
+    f.gh = HEAD ? decay[t * (uint32_t)H + h] : 1.f;
   };
   auto stash = [&](const Chunk& f, int buf) {
 #pragma unroll
     for (int e = 0; e < NF; ++e) {
       const int idx = tid + NT * e, c = (idx % (DKP / 4)) * 4;
       if (TC * DKP / 4 % NT == 0 || idx < TC * DKP / 4) {
-        float4 q = f.q[e], k = f.k[e], w = f.g[e];
+        float4 q = f.q[e], k = f.k[e], w = f.g[HEAD ? 0 : e];
         if (c + 4 > dk) {                                     // channels past dk: nothing to read or write, no decay
           if (c + 0 >= dk) { q.x = k.x = 0.f; w.x = 1.f; }
           if (c + 1 >= dk) { q.y = k.y = 0.f; w.y = 1.f; }
@@ -198,39 +212,42 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
         }
         reinterpret_cast<float4*>(&sq[buf][0][0])[idx] = q;
         reinterpret_cast<float4*>(&sk[buf][0][0])[idx] = k;
-        reinterpret_cast<float4*>(&sg[buf][0][0])[idx] = w;
+        if (!HEAD) reinterpret_cast<float4*>(&sg[buf][0][0])[idx] = w;
       }
     }
     (&sv[buf][0][0])[tid] = to_f32(f.v);
     sbx[buf][tid % TC] = float2{f.b, f.x};                    // (several threads write the same)
+    if (HEAD) sgh[buf][tid % TC] = f.gh;
   };
   struct Token {
-    float4 q[R / 4], k[R / 4], g[R / 4];
-    float v;
+    float4 q[R / 4], k[R / 4], g[HEAD ? 1 : R / 4];
+    float v, gh;
     float2 bx;
   };
   auto take = [&](Token& o, int buf, int tt) {
     if (tt > TC - 1) tt = TC - 1;                           // past the chunk: not used
 #pragma unroll
     for (int i = 0; i < R / 4; ++i) {
-      o.g[i] = *reinterpret_cast<const float4*>(&sg[buf][tt][4 * LANES * i + 4 * lane]);
+      if (!HEAD) o.g[i] = *reinterpret_cast<const float4*>(&sg[buf][tt][4 * LANES * i + 4 * lane]);
       o.k[i] = *reinterpret_cast<const float4*>(&sk[buf][tt][4 * LANES * i + 4 * lane]);
       o.q[i] = *reinterpret_cast<const float4*>(&sq[buf][tt][4 * LANES * i + 4 * lane]);
     }
     o.v = sv[buf][tt][cl];
     o.bx = sbx[buf][tt];
+    o.gh = HEAD ? sgh[buf][tt] : 1.f;
   };
   float kept = 0.f;                     // lane l keeps the readout of the chunk's token l
   auto token = [&](const Token& o, int tt) {
     float w[4] = {0.f, 0.f, 0.f, 0.f}, r[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int i = 0; i < R / 4; ++i) {
-      const float gs[4] = {o.g[i].x, o.g[i].y, o.g[i].z, o.g[i].w};
+      const float4 g4 = o.g[HEAD ? 0 : i];
+      const float gs[4] = {g4.x, g4.y, g4.z, g4.w};
       const float ks[4] = {o.k[i].x, o.k[i].y, o.k[i].z, o.k[i].w};
       const float qs[4] = {o.q[i].x, o.q[i].y, o.q[i].z, o.q[i].w};
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
-        S[4 * i + e] *= gs[e];
+        S[4 * i + e] *= HEAD ? o.gh : gs[e];
         w[e] = fmaf(S[4 * i + e], ks[e], w[e]);
         r[e] = fmaf(S[4 * i + e], qs[e], r[e]);
       }
@@ -249,7 +266,7 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
     kept = lane == tt ? out : kept;
   };
   {
-    Chunk f;
+    Chunk f{};
     fetch(f, start);
     stash(f, 0);
   }
@@ -257,9 +274,9 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
   int buf = 0;
   for (int t0 = start; t0 < end; t0 += TC, buf ^= 1) {
     const int n = end - t0 < TC ? end - t0 : TC;
-    Chunk f;
+    Chunk f{};
     fetch(f, t0 + TC);                  // behind the last chunk: its last token again, for nothing
-    Token a, c;
+    Token a{}, c{};
     // the next token's operands are asked for in front of this token's arithmetic, and stay there
     __builtin_amdgcn_sched_barrier(0);
     take(a, buf, 0);
@@ -295,11 +312,11 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
 
 // qn, kn, decay, beta, kq: what ta_delta_prepare left. v: [nt] rows, v_stride apart, of H*dv values in
 // the engine's type. state [slots, H, dk, dv] float32; o_out [nt, H, dv] float32. lanes that share a value
-// column (16 or 32; 0: chosen by the number of heads and sequences).
+// column (16 or 32; 0: chosen by the number of heads and sequences). per_head: decay is [nt, H].
 extern "C" int ta_delta_recurrent(hipStream_t stream, int dtype, const float* qn, const float* kn, const float* decay,
                                   const void* v, int v_stride, const float* beta, const float* kq, float* state,
                                   const int* cu_q, const int* slots, int batch, int nt, int H, int G, int dk, int dv,
-                                  int lanes, float* o_out) {
+                                  int lanes, int per_head, float* o_out) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch, "ta_delta_recurrent: bad batch %d / tokens %d", batch, nt);
   TA_REQUIRE(G >= 1 && H >= 1 && H % G == 0 && dk >= 1 && dk <= 256 && dv >= 1 && v_stride >= H * dv,
              "ta_delta_recurrent: %d heads in %d groups of %d / %d", H, G, dk, dv);
@@ -312,12 +329,13 @@ extern "C" int ta_delta_recurrent(hipStream_t stream, int dtype, const float* qn
   const int cols = 256 / lanes;
   TA_REQUIRE((dv + cols - 1) / cols <= 65535, "ta_delta_recurrent: values of %d", dv);
   dim3 g(H, (dv + cols - 1) / cols, batch);
-  const bool vec = dk % 4 == 0 && (((uintptr_t)qn | (uintptr_t)kn | (uintptr_t)decay) & 15) == 0;
-#define DR_RUN(T, L, RR, VE)                                                                              \
-  delta_recurrent_kernel<T, L, RR, VE><<<g, 256, 0, stream>>>(qn, kn, decay, (const T*)v, v_stride, beta, kq, \
+  const bool vec = dk % 4 == 0 && (((uintptr_t)qn | (uintptr_t)kn | (per_head ? 0 : (uintptr_t)decay)) & 15) == 0;
+#define DR_RUN(T, L, RR, VE, HD)                                                                          \
+  delta_recurrent_kernel<T, L, RR, VE, HD><<<g, 256, 0, stream>>>(qn, kn, decay, (const T*)v, v_stride, beta, kq, \
                                                               state, cu_q, slots, H, G, dk, dv, o_out)
 #define DR_BY_VEC(T, L, RR) \
-  if (vec) DR_RUN(T, L, RR, true); else DR_RUN(T, L, RR, false)
+  if (per_head) { if (vec) DR_RUN(T, L, RR, true, true); else DR_RUN(T, L, RR, false, true); } \
+  else { if (vec) DR_RUN(T, L, RR, true, false); else DR_RUN(T, L, RR, false, false); }
 #define DR_BY_WIDTH(T)                                                  \
   if (dk <= 64) { DR_BY_VEC(T, 16, 4); }                                \
   else if (dk <= 128) {                                                 \
@@ -380,7 +398,8 @@ __global__ __launch_bounds__(DS_NT) void delta_step_kernel(
     const T* __restrict__ qkv, int stride, const T* __restrict__ proj, int pstride, int aoff, int ra, int goff, int rg,
     int boff, const TW* __restrict__ a2, const TW* __restrict__ g2, const float* __restrict__ dt_bias,
     const float* __restrict__ a_log, float* __restrict__ state, const int* __restrict__ slots, int H, int G, int dk,
-    int dv, float qscale, const float* __restrict__ norm_w, float eps, int a_vec, int g_vec, T* __restrict__ out) {
+    int dv, float qscale, const float* __restrict__ norm_w, float eps, int a_vec, int g_vec, int gate_act,
+    T* __restrict__ out) {
   extern __shared__ float lds[];
   const int CV = dv / VW, RG = DS_NT / CV;           // column groups; row groups
   float* qs = lds;                                   // [dk]
@@ -440,15 +459,22 @@ __global__ __launch_bounds__(DS_NT) void delta_step_kernel(
   sx = wave_sum(sx);
   const float fq = qscale * rsqrtf(sq + DR_UNIT_EPS), fk = rsqrtf(sk + DR_UNIT_EPS);
   const float kq = sx * fq * fk;
+  auto gate_of = [&](float z) { return gate_act == 1 ? dr_sigmoid(z) : z * dr_sigmoid(z); };
+  if (ra == 0) {                                     // one decay for the head
+    const float g = expf(-rate * dr_softplus(to_f32(prow[aoff + h]) + dt_bias[h]));
+    for (int c = tid; c < dk; c += DS_NT) gs[c] = g;
+  }
+  if (rg == 0)                                       // the gate as projected
+    for (int j = tid; j < dv; j += DS_NT) gate[j] = gate_of(to_f32(prow[goff + h * dv + j]));
   // (whole groups of four lanes take a row; the loop's bound is the same for the four)
-  for (int i = tid / 4; i < dk + dv; i += DS_NT / 4) {
+  for (int i = tid / 4 + (ra == 0 ? dk : 0); i < (rg == 0 ? dk : dk + dv); i += DS_NT / 4) {
     const bool dec = i < dk;
     const int j = dec ? i : i - dk;
     const float s = dec ? ds_row_dot<TW>(a2 + ((size_t)h * dk + j) * ra, la, ra, tid % 4, a_vec)
                         : ds_row_dot<TW>(g2 + ((size_t)h * dv + j) * rg, lg, rg, tid % 4, g_vec);
     if (tid % 4 == 0) {
       if (dec) gs[j] = expf(-rate * dr_softplus(s + dt_bias[h * dk + j]));
-      else gate[j] = dr_sigmoid(s);
+      else gate[j] = gate_of(s);
     }
   }
   __syncthreads();
@@ -528,23 +554,27 @@ static size_t delta_step_lds(int dk, int dv, int ra, int rg) {
   return ((size_t)3 * dk + 2 * dv + ra + rg + (size_t)2 * (DS_NT / cv) * dv) * sizeof(float);
 }
 
-// Whether ta_delta_step takes heads of dk x dv with low-rank inputs of ra and rg.
+// Whether ta_delta_step takes heads of dk x dv with low-rank inputs of ra and rg (0: none).
 extern "C" int ta_delta_step_fits(int dk, int dv, int ra, int rg) {
-  return dk >= 1 && ra >= 1 && rg >= 1 && delta_step_rows(dk, dv) > 0 && delta_step_lds(dk, dv, ra, rg) <= 60000;
+  return dk >= 1 && ra >= 0 && rg >= 0 && delta_step_rows(dk, dv) > 0 && delta_step_lds(dk, dv, ra, rg) <= 60000;
 }
 
 // qkv: [batch] rows, stride apart, of [q: G*dk | k: G*dk | v: H*dv] behind convolution and activation;
 // proj: [batch] rows, pstride apart, holding the decay's low-rank input (ra) at aoff, the gate's (rg) at
 // goff and the step sizes' (H) at boff; a2 [H*dk, ra], g2 [H*dv, rg]; state [slots, H, dk, dv] float32;
-// norm_w [dv]; out [batch, H*dv] = the readout over its root mean square per head, times norm_w, gated.
+// norm_w [dv]; out [batch, H*dv] = the readout over its root mean square per head, times norm_w, gated
+// (gate_act 0: silu, 1: sigmoid). ra 0: the rows hold H decay inputs at aoff, one per head, and dt_bias H
+// numbers; rg 0: they hold the gates (H*dv) at goff.
 extern "C" int ta_delta_step(hipStream_t stream, int dtype, int wdtype, const void* qkv, int stride, const void* proj,
                              int pstride, int aoff, int ra, int goff, int rg, int boff, const void* a2, const void* g2,
                              const float* dt_bias, const float* a_log, float* state, const int* slots, int batch, int H,
-                             int G, int dk, int dv, float qscale, const float* norm_w, float eps, void* out) {
+                             int G, int dk, int dv, float qscale, const float* norm_w, float eps, int gate_act,
+                             void* out) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && G >= 1 && H >= 1 && H % G == 0, "ta_delta_step: batch %d, %d heads in %d groups", batch, H, G);
   TA_REQUIRE(ta_delta_step_fits(dk, dv, ra, rg), "ta_delta_step: heads of %d x %d, ranks %d / %d", dk, dv, ra, rg);
-  TA_REQUIRE(stride >= 2 * G * dk + H * dv && aoff >= 0 && goff >= 0 && boff >= 0 && pstride >= aoff + ra &&
-             pstride >= goff + rg && pstride >= boff + H, "ta_delta_step: rows of %d / %d are too short", stride, pstride);
+  TA_REQUIRE(stride >= 2 * G * dk + H * dv && aoff >= 0 && goff >= 0 && boff >= 0 &&
+             pstride >= aoff + (ra ? ra : H) && pstride >= goff + (rg ? rg : H * dv) && pstride >= boff + H, "ta_delta_step: rows of %d / %d are too short", stride, pstride);
+  TA_REQUIRE(gate_act == 0 || gate_act == 1, "ta_delta_step: unknown gate activation %d", gate_act);
   const int rows = delta_step_rows(dk, dv);
   const size_t lds = delta_step_lds(dk, dv, ra, rg);
   const int a_vec = ra % 8 == 0 && (uintptr_t)a2 % 16 == 0, g_vec = rg % 8 == 0 && (uintptr_t)g2 % 16 == 0;
@@ -554,7 +584,7 @@ extern "C" int ta_delta_step(hipStream_t stream, int dtype, int wdtype, const vo
 #define DS_RUN(T, TW, VWV, RW)                                                                                       \
   delta_step_kernel<T, TW, VWV, RW><<<g, DS_NT, lds, stream>>>(                                                      \
       (const T*)qkv, stride, (const T*)proj, pstride, aoff, ra, goff, rg, boff, (const TW*)a2, (const TW*)g2, dt_bias, \
-      a_log, state, slots, H, G, dk, dv, qscale, norm_w, eps, a_vec, g_vec, (T*)out)
+      a_log, state, slots, H, G, dk, dv, qscale, norm_w, eps, a_vec, g_vec, gate_act, (T*)out)
 #define DS_BY_ROWS(T, TW, VWV)                 \
   switch (rows) {                              \
     case 4: DS_RUN(T, TW, VWV, 4); break;      \

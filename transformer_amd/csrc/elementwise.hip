@@ -82,6 +82,44 @@ extern "C" int ta_embed(hipStream_t stream, int dtype, const void* table, int vo
   return ta_check_launch("ta_embed");
 }
 
+// x[t, :] += table[position[t], :]: a learned row per position. Positions that the host has checked never
+// fall outside the table; one that does makes its row NaN, as a token does above.
+template <typename T, int V>
+__global__ __launch_bounds__(256) void rows_add_kernel(const T* __restrict__ table, const int* __restrict__ index,
+                                                       float* __restrict__ x, int d, int rows) {
+  const int t = blockIdx.x;
+  const int id = index[t];
+  const bool ok = id >= 0 && id < rows;
+  const T* row = table + (size_t)(ok ? id : 0) * d;
+  float* out = x + (size_t)t * d;
+  struct alignas(V * sizeof(T)) Piece { T v[V]; };
+  struct alignas(V * sizeof(float)) Wide { float v[V]; };
+  for (int i = threadIdx.x * V; i < d; i += 256 * V) {
+    const Piece a = *reinterpret_cast<const Piece*>(row + i);
+    Wide o = *reinterpret_cast<const Wide*>(out + i);
+#pragma unroll
+    for (int k = 0; k < V; ++k) o.v[k] = ok ? o.v[k] + to_f32(a.v[k]) : __builtin_nanf("");
+    *reinterpret_cast<Wide*>(out + i) = o;
+  }
+}
+
+// table [rows, d]; index int32 [nt] on the device; x float32 [nt, d], in place.
+extern "C" int ta_rows_add(hipStream_t stream, int dtype, const void* table, int rows, int d, const int* index, int nt,
+                           float* x) {
+  TA_REQUIRE(dtype == TA_F32 || dtype == TA_BF16, "ta_rows_add: unknown dtype %d", dtype);
+  TA_REQUIRE(rows > 0 && d > 0 && nt >= 0, "ta_rows_add: bad sizes rows=%d d=%d nt=%d", rows, d, nt);
+  if (nt == 0) return 0;
+  const bool four = d % 4 == 0 && (((uintptr_t)table | (uintptr_t)x) & 15) == 0;
+#define ROWS_ADD(T, V) rows_add_kernel<T, V><<<nt, 256, 0, stream>>>((const T*)table, index, x, d, rows)
+  if (dtype == TA_F32) {
+    if (four) ROWS_ADD(float, 4); else ROWS_ADD(float, 1);
+  } else {
+    if (four) ROWS_ADD(bf16_t, 4); else ROWS_ADD(bf16_t, 1);
+  }
+#undef ROWS_ADD
+  return ta_check_launch("ta_rows_add");
+}
+
 // ------------------------------------------------------------------ add + RMS norm
 // For output row i (source row r = rows ? rows[i] : i):
 //   v = x[r] + delta[r] + delta_bias        (terms that are null are left out)

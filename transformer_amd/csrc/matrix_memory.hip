@@ -1,0 +1,261 @@
+// The matrix memory of xLSTM ("mLSTM"): per head a state S [dk][dv], a normaliser n [dk] and a running
+// maximum m (0 at a sequence's start), with exponential gates that are kept as logarithms:
+//
+//     i_t = cap tanh((a_t + bi) / cap),  f_t = log sigmoid(cap tanh((b_t + bf) / cap))
+//     m_t = max(f_t + m_(t-1), i_t),  keep_t = exp(f_t + m_(t-1) - m_t),  write_t = exp(i_t - m_t)
+//     S_t = keep_t S_(t-1) + write_t k_t v_t^T,  n_t = keep_t n_(t-1) + write_t k_t
+//     o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
+//
+//   memory_gates : keep, write and exp(-m) of every token and head; the running maximum of 64 tokens at
+//                  once by a scan over a wave
+//   memory_step  : a step of single tokens in one kernel: gates, the state's update, the readout with its
+//                  denominator, the head's norm and the output gate
+//
+// (The recurrence over a prompt is the kernel of gated linear attention with keep as the decay, write as a
+// factor on the key, and the normaliser as one more value column, see recurrent.hip.)
+//
+// keep is formed as exp(f - (m_t - m_(t-1))): where m_t is the rounded f + m_(t-1), the difference of the
+// two maxima is exact and keep makes up for that rounding.
+#include "common.h"
+
+#define MM_FLOOR_EPS 1e-6f      // beside the denominator
+
+__device__ __forceinline__ float mm_cap(float z, float cap) { return cap * tanhf(z / cap); }
+__device__ __forceinline__ float mm_log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+
+// ------------------------------------------------------------------ gates of a step
+// One wave per (head, sequence). Elements of the scan are (sum of f, best of i_j + f_(j+1) + .. + f_t); two
+// neighbours join to (F1 + F2, max(M1 + F2, M2)), and m_t = max(F + m before the turn, M).
+template <typename T>
+__global__ __launch_bounds__(64) void memory_gates_kernel(
+    const T* __restrict__ proj, int stride, int ioff, int foff, const float* __restrict__ ibias,
+    const float* __restrict__ fbias, float cap, float* __restrict__ m_state, const int* __restrict__ cu_q,
+    const int* __restrict__ slots, int H, float* __restrict__ keep, float* __restrict__ write, float* __restrict__ floor_) {
+  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
+  const int start = cu_q[b], end = cu_q[b + 1];
+  if (start >= end) return;
+  float* ms = m_state + (size_t)slots[b] * H + h;
+  float m0 = *ms;
+  const float bi = ibias[h], bf = fbias[h];
+  // the next turn's inputs are on their way while this turn is worked on
+  auto at = [&](int t) { return (size_t)(t < end ? t : end - 1) * stride; };
+  T ri = proj[at(start + lane) + ioff + h], rf = proj[at(start + lane) + foff + h];
+  for (int t0 = start; t0 < end; t0 += TA_WAVE) {
+    const int t = t0 + lane;
+    const bool on = t < end;
+    const float i = on ? mm_cap(to_f32(ri) + bi, cap) : -INFINITY;
+    const float f = on ? mm_log_sigmoid(mm_cap(to_f32(rf) + bf, cap)) : 0.f;
+    if (t0 + TA_WAVE < end) {
+      ri = proj[at(t + TA_WAVE) + ioff + h];
+      rf = proj[at(t + TA_WAVE) + foff + h];
+    }
+    float F = f, M = i;
+#pragma unroll
+    for (int o = 1; o < TA_WAVE; o <<= 1) {
+      const float Fp = __shfl_up(F, o, TA_WAVE), Mp = __shfl_up(M, o, TA_WAVE);
+      if (lane >= o) {
+        M = fmaxf(Mp + F, M);
+        F += Fp;
+      }
+    }
+    const float m = fmaxf(F + m0, M);
+    const float up = __shfl_up(m, 1, TA_WAVE);
+    const float before = lane == 0 ? m0 : up;
+    if (on) {
+      const size_t e = (size_t)t * H + h;
+      keep[e] = expf(f - (m - before));
+      write[e] = expf(i - m);
+      floor_[e] = expf(-m);
+    }
+    m0 = __shfl(m, TA_WAVE - 1, TA_WAVE);       // (lanes past the end carry the last token's)
+  }
+  if (lane == 0) *ms = m0;
+}
+
+// proj: [nt] rows, stride apart, with the input gates' numbers (H) at column ioff and the forget gates' at
+// foff; ibias, fbias [H]; m_state [slots, H] float32, moved on; keep, write, floor_ [nt, H] float32.
+extern "C" int ta_memory_gates(hipStream_t stream, int dtype, const void* proj, int stride, int ioff, int foff,
+                               const float* ibias, const float* fbias, float cap, float* m_state, const int* cu_q,
+                               const int* slots, int batch, int nt, int H, float* keep, float* write, float* floor_) {
+  TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch && H >= 1, "ta_memory_gates: batch %d, %d tokens, %d heads", batch, nt, H);
+  TA_REQUIRE(ioff >= 0 && foff >= 0 && stride >= ioff + H && stride >= foff + H, "ta_memory_gates: rows of %d are too short", stride);
+  TA_REQUIRE(cap > 0.f, "ta_memory_gates: the cap must be positive, got %g", (double)cap);
+  dim3 g(H, batch);
+  if (dtype == TA_F32)
+    memory_gates_kernel<float><<<g, 64, 0, stream>>>((const float*)proj, stride, ioff, foff, ibias, fbias, cap, m_state,
+                                                     cu_q, slots, H, keep, write, floor_);
+  else if (dtype == TA_BF16)
+    memory_gates_kernel<bf16_t><<<g, 64, 0, stream>>>((const bf16_t*)proj, stride, ioff, foff, ibias, fbias, cap, m_state,
+                                                      cu_q, slots, H, keep, write, floor_);
+  else return ta_fail("ta_memory_gates: unknown dtype %d", dtype);
+  return ta_check_launch("ta_memory_gates");
+}
+
+// ------------------------------------------------------------------ steps of single tokens
+// One workgroup of MS_NT threads per (head, sequence). A thread keeps VW neighbouring value columns of every
+// RG-th key channel; the whole state is asked for before anything else is done.
+#define MS_NT 512
+
+template <typename T, int VW, int ROWS>
+__global__ __launch_bounds__(MS_NT) void memory_step_kernel(
+    const T* __restrict__ proj, int stride, int qoff, int koff, int voff, int goff, int ioff, int foff,
+    const float* __restrict__ ibias, const float* __restrict__ fbias, float cap, float* __restrict__ state,
+    float* __restrict__ n_state, float* __restrict__ m_state, const int* __restrict__ slots, int H, int dk, int dv,
+    float qscale, const float* __restrict__ norm_w, float eps, T* __restrict__ out) {
+  extern __shared__ float lds[];
+  const int CV = dv / VW, RG = MS_NT / CV;           // column groups; row groups
+  float* qs = lds;                                   // [dk]
+  float* ks = qs + dk;                               // [dk], times the write weight
+  float* pr = ks + dk;                               // [RG][dv]
+  __shared__ float red[MS_NT / TA_WAVE], redn[MS_NT / TA_WAVE];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const size_t slot = (size_t)slots[b];
+  float* st = state + (slot * H + h) * dk * (size_t)dv;
+  float* ns = n_state + (slot * H + h) * dk;
+  const int r0 = tid / CV, c0 = (tid % CV) * VW;
+  const bool on = r0 < RG;
+  float S[ROWS][VW];
+#pragma unroll
+  for (int i = 0; i < ROWS; ++i) {
+    const int row = r0 + RG * i;
+    const bool ok = on && row < dk;
+    const float* p = st + (size_t)(ok ? row : 0) * dv + (on ? c0 : 0);
+    if (VW == 4) {
+      const float4 a = *reinterpret_cast<const float4*>(p);
+      S[i][0] = a.x;
+      S[i][VW > 1 ? 1 : 0] = VW > 1 ? a.y : S[i][0];
+      S[i][VW > 2 ? 2 : 0] = VW > 2 ? a.z : S[i][0];
+      S[i][VW > 3 ? 3 : 0] = VW > 3 ? a.w : S[i][0];
+    } else {
+      S[i][0] = p[0];
+    }
+  }
+  const T* row = proj + (size_t)b * stride;
+  float v[VW];
+#pragma unroll
+  for (int e = 0; e < VW; ++e) v[e] = on ? to_f32(row[voff + h * dv + c0 + e]) : 0.f;
+  // the gates, by every thread for itself
+  const float i = mm_cap(to_f32(row[ioff + h]) + ibias[h], cap);
+  const float f = mm_log_sigmoid(mm_cap(to_f32(row[foff + h]) + fbias[h], cap));
+  const float before = m_state[slot * H + h];
+  const float m = fmaxf(f + before, i);
+  const float keep = expf(f - (m - before)), write = expf(i - m);
+  // the normaliser and its product with q
+  float dot = 0.f;
+  for (int c = tid; c < dk; c += MS_NT) {
+    const float q = to_f32(row[qoff + h * dk + c]) * qscale, k = to_f32(row[koff + h * dk + c]) * write;
+    const float n = fmaf(keep, ns[c], k);
+    qs[c] = q;
+    ks[c] = k;
+    ns[c] = n;
+    dot = fmaf(n, q, dot);
+  }
+  dot = wave_sum(dot);
+  if (tid % TA_WAVE == 0) redn[tid / TA_WAVE] = dot;
+  __syncthreads();                                   // (every thread has read m_state before one writes it)
+  if (tid == 0) m_state[slot * H + h] = m;
+  // ---- the update and the readout
+  float r[VW];
+#pragma unroll
+  for (int e = 0; e < VW; ++e) r[e] = 0.f;
+#pragma unroll
+  for (int i2 = 0; i2 < ROWS; ++i2) {
+    const int rw = r0 + RG * i2;
+    if (on && rw < dk) {
+      const float k = ks[rw], q = qs[rw];
+#pragma unroll
+      for (int e = 0; e < VW; ++e) {
+        S[i2][e] = fmaf(keep, S[i2][e], k * v[e]);
+        r[e] = fmaf(S[i2][e], q, r[e]);
+      }
+      float* p = st + (size_t)rw * dv + c0;
+      if (VW == 4) *reinterpret_cast<float4*>(p) = float4{S[i2][0], S[i2][VW > 1 ? 1 : 0], S[i2][VW > 2 ? 2 : 0], S[i2][VW > 3 ? 3 : 0]};
+      else p[0] = S[i2][0];
+    }
+  }
+  if (on) {
+#pragma unroll
+    for (int e = 0; e < VW; ++e) pr[r0 * dv + c0 + e] = r[e];
+  }
+  __syncthreads();
+  float below = 0.f;
+#pragma unroll
+  for (int w = 0; w < MS_NT / TA_WAVE; ++w) below += redn[w];
+  below = 1.0f / (fmaxf(fabsf(below), expf(-m)) + MM_FLOOR_EPS);
+  float ss = 0.f;
+  for (int j = tid; j < dv; j += MS_NT) {            // row groups in order
+    float o = 0.f;
+    for (int g = 0; g < RG; ++g) o += pr[g * dv + j];
+    o *= below;
+    pr[j] = o;                                       // column j of row group 0 is this thread's alone now
+    ss = fmaf(o, o, ss);
+  }
+  ss = wave_sum(ss);
+  if (tid % TA_WAVE == 0) red[tid / TA_WAVE] = ss;
+  __syncthreads();
+  float tot = 0.f;
+#pragma unroll
+  for (int w = 0; w < MS_NT / TA_WAVE; ++w) tot += red[w];
+  const float fac = rsqrtf(tot / (float)dv + eps);
+  for (int j = tid; j < dv; j += MS_NT) {
+    const float g = to_f32(row[goff + h * dv + j]);
+    out[(size_t)b * H * dv + (size_t)h * dv + j] = from_f32<T>(pr[j] * fac * norm_w[h * dv + j] / (1.0f + expf(-g)));
+  }
+}
+
+static int memory_step_rows(int dk, int dv) {         // key channels a thread keeps; 0: not taken
+  const int cv = dv % 4 == 0 ? dv / 4 : dv;
+  if (cv < 1 || cv > MS_NT) return 0;
+  const int rg = MS_NT / cv;
+  const int rows = (dk + rg - 1) / rg;
+  return rows <= 4 ? 4 : rows <= 8 ? 8 : rows <= 16 ? 16 : rows <= 32 ? 32 : 0;
+}
+static size_t memory_step_lds(int dk, int dv) {
+  const int cv = dv % 4 == 0 ? dv / 4 : dv;
+  return ((size_t)2 * dk + (size_t)(MS_NT / cv) * dv) * sizeof(float);
+}
+
+// Whether ta_memory_step takes heads of dk x dv.
+extern "C" int ta_memory_step_fits(int dk, int dv) {
+  return dk >= 1 && dv >= 1 && memory_step_rows(dk, dv) > 0 && memory_step_lds(dk, dv) <= 60000;
+}
+
+// proj: [batch] rows, stride apart, with q and k (H*dk each), v and the output gate (H*dv each), the input and
+// the forget gates' numbers (H each) at columns qoff, koff, voff, goff, ioff, foff. state [slots, H, dk, dv],
+// n_state [slots, H, dk], m_state [slots, H] float32; norm_w [H*dv]; out [batch, H*dv] = the readout over its
+// root mean square per head, times norm_w, times sigmoid(gate).
+extern "C" int ta_memory_step(hipStream_t stream, int dtype, const void* proj, int stride, int qoff, int koff, int voff,
+                              int goff, int ioff, int foff, const float* ibias, const float* fbias, float cap,
+                              float* state, float* n_state, float* m_state, const int* slots, int batch, int H, int dk,
+                              int dv, float qscale, const float* norm_w, float eps, void* out) {
+  TA_REQUIRE(batch > 0 && batch <= 65535 && H >= 1 && H <= 65535, "ta_memory_step: batch %d, %d heads", batch, H);
+  TA_REQUIRE(ta_memory_step_fits(dk, dv), "ta_memory_step: heads of %d x %d", dk, dv);
+  TA_REQUIRE(qoff >= 0 && koff >= 0 && voff >= 0 && goff >= 0 && ioff >= 0 && foff >= 0 && stride >= qoff + H * dk &&
+             stride >= koff + H * dk && stride >= voff + H * dv && stride >= goff + H * dv && stride >= ioff + H &&
+             stride >= foff + H, "ta_memory_step: rows of %d are too short", stride);
+  TA_REQUIRE(cap > 0.f, "ta_memory_step: the cap must be positive, got %g", (double)cap);
+  TA_REQUIRE(dv % 4 != 0 || (uintptr_t)state % 16 == 0, "ta_memory_step: the state must be 16-byte aligned");
+  const int rows = memory_step_rows(dk, dv);
+  const size_t lds = memory_step_lds(dk, dv);
+  dim3 g(H, batch);
+#define MS_RUN(T, VWV, RW)                                                                                             \
+  memory_step_kernel<T, VWV, RW><<<g, MS_NT, lds, stream>>>((const T*)proj, stride, qoff, koff, voff, goff, ioff, foff, \
+                                                            ibias, fbias, cap, state, n_state, m_state, slots, H, dk,  \
+                                                            dv, qscale, norm_w, eps, (T*)out)
+#define MS_BY_ROWS(T, VWV)                 \
+  switch (rows) {                          \
+    case 4: MS_RUN(T, VWV, 4); break;      \
+    case 8: MS_RUN(T, VWV, 8); break;      \
+    case 16: MS_RUN(T, VWV, 16); break;    \
+    default: MS_RUN(T, VWV, 32); break;    \
+  }
+#define MS_BY_COLS(T) \
+  if (dv % 4 == 0) { MS_BY_ROWS(T, 4) } else { MS_BY_ROWS(T, 1) }
+  if (dtype == TA_F32) { MS_BY_COLS(float) }
+  else if (dtype == TA_BF16) { MS_BY_COLS(bf16_t) }
+  else return ta_fail("ta_memory_step: unknown dtype %d", dtype);
+#undef MS_BY_COLS
+#undef MS_BY_ROWS
+#undef MS_RUN
+  return ta_check_launch("ta_memory_step");
+}

@@ -15,6 +15,9 @@
 //   moe_combine : delta[t] = sum of the token's pairs' rows (times the weight when it acts on
 //                 the output) + sigmoid(shared gate) * the shared expert's rows
 //
+// Choices from E on are identity experts: they have no rows and no matrices, and moe_combine adds the
+// token's own row times the pair's weight for them.
+//
 // Router scores, weights and all sums are float32.
 #include "common.h"
 
@@ -26,12 +29,15 @@
 // (with mode 1 that is the softmax over the chosen logits alone). bias [E] or null: added to
 // the logits first. groups > 1: the experts form that many equal groups of neighbours, a group
 // counts as its largest score, and only experts of the `keep` best groups (the lowest index
-// among equals) can be chosen.
+// among equals) can be chosen. correction [E] or null: the choice compares score + correction, the
+// weights are the scores without it. factor: the weights are multiplied by it last.
 __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__ logits, int ld, int E, int top,
                                                        int mode, int renorm, int* __restrict__ chosen,
                                                        float* __restrict__ weight,
-                                                       const float* __restrict__ bias, int groups, int keep) {
-  extern __shared__ float sc[];           // [E], then a score per group [groups]
+                                                       const float* __restrict__ bias, int groups, int keep,
+                                                       const float* __restrict__ correction, float factor) {
+  extern __shared__ float sc[];           // [E], then a score per group [groups], then the plain scores [E]
+  float* plain = sc + E + groups;         // (with a correction only)
   const size_t t = blockIdx.x;
   const int lane = threadIdx.x;
   float mx = -INFINITY;
@@ -45,6 +51,13 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
     sum += s;
   }
   sum = wave_sum(sum);
+  if (correction) {                       // (a lane meets the entries that it wrote itself)
+    for (int e = lane; e < E; e += 64) {
+      const float s = mode == 0 ? sc[e] : sc[e] / sum;
+      plain[e] = s;
+      sc[e] = s + correction[e];
+    }
+  }
   __syncthreads();
   if (groups > 1) {
     float* gs = sc + E;
@@ -79,10 +92,10 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
       const int oa = __shfl_xor(at, o, TA_WAVE);
       if (ob > best || (ob == best && oa < at)) { best = ob; at = oa; }
     }
-    const float w = mode == 0 ? best : best / sum;
+    const float w = correction ? plain[at] : mode == 0 ? best : best / sum;
     if (lane == 0) {
       chosen[t * top + j] = at;
-      weight[t * top + j] = w;
+      weight[t * top + j] = renorm ? w : w * factor;
     }
     total += w;
     __syncthreads();
@@ -91,35 +104,29 @@ __global__ __launch_bounds__(64) void moe_route_kernel(const float* __restrict__
   }
   if (renorm) {
     __syncthreads();
-    for (int j = lane; j < top; j += 64) weight[t * top + j] /= total;
+    for (int j = lane; j < top; j += 64) weight[t * top + j] = weight[t * top + j] / total * factor;
   }
 }
 
-extern "C" int ta_moe_route_groups(hipStream_t stream, const float* logits, const float* bias, int ld, int nt, int E,
-                                   int top, int mode, int renorm, int groups, int keep, int* chosen, float* weight) {
+extern "C" int ta_moe_route(hipStream_t stream, const float* logits, const float* bias, int ld, int nt, int E,
+                            int top, int mode, int renorm, int groups, int keep, const float* correction,
+                            float factor, int* chosen, float* weight) {
   TA_REQUIRE(nt >= 0 && E >= 1 && E <= 8192 && top >= 1 && top <= E && ld >= E && (mode == 0 || mode == 1),
              "ta_moe_route: bad sizes nt=%d experts=%d top=%d ld=%d", nt, E, top, ld);
   TA_REQUIRE(groups >= 1 && E % groups == 0 && keep >= 1 && keep <= groups && top <= keep * (E / groups),
              "ta_moe_route: %d experts in %d groups of which %d stay do not hold %d choices", E, groups, keep, top);
   if (nt == 0) return 0;
-  moe_route_kernel<<<nt, 64, (size_t)(E + groups) * sizeof(float), stream>>>(logits, ld, E, top, mode, renorm, chosen,
-                                                                             weight, bias, groups, keep);
+  const size_t lds = ((size_t)E + groups + (correction ? E : 0)) * sizeof(float);
+  TA_REQUIRE(lds <= 65536, "ta_moe_route: %d experts in %d groups do not fit the LDS", E, groups);
+  moe_route_kernel<<<nt, 64, lds, stream>>>(logits, ld, E, top, mode, renorm, chosen, weight, bias, groups, keep,
+                                            correction, factor);
   return ta_check_launch("ta_moe_route");
-}
-
-extern "C" int ta_moe_route_bias(hipStream_t stream, const float* logits, const float* bias, int ld, int nt, int E,
-                                 int top, int mode, int renorm, int* chosen, float* weight) {
-  return ta_moe_route_groups(stream, logits, bias, ld, nt, E, top, mode, renorm, 1, 1, chosen, weight);
-}
-
-extern "C" int ta_moe_route(hipStream_t stream, const float* logits, int ld, int nt, int E, int top, int mode,
-                            int renorm, int* chosen, float* weight) {
-  return ta_moe_route_bias(stream, logits, nullptr, ld, nt, E, top, mode, renorm, chosen, weight);
 }
 
 // ------------------------------------------------------------------ ordering the pairs by expert
 // One workgroup. row_pair: [max_rows] pair index of every ordered row, -1 for a row that only
-// fills a tile; tile_expert: [max_rows / 16], -1 for a tile past the last; pair_row: [pairs].
+// fills a tile; tile_expert: [max_rows / 16], -1 for a tile past the last; pair_row: [pairs],
+// -1 for a pair whose choice is no expert with matrices (E or more).
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ chosen, int pairs, int E,
                                                         int max_rows, int* __restrict__ row_pair,
                                                         int* __restrict__ tile_expert, int* __restrict__ pair_row) {
@@ -129,7 +136,8 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   for (int e = threadIdx.x; e < E; e += 1024) count[e] = 0;
   for (int i = threadIdx.x; i < max_rows; i += 1024) row_pair[i] = -1;
   __syncthreads();
-  for (int i = threadIdx.x; i < pairs; i += 1024) atomicAdd(&count[chosen[i]], 1);
+  for (int i = threadIdx.x; i < pairs; i += 1024)
+    if (chosen[i] < E) atomicAdd(&count[chosen[i]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0;
@@ -158,6 +166,10 @@ __global__ __launch_bounds__(1024) void moe_plan_kernel(const int* __restrict__ 
   // the order of an expert's rows among themselves does not matter: every row is computed alone
   for (int i = threadIdx.x; i < pairs; i += 1024) {
     const int e = chosen[i];
+    if (e >= E) {
+      pair_row[i] = -1;
+      continue;
+    }
     const int r = start[e] + atomicAdd(&count[e], 1);
     row_pair[r] = i;
     pair_row[i] = r;
@@ -667,13 +679,15 @@ extern "C" int ta_moe_gemm(hipStream_t stream, int dtype, int out_dtype, const v
 }
 
 // ------------------------------------------------------------------ putting the rows back
+template <typename T>
 __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restrict__ rows, int d, int top,
                                                           const int* __restrict__ pair_row,
                                                           const float* __restrict__ weight,
                                                           const float* __restrict__ shared, int planes, size_t plane,
                                                           const float* __restrict__ shared_gate, int gate_ld,
                                                           float* __restrict__ delta,
-                                                          const float* __restrict__ extra, int xplanes, size_t xplane) {
+                                                          const float* __restrict__ extra, int xplanes, size_t xplane,
+                                                          const T* __restrict__ h) {
   extern __shared__ float cmb[];          // [top] rows of the token's pairs, [top] their weights
   int* prow = reinterpret_cast<int*>(cmb);
   float* pw = cmb + top;
@@ -687,7 +701,12 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
   __syncthreads();
   for (int c = threadIdx.x; c < d; c += 256) {
     float s = 0.f;
-    for (int j = 0; j < top; ++j) s = fmaf(rows[(size_t)prow[j] * d + c], pw[j], s);
+    const float own = h ? to_f32(h[t * d + c]) : 0.f;        // what an identity expert gives
+    for (int j = 0; j < top; ++j) {
+      const int r = prow[j];
+      const float y = rows[(size_t)(r >= 0 ? r : 0) * d + c];
+      s = fmaf(r >= 0 ? y : own, pw[j], s);
+    }
     if (shared) {
       float v = shared[t * d + c];
       for (int p = 1; p < planes; ++p) v += shared[t * d + c + p * plane];
@@ -704,24 +723,24 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 // shared expert's result; shared_gate (or null): its gate's pre-activation, one number per
 // token, element 0 of a row of gate_ld float32. delta: [nt, d] float32.
 // extra (or null): [xplanes, nt, d] float32 planes, ``xplane`` elements apart, added as they are.
-extern "C" int ta_moe_combine_extra(hipStream_t stream, const float* rows, int d, int top, const int* pair_row,
-                                    const float* weight, const float* shared, int planes, long long plane,
-                                    const float* shared_gate, int gate_ld, const float* extra, int xplanes,
-                                    long long xplane, float* delta, int nt) {
+// h (or null; float32 or bfloat16 by h_dtype): [nt, d] the rows that identity experts (pairs without a row)
+// hand back.
+extern "C" int ta_moe_combine(hipStream_t stream, const float* rows, int d, int top, const int* pair_row,
+                              const float* weight, const float* shared, int planes, long long plane,
+                              const float* shared_gate, int gate_ld, const float* extra, int xplanes,
+                              long long xplane, int h_dtype, const void* h, float* delta, int nt) {
+  TA_REQUIRE(h_dtype == TA_F32 || h_dtype == TA_BF16, "ta_moe_combine: unknown dtype %d", h_dtype);
   TA_REQUIRE(nt >= 0 && d > 0 && top >= 1 && planes >= 1 && planes <= TA_MAX_PLANES, "ta_moe_combine: bad sizes");
   TA_REQUIRE(!extra || (xplanes >= 1 && xplanes <= TA_MAX_PLANES && (xplanes == 1 || xplane > 0)),
              "ta_moe_combine: %d planes of the further addend", xplanes);
   if (nt == 0) return 0;
-  moe_combine_kernel<<<nt, 256, (size_t)2 * top * sizeof(float), stream>>>(rows, d, top, pair_row, weight, shared, planes, (size_t)plane,
-                                             shared_gate, gate_ld, delta, extra, xplanes, (size_t)xplane);
+#define MOE_COMBINE(T)                                                                                          \
+  moe_combine_kernel<T><<<nt, 256, (size_t)2 * top * sizeof(float), stream>>>(                                  \
+      rows, d, top, pair_row, weight, shared, planes, (size_t)plane, shared_gate, gate_ld, delta, extra, xplanes, \
+      (size_t)xplane, (const T*)h)
+  if (h_dtype == TA_F32) MOE_COMBINE(float); else MOE_COMBINE(bf16_t);
+#undef MOE_COMBINE
   return ta_check_launch("ta_moe_combine");
-}
-
-extern "C" int ta_moe_combine(hipStream_t stream, const float* rows, int d, int top, const int* pair_row,
-                              const float* weight, const float* shared, int planes, long long plane,
-                              const float* shared_gate, int gate_ld, float* delta, int nt) {
-  return ta_moe_combine_extra(stream, rows, d, top, pair_row, weight, shared, planes, plane, shared_gate, gate_ld,
-                              nullptr, 0, 0, delta, nt);
 }
 
 // ------------------------------------------------------------------ the limited gated activation

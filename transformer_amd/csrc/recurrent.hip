@@ -19,6 +19,10 @@
 //   `ssm_steps` forms step sizes and decays, the recurrence is `gla_recurrent` with q = C, k = B, v = x
 //   (the heads of a group read the same B and C), `gated_group_norm` adds D x, gates and norms.
 //
+// Matrix memory (matrix_memory.hip): the same recurrence with one decay and one key factor per (token,
+//   head) and a normaliser n_t, which decays and is written as S is and whose product with q is the
+//   readout's denominator: it is one more value column whose value is always 1.
+//
 // Short causal convolution (`causal_conv`): per channel over a sequence's tokens, with the last
 //   inputs of every sequence kept between steps; used in front of the state space and by the
 //   attention variant that convolves its q, k and v.
@@ -571,16 +575,19 @@ struct GlaOperands {  // what one thread brings in for a chunk
   float q[GLA_TC * GLA_RT / 256], k[GLA_TC * GLA_RT / 256], a[GLA_TC * GLA_RT / 256], v[GLA_TC * GLA_CT / 256];
 };
 
+// NORM: column dv stands for the normaliser: its value is 1, its state is n_state [slots, H, dk], and its
+// readout goes to the planes of den_out [nt, H].
 // BONUS: the readout comes BEFORE the update and gives the current token a weight of its own,
 // o_t = (S_{t-1} + diag(bonus) k_t v_t^T)^T q_t, then S_t = diag(alpha_t) S_{t-1} + k_t v_t^T.
-template <typename T, int GLA_TC, bool BONUS>
+template <typename T, int GLA_TC, bool BONUS, bool NORM = false>
 __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     const T* __restrict__ proj, int stride, int qoff, int koff, int voff, const float* __restrict__ alpha,
     float qscale, float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ slots,
     int H, int dk, int dv, int col_tiles, size_t plane, float* __restrict__ o_out,
     const float* __restrict__ bonus, const float* __restrict__ head_decay,
     int qk_share = 1, const float* __restrict__ tok_decay = nullptr,
-    const float* __restrict__ tok_kscale = nullptr) {
+    const float* __restrict__ tok_kscale = nullptr, float* __restrict__ n_state = nullptr,
+    float* __restrict__ den_out = nullptr) {
   __shared__ float sq[GLA_TC][GLA_RT], sk[GLA_TC][GLA_RT], sa[GLA_TC][GLA_RT];
   __shared__ float sv[GLA_TC][GLA_CT];
   __shared__ float part[GLA_TC][4][GLA_CT];
@@ -600,6 +607,7 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     for (int c = 0; c < 2; ++c) {
       const int i = row0 + rg * 4 + r, j = col0 + cg * 2 + c;
       S[r][c] = (i < dk && j < dv) ? st[(size_t)i * dv + j] : 0.f;
+      if (NORM && i < dk && j == dv) S[r][c] = n_state[(slot * H + h) * dk + i];
     }
   float bu[4] = {0.f, 0.f, 0.f, 0.f};
   if (BONUS) {
@@ -637,7 +645,7 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
       const int idx = tid + 256 * e, tt = idx / GLA_CT, j = col0 + idx % GLA_CT;
       const bool ok = t0 + tt < end && j < dv;
       const float vv = to_f32(proj[(size_t)(ok ? t0 + tt : start) * stride + voff + h * dv + (ok ? j : 0)]);
-      o.v[e] = ok ? vv : 0.f;
+      o.v[e] = ok ? vv : (NORM && j == dv) ? 1.f : 0.f;
     }
   };
   auto turn = [&](GlaOperands<GLA_TC>& o, int t0) {
@@ -705,6 +713,9 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
       if (col0 + c < dv)
         o_out[rpart * plane + ((size_t)(t0 + tt) * H + h) * dv + col0 + c] =
             (part[tt][0][c] + part[tt][1][c]) + (part[tt][2][c] + part[tt][3][c]);
+      if (NORM && col0 + c == dv)
+        den_out[rpart * (plane / dv) + (size_t)(t0 + tt) * H + h] =
+            (part[tt][0][c] + part[tt][1][c]) + (part[tt][2][c] + part[tt][3][c]);
     }
     // The next turn's stores into sq/sk/sa/sv follow the barrier above, which every thread
     // passes only after its last read of them; `part` is read here and written again only
@@ -723,6 +734,7 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     for (int c = 0; c < 2; ++c) {
       const int i = row0 + rg * 4 + r, j = col0 + cg * 2 + c;
       if (i < dk && j < dv) st[(size_t)i * dv + j] = S[r][c];
+      if (NORM && i < dk && j == dv) n_state[(slot * H + h) * dk + i] = S[r][c];
     }
 }
 
@@ -738,13 +750,14 @@ static int gla_recurrent_launch(hipStream_t stream, int dtype, int wdtype, const
                                 float* state, const int* cu_q, const int* slots, int batch, int nt, int H, int dk,
                                 int dv, float* o_out, int mode, const float* bonus,
                                 const float* head_decay = nullptr, int qk_share = 1,
-                                const float* tok_decay = nullptr, const float* tok_kscale = nullptr) {
+                                const float* tok_decay = nullptr, const float* tok_kscale = nullptr,
+                                float* n_state = nullptr, float* den_out = nullptr) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && H > 0 && H <= 65535 && nt >= batch,
              "ta_gla_recurrent: bad batch %d / heads %d / tokens %d", batch, H, nt);
   TA_REQUIRE(qk_share >= 1 && H % qk_share == 0, "ta_gla_recurrent: %d heads do not form groups of %d", H, qk_share);
   TA_REQUIRE(dk >= 1 && dv >= 1 && (head_decay || tok_decay || (rank >= 1 && rank <= 8192)),
              "ta_gla_recurrent: bad widths %d / %d / %d", dk, dv, rank);
-  const int parts = (dk + GLA_RT - 1) / GLA_RT, tiles = (dv + GLA_CT - 1) / GLA_CT;
+  const int parts = (dk + GLA_RT - 1) / GLA_RT, tiles = (dv + (n_state ? 1 : 0) + GLA_CT - 1) / GLA_CT;
   TA_REQUIRE(parts * tiles <= 65535, "ta_gla_recurrent: heads of %d x %d are too large", dk, dv);
   const int n = H * dk;
   dim3 gd(nt, (n + 255) / 256 < 64 ? (n + 255) / 256 : 64);
@@ -761,11 +774,17 @@ static int gla_recurrent_launch(hipStream_t stream, int dtype, int wdtype, const
   dim3 g(batch, H, parts * tiles);
   const size_t plane = (size_t)nt * H * dv;
   const bool few = nt <= 8 * batch;         // at most 8 tokens a sequence on average: short chunks
-#define GLA_RUN(T, TC, B)                                                                                   \
-  gla_recurrent_kernel<T, TC, B><<<g, 256, 0, stream>>>((const T*)proj, stride, qoff, koff, voff, alpha, qscale, \
+#define GLA_RUN(T, TC, ...)                                                                                 \
+  gla_recurrent_kernel<T, TC, __VA_ARGS__><<<g, 256, 0, stream>>>((const T*)proj, stride, qoff, koff, voff, alpha, qscale, \
                                                         state, cu_q, slots, H, dk, dv, tiles, plane, o_out, bonus, \
-                                                        head_decay, qk_share, tok_decay, tok_kscale)
-  if (bonus) {
+                                                        head_decay, qk_share, tok_decay, tok_kscale, n_state, den_out)
+  if (n_state) {
+    if (dtype == TA_F32) {
+      if (few) GLA_RUN(float, 8, false, true); else GLA_RUN(float, 32, false, true);
+    } else {
+      if (few) GLA_RUN(bf16_t, 8, false, true); else GLA_RUN(bf16_t, 32, false, true);
+    }
+  } else if (bonus) {
     if (dtype == TA_F32) {
       if (few) GLA_RUN(float, 8, true); else GLA_RUN(float, 32, true);
     } else {
@@ -816,21 +835,49 @@ extern "C" int ta_decay_recurrent(hipStream_t stream, int dtype, const void* pro
                               nullptr, head_decay);
 }
 
+// The recurrence of the matrix memory: keep and write [nt, H] float32 (ta_memory_gates), q, k, v at column
+// offsets of the rows of ``proj``, the query times qscale; n_state [slots, H, dk] float32. o_out
+// [ta_gla_row_parts(dk), nt, H, dv] and den_out [ta_gla_row_parts(dk), nt, H]: planes that add up to S_t^T q
+// and n_t . q.
+extern "C" int ta_memory_recurrent(hipStream_t stream, int dtype, const void* proj, int stride, int qoff, int koff,
+                                   int voff, float qscale, const float* keep, const float* write, float* state,
+                                   float* n_state, const int* cu_q, const int* slots, int batch, int nt, int H, int dk,
+                                   int dv, float* o_out, float* den_out) {
+  TA_REQUIRE(keep != nullptr && write != nullptr && n_state != nullptr && den_out != nullptr,
+             "ta_memory_recurrent: weights, normaliser and denominators are required");
+  return gla_recurrent_launch(stream, dtype, dtype, proj, stride, qoff, koff, voff, nullptr, 0, 0, 0, nullptr, nullptr,
+                              1.0f, qscale, nullptr, state, cu_q, slots, batch, nt, H, dk, dv, o_out, 0, nullptr,
+                              nullptr, 1, keep, write, n_state, den_out);
+}
+
 // ------------------------------------------------------------------ gla: head norm and output gate
+// Where a readout has a denominator, den [parts, nt, H] are the planes of n . q and floor_ [nt, H] what its
+// absolute value does not fall below: the readout is divided by max(|n . q|, floor) + 1e-6 before its norm.
+__device__ __forceinline__ float readout_factor(const float* __restrict__ den, const float* __restrict__ floor_,
+                                                int parts, size_t plane, size_t at) {
+  if (den == nullptr) return 1.f;
+  float d = den[at];
+  for (int p = 1; p < parts; ++p) d += den[p * plane + at];
+  return 1.0f / (fmaxf(fabsf(d), floor_[at]) + 1e-6f);
+}
+
 template <typename T>
 __global__ __launch_bounds__(64) void gla_out_kernel(const float* __restrict__ o, int parts, size_t plane,
                                                      const T* __restrict__ proj,
                                                      int stride, int goff, const float* __restrict__ w,
                                                      int wstride, float eps, int H, int dv, T* __restrict__ out,
-                                                     int gate_act) {
+                                                     int gate_act, const float* __restrict__ den,
+                                                     const float* __restrict__ floor_) {
   extern __shared__ float row[];          // [dv]
   const size_t t = blockIdx.x;
   const int h = blockIdx.y;
   const float* src = o + (t * H + h) * dv;
+  const float by = readout_factor(den, floor_, parts, plane / dv, t * H + h);
   float ss = 0.f;
   for (int c = threadIdx.x; c < dv; c += 64) {
     float v = src[c];
     for (int p = 1; p < parts; ++p) v += src[p * plane + c];
+    v *= by;
     row[c] = v;
     ss += v * v;
   }
@@ -851,7 +898,9 @@ template <typename T>
 __global__ __launch_bounds__(512) void gla_out_wide_kernel(const float* __restrict__ o, int parts, size_t plane,
                                                            const T* __restrict__ proj, int stride,
                                                            const float* __restrict__ w, int wstride, float eps,
-                                                           int H, int dv, T* __restrict__ out, int gate_act) {
+                                                           int H, int dv, T* __restrict__ out, int gate_act,
+                                                           const float* __restrict__ den,
+                                                           const float* __restrict__ floor_) {
   constexpr int PER = 8;                  // columns a thread can own: rows of up to 512 * PER
   __shared__ float red[8];
   const size_t t = blockIdx.x;
@@ -880,9 +929,13 @@ __global__ __launch_bounds__(512) void gla_out_wide_kernel(const float* __restri
     g[i] = c < dv ? to_f32(proj[t * stride + h * dv + c]) : 0.f;
     wc[i] = (c < dv && w) ? w[h * wstride + c] : 1.0f;
   }
+  const float by = readout_factor(den, floor_, parts, plane / dv, t * H + h);
   float ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < PER; ++i) ss += v[i] * v[i];
+  for (int i = 0; i < PER; ++i) {
+    v[i] *= by;
+    ss += v[i] * v[i];
+  }
   ss = wave_sum(ss);
   if (threadIdx.x % TA_WAVE == 0) red[threadIdx.x / TA_WAVE] = ss;
   __syncthreads();
@@ -900,42 +953,38 @@ __global__ __launch_bounds__(512) void gla_out_wide_kernel(const float* __restri
 // o: [parts, nt, H, dv] float32 planes that add up to the readout; the gate's pre-activation sits
 // at element goff of proj, ``stride`` elements between tokens; w [dv] shared by the heads
 // (wstride 0) or [H, dv] (wstride dv); out [nt, H*dv] = rms_norm(o per head) * w * silu(gate).
-// gate_act 0: silu(gate); 1: sigmoid(gate). w may be null (no weight).
+// gate_act 0: silu(gate); 1: sigmoid(gate). w may be null (no weight). den, floor_: null, or the readout's
+// denominators (see readout_factor).
 extern "C" int ta_gla_out_act(hipStream_t stream, int dtype, const float* o, int parts, const void* proj, int stride,
                               long long goff, const float* w, int wstride, float eps, int nt, int H, int dv,
-                              int gate_act, void* out) {
+                              int gate_act, const float* den, const float* floor_, void* out) {
   TA_REQUIRE(nt >= 0 && H > 0 && H <= 65535 && dv > 0 && dv <= 15000 && parts >= 1, "ta_gla_out: bad sizes");
   TA_REQUIRE(gate_act == 0 || gate_act == 1, "ta_gla_out: unknown gate activation %d", gate_act);
+  TA_REQUIRE((den == nullptr) == (floor_ == nullptr), "ta_gla_out: denominators come with their floor");
   TA_REQUIRE(wstride == 0 || wstride == dv, "ta_gla_out: weight rows of %d for heads of %d", wstride, dv);
   if (nt == 0) return 0;
   dim3 g(nt, H);
   const size_t plane = (size_t)nt * H * dv, lds = (size_t)dv * sizeof(float);
   if (dv > 512 && dv <= 4096 && (dtype == TA_F32 || dtype == TA_BF16)) {
     if (dtype == TA_F32)
-      gla_out_wide_kernel<float><<<g, 512, 0, stream>>>(o, parts, plane, (const float*)proj + goff, stride, w, wstride, eps, H, dv, (float*)out, gate_act);
+      gla_out_wide_kernel<float><<<g, 512, 0, stream>>>(o, parts, plane, (const float*)proj + goff, stride, w, wstride, eps, H, dv, (float*)out, gate_act, den, floor_);
     else
-      gla_out_wide_kernel<bf16_t><<<g, 512, 0, stream>>>(o, parts, plane, (const bf16_t*)proj + goff, stride, w, wstride, eps, H, dv, (bf16_t*)out, gate_act);
+      gla_out_wide_kernel<bf16_t><<<g, 512, 0, stream>>>(o, parts, plane, (const bf16_t*)proj + goff, stride, w, wstride, eps, H, dv, (bf16_t*)out, gate_act, den, floor_);
     return ta_check_launch("ta_gla_out");
   }
   if (dtype == TA_F32)
-    gla_out_kernel<float><<<g, 64, lds, stream>>>(o, parts, plane, (const float*)proj + goff, stride, 0, w, wstride, eps, H, dv, (float*)out, gate_act);
+    gla_out_kernel<float><<<g, 64, lds, stream>>>(o, parts, plane, (const float*)proj + goff, stride, 0, w, wstride, eps, H, dv, (float*)out, gate_act, den, floor_);
   else if (dtype == TA_BF16)
-    gla_out_kernel<bf16_t><<<g, 64, lds, stream>>>(o, parts, plane, (const bf16_t*)proj + goff, stride, 0, w, wstride, eps, H, dv, (bf16_t*)out, gate_act);
+    gla_out_kernel<bf16_t><<<g, 64, lds, stream>>>(o, parts, plane, (const bf16_t*)proj + goff, stride, 0, w, wstride, eps, H, dv, (bf16_t*)out, gate_act, den, floor_);
   else
     return ta_fail("ta_gla_out: unknown dtype %d", dtype);
   return ta_check_launch("ta_gla_out");
 }
 
-extern "C" int ta_gla_out_w(hipStream_t stream, int dtype, const float* o, int parts, const void* proj, int stride,
-                            long long goff, const float* w, int wstride, float eps, int nt, int H, int dv,
-                            void* out) {
-  TA_REQUIRE(w != nullptr, "ta_gla_out: the weight is required");
-  return ta_gla_out_act(stream, dtype, o, parts, proj, stride, goff, w, wstride, eps, nt, H, dv, 0, out);
-}
-
 extern "C" int ta_gla_out(hipStream_t stream, int dtype, const float* o, int parts, const void* proj, int stride,
                           int goff, const float* w, float eps, int nt, int H, int dv, void* out) {
-  return ta_gla_out_w(stream, dtype, o, parts, proj, stride, goff, w, 0, eps, nt, H, dv, out);
+  TA_REQUIRE(w != nullptr, "ta_gla_out: the weight is required");
+  return ta_gla_out_act(stream, dtype, o, parts, proj, stride, goff, w, 0, eps, nt, H, dv, 0, nullptr, nullptr, out);
 }
 
 // ------------------------------------------------------------------ short causal convolution

@@ -197,6 +197,9 @@ class DecoderModel:
                 self._run_extra("after_embed", x, ctx, cache)
         if self.dump is not None:
             self.dump("embed", x)
+        entered = None                       # what the embedding gave, where a later run adds it again
+        if any(run.reenter for run in s.schedule):
+            entered = kernels.weighted_sum([x], [1.0], self.ws.take("model.entered", x.shape, torch.float32))
         pending = (None, None)
         for i, run in enumerate(s.schedule):
             block = self.blocks[run.block]
@@ -205,8 +208,11 @@ class DecoderModel:
             kw = {}
             if run.opening is not None:
                 pending = self._open(x, pending, self.w["stream_rows"][run.opening])
+            if run.reenter:
+                pending = self._reenter(x, pending, entered)
             # the block in front may prepare the next block's norm, unless something is added in between
-            if getattr(block, "folds_norms", False) and i + 1 < len(s.schedule) and s.schedule[i + 1].opening is None:
+            if getattr(block, "folds_norms", False) and i + 1 < len(s.schedule) and s.schedule[i + 1].opening is None \
+                    and not s.schedule[i + 1].reenter:
                 kw["after"] = self.blocks[s.schedule[i + 1].block]    # it may prepare that block's norm
             pending = block.run(x, pending, ctx, cache, self.cache_layer[i],
                                 writes_cache=run.cache_of is None, **kw)
@@ -233,6 +239,14 @@ class DecoderModel:
         if isinstance(pending, tuple) and pending[1] is None and not isinstance(pending[0], kernels.GatedDelta):
             return pending[0], row
         kernels.stream_add(x, bias=row)
+        return pending
+
+    @staticmethod
+    def _reenter(x, pending, rows):
+        """``rows`` [nt, hidden] for the stream: where nothing else is pending the next norm adds them."""
+        if isinstance(pending, tuple) and pending[0] is None:
+            return rows, pending[1]
+        kernels.stream_add(x, delta=rows)
         return pending
 
     def _run_extra(self, name, t, ctx, cache):

@@ -108,6 +108,17 @@ def embed(table: torch.Tensor, tokens: torch.Tensor, out: torch.Tensor) -> torch
     return out
 
 
+def rows_add(table: torch.Tensor, index: torch.Tensor, x: torch.Tensor) -> torch.Tensor:
+    """x[t] += table[index[t]] in float32, in place. index: int32 [nt]; x: float32 [nt, d]."""
+    _dev(table, "table"); _dev(index, "index", torch.int32); _dev(x, "x", torch.float32)
+    rows, d = table.shape
+    if x.shape != (index.numel(), d):
+        raise KernelError(f"rows_add: x is {tuple(x.shape)}, expected {(index.numel(), d)}")
+    _check(library().ta_rows_add(_stream(), c_int(_code(table.dtype)), _ptr(table), c_int(rows), c_int(d), _ptr(index),
+                                 c_int(index.numel()), _ptr(x)))
+    return x
+
+
 # ------------------------------------------------------------------ add + norm
 def add_rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.Tensor,
                 delta: Optional[torch.Tensor] = None, delta_bias: Optional[torch.Tensor] = None,
@@ -359,11 +370,19 @@ def key_unit_count(batch: int, num_kv_heads: int) -> int:
 UNIT_INTS = 8      # int32 values in a unit's record, fixed in csrc/common.h (TA_UNIT_INTS)
 
 
-def seen_pages(length: int, window: Optional[int], keep_first: int = 0):
+def first_key(length: int, window: Optional[int], chunk: Optional[int] = None) -> int:
+    """The first key that a token at position ``length`` - 1 sees: of its window, of its chunk (chunks are
+    counted from position 0), or of all."""
+    if chunk:
+        return max(int(length) - 1, 0) // chunk * chunk
+    return max(0, int(length) - window) if window else 0
+
+
+def seen_pages(length: int, window: Optional[int], keep_first: int = 0, chunk: Optional[int] = None):
     """Page ranges [(first, pages), ...] that a single token at position ``length`` - 1 reads: the pages of
-    its window behind those of the sequence's kept first keys (one range where the two meet)."""
+    its window (or chunk) behind those of the sequence's kept first keys (one range where the two meet)."""
     n = max(1, -(-int(length) // PAGE))
-    first = max(0, int(length) - window) // PAGE if window else 0
+    first = first_key(length, window, chunk) // PAGE
     kept = min(-(-int(keep_first) // PAGE), first)
     if kept == first:
         return [(0, n)]
@@ -371,7 +390,7 @@ def seen_pages(length: int, window: Optional[int], keep_first: int = 0):
 
 
 def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tables=None,
-                   window: Optional[int] = None, keep_first: int = 0):
+                   window: Optional[int] = None, keep_first: int = 0, chunk: Optional[int] = None):
     """Cuts sequences of ``kv_lens`` tokens (this step's token included) into at most
     ``n_units`` runs of pages of about equal length, none shorter than ``min_pages`` unless
     it is a whole sequence: a CU can ask only so much of the memory in a given time, so the
@@ -379,7 +398,7 @@ def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tab
     first page, pages, the sequence's length, page numbers of the unit's first two pages (from
     ``tables[b]``, the sequence's row of the block table; 0 without), units of the sequence,
     0), spare units holding 0 pages, and seq_units [batch, 2] = (first unit, units); a
-    sequence's units follow one another and cover its pages in order. With a window only the pages
+    sequence's units follow one another and cover its pages in order. With a window or chunks only the pages
     that the token sees are dealt out (``seen_pages``), unless there are too few units. Pure host."""
     import heapq
     import numpy as np
@@ -387,7 +406,7 @@ def plan_key_units(kv_lens: Sequence[int], n_units: int, min_pages: int = 0, tab
     B = len(kv_lens)
     if n_units < B:
         raise KernelError(f"{n_units} units of work cannot hold {B} sequences")
-    ranges = [(b, first, n) for b in range(B) for first, n in seen_pages(kv_lens[b], window, keep_first)]
+    ranges = [(b, first, n) for b in range(B) for first, n in seen_pages(kv_lens[b], window, keep_first, chunk)]
     if n_units < len(ranges):
         ranges = [(b, first, n) for b in range(B) for first, n in seen_pages(kv_lens[b], None)]
     pages = [r[2] for r in ranges]
@@ -1407,11 +1426,13 @@ _GATE_ACTS = {"silu": 0, "sigmoid": 1}
 
 def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, heads: int, value_dim: int,
                    weight: Optional[torch.Tensor], eps: float, out: torch.Tensor,
-                   gate_act: str = "silu") -> torch.Tensor:
+                   gate_act: str = "silu", den: Optional[torch.Tensor] = None,
+                   floor: Optional[torch.Tensor] = None) -> torch.Tensor:
     """out = rms_norm(o per head) * weight * act(gate): o [parts, nt, H, dv] float32 planes that
     add up, gate [nt, H*dv] (contiguous rows), weight [dv] for all heads, [H*dv], or None (the
     plain division by the root mean square); act "silu" or "sigmoid". A norm over all heads at
-    once is the call with heads = 1 and value_dim = the whole row."""
+    once is the call with heads = 1 and value_dim = the whole row. den [parts, nt, H] planes and floor
+    [nt, H], float32: o is first divided by max(|sum of den|, floor) + 1e-6."""
     _dev(o, "o", torch.float32); _dev(gate, "gate", contiguous=False); _dev(out, "out", gate.dtype)
     if weight is not None:
         _dev(weight, "weight", torch.float32)
@@ -1423,10 +1444,17 @@ def head_norm_gate(o: torch.Tensor, gate: torch.Tensor, heads: int, value_dim: i
             or (weight is not None and weight.numel() not in (dv, H * dv)):
         raise KernelError(f"head_norm_gate: o {tuple(o.shape)} gate {tuple(gate.shape)} out {tuple(out.shape)} "
                           f"weight {None if weight is None else tuple(weight.shape)}")
+    if (den is None) != (floor is None):
+        raise KernelError("head_norm_gate: denominators come with their floor")
+    if den is not None:
+        _dev(den, "den", torch.float32); _dev(floor, "floor", torch.float32)
+        if den.shape != (o.shape[0], nt, H) or floor.shape != (nt, H):
+            raise KernelError(f"head_norm_gate: den {tuple(den.shape)} floor {tuple(floor.shape)} for o {tuple(o.shape)}")
     wstride = dv if weight is not None and weight.numel() == H * dv and H > 1 else 0
     _check(library().ta_gla_out_act(_stream(), c_int(_code(gate.dtype)), _ptr(o), c_int(o.shape[0]), _ptr(gate),
                                     c_int(gs), c_longlong(0), _ptr(weight), c_int(wstride), c_float(eps),
-                                    c_int(nt), c_int(H), c_int(dv), c_int(_GATE_ACTS[gate_act]), _ptr(out)))
+                                    c_int(nt), c_int(H), c_int(dv), c_int(_GATE_ACTS[gate_act]), _ptr(den), _ptr(floor),
+                                    _ptr(out)))
     return out
 
 
@@ -1631,13 +1659,14 @@ def moe_max_rows(pairs: int, experts: int) -> int:
 
 def moe_route(logits: torch.Tensor, experts: int, top: int, chosen: torch.Tensor, weight: torch.Tensor,
               score: str = "sigmoid", renormalize: bool = False, bias: Optional[torch.Tensor] = None,
-              groups: int = 1, keep_groups: int = 1):
+              groups: int = 1, keep_groups: int = 1, correction: Optional[torch.Tensor] = None, factor: float = 1.0):
     """chosen [nt, top] int32, weight [nt, top] float32: the ``top`` largest scores of the
     first ``experts`` columns of logits [nt, >= experts] float32 (lowest index among equals).
     bias [experts] float32: added to the logits first. "softmax" with ``renormalize`` is the
     softmax over the chosen logits alone. groups > 1: the experts form that many equal groups of
     neighbours, a group counts as its largest score, and only experts of the ``keep_groups`` best
-    groups can be chosen."""
+    groups can be chosen. correction [experts] float32: the choice compares score + correction, the weights
+    are the scores without it. factor: multiplies the weights (behind ``renormalize``)."""
     _dev(logits, "logits", torch.float32, contiguous=False)
     nt, ld = _rows2d(logits, "logits")
     _dev(chosen, "chosen", torch.int32); _dev(weight, "weight", torch.float32)
@@ -1650,15 +1679,20 @@ def moe_route(logits: torch.Tensor, experts: int, top: int, chosen: torch.Tensor
     if groups < 1 or experts % groups or not 1 <= keep_groups <= groups or top > keep_groups * (experts // groups):
         raise KernelError(f"moe_route: {experts} experts in {groups} groups of which {keep_groups} stay "
                           f"do not hold {top} choices")
-    _check(library().ta_moe_route_groups(_stream(), _ptr(logits), _ptr(bias), c_int(ld), c_int(nt), c_int(experts),
-                                         c_int(top), c_int(_ROUTE_MODES[score]), c_int(int(renormalize)),
-                                         c_int(groups), c_int(keep_groups), _ptr(chosen), _ptr(weight)))
+    if correction is not None:
+        _dev(correction, "correction", torch.float32)
+        if correction.shape != (experts,):
+            raise KernelError(f"moe_route: correction is {tuple(correction.shape)}, expected {(experts,)}")
+    _check(library().ta_moe_route(_stream(), _ptr(logits), _ptr(bias), c_int(ld), c_int(nt), c_int(experts),
+                                  c_int(top), c_int(_ROUTE_MODES[score]), c_int(int(renormalize)), c_int(groups),
+                                  c_int(keep_groups), _ptr(correction), c_float(factor), _ptr(chosen), _ptr(weight)))
     return chosen, weight
 
 
 def moe_plan(chosen: torch.Tensor, experts: int, row_pair: torch.Tensor, tile_expert: torch.Tensor,
              pair_row: torch.Tensor):
-    """Orders the (token, choice) pairs by expert; see ``moe_max_rows`` for row_pair's size."""
+    """Orders the (token, choice) pairs by expert; see ``moe_max_rows`` for row_pair's size. A choice of
+    ``experts`` or more gets no row (pair_row -1): an expert without matrices."""
     _dev(chosen, "chosen", torch.int32); _dev(row_pair, "row_pair", torch.int32)
     _dev(tile_expert, "tile_expert", torch.int32); _dev(pair_row, "pair_row", torch.int32)
     pairs = chosen.numel()
@@ -1703,11 +1737,12 @@ def moe_gemm(a: torch.Tensor, w: torch.Tensor, tile_expert: torch.Tensor, out: t
 
 
 def moe_combine(rows: torch.Tensor, top: int, pair_row: torch.Tensor, weight, shared, shared_gate,
-                delta: torch.Tensor, extra: Optional[torch.Tensor] = None) -> torch.Tensor:
+                delta: torch.Tensor, extra: Optional[torch.Tensor] = None,
+                own: Optional[torch.Tensor] = None) -> torch.Tensor:
     """delta[t] = sum over the token's pairs of rows[pair_row] (* weight) + sigmoid(shared_gate[t,
     0]) * shared[t] (+ extra[t]); shared and extra [nt, d] or [planes, nt, d] float32;
     shared_gate float32 [nt, >= 1]. ``extra``: what another sublayer adds to the stream beside
-    this one."""
+    this one. own [nt, d]: the token's own row, which stands for a pair without a row (pair_row -1)."""
     _dev(rows, "rows", torch.float32); _dev(pair_row, "pair_row", torch.int32); _dev(delta, "delta", torch.float32)
     nt, d = delta.shape
     if rows.shape[1] != d or pair_row.numel() != nt * top:
@@ -1735,10 +1770,15 @@ def moe_combine(rows: torch.Tensor, top: int, pair_row: torch.Tensor, weight, sh
             xplanes = 1
         else:
             raise KernelError(f"moe_combine: extra is {tuple(extra.shape)}")
-    _check(library().ta_moe_combine_extra(_stream(), _ptr(rows), c_int(d), c_int(top), _ptr(pair_row), _ptr(weight),
-                                          _ptr(shared), c_int(planes), c_longlong(plane), _ptr(shared_gate),
-                                          c_int(gl), _ptr(extra), c_int(xplanes), c_longlong(xplane), _ptr(delta),
-                                          c_int(nt)))
+    if own is not None:
+        _dev(own, "own")
+        if own.shape != delta.shape:
+            raise KernelError(f"moe_combine: own is {tuple(own.shape)}")
+    _check(library().ta_moe_combine(_stream(), _ptr(rows), c_int(d), c_int(top), _ptr(pair_row), _ptr(weight),
+                                    _ptr(shared), c_int(planes), c_longlong(plane), _ptr(shared_gate),
+                                    c_int(gl), _ptr(extra), c_int(xplanes), c_longlong(xplane),
+                                    c_int(_code(torch.float32 if own is None else own.dtype)), _ptr(own), _ptr(delta),
+                                    c_int(nt)))
     return delta
 
 
@@ -1762,7 +1802,7 @@ def qk_rotate_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_di
     cols = num_heads * key_dim + own * (key_dim + value_dim)
     if qkv.shape[1] != cols:
         raise KernelError(f"qk_rotate_store: rows of {qkv.shape[1]}, expected {cols}")
-    if style not in _ROT_STYLES or key_dim % 2 or rot % 2 or not 0 <= rot <= key_dim:
+    if style not in _ROT_STYLES or (key_dim % 2 and (rot or bias is not None)) or rot % 2 or not 0 <= rot <= key_dim:
         raise KernelError(f"qk_rotate_store: {rot} rotated coordinates of heads of {key_dim}, pairing {style!r}")
     if bias is not None:
         _dev(bias, "bias", torch.float32)
@@ -1794,14 +1834,16 @@ def qk_rotate_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, key_di
 
 def attention_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, num_heads, num_kv_heads, key_dim,
                    value_dim, scale, window=None, softcap: Optional[float] = None, sink=None,
-                   gate: Optional[torch.Tensor] = None, gate_dim: Optional[int] = None, keep_first: int = 0):
+                   gate: Optional[torch.Tensor] = None, gate_dim: Optional[int] = None, keep_first: int = 0,
+                   chunk: Optional[int] = None):
     """``attention_generic_dv`` with the options of a capped, sunk and gated softmax. softcap: score <-
     softcap * tanh(score / softcap) after the scale. sink: None; "unit": the denominator holds one more
     term exp(0) = 1; a float32 tensor [heads]: one more term exp(sink[head]). gate: rows [nt, >= heads *
     value_dim] of q's type whose sigmoid multiplies the result element by element. gate_dim: columns per
     head of the gate's rows where that is less than value_dim (a cache whose value rows are padded): the
     result's columns beyond it are not gated; 0: the gate's rows [nt, >= heads] hold one number per head.
-    keep_first: with a window, that many first keys of a sequence are seen as well."""
+    keep_first: with a window, that many first keys of a sequence are seen as well. chunk: instead of a
+    window, a query at position p sees the keys from (p // chunk) * chunk on."""
     _dev(q, "q", contiguous=False); _dev(out, "out", q.dtype, contiguous=False)
     nt, qs = _rows2d(q, "q")
     nto, os_ = _rows2d(out, "out")
@@ -1824,7 +1866,7 @@ def attention_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, nu
         _ptr(vcache), _ptr(block_table), c_int(block_table.shape[1]), _ptr(cu_q), _ptr(pos0),
         c_int(B), c_int(max_qlen), c_int(num_heads), c_int(num_kv_heads), c_int(key_dim),
         c_int(value_dim), c_float(scale), c_int(window or 0), c_float(cap), c_int(mode),
-        _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window))))
+        _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window)), c_int(_chunk(chunk, window))))
     return out
 
 
@@ -1833,6 +1875,14 @@ def _kept(keep_first, window) -> int:
     if keep_first < 0:
         raise KernelError(f"attention: {keep_first} kept first keys")
     return int(keep_first) if window else 0
+
+
+def _chunk(chunk, window) -> int:
+    if chunk is None:
+        return 0
+    if chunk < 1 or window:
+        raise KernelError(f"attention: chunks of {chunk} keys beside a window of {window}")
+    return int(chunk)
 
 
 def _sink_args(what, q, num_heads, value_dim, softcap, sink, gate):
@@ -1860,7 +1910,7 @@ def _sink_args(what, q, num_heads, value_dim, softcap, sink, gate):
 
 def attention_rows_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qlen, num_heads, num_kv_heads,
                         head_dim, scale, window=None, softcap=None, sink=None, gate=None, gate_dim=None,
-                        exact=True, through_lds=None, keep_first=0):
+                        exact=True, through_lds=None, keep_first=0, chunk=None):
     """``attention_rows`` (matrix cores, bfloat16, values as wide as the keys) with the options of
     ``attention_sink``. gate_dim: columns per head of the gate's rows (the values' own width where the
     cache pads them to the keys'; 0: one number per head); out's columns beyond it are not gated. exact: the softmax weights
@@ -1877,13 +1927,13 @@ def attention_rows_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_qle
         _ptr(block_table), c_int(block_table.shape[1]), _ptr(cu_q), _ptr(pos0), c_int(B),
         c_int(max_qlen), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim), c_float(scale),
         c_int(window or 0), c_int(int(through_lds)), c_float(cap), c_int(int(exact)), c_int(mode), _ptr(sink_t),
-        _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window))))
+        _ptr(gate), c_int(gs), c_int(gd), c_int(_kept(keep_first, window)), c_int(_chunk(chunk, window))))
     return out
 
 
 def attention_keys_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_kv_len, num_heads, num_kv_heads,
                         head_dim, scale, window=None, softcap=None, sink=None, gate=None, gate_dim=None,
-                        exact=True, units=None, seq_units=None, keep_first=0):
+                        exact=True, units=None, seq_units=None, keep_first=0, chunk=None):
     """``attention_keys`` (single tokens on the matrix cores; q holds rotated heads, the cache the step's
     keys and values) with the options of ``attention_rows_sink``: the kernel whose four waves take a
     unit's pages in turn, and the merge, which adds the sink's share and applies the gate."""
@@ -1912,7 +1962,7 @@ def attention_keys_sink(q, out, kcache, vcache, block_table, cu_q, pos0, max_kv_
         c_int(block_table.shape[1]), _ptr(pos0), c_int(B), c_int(num_heads), c_int(num_kv_heads), c_int(head_dim),
         c_float(scale), c_int(window or 0), _ptr(units), _ptr(seq_units), c_int(n_units), c_int(4), _ptr(scratch),
         c_float(cap), c_int(int(exact)), c_int(mode), _ptr(sink_t), _ptr(gate), c_int(gs), c_int(gd),
-        c_int(_kept(keep_first, window))))
+        c_int(_kept(keep_first, window)), c_int(_chunk(chunk, window))))
     return out
 
 
@@ -2083,39 +2133,46 @@ def delta_prepare(qkv: torch.Tensor, z: torch.Tensor, dt_bias, a_log, b_raw: tor
     """What the delta rule needs of every token, float32: from rows [q | k | ...] of ``qkv`` (groups x
     key_dim each, behind convolution and activation) unit vectors per group, qn = q_scale * q / |q| and
     kn = k / |k| ([nt, groups, key_dim]; |x|^2 = sum of squares + 1e-6), and kq = kn . qn [nt, groups];
-    decay [nt, heads, key_dim] = exp(-exp(a_log[h]) * softplus(z + dt_bias)), z [nt, heads * key_dim];
-    beta [nt, heads] = sigmoid(b_raw)."""
-    _dev(qkv, "qkv", contiguous=False); _dev(z, "z", torch.float32); _dev(b_raw, "b_raw", qkv.dtype, contiguous=False)
+    decay [nt, heads, key_dim] = exp(-exp(a_log[h]) * softplus(z + dt_bias)), z [nt, heads * key_dim] float32, or
+    decay [nt, heads] (one per head), z [nt, heads] columns in the type of ``qkv``; beta [nt, heads] =
+    sigmoid(b_raw)."""
+    per_head = decay.dim() == 2
+    _dev(qkv, "qkv", contiguous=False); _dev(b_raw, "b_raw", qkv.dtype, contiguous=False)
+    _dev(z, "z", qkv.dtype if per_head else torch.float32, contiguous=False)
     nt, stride = _rows2d(qkv, "qkv")
     nb, bs = _rows2d(b_raw, "b_raw")
+    nz, zs = _rows2d(z, "z")
     G, H, dk = groups, heads, key_dim
-    for t, n, shape in ((dt_bias, "dt_bias", (H * dk,)), (a_log, "a_log", (H,)), (z, "z", (nt, H * dk)),
-                        (qn, "qn", (nt, G, dk)), (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H, dk)),
+    n_z = H if per_head else H * dk
+    for t, n, shape in ((dt_bias, "dt_bias", (n_z,)), (a_log, "a_log", (H,)), (qn, "qn", (nt, G, dk)),
+                        (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H) if per_head else (nt, H, dk)),
                         (beta, "beta", (nt, H)), (kq, "kq", (nt, G))):
         _dev(t, n, torch.float32)
         if tuple(t.shape) != shape:
             raise KernelError(f"delta_prepare: {n} is {tuple(t.shape)}, expected {shape}")
-    if nb != nt or b_raw.shape[1] != H or qkv.shape[1] < 2 * G * dk or G < 1 or H % G:
-        raise KernelError(f"delta_prepare: qkv {tuple(qkv.shape)} / b_raw {tuple(b_raw.shape)} for {H} heads in {G} groups of {dk}")
+    if nb != nt or b_raw.shape[1] != H or tuple(z.shape) != (nt, n_z) or qkv.shape[1] < 2 * G * dk or G < 1 or H % G:
+        raise KernelError(f"delta_prepare: qkv {tuple(qkv.shape)} / z {tuple(z.shape)} / b_raw {tuple(b_raw.shape)} for "
+                          f"{H} heads in {G} groups of {dk}")
     _check(library().ta_delta_prepare(
-        _stream(), c_int(_code(qkv.dtype)), _ptr(qkv), c_int(stride), _ptr(z), _ptr(dt_bias), _ptr(a_log), _ptr(b_raw),
-        c_int(bs), c_int(nt), c_int(G), c_int(H), c_int(dk), c_float(q_scale), _ptr(qn), _ptr(kn), _ptr(decay),
-        _ptr(beta), _ptr(kq)))
+        _stream(), c_int(_code(qkv.dtype)), _ptr(qkv), c_int(stride), _ptr(z), c_int(zs), c_int(int(per_head)),
+        _ptr(dt_bias), _ptr(a_log), _ptr(b_raw), c_int(bs), c_int(nt), c_int(G), c_int(H), c_int(dk), c_float(q_scale),
+        _ptr(qn), _ptr(kn), _ptr(decay), _ptr(beta), _ptr(kq)))
 
 
 def delta_recurrent(qn: torch.Tensor, kn: torch.Tensor, decay: torch.Tensor, v: torch.Tensor, beta: torch.Tensor,
                     kq: torch.Tensor, state: torch.Tensor, cu_q, slots, o_out: torch.Tensor, lanes: int = 0) -> torch.Tensor:
     """The delta rule along every sequence: S <- diag(decay) S; u = beta (v - S^T k); S <- S + k u^T; o =
-    S^T q, head h with the q and k of group h // (heads / groups). qn, kn [nt, G, dk], decay [nt, H, dk],
-    beta [nt, H], kq [nt, G] (k . q) float32; v [nt, H * dv] rows in the engine's type; ``state`` [slots, H,
-    dk, dv] float32; o_out [nt, H, dv] float32. lanes that share a column: 16 or 32 (0: chosen by the shape)."""
+    S^T q, head h with the q and k of group h // (heads / groups). qn, kn [nt, G, dk], decay [nt, H, dk] or one
+    per head [nt, H], beta [nt, H], kq [nt, G] (k . q) float32; v [nt, H * dv] rows in the engine's type;
+    ``state`` [slots, H, dk, dv] float32; o_out [nt, H, dv] float32. lanes that share a column: 16 or 32 (0:
+    chosen by the shape)."""
     nt, G, dk = qn.shape
-    H = decay.shape[1]
+    H, per_head = decay.shape[1], decay.dim() == 2
     _dev(v, "v", contiguous=False); _dev(state, "state", torch.float32)
     nv, vs = _rows2d(v, "v")
     batch = _step_tables(cu_q, slots, nt, "delta_recurrent")
     dv = state.shape[3] if state.dim() == 4 else -1
-    for t, n, shape in ((qn, "qn", (nt, G, dk)), (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H, dk)),
+    for t, n, shape in ((qn, "qn", (nt, G, dk)), (kn, "kn", (nt, G, dk)), (decay, "decay", (nt, H) if per_head else (nt, H, dk)),
                         (beta, "beta", (nt, H)), (kq, "kq", (nt, G)), (o_out, "o_out", (nt, H, dv))):
         _dev(t, n, torch.float32)
         if tuple(t.shape) != shape:
@@ -2127,42 +2184,143 @@ def delta_recurrent(qn: torch.Tensor, kn: torch.Tensor, decay: torch.Tensor, v: 
     _check(library().ta_delta_recurrent(
         _stream(), c_int(_code(v.dtype)), _ptr(qn), _ptr(kn), _ptr(decay), _ptr(v), c_int(vs), _ptr(beta), _ptr(kq),
         _ptr(state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(H), c_int(G), c_int(dk), c_int(dv),
-        c_int(lanes), _ptr(o_out)))
+        c_int(lanes), c_int(int(per_head)), _ptr(o_out)))
     return o_out
 
 
 def delta_step_fits(key_dim: int, value_dim: int, decay_rank: int, gate_rank: int) -> bool:
-    """Whether ``delta_step`` takes heads of this size."""
+    """Whether ``delta_step`` takes heads of this size (ranks 0: no low-rank product)."""
     return bool(library().ta_delta_step_fits(c_int(key_dim), c_int(value_dim), c_int(decay_rank), c_int(gate_rank)))
 
 
 def delta_step(qkv: torch.Tensor, proj: torch.Tensor, a_off: int, g_off: int, b_off: int, decay_w, gate_w, dt_bias, a_log,
                state: torch.Tensor, slots, heads: int, groups: int, q_scale: float, norm_w, eps: float,
-               out: torch.Tensor) -> torch.Tensor:
+               out: torch.Tensor, gate_act: str = "sigmoid") -> torch.Tensor:
     """A step of single tokens of the delta rule in one kernel (row b belongs to sequence b): qkv rows
     [q | k | v] behind convolution and activation; the rows of ``proj`` hold the decay's low-rank input at
     column a_off, the output gate's at g_off and the step sizes' at b_off; decay_w [H*dk, ra], gate_w
-    [H*dv, rg]. out [batch, H*dv] = o / rms(o per head) * norm_w * sigmoid(gate)."""
+    [H*dv, rg]. decay_w None: one decay per head, its H inputs at a_off, dt_bias [H]; gate_w None: the gates
+    (H*dv) themselves at g_off. out [batch, H*dv] = o / rms(o per head) * norm_w * act(gate)."""
     _dev(qkv, "qkv", contiguous=False); _dev(proj, "proj", qkv.dtype, contiguous=False); _dev(out, "out", qkv.dtype)
     B, stride = _rows2d(qkv, "qkv")
     Bp, ps = _rows2d(proj, "proj")
-    _dev(state, "state", torch.float32); _dev(slots, "slots", torch.int32); _dev(decay_w, "decay_w"); _dev(gate_w, "gate_w")
-    if state.dim() != 4 or state.shape[1] != heads or decay_w.dtype != gate_w.dtype:
-        raise KernelError(f"delta_step: state {tuple(state.shape)} for {heads} heads, weights {decay_w.dtype} / {gate_w.dtype}")
+    _dev(state, "state", torch.float32); _dev(slots, "slots", torch.int32)
+    if state.dim() != 4 or state.shape[1] != heads or gate_act not in _GATE_ACTS:
+        raise KernelError(f"delta_step: state {tuple(state.shape)} for {heads} heads, gate activation {gate_act!r}")
     dk, dv, H, G = state.shape[2], state.shape[3], heads, groups
-    ra, rg = decay_w.shape[1], gate_w.shape[1]
-    for t, n, shape in ((dt_bias, "dt_bias", (H * dk,)), (a_log, "a_log", (H,)), (norm_w, "norm_w", (dv,))):
+    wcodes, ranks = [], []
+    for w, n, rows in ((decay_w, "decay_w", H * dk), (gate_w, "gate_w", H * dv)):
+        if w is None:
+            ranks.append(0)
+            continue
+        _dev(w, n)
+        if w.dim() != 2 or w.shape[0] != rows:
+            raise KernelError(f"delta_step: {n} is {tuple(w.shape)}, expected {rows} rows")
+        ranks.append(w.shape[1])
+        wcodes.append(_wcode(w, qkv.dtype, "delta_step"))
+    if len(set(wcodes)) > 1:
+        raise KernelError(f"delta_step: weights {decay_w.dtype} / {gate_w.dtype}")
+    ra, rg = ranks
+    for t, n, shape in ((dt_bias, "dt_bias", (H * dk,) if ra else (H,)), (a_log, "a_log", (H,)), (norm_w, "norm_w", (dv,))):
         _dev(t, n, torch.float32)
         if tuple(t.shape) != shape:
             raise KernelError(f"delta_step: {n} is {tuple(t.shape)}, expected {shape}")
-    if Bp != B or slots.numel() != B or qkv.shape[1] != 2 * G * dk + H * dv or decay_w.shape[0] != H * dk or \
-            gate_w.shape[0] != H * dv or out.shape != (B, H * dv) or H % G or min(a_off, g_off, b_off) < 0 or \
-            max(a_off + ra, g_off + rg, b_off + H) > proj.shape[1]:
+    if Bp != B or slots.numel() != B or qkv.shape[1] != 2 * G * dk + H * dv or out.shape != (B, H * dv) or H % G or \
+            min(a_off, g_off, b_off) < 0 or max(a_off + (ra or H), g_off + (rg or H * dv), b_off + H) > proj.shape[1]:
         raise KernelError(f"delta_step: qkv {tuple(qkv.shape)} proj {tuple(proj.shape)} out {tuple(out.shape)} for {H} "
                           f"heads in {G} groups of {dk} / {dv}, ranks {ra} / {rg}")
     _check(library().ta_delta_step(
-        _stream(), c_int(_code(qkv.dtype)), c_int(_wcode(decay_w, qkv.dtype, "delta_step")), _ptr(qkv), c_int(stride),
+        _stream(), c_int(_code(qkv.dtype)), c_int(wcodes[0] if wcodes else _code(qkv.dtype)), _ptr(qkv), c_int(stride),
         _ptr(proj), c_int(ps), c_int(a_off), c_int(ra), c_int(g_off), c_int(rg), c_int(b_off), _ptr(decay_w), _ptr(gate_w),
         _ptr(dt_bias), _ptr(a_log), _ptr(state), _ptr(slots), c_int(B), c_int(H), c_int(G), c_int(dk), c_int(dv),
-        c_float(q_scale), _ptr(norm_w), c_float(eps), _ptr(out)))
+        c_float(q_scale), _ptr(norm_w), c_float(eps), c_int(_GATE_ACTS[gate_act]), _ptr(out)))
+    return out
+
+
+# ------------------------------------------------------------------ matrix memory
+def _memory_columns(what, proj, offs, H, dk, dv):
+    """Checks that q, k, v, gate, i, f (or the first of them) lie inside the rows of ``proj``."""
+    for off, n in zip(offs, (H * dk, H * dk, H * dv, H * dv, H, H)):
+        if off < 0 or off + n > proj.shape[1]:
+            raise KernelError(f"{what}: columns {off}..{off + n} of rows of {proj.shape[1]}")
+
+
+def memory_gates(proj: torch.Tensor, i_off: int, f_off: int, i_bias, f_bias, cap: float, m_state: torch.Tensor, cu_q,
+                 slots, keep: torch.Tensor, write: torch.Tensor, floor: torch.Tensor) -> None:
+    """The gates of the matrix memory, float32 [nt, H] each: with i = cap tanh((proj[i_off + h] + i_bias) / cap), f =
+    log sigmoid(cap tanh((proj[f_off + h] + f_bias) / cap)) and the running maximum m <- max(f + m, i) of every
+    sequence (``m_state`` [slots, H], moved on): keep = exp(f + m_before - m), write = exp(i - m), floor = exp(-m)."""
+    _dev(proj, "proj", contiguous=False)
+    nt, stride = _rows2d(proj, "proj")
+    batch = _step_tables(cu_q, slots, nt, "memory_gates")
+    _dev(m_state, "m_state", torch.float32)
+    H = m_state.shape[1] if m_state.dim() == 2 else -1
+    for t, n, shape in ((i_bias, "i_bias", (H,)), (f_bias, "f_bias", (H,)), (keep, "keep", (nt, H)),
+                        (write, "write", (nt, H)), (floor, "floor", (nt, H))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"memory_gates: {n} is {tuple(t.shape)}, expected {shape}")
+    if min(i_off, f_off) < 0 or max(i_off, f_off) + H > proj.shape[1]:
+        raise KernelError(f"memory_gates: columns {i_off} / {f_off} of rows of {proj.shape[1]} for {H} heads")
+    _check(library().ta_memory_gates(
+        _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), c_int(i_off), c_int(f_off), _ptr(i_bias),
+        _ptr(f_bias), c_float(cap), _ptr(m_state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(H), _ptr(keep),
+        _ptr(write), _ptr(floor)))
+
+
+def memory_recurrent(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_scale: float, keep: torch.Tensor,
+                     write: torch.Tensor, state: torch.Tensor, n_state: torch.Tensor, cu_q, slots, o_out: torch.Tensor,
+                     den_out: torch.Tensor) -> torch.Tensor:
+    """The matrix memory along every sequence: S <- keep S + write k v^T, n <- keep n + write k, o = S^T (q_scale q),
+    den = n . (q_scale q). ``state`` [slots, H, dk, dv], ``n_state`` [slots, H, dk] float32; o_out
+    [gla_row_parts(dk), nt, H, dv] and den_out [gla_row_parts(dk), nt, H] float32 planes that add up."""
+    _dev(proj, "proj", contiguous=False); _dev(state, "state", torch.float32)
+    nt, stride = _rows2d(proj, "proj")
+    batch = _step_tables(cu_q, slots, nt, "memory_recurrent")
+    if state.dim() != 4:
+        raise KernelError(f"memory_recurrent: state is {tuple(state.shape)}")
+    S, H, dk, dv = state.shape
+    parts = gla_row_parts(dk)
+    for t, n, shape in ((keep, "keep", (nt, H)), (write, "write", (nt, H)), (n_state, "n_state", (S, H, dk)),
+                        (o_out, "o_out", (parts, nt, H, dv)), (den_out, "den_out", (parts, nt, H))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"memory_recurrent: {n} is {tuple(t.shape)}, expected {shape}")
+    _memory_columns("memory_recurrent", proj, (q_off, k_off, v_off), H, dk, dv)
+    _check(library().ta_memory_recurrent(
+        _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), c_int(q_off), c_int(k_off), c_int(v_off),
+        c_float(q_scale), _ptr(keep), _ptr(write), _ptr(state), _ptr(n_state), _ptr(cu_q), _ptr(slots), c_int(batch),
+        c_int(nt), c_int(H), c_int(dk), c_int(dv), _ptr(o_out), _ptr(den_out)))
+    return o_out
+
+
+def memory_step_fits(key_dim: int, value_dim: int) -> bool:
+    """Whether ``memory_step`` takes heads of this size."""
+    return bool(library().ta_memory_step_fits(c_int(key_dim), c_int(value_dim)))
+
+
+def memory_step(proj: torch.Tensor, offsets: Sequence[int], i_bias, f_bias, cap: float, state: torch.Tensor,
+                n_state: torch.Tensor, m_state: torch.Tensor, slots, q_scale: float, norm_w, eps: float,
+                out: torch.Tensor) -> torch.Tensor:
+    """A step of single tokens of the matrix memory in one kernel (row b belongs to sequence b). offsets: columns
+    of q, k, v, the output gate, the input and the forget gates in the rows of ``proj``. out [batch, H*dv] = o /
+    rms(o per head) * norm_w * sigmoid(gate), o = S^T q / (max(|n . q|, exp(-m)) + 1e-6)."""
+    _dev(proj, "proj", contiguous=False); _dev(state, "state", torch.float32); _dev(out, "out", proj.dtype)
+    B, stride = _rows2d(proj, "proj")
+    _dev(slots, "slots", torch.int32)
+    if state.dim() != 4 or len(offsets) != 6:
+        raise KernelError(f"memory_step: state {tuple(state.shape)}, offsets {tuple(offsets)}")
+    S, H, dk, dv = state.shape
+    for t, n, shape in ((i_bias, "i_bias", (H,)), (f_bias, "f_bias", (H,)), (n_state, "n_state", (S, H, dk)),
+                        (m_state, "m_state", (S, H)), (norm_w, "norm_w", (H * dv,))):
+        _dev(t, n, torch.float32)
+        if tuple(t.shape) != shape:
+            raise KernelError(f"memory_step: {n} is {tuple(t.shape)}, expected {shape}")
+    if slots.numel() != B or out.shape != (B, H * dv):
+        raise KernelError(f"memory_step: {slots.numel()} slots, out {tuple(out.shape)} for {B} rows of {H} heads of {dv}")
+    _memory_columns("memory_step", proj, offsets, H, dk, dv)
+    _check(library().ta_memory_step(
+        _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), *[c_int(int(o)) for o in offsets], _ptr(i_bias),
+        _ptr(f_bias), c_float(cap), _ptr(state), _ptr(n_state), _ptr(m_state), _ptr(slots), c_int(B), c_int(H), c_int(dk),
+        c_int(dv), c_float(q_scale), _ptr(norm_w), c_float(eps), _ptr(out)))
     return out

@@ -28,10 +28,11 @@ class KeyUnitPlanner:
     """The work plan of the single-token attention kernels, made on the host with every step's
     tables: the sequences of the step cut into units of work of about equal length
     (``kernels.plan_key_units``). Mixers with the same number of kv heads (and, where the plan leaves
-    out pages that no token of the step sees, the same window and kept first keys) share one plan."""
+    out pages that no token of the step sees, the same window or chunk and kept first keys) share one plan."""
     num_kv_heads: int
     window: int = 0
     keep_first: int = 0
+    chunk: int = 0
 
     def ints(self, batch: int) -> int:
         return kernels.UNIT_INTS * kernels.key_unit_count(batch, self.num_kv_heads) + 2 * batch
@@ -39,7 +40,7 @@ class KeyUnitPlanner:
     def tables(self, kv_lens, block_table):
         units, seq_units = kernels.plan_key_units(
             kv_lens, kernels.key_unit_count(len(kv_lens), self.num_kv_heads), tables=block_table,
-            window=self.window or None, keep_first=self.keep_first)
+            window=self.window or None, keep_first=self.keep_first, chunk=self.chunk or None)
         return {"units": units, "seq_units": seq_units}
 
 
@@ -251,7 +252,7 @@ register_part("attention_normed", NormedAttention)
 
 
 class SinkAttention(Part):
-    """Softmax attention with key and value widths of their own, capped scores, a window and one
+    """Softmax attention with key and value widths of their own, capped scores, a window or chunks and one
     more term in the softmax denominator (``SinkAttentionSpec``).
 
     One merged product gives [q | k | v | gate] (k and v only where the layer has keys and values of
@@ -277,6 +278,8 @@ class SinkAttention(Part):
             raise PartError(f"{s.rot_dims} rotated coordinates ({s.rot_style!r}) do not fit heads of {s.key_dim}")
         if s.window is not None and s.window < 1:
             raise PartError(f"attention window must be >= 1, got {s.window}")
+        if s.chunk is not None and (s.chunk < 1 or s.window is not None or s.cache_window is not None or not s.own_kv):
+            raise PartError(f"chunks of {s.chunk} keys go without a window and with keys of the layer's own")
         if s.cache_window is not None and (s.cache_window < 0 or
                                            (s.cache_window > 0 and (s.window is None or s.cache_window < s.window))):
             raise PartError(f"a cache kept for {s.cache_window} tokens does not serve a window of {s.window}")
@@ -339,7 +342,7 @@ class SinkAttention(Part):
 
     def step_planner(self):
         if self._on_matrix_cores() and kernels.keys_sink_fits(self.nq, self.nkv, self.dk):
-            return KeyUnitPlanner(self.nkv, self._cache_window() or 0, self.spec.keep_first)
+            return KeyUnitPlanner(self.nkv, self._cache_window() or 0, self.spec.keep_first, self.spec.chunk or 0)
         return None
 
     def bind(self, tensors):
@@ -358,7 +361,8 @@ class SinkAttention(Part):
 
     def cache_need(self):
         s = self.spec
-        kv = KVNeed(self.nkv, self.dk, self._cache_window(), self.dk if self._pads_values() else self.dv, s.keep_first)
+        kv = KVNeed(self.nkv, self.dk, self._cache_window(), self.dk if self._pads_values() else self.dv, s.keep_first,
+                    s.chunk)
         if s.conv_taps > 1:
             from ..cache.storage import StateNeed
             return [kv, StateNeed((s.conv_taps - 1, self.qkv_width), torch.float32)]
@@ -410,7 +414,7 @@ class SinkAttention(Part):
             o = ctx.ws.take("attention.o", (nt, self.nq * vd), self.dtype)
             kernels.attention_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_qlen, self.nq,
                                    self.nkv, self.dk, vd, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
-                                   keep_first=s.keep_first)
+                                   keep_first=s.keep_first, chunk=s.chunk)
             return finish(o, w, ctx.ws, "attention.delta", fold, into)
         # matrix cores: scores and sums in float32, the softmax weights kept at 32 bits by three pieces
         o = ctx.ws.take("attention.o", (nt, self.nq * self.dk), self.dtype)
@@ -421,11 +425,11 @@ class SinkAttention(Part):
         if ctx.all_single and plan:
             kernels.attention_keys_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_kv_len, self.nq,
                                         self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
-                                        keep_first=s.keep_first, units=plan.get("units"), seq_units=plan.get("seq_units"))
+                                        keep_first=s.keep_first, chunk=s.chunk, units=plan.get("units"), seq_units=plan.get("seq_units"))
         else:
             kernels.attention_rows_sink(qkv, o, kc, vc, meta.block_table, ctx.cu_q, ctx.pos0, ctx.max_qlen, self.nq,
                                         self.nkv, self.dk, float(s.scale), s.window, s.softcap, sink, gate, self.gate_dim,
-                                        keep_first=s.keep_first)
+                                        keep_first=s.keep_first, chunk=s.chunk)
         return finish(o, w, ctx.ws, "attention.delta", fold, into)
 
 

@@ -68,6 +68,22 @@ class EmbedScale(Part):
         return x
 
 
+class LearnedPositions(Part):
+    """x_t += table[position of t]."""
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        if spec.positions < 1:
+            raise PartError(f"a table of {spec.positions} positions")
+        self.spec = spec
+
+    def params(self):
+        return {"table": Param((self.spec.positions, self.spec.hidden), "matrix")}
+
+    def run(self, x, ctx):
+        return kernels.rows_add(self.w["table"], ctx.positions, x)
+
+
 class TokenSideTable(Part):
     """Gathers the step's rows of a second table indexed by token, as float32, into
     ``ctx.shared[TokenSideTable.KEY]`` [nt, width]; the blocks' token-side parts read their
@@ -112,5 +128,6 @@ class Chain(Part):
 
 
 register_part("embed_scale", EmbedScale)
+register_part("learned_positions", LearnedPositions)
 register_part("token_side_table", TokenSideTable)
 register_part("chain", Chain)

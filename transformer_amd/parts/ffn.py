@@ -140,7 +140,9 @@ class RoutedMLP(Part):
 
     def __init__(self, spec, dtype, device):
         s = spec
-        if not 1 <= s.top <= s.experts or s.intermediate < 1:
+        self.identity = int(getattr(s, "identity", 0))           # router outputs whose expert is the input itself
+        self.outputs = s.experts + self.identity                 # of the router
+        if s.experts < 1 or self.identity < 0 or not 1 <= s.top <= self.outputs or s.intermediate < 1:
             raise PartError(f"routed feed-forward: top {s.top} of {s.experts} experts of {s.intermediate}")
         form = getattr(s, "form", "mlp")
         if form not in ("mlp", "limited_glu", "glu"):
@@ -149,8 +151,8 @@ class RoutedMLP(Part):
         self.glu = form == "glu"                  # act(gate) * up, no limits
         self.two = self.limited or self.glu       # an expert's first matrix is [gate rows | up rows]
         self.groups, self.keep_groups = int(getattr(s, "groups", 1)), int(getattr(s, "keep_groups", 1))
-        if self.groups < 1 or s.experts % self.groups or not 1 <= self.keep_groups <= self.groups or \
-                s.top > self.keep_groups * (s.experts // self.groups):
+        if self.groups < 1 or self.outputs % self.groups or not 1 <= self.keep_groups <= self.groups or \
+                s.top > self.keep_groups * (self.outputs // self.groups):
             raise PartError(f"routed feed-forward: {s.experts} experts in {self.groups} groups of which "
                             f"{self.keep_groups} stay do not hold {s.top} choices")
         if self.glu:
@@ -167,16 +169,20 @@ class RoutedMLP(Part):
             raise PartError(f"routed feed-forward: score {s.score!r}, weight on {s.weight_on!r}")
         self.spec, self.dtype = s, dtype
         self.gated_shared = s.shared_intermediate is not None and s.shared_gate
+        if self.identity and s.weight_on == "input":
+            raise PartError("routed feed-forward: identity experts go with weights on the experts' results")
 
     def params(self):
         s = self.spec
         # limited_glu, glu: an expert's first matrix is [gate rows | up rows]
         first, k = ("gate_up", 2) if self.two else ("up", 1)
-        p = {"router.weight": Param((s.experts + int(self.gated_shared), s.hidden), "matrix"),
+        p = {"router.weight": Param((self.outputs + int(self.gated_shared), s.hidden), "matrix"),
              f"experts.{first}.weight": Param((s.experts * k * s.intermediate, s.hidden), "matrix"),
              "experts.down.weight": Param((s.experts * s.hidden, s.intermediate), "matrix")}
         if getattr(s, "router_bias", False):
-            p["router.bias"] = Param((s.experts,), "vector")
+            p["router.bias"] = Param((self.outputs,), "vector")
+        if getattr(s, "correction", False):
+            p["router.correction"] = Param((self.outputs,), "vector", init="zero")
         if s.shared_intermediate is not None:
             p[f"shared.{first}.weight"] = Param((k * s.shared_intermediate, s.hidden), "matrix")
             p["shared.down.weight"] = Param((s.hidden, s.shared_intermediate), "matrix")
@@ -205,11 +211,13 @@ class RoutedMLP(Part):
         s, nt, d = self.spec, h.shape[0], self.spec.hidden
         E, top, ff = s.experts, s.top, s.intermediate
         ws = ctx.ws
-        logits = linear(h, self.w["router.weight"], ws.take("moe.logits", (nt, E + int(self.gated_shared)), torch.float32))
+        R = self.outputs
+        logits = linear(h, self.w["router.weight"], ws.take("moe.logits", (nt, R + int(self.gated_shared)), torch.float32))
         chosen = ws.take("moe.chosen", (nt, top), torch.int32)
         weight = ws.take("moe.weight", (nt, top), torch.float32)
-        kernels.moe_route(logits, E, top, chosen, weight, s.score, s.renormalize, bias=self.w.get("router.bias"),
-                          groups=self.groups, keep_groups=self.keep_groups)
+        kernels.moe_route(logits, R, top, chosen, weight, s.score, s.renormalize, bias=self.w.get("router.bias"),
+                          groups=self.groups, keep_groups=self.keep_groups, correction=self.w.get("router.correction"),
+                          factor=float(getattr(s, "factor", 1.0)))
         if getattr(ctx, "dump", None) is not None:
             ctx.dump("experts", chosen)
         rows = kernels.moe_max_rows(nt * top, E)
@@ -232,8 +240,9 @@ class RoutedMLP(Part):
                             getattr(s, "shared_limit", 0.0))
             shared = linear_delta(u, self.w["shared.down.weight"], ws, "moe.shared")
         delta = kernels.moe_combine(out, top, pair_row, None if on_input else weight, shared,
-                                    logits[:, E:] if self.gated_shared else None,
-                                    ws.take("moe.delta", (nt, d), torch.float32), extra=extra)
+                                    logits[:, R:] if self.gated_shared else None,
+                                    ws.take("moe.delta", (nt, d), torch.float32), extra=extra,
+                                    own=h if self.identity else None)
         return delta, None
 
 

@@ -302,43 +302,56 @@ class StateSpace(Part):
 
 
 class GatedDelta(Part):
-    """The gated delta rule with a decay per head and key channel (``GatedDeltaSpec``).
+    """The gated delta rule with a decay per head and key channel, or per head (``GatedDeltaSpec``).
 
-    One product gives [q | k | v | decay input | gate input | step sizes]; ``kernels.causal_conv`` runs the
+    One product gives [q | k | v | decay input | gate input | step sizes], or [q | k | v | gate | decays | step
+    sizes] where the gate is no low-rank product; ``kernels.causal_conv`` runs the
     convolution with silu over [q | k | v] (its memory is the second piece of state). A step of single
     tokens then takes ONE kernel to the normed and gated readout (``kernels.delta_step``); longer steps
-    form the two low-rank products, ``kernels.delta_prepare`` makes unit vectors, decays and step sizes of
+    form the low-rank products, ``kernels.delta_prepare`` makes unit vectors, decays and step sizes of
     all tokens, ``kernels.delta_recurrent`` walks them, and the head norm with its gate follows. State,
     decays, step sizes, unit vectors and readout stay float32."""
     graph_safe = True
 
     def __init__(self, spec, dtype, device):
         s = spec
-        if min(s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim, s.taps, s.decay_rank, s.gate_rank) < 1 \
-                or s.num_heads % s.num_kv_heads:
+        ranks = [r for r in (s.decay_rank, s.gate_rank) if r is not None]
+        if min(s.num_heads, s.num_kv_heads, s.key_dim, s.value_dim, s.taps, *ranks) < 1 or s.num_heads % s.num_kv_heads:
             raise PartError(f"delta rule: {s.num_heads} heads of {s.key_dim} / {s.value_dim} in {s.num_kv_heads} groups, "
                             f"{s.taps} taps, ranks {s.decay_rank} / {s.gate_rank}")
         if s.key_dim > kernels.DELTA_MAX_KEY_DIM:
             raise PartError(f"delta rule: key widths up to {kernels.DELTA_MAX_KEY_DIM}, not {s.key_dim}")
+        if s.gate_activation not in ("silu", "sigmoid"):
+            raise PartError(f"delta rule: unknown gate activation {s.gate_activation!r}")
         self.spec, self.dtype = s, dtype
         self.nk, self.nv = s.num_kv_heads * s.key_dim, s.num_heads * s.value_dim
         self.conv_width = 2 * self.nk + self.nv
-        self.a_off = self.conv_width
-        self.g_off = self.a_off + s.decay_rank
-        self.b_off = self.g_off + s.gate_rank
+        # columns of the decay's and the gate's inputs: a full gate comes first, so that it starts where v ends
+        self.a_width = s.num_heads if s.decay_rank is None else s.decay_rank
+        self.g_width = self.nv if s.gate_rank is None else s.gate_rank
+        if s.gate_rank is None:
+            self.g_off = self.conv_width
+            self.a_off = self.g_off + self.g_width
+        else:
+            self.a_off = self.conv_width
+            self.g_off = self.a_off + self.a_width
+        self.b_off = self.conv_width + self.a_width + self.g_width
         self.width = self.b_off + s.num_heads
 
     def params(self):
         s = self.spec
         H = s.num_heads
-        return {"in.weight": Param((self.width, s.hidden), "matrix"),     # q, k, v, decay input, gate input, step sizes
-                "conv.weight": Param((self.conv_width, s.taps), "vector"),
-                "decay.weight": Param((H * s.key_dim, s.decay_rank), "matrix"),
-                "gate.weight": Param((self.nv, s.gate_rank), "matrix"),
-                "dt_bias": Param((H * s.key_dim,), "vector", init="zero"),
-                "A_log": Param((H,), "vector", init="zero"),
-                "norm.weight": Param((s.value_dim,), "vector", init="around_one"),
-                "out.weight": Param((s.hidden, self.nv), "matrix")}
+        p = {"in.weight": Param((self.width, s.hidden), "matrix"),     # q, k, v, decay and gate inputs, step sizes
+             "conv.weight": Param((self.conv_width, s.taps), "vector"),
+             "dt_bias": Param((H if s.decay_rank is None else H * s.key_dim,), "vector", init="zero"),
+             "A_log": Param((H,), "vector", init="zero"),
+             "norm.weight": Param((s.value_dim,), "vector", init="around_one"),
+             "out.weight": Param((s.hidden, self.nv), "matrix")}
+        if s.decay_rank is not None:
+            p["decay.weight"] = Param((H * s.key_dim, s.decay_rank), "matrix")
+        if s.gate_rank is not None:
+            p["gate.weight"] = Param((self.nv, s.gate_rank), "matrix")
+        return p
 
     def cache_need(self):
         s = self.spec
@@ -376,23 +389,95 @@ class GatedDelta(Part):
                             activation="silu")
         y = take("delta.y", (nt, self.nv), self.dtype)
         q_scale = float(dk) ** -0.5
-        if ctx.all_single and kernels.delta_step_fits(dk, dv, s.decay_rank, s.gate_rank):
-            kernels.delta_step(qkv, proj, self.a_off, self.g_off, self.b_off, self.w["decay.weight"], self.w["gate.weight"],
-                               self.w["dt_bias"], self.w["A_log"], state, ctx.slots, H, G, q_scale, self.w["norm.weight"],
-                               float(s.eps), y)
+        if ctx.all_single and kernels.delta_step_fits(dk, dv, s.decay_rank or 0, s.gate_rank or 0):
+            kernels.delta_step(qkv, proj, self.a_off, self.g_off, self.b_off, self.w.get("decay.weight"),
+                               self.w.get("gate.weight"), self.w["dt_bias"], self.w["A_log"], state, ctx.slots, H, G,
+                               q_scale, self.w["norm.weight"], float(s.eps), y, s.gate_activation)
             return finish(y, self.w["out.weight"], ctx.ws, "delta.delta", fold, into)
-        z = self._low_rank(proj[:, self.a_off:self.g_off], self.w["decay.weight"], take("delta.z", (nt, H * dk), f32))
-        gate = self._low_rank(proj[:, self.g_off:self.b_off], self.w["gate.weight"], take("delta.gate", (nt, self.nv), self.dtype))
+        z, gate = proj[:, self.a_off:self.a_off + self.a_width], proj[:, self.g_off:self.g_off + self.g_width]
+        if s.decay_rank is not None:
+            z = self._low_rank(z, self.w["decay.weight"], take("delta.z", (nt, H * dk), f32))
+        if s.gate_rank is not None:
+            gate = self._low_rank(gate, self.w["gate.weight"], take("delta.gate", (nt, self.nv), self.dtype))
         qn, kn = take("delta.qn", (nt, G, dk), f32), take("delta.kn", (nt, G, dk), f32)
-        decay, beta, kq = take("delta.decay", (nt, H, dk), f32), take("delta.beta", (nt, H), f32), take("delta.kq", (nt, G), f32)
+        decay = take("delta.decay", (nt, H) if s.decay_rank is None else (nt, H, dk), f32)
+        beta, kq = take("delta.beta", (nt, H), f32), take("delta.kq", (nt, G), f32)
         kernels.delta_prepare(qkv, z, self.w["dt_bias"], self.w["A_log"], proj[:, self.b_off:self.width], G, H, dk, q_scale,
                               qn, kn, decay, beta, kq)
         o = kernels.delta_recurrent(qn, kn, decay, qkv[:, 2 * self.nk:], beta, kq, state, ctx.cu_q, ctx.slots,
                                     take("delta.o", (nt, H, dv), f32))
-        kernels.head_norm_gate(o.unsqueeze(0), gate, H, dv, self.w["norm.weight"], float(s.eps), y, "sigmoid")
+        kernels.head_norm_gate(o.unsqueeze(0), gate, H, dv, self.w["norm.weight"], float(s.eps), y,
+                               s.gate_activation)
         return finish(y, self.w["out.weight"], ctx.ws, "delta.delta", fold, into)
 
 
+class MatrixMemory(Part):
+    """The matrix memory with exponential gates, a running maximum and a normaliser (``MatrixMemorySpec``).
+
+    One product gives [q | k | v | output gate | input gates | forget gates]. A step of single tokens then takes
+    ONE kernel to the normed and gated readout (``kernels.memory_step``). Longer steps, and heads too large for
+    it: ``kernels.memory_gates`` forms the weights of all tokens by a scan over the running maximum,
+    ``kernels.memory_recurrent`` walks the tokens with the normaliser as one more value column, and the head norm
+    divides by the denominator first. State, normaliser, maximum, gates and readout stay float32."""
+    graph_safe = True
+
+    def __init__(self, spec, dtype, device):
+        s = spec
+        if min(s.num_heads, s.key_dim, s.value_dim) < 1 or not s.gate_cap > 0:
+            raise PartError(f"matrix memory: {s.num_heads} heads of {s.key_dim} / {s.value_dim}, gates capped at {s.gate_cap}")
+        self.spec, self.dtype = s, dtype
+        self.nk, self.nv = s.num_heads * s.key_dim, s.num_heads * s.value_dim
+        i_off = 2 * self.nk + 2 * self.nv
+        self.offsets = (0, self.nk, 2 * self.nk, 2 * self.nk + self.nv, i_off, i_off + s.num_heads)   # q, k, v, g, i, f
+        self.width = i_off + 2 * s.num_heads
+
+    def params(self):
+        s = self.spec
+        return {"in.weight": Param((self.width, s.hidden), "matrix"),     # q, k, v, output gate, input and forget gates
+                "i.bias": Param((s.num_heads,), "vector"),
+                "f.bias": Param((s.num_heads,), "vector"),
+                "norm.weight": Param((self.nv,), "vector", init="around_one"),
+                "out.weight": Param((s.hidden, self.nv), "matrix")}
+
+    def cache_need(self):
+        s = self.spec
+        H, f32 = s.num_heads, torch.float32
+        return [StateNeed((H, s.key_dim, s.value_dim), f32), StateNeed((H, s.key_dim), f32), StateNeed((H,), f32)]
+
+    # as in ``GatedDelta``
+    def can_add(self, nt: int) -> bool:
+        return adds_in_place(nt, self.w["out.weight"])
+
+    def takes_scaled(self, nt: int) -> bool:
+        return kernels.skinny_takes(nt, self.w["in.weight"])
+
+    def can_fold(self, nt: int) -> bool:
+        return kernels.skinny_folds(nt, self.w["out.weight"])
+
+    def run(self, h, ctx, cache, layer, writes_cache=True, scale=None, fold=None, into=None):
+        s, nt = self.spec, h.shape[0]
+        H, dk, dv = s.num_heads, s.key_dim, s.value_dim
+        take, f32 = ctx.ws.take, torch.float32
+        state, n_state, m_state = (cache.layer_state(l) for l in layer)
+        proj = linear(h, self.w["in.weight"], aligned_rows(ctx.ws, "memory.in", nt, self.width, self.dtype), scale=scale)
+        y = take("memory.y", (nt, self.nv), self.dtype)
+        q_off, k_off, v_off, g_off, i_off, f_off = self.offsets
+        q_scale, biases = float(dk) ** -0.5, (self.w["i.bias"], self.w["f.bias"])
+        if ctx.all_single and kernels.memory_step_fits(dk, dv):
+            kernels.memory_step(proj, self.offsets, *biases, float(s.gate_cap), state, n_state, m_state, ctx.slots, q_scale,
+                                self.w["norm.weight"], float(s.eps), y)
+            return finish(y, self.w["out.weight"], ctx.ws, "memory.delta", fold, into)
+        keep, write, floor = (take(f"memory.{n}", (nt, H), f32) for n in ("keep", "write", "floor"))
+        kernels.memory_gates(proj, i_off, f_off, *biases, float(s.gate_cap), m_state, ctx.cu_q, ctx.slots, keep, write, floor)
+        parts = kernels.gla_row_parts(dk)
+        o, den = take("memory.o", (parts, nt, H, dv), f32), take("memory.den", (parts, nt, H), f32)
+        kernels.memory_recurrent(proj, q_off, k_off, v_off, q_scale, keep, write, state, n_state, ctx.cu_q, ctx.slots, o, den)
+        kernels.head_norm_gate(o, proj[:, g_off:g_off + self.nv], H, dv, self.w["norm.weight"], float(s.eps), y, "sigmoid",
+                               den=den, floor=floor)
+        return finish(y, self.w["out.weight"], ctx.ws, "memory.delta", fold, into)
+
+
+register_part("matrix_memory", MatrixMemory)
 register_part("gated_delta", GatedDelta)
 register_part("state_space", StateSpace)
 register_part("diagonal_recurrence", DiagonalRecurrence)
