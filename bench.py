@@ -348,6 +348,43 @@ def zirutar_shapes():
             "w4096": shape(4096, 32, 8, 1536, 512, 1024, 128, 128, 14336, 32000)}
 
 
+def linonex_shapes():
+    """Layer sizes that resemble real models' (random weights): Linonex models whose layers are all
+    matrix memory or all parallel (chunked attention beside a delta rule), each with the dense and with the
+    routed feed-forward, the mixed order, and the closest layers of the other decoders at the same width and
+    heads: the Vametar decoder's gated linear attention (the matrix memory's heads), the Zirutar decoder's
+    delta rule, the Saredra decoder's parallel layer with routed experts of the same sizes, and the Llama
+    layer."""
+    def shape(width, heads, kv, mem, mem_dim, chunk, experts, top, eff, ff, vocab):
+        dense = {"kind": "dense", "ff": ff}
+        moe = {"kind": "moe", "expert": {"ff": eff}, "router": {"experts": experts, "identity": experts // 8, "scale": 2.0, "top": top}}
+        memory = {"heads": mem, "dim": mem_dim, "vdim": 2 * mem_dim, "gate_cap": 15.0}
+        sides = {"left": {"heads": heads, "kv_heads": kv, "dim": 128, "vdim": 128, "conv": 4, "scale": 128 ** -0.5,
+                          "softcap": 30.0, "mask": {"size": chunk}},
+                 "right": {"heads": heads, "kv_heads": heads, "dim": 128, "vdim": 128, "conv": 4}}
+        lay = lambda kind, mlp: {"type": kind, "mlp": mlp, "mixer": memory if kind == "mlstm" else sides}
+        base = {"architecture": "Linonex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "max_positions": 1 << 16}
+        kinds = {"mlstm": [lay("mlstm", dense)] * 4, "parallel": [lay("parallel", dense)] * 4,
+                 "mlstm_moe": [lay("mlstm", moe)] * 4, "parallel_moe": [lay("parallel", moe)] * 4,
+                 "mixed": [lay("mlstm", dense), lay("parallel", moe), lay("parallel", dense), lay("mlstm", moe)]}
+        sar = saredra_shapes()[f"w{width}"]
+        smoe = {"kind": "moe", "router": {"experts": experts, "top": top}, "expert": {"ff": eff}}
+        spar = {**sar[1]["parallel"][0], "mlp": smoe}
+        zi = zirutar_shapes()[f"w{width}"]
+        zdelta = {**zi[1]["delta"][0], "mlp": {**dense, "limit": 7.0}}
+        vam = zi[2]["vametar_gla"][1]
+        near = {
+            "vametar_gla": ("Vametar", {**vam, "layers": [{"type": "gla", "mlp": dense, "mixer": {
+                "heads": mem, "dim": mem_dim, "vdim": 2 * mem_dim, "tau": 16.0, "rank": 16}}] * 4}),
+            "zirutar_delta": ("Zirutar", {**zi[0], "layers": [zdelta] * 4}),
+            "saredra_parallel": ("Saredra", {**sar[0], "layers": [spar] * 4}),
+            "llama": zi[2]["llama"],
+        }
+        return base, kinds, near
+    return {"w2048": shape(2048, 16, 4, 8, 128, 1024, 32, 4, 1024, 8192, 32000),
+            "w4096": shape(4096, 32, 8, 8, 256, 1024, 64, 6, 1408, 14336, 32000)}
+
+
 def _routed_parts(model):
     return [b.ffn for b in model.blocks if getattr(getattr(b, "ffn", None), "spec", None) is not None
             and getattr(b.ffn.spec, "kind", "") == "routed_mlp"]
@@ -390,9 +427,9 @@ def generic_step_bytes(model, contexts):
         sp = f.spec
         w -= max(0, sp.experts - len(contexts) * sp.top) * _expert_entries(sp) * item
     windowed = 0
-    for need in model.cache_needs:       # a window bounds what a layer reads of a sequence
-        if isinstance(need, KVNeed) and need.window is not None:
-            windowed += sum(max(0, c - need.window - need.keep_first) for c in contexts) * need.num_kv_heads * \
+    for need in model.cache_needs:       # a window (or chunk) bounds what a layer reads of a sequence
+        if isinstance(need, KVNeed) and need.span is not None:
+            windowed += sum(max(0, need.first_key(c) - need.keep_first) for c in contexts) * need.num_kv_heads * \
                 (need.head_dim + need.value_dim) * item
     return w + sum(contexts) * per_token - windowed + len(contexts) * per_seq
 
@@ -411,9 +448,13 @@ def generic_prefill_flops(model, T):
     fl = 2 * T * mats + 2 * model.spec.hidden * model.spec.vocab
     for m in (x for blk in model.blocks for x in _leaf_mixers(blk.mixer)):
         need = m.cache_need()
+        need = need[0] if isinstance(need, (list, tuple)) and need else need
         if isinstance(need, KVNeed):
             window = getattr(m.spec, "window", None)
             pairs = T * (T + 1) // 2 if window is None or window >= T else window * (window + 1) // 2 + (T - window) * window
+            chunk = getattr(m.spec, "chunk", None)
+            if chunk is not None:
+                pairs = T // chunk * (chunk * (chunk + 1) // 2) + (T % chunk) * (T % chunk + 1) // 2
             if hasattr(m, "nq"):
                 fl += 2 * m.nq * (need.head_dim + need.value_dim) * pairs
             else:                        # one latent row per token: scores over its whole width, sums over the latent
@@ -600,11 +641,11 @@ def main():
                     help="tokens of the prompt whose step is timed (the line's \"prefill\")")
     ap.add_argument("--prefill-only", action="store_true",
                     help="run only the 2,048-token prefill (for profiling); prints its own line")
-    ap.add_argument("--design", default=None, choices=["vametar", "kunitar", "luduvik", "saredra", "zirutar"],
+    ap.add_argument("--design", default=None, choices=["vametar", "kunitar", "luduvik", "saredra", "zirutar", "linonex"],
                     help="instead of the default workload: prefill and decode of this design at a few "
                          "layer sizes, beside the Llama decoder at the same sizes (a line of its own)")
     ap.add_argument("--design-size", default=None, help="with --design: only these sizes (w2048,w4096)")
-    ap.add_argument("--design-case", default=None, help="with --design kunitar, luduvik, saredra or zirutar: only these rows (llama,latent,...)")
+    ap.add_argument("--design-case", default=None, help="with --design kunitar, luduvik, saredra, zirutar or linonex: only these rows (llama,latent,...)")
     a = ap.parse_args()
     if a.design == "kunitar" and a.gpus == 1:
         return bench_kunitar(a)
@@ -614,6 +655,8 @@ def main():
         return bench_beside(a, "saredra", "Saredra", saredra_shapes())
     if a.design == "zirutar" and a.gpus == 1:
         return bench_beside(a, "zirutar", "Zirutar", zirutar_shapes())
+    if a.design == "linonex" and a.gpus == 1:
+        return bench_beside(a, "linonex", "Linonex", linonex_shapes())
     if a.design and a.gpus == 1:
         return bench_design(a)
     if a.gpus != 1:

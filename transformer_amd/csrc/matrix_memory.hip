@@ -6,8 +6,8 @@
 //     S_t = keep_t S_(t-1) + write_t k_t v_t^T,  n_t = keep_t n_(t-1) + write_t k_t
 //     o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6)
 //
-//   memory_gates : keep, write and exp(-m) of every token and head; the running maximum of 64 tokens at
-//                  once by a scan over a wave
+//   memory_gates : keep, write and exp(-m) of every token and head; the running maximum by a scan over
+//                  the waves of a workgroup
 //   memory_step  : a step of single tokens in one kernel: gates, the state's update, the readout with its
 //                  denominator, the head's norm and the output gate
 //
@@ -24,14 +24,17 @@ __device__ __forceinline__ float mm_cap(float z, float cap) { return cap * tanhf
 __device__ __forceinline__ float mm_log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
 
 // ------------------------------------------------------------------ gates of a step
-// One wave per (head, sequence). Elements of the scan are (sum of f, best of i_j + f_(j+1) + .. + f_t); two
-// neighbours join to (F1 + F2, max(M1 + F2, M2)), and m_t = max(F + m before the turn, M).
-template <typename T>
-__global__ __launch_bounds__(64) void memory_gates_kernel(
+// One workgroup of WAVES waves per (head, sequence), a token a thread. Elements of the scan are (sum of f, best
+// of i_j + f_(j+1) + .. + f_t); two neighbours join to (F1 + F2, max(M1 + F2, M2)), and m_t = max(F + m before
+// the turn, M). A wave scans its 64 tokens; the waves' totals are joined in order by every wave for itself.
+template <typename T, int WAVES>
+__global__ __launch_bounds__(WAVES * TA_WAVE) void memory_gates_kernel(
     const T* __restrict__ proj, int stride, int ioff, int foff, const float* __restrict__ ibias,
     const float* __restrict__ fbias, float cap, float* __restrict__ m_state, const int* __restrict__ cu_q,
     const int* __restrict__ slots, int H, float* __restrict__ keep, float* __restrict__ write, float* __restrict__ floor_) {
-  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x;
+  constexpr int NT = WAVES * TA_WAVE;
+  __shared__ float2 total[2][WAVES];                // a turn's waves: sum of f, best
+  const int h = blockIdx.x, b = blockIdx.y, lane = threadIdx.x % TA_WAVE, wave = threadIdx.x / TA_WAVE;
   const int start = cu_q[b], end = cu_q[b + 1];
   if (start >= end) return;
   float* ms = m_state + (size_t)slots[b] * H + h;
@@ -39,15 +42,16 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(
   const float bi = ibias[h], bf = fbias[h];
   // the next turn's inputs are on their way while this turn is worked on
   auto at = [&](int t) { return (size_t)(t < end ? t : end - 1) * stride; };
-  T ri = proj[at(start + lane) + ioff + h], rf = proj[at(start + lane) + foff + h];
-  for (int t0 = start; t0 < end; t0 += TA_WAVE) {
-    const int t = t0 + lane;
+  T ri = proj[at(start + threadIdx.x) + ioff + h], rf = proj[at(start + threadIdx.x) + foff + h];
+  int buf = 0;
+  for (int t0 = start; t0 < end; t0 += NT, buf ^= 1) {
+    const int t = t0 + threadIdx.x;
     const bool on = t < end;
     const float i = on ? mm_cap(to_f32(ri) + bi, cap) : -INFINITY;
     const float f = on ? mm_log_sigmoid(mm_cap(to_f32(rf) + bf, cap)) : 0.f;
-    if (t0 + TA_WAVE < end) {
-      ri = proj[at(t + TA_WAVE) + ioff + h];
-      rf = proj[at(t + TA_WAVE) + foff + h];
+    if (t0 + NT < end) {
+      ri = proj[at(t + NT) + ioff + h];
+      rf = proj[at(t + NT) + foff + h];
     }
     float F = f, M = i;
 #pragma unroll
@@ -58,36 +62,53 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(
         F += Fp;
       }
     }
-    const float m = fmaxf(F + m0, M);
+    float mine = m0;                                // the maximum in front of this wave's tokens
+    if (WAVES > 1) {
+      if (lane == TA_WAVE - 1) total[buf][wave] = float2{F, M};
+      __syncthreads();                              // (a buffer's readers are behind the next turn's barrier)
+      float run = m0;
+#pragma unroll
+      for (int w = 0; w < WAVES; ++w) {
+        if (w == wave) mine = run;
+        const float2 e = total[buf][w];
+        run = fmaxf(e.x + run, e.y);
+      }
+      m0 = run;
+    }
+    const float m = fmaxf(F + mine, M);
     const float up = __shfl_up(m, 1, TA_WAVE);
-    const float before = lane == 0 ? m0 : up;
+    const float before = lane == 0 ? mine : up;
     if (on) {
       const size_t e = (size_t)t * H + h;
       keep[e] = expf(f - (m - before));
       write[e] = expf(i - m);
       floor_[e] = expf(-m);
     }
-    m0 = __shfl(m, TA_WAVE - 1, TA_WAVE);       // (lanes past the end carry the last token's)
+    if (WAVES == 1) m0 = __shfl(m, TA_WAVE - 1, TA_WAVE);       // (lanes past the end carry the last token's)
   }
-  if (lane == 0) *ms = m0;
+  if (threadIdx.x == 0) *ms = m0;
 }
 
 // proj: [nt] rows, stride apart, with the input gates' numbers (H) at column ioff and the forget gates' at
-// foff; ibias, fbias [H]; m_state [slots, H] float32, moved on; keep, write, floor_ [nt, H] float32.
+// foff; ibias, fbias [H]; m_state [slots, H] float32, moved on; keep, write, floor_ [nt, H] float32. max_qlen: the
+// most tokens a sequence brings (chooses the launch alone).
 extern "C" int ta_memory_gates(hipStream_t stream, int dtype, const void* proj, int stride, int ioff, int foff,
                                const float* ibias, const float* fbias, float cap, float* m_state, const int* cu_q,
-                               const int* slots, int batch, int nt, int H, float* keep, float* write, float* floor_) {
+                               const int* slots, int batch, int nt, int max_qlen, int H, float* keep, float* write, float* floor_) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch && H >= 1, "ta_memory_gates: batch %d, %d tokens, %d heads", batch, nt, H);
   TA_REQUIRE(ioff >= 0 && foff >= 0 && stride >= ioff + H && stride >= foff + H, "ta_memory_gates: rows of %d are too short", stride);
   TA_REQUIRE(cap > 0.f, "ta_memory_gates: the cap must be positive, got %g", (double)cap);
   dim3 g(H, batch);
-  if (dtype == TA_F32)
-    memory_gates_kernel<float><<<g, 64, 0, stream>>>((const float*)proj, stride, ioff, foff, ibias, fbias, cap, m_state,
-                                                     cu_q, slots, H, keep, write, floor_);
-  else if (dtype == TA_BF16)
-    memory_gates_kernel<bf16_t><<<g, 64, 0, stream>>>((const bf16_t*)proj, stride, ioff, foff, ibias, fbias, cap, m_state,
-                                                      cu_q, slots, H, keep, write, floor_);
+#define MG_RUN(T, W)                                                                                               \
+  memory_gates_kernel<T, W><<<g, W * TA_WAVE, 0, stream>>>((const T*)proj, stride, ioff, foff, ibias, fbias, cap, \
+                                                           m_state, cu_q, slots, H, keep, write, floor_)
+#define MG_BY_LEN(T) \
+  if (max_qlen <= TA_WAVE) MG_RUN(T, 1); else if (max_qlen <= 4 * TA_WAVE) MG_RUN(T, 4); else MG_RUN(T, 16)
+  if (dtype == TA_F32) { MG_BY_LEN(float); }
+  else if (dtype == TA_BF16) { MG_BY_LEN(bf16_t); }
   else return ta_fail("ta_memory_gates: unknown dtype %d", dtype);
+#undef MG_BY_LEN
+#undef MG_RUN
   return ta_check_launch("ta_memory_gates");
 }
 

@@ -2246,7 +2246,7 @@ def _memory_columns(what, proj, offs, H, dk, dv):
 
 
 def memory_gates(proj: torch.Tensor, i_off: int, f_off: int, i_bias, f_bias, cap: float, m_state: torch.Tensor, cu_q,
-                 slots, keep: torch.Tensor, write: torch.Tensor, floor: torch.Tensor) -> None:
+                 slots, max_qlen: int, keep: torch.Tensor, write: torch.Tensor, floor: torch.Tensor) -> None:
     """The gates of the matrix memory, float32 [nt, H] each: with i = cap tanh((proj[i_off + h] + i_bias) / cap), f =
     log sigmoid(cap tanh((proj[f_off + h] + f_bias) / cap)) and the running maximum m <- max(f + m, i) of every
     sequence (``m_state`` [slots, H], moved on): keep = exp(f + m_before - m), write = exp(i - m), floor = exp(-m)."""
@@ -2264,8 +2264,8 @@ def memory_gates(proj: torch.Tensor, i_off: int, f_off: int, i_bias, f_bias, cap
         raise KernelError(f"memory_gates: columns {i_off} / {f_off} of rows of {proj.shape[1]} for {H} heads")
     _check(library().ta_memory_gates(
         _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), c_int(i_off), c_int(f_off), _ptr(i_bias),
-        _ptr(f_bias), c_float(cap), _ptr(m_state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(H), _ptr(keep),
-        _ptr(write), _ptr(floor)))
+        _ptr(f_bias), c_float(cap), _ptr(m_state), _ptr(cu_q), _ptr(slots), c_int(batch), c_int(nt), c_int(int(max_qlen)),
+        c_int(H), _ptr(keep), _ptr(write), _ptr(floor)))
 
 
 def memory_recurrent(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_scale: float, keep: torch.Tensor,

@@ -271,7 +271,8 @@ class SinkAttention(Part):
         s = spec
         if s.num_heads % s.num_kv_heads:
             raise PartError(f"{s.num_heads} heads do not divide into {s.num_kv_heads} kv heads")
-        odd_ok = s.unit_norm or s.values_from_keys
+        # (the kernel that adds biases and turns works on pairs of coordinates)
+        odd_ok = s.unit_norm or s.values_from_keys or (not s.rot_dims and (not s.qkv_bias or s.conv_taps > 0))
         if not (1 <= s.key_dim <= 256 and (odd_ok or s.key_dim % 2 == 0) and 1 <= s.value_dim <= 256):
             raise PartError(f"attention takes even key widths and value widths in [1, 256], not {s.key_dim} / {s.value_dim}")
         if s.rot_dims % 2 or not 0 <= s.rot_dims <= s.key_dim or s.rot_style not in ("half", "interleaved"):

@@ -468,7 +468,8 @@ class MatrixMemory(Part):
                                 self.w["norm.weight"], float(s.eps), y)
             return finish(y, self.w["out.weight"], ctx.ws, "memory.delta", fold, into)
         keep, write, floor = (take(f"memory.{n}", (nt, H), f32) for n in ("keep", "write", "floor"))
-        kernels.memory_gates(proj, i_off, f_off, *biases, float(s.gate_cap), m_state, ctx.cu_q, ctx.slots, keep, write, floor)
+        kernels.memory_gates(proj, i_off, f_off, *biases, float(s.gate_cap), m_state, ctx.cu_q, ctx.slots,
+                             ctx.max_qlen, keep, write, floor)
         parts = kernels.gla_row_parts(dk)
         o, den = take("memory.o", (parts, nt, H, dv), f32), take("memory.den", (parts, nt, H), f32)
         kernels.memory_recurrent(proj, q_off, k_off, v_off, q_scale, keep, write, state, n_state, ctx.cu_q, ctx.slots, o, den)
