@@ -145,8 +145,8 @@ EDGES = [(0, None), (63, None), (298, None), (200, 100), (199, 100), (256, 64), 
          (150, 150), (149, 150), (0, 300), (297, 27), (296, 27), (280, 70), (279, 70)]
 
 
-@pytest.mark.parametrize("kernel", ["vector32", "vector16", "matrix", "matrix_lds"])
-@pytest.mark.parametrize("where", ["prompt", "decode", "planned"])
+@pytest.mark.parametrize("where,kernel", [(w, k) for k in ("vector32", "vector16", "matrix") for w in ("prompt", "decode")] +
+                         [("prompt", "matrix_lds"), ("planned", "matrix")])
 @pytest.mark.parametrize("mark,chunk", EDGES)
 def test_one_key_stands_out(where, kernel, mark, chunk):
     """The last query points at ONE earlier key (the first, the last and the first of a page, the first of its
@@ -155,8 +155,6 @@ def test_one_key_stands_out(where, kernel, mark, chunk):
     from transformer_amd import kernels as K
     from transformer_amd.kernels import PAGE
     dtype = "float32" if kernel == "vector32" else "bfloat16"
-    if where == "planned" and kernel != "matrix" or where == "decode" and kernel == "matrix_lds":
-        pytest.skip("one kernel serves single tokens")
     H, G, dh, T = 4, 2, 32, 300
     rng = np.random.default_rng(mark)
     q, k = 0.05 * rng.standard_normal((T, H * dh)), 0.3 * rng.standard_normal((T, G * dh))
@@ -305,6 +303,43 @@ def test_memory_gates_alone(lens):
             m = new
         np.testing.assert_allclose(_np(state[slots[b]]), m, atol=3e-5)
     assert float(state[4].min()) == 7.0
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("lanes", [0, 16, 32])
+@pytest.mark.parametrize("geom", [(3, 32, 16), (2, 128, 40), (2, 47, 5), (2, 192, 33), (1, 256, 70), (8, 64, 64), (1, 300, 9), (1, 1000, 6), (2, 3, 15)])
+def test_matrix_memory_recurrence_alone(geom, lanes, dtype):
+    """The recurrence's kernel on weights of its own (keep down to 0 and up to 1), rows whose heads do and do not
+    start on whole pieces, sequences that end inside, at and behind the edge of a chunk of tokens."""
+    from transformer_amd import kernels as K
+    H, dk, dv = geom
+    rng = np.random.default_rng(dk)
+    lens = [1, 16, 17, 50, 3]
+    nt, n = sum(lens), 2 * H * dk + H * dv
+    rows = _bf(rng.standard_normal((nt, n + 5)), dtype)
+    keep, write = rng.uniform(0.5, 1.0, (nt, H)), rng.uniform(0, 1, (nt, H))
+    keep[::3], keep[::5], write[::4] = 1.0, 0.0, 0.0
+    S0, n0 = rng.standard_normal((len(lens), H, dk, dv)), rng.standard_normal((len(lens), H, dk))
+    state, norm = torch.zeros((7, H, dk, dv), device=DEV), torch.zeros((7, H, dk), device=DEV)
+    slots = [4, 0, 5, 2, 6]
+    for s, a, c in zip(slots, S0, n0):
+        state[s], norm[s] = _t(a), _t(c)
+    cu = np.concatenate([[0], np.cumsum(lens)])
+    o, den = torch.full((nt, H, dv), float("nan"), device=DEV), torch.full((nt, H), float("nan"), device=DEV)
+    off, scale = (1 if H == 2 else 4), dk ** -0.5
+    K.memory_recurrent(_t(rows, TD[dtype]), off, off + H * dk, off + 2 * H * dk, scale, _t(keep), _t(write), state, norm,
+                       _t(cu, torch.int32), _t(slots, torch.int32), o, den, lanes=lanes)
+    q, k, v = (rows[:, a:b].reshape(nt, H, -1) for a, b in ((off, off + H * dk), (off + H * dk, off + 2 * H * dk), (off + 2 * H * dk, off + n)))
+    for i in range(len(lens)):
+        S, nn = S0[i], n0[i]
+        for t in range(cu[i], cu[i + 1]):
+            S = keep[t][:, None, None] * S + write[t][:, None, None] * k[t][:, :, None] * v[t][:, None, :]
+            nn = keep[t][:, None] * nn + write[t][:, None] * k[t]
+            np.testing.assert_allclose(_np(o[t]), scale * np.einsum("hkv,hk->hv", S, q[t]), atol=1e-3)
+            np.testing.assert_allclose(_np(den[t]), scale * (nn * q[t]).sum(-1), atol=1e-3)
+        np.testing.assert_allclose(_np(state[slots[i]]), S, atol=1e-3)
+        np.testing.assert_allclose(_np(norm[slots[i]]), nn, atol=1e-3)
+    assert float(state[[1, 3]].abs().max()) == 0.0 and float(norm[[1, 3]].abs().max()) == 0.0
 
 
 @pytest.mark.parametrize("where", ["prompt", "decode"])

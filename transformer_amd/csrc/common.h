@@ -77,6 +77,40 @@ __device__ __forceinline__ float wave_max(float v) {
   return v;
 }
 
+// Sums over 16, 32 or 64 neighbouring lanes that leave the same bits in each of them.
+template <int CTRL>
+__device__ __forceinline__ float ta_dpp(float x) {
+  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float ta_sum16(float x) {       // pairs, quads, halves of a row, rows
+  x += ta_dpp<0xB1>(x);      // lanes 1 apart
+  x += ta_dpp<0x4E>(x);      // 2 apart
+  x += ta_dpp<0x141>(x);     // mirrored in eights
+  x += ta_dpp<0x140>(x);     // mirrored in sixteens
+  return x;
+}
+// two sums at once
+template <int LANES>
+__device__ __forceinline__ void ta_sums2(float& w, float& r) {
+  static_assert(LANES == 16 || LANES == 32 || LANES == 64, "lanes that share a sum");
+  if (LANES == 16) {
+    w = ta_sum16(w);
+    r = ta_sum16(r);
+    return;
+  }
+  // rows of 16 lanes trade places: the even ones are left with what both rows have of w, the odd ones with
+  // theirs of r, one exchange sums either, and a second trade hands both to all lanes
+  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(w), __float_as_uint(r), false, false);
+  float t = ta_sum16(__uint_as_float(a[0]) + __uint_as_float(a[1]));
+  if (LANES == 64) {
+    const auto h = __builtin_amdgcn_permlane32_swap(__float_as_uint(t), __float_as_uint(t), false, false);
+    t = __uint_as_float(h[0]) + __uint_as_float(h[1]);
+  }
+  const auto c = __builtin_amdgcn_permlane16_swap(__float_as_uint(t), __float_as_uint(t), false, false);
+  w = __uint_as_float(c[0]);
+  r = __uint_as_float(c[1]);
+}
+
 // ---------------------------------------------------------------- host side
 int ta_fail(const char* fmt, ...);            // records the message, returns 1
 int ta_check_launch(const char* what);        // hipGetLastError -> message

@@ -106,36 +106,6 @@ extern "C" int ta_delta_prepare(hipStream_t stream, int dtype, const void* qkv, 
 // token's leave LDS a token ahead.
 #define DR_FEW_COLUMNS 3072
 
-template <int CTRL>
-__device__ __forceinline__ float dr_dpp(float x) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(x), CTRL, 0xf, 0xf, true));
-}
-// the sum over 16 neighbouring lanes, the same bits in each: pairs, quads, halves of a row, rows
-__device__ __forceinline__ float dr_sum16(float x) {
-  x += dr_dpp<0xB1>(x);      // lanes 1 apart
-  x += dr_dpp<0x4E>(x);      // 2 apart
-  x += dr_dpp<0x141>(x);     // mirrored in eights
-  x += dr_dpp<0x140>(x);     // mirrored in sixteens
-  return x;
-}
-
-// both sums over the lanes of a column, the same bits in each of them
-template <int LANES>
-__device__ __forceinline__ void dr_sums(float& w, float& r) {
-  if (LANES == 16) {
-    w = dr_sum16(w);
-    r = dr_sum16(r);
-    return;
-  }
-  // rows of 16 lanes trade places: the even ones are left with what both rows have of w, the odd ones with
-  // theirs of r, one exchange sums either, and a second trade hands both to all lanes
-  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(w), __float_as_uint(r), false, false);
-  const float t = dr_sum16(__uint_as_float(a[0]) + __uint_as_float(a[1]));
-  const auto c = __builtin_amdgcn_permlane16_swap(__float_as_uint(t), __float_as_uint(t), false, false);
-  w = __uint_as_float(c[0]);
-  r = __uint_as_float(c[1]);
-}
-
 // HEAD: one decay per token and head, [nt, H]; it travels with the step size.
 template <typename T, int LANES, int R, bool VEC, bool HEAD>
 __global__ __launch_bounds__(256) void delta_recurrent_kernel(
@@ -253,7 +223,7 @@ __global__ __launch_bounds__(256) void delta_recurrent_kernel(
       }
     }
     float ws = (w[0] + w[1]) + (w[2] + w[3]), rs = (r[0] + r[1]) + (r[2] + r[3]);
-    dr_sums<LANES>(ws, rs);
+    ta_sums2<LANES>(ws, rs);
     const float u = o.bx.x * (o.v - ws);
 #pragma unroll
     for (int i = 0; i < R / 4; ++i) {

@@ -8,11 +8,10 @@
 //
 //   memory_gates : keep, write and exp(-m) of every token and head; the running maximum by a scan over
 //                  the waves of a workgroup
+//   memory_recurrent : walks a sequence's tokens in order with S in registers; the normaliser is one more value
+//                  column whose value is always 1
 //   memory_step  : a step of single tokens in one kernel: gates, the state's update, the readout with its
 //                  denominator, the head's norm and the output gate
-//
-// (The recurrence over a prompt is the kernel of gated linear attention with keep as the decay, write as a
-// factor on the key, and the normaliser as one more value column, see recurrent.hip.)
 //
 // keep is formed as exp(f - (m_t - m_(t-1))): where m_t is the rounded f + m_(t-1), the difference of the
 // two maxima is exact and keep makes up for that rounding.
@@ -110,6 +109,214 @@ extern "C" int ta_memory_gates(hipStream_t stream, int dtype, const void* proj, 
 #undef MG_BY_LEN
 #undef MG_RUN
   return ta_check_launch("ta_memory_gates");
+}
+
+// ------------------------------------------------------------------ prompts
+// LANES (16, 32 or 64) lanes share a value column, each with R of its key channels (in runs of four: run i of lane
+// l holds channels 4 LANES i + 4 l ..+3, so that a wave's operand reads from LDS meet every bank once); a wave owns
+// 64 / LANES columns. Operands of the next chunk of tokens are on their way to registers while this chunk is worked
+// on out of one of two LDS buffers; keys wait in LDS already times their write weight, and the next token's
+// operands leave LDS a token ahead. Two tokens' readouts are summed over the lanes together, outside the chain of
+// updates.
+template <typename T, int LANES, int R, bool VEC>
+__global__ __launch_bounds__(256) void memory_recurrent_kernel(
+    const T* __restrict__ proj, int stride, int qoff, int koff, int voff, float qscale, const float* __restrict__ keep,
+    const float* __restrict__ write, float* __restrict__ state, float* __restrict__ n_state,
+    const int* __restrict__ cu_q, const int* __restrict__ slots, int H, int dk, int dv, float* __restrict__ o_out,
+    float* __restrict__ den_out) {
+  constexpr int DKP = LANES * R, NT = 256, COLS = NT / LANES;
+  constexpr int TC = DKP <= 128 ? 16 : 2048 / DKP;   // tokens of a chunk (even, at most LANES: see `kept`)
+  constexpr int NF = (TC * DKP / 4 + NT - 1) / NT;   // runs of four that a thread brings in of each operand
+  __shared__ __attribute__((aligned(16))) float sq[2][TC][DKP], sk[2][TC][DKP];
+  __shared__ float sv[2][TC][COLS];                  // (TC * COLS is at most NT)
+  __shared__ float sg[2][TC];
+  const int h = blockIdx.x, col0 = blockIdx.y * COLS, b = blockIdx.z;
+  const int start = cu_q[b], end = cu_q[b + 1];
+  if (start >= end) return;
+  const int tid = threadIdx.x, lane = tid % LANES, cl = tid / LANES;
+  const int col = col0 + cl;                         // dv: the normaliser
+  const size_t head = (size_t)slots[b] * H + h;
+  float* st = col < dv ? state + head * dk * (size_t)dv + col : n_state + head * dk;
+  const size_t sstep = col < dv ? dv : 1;
+  const bool mine = col <= dv;
+  float S[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = 4 * LANES * (i / 4) + 4 * lane + i % 4;
+    S[i] = (mine && row < dk) ? st[row * sstep] : 0.f;
+  }
+  struct alignas(4 * sizeof(T)) Run { T x[4]; };
+  struct Chunk {
+    Run q[NF], k[NF];
+    float w[NF], g;
+    T v;
+  };
+  // every load is issued without a condition (a channel past dk, a column past dv, a token past the sequence's
+  // end read what is there and are replaced), so that none is waited for before its chunk goes to LDS
+  auto run4 = [&](const T* p, int c) {
+    if (VEC) return *reinterpret_cast<const Run*>(p + (c < dk ? c : 0));
+    Run r;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) r.x[e] = p[c + e < dk ? c + e : 0];
+    return r;
+  };
+  auto fetch = [&](Chunk& f, int t0) {
+#pragma unroll
+    for (int e = 0; e < NF; ++e) {
+      const int idx = tid + NT * e, tt = idx / (DKP / 4), c = (idx % (DKP / 4)) * 4;
+      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
+      const T* row = proj + t * stride + h * dk;
+      f.q[e] = run4(row + qoff, c);
+      f.k[e] = run4(row + koff, c);
+      f.w[e] = write[t * H + h];
+    }
+    {
+      const int tt = tid / COLS, c = col0 + tid % COLS;
+      const size_t t = t0 + tt < end ? t0 + tt : end - 1;
+      f.v = proj[t * stride + voff + h * dv + (c < dv ? c : 0)];
+    }
+    const size_t t = t0 + tid % TC < end ? t0 + tid % TC : end - 1;
+    f.g = keep[t * H + h];
+  };
+  auto stash = [&](const Chunk& f, int t0, int buf) {
+#pragma unroll
+    for (int e = 0; e < NF; ++e) {
+      const int idx = tid + NT * e, tt = idx / (DKP / 4), c = (idx % (DKP / 4)) * 4;
+      if (TC * DKP / 4 % NT == 0 || idx < TC * DKP / 4) {
+        const float w = t0 + tt < end ? f.w[e] : 0.f;         // a token past the end writes nothing
+        float q[4], k[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const bool ok = c + j < dk;
+          q[j] = ok ? to_f32(f.q[e].x[j]) * qscale : 0.f;
+          k[j] = ok ? to_f32(f.k[e].x[j]) * w : 0.f;
+        }
+        reinterpret_cast<float4*>(&sq[buf][0][0])[idx] = float4{q[0], q[1], q[2], q[3]};
+        reinterpret_cast<float4*>(&sk[buf][0][0])[idx] = float4{k[0], k[1], k[2], k[3]};
+      }
+    }
+    if (TC * COLS == NT || tid < TC * COLS) (&sv[buf][0][0])[tid] = col0 + tid % COLS == dv ? 1.f : to_f32(f.v);
+    if (tid < TC) sg[buf][tid] = t0 + tid < end ? f.g : 1.f;
+  };
+  struct Token {
+    float4 q[R / 4], k[R / 4];
+    float v, g;
+  };
+  auto take = [&](Token& o, int buf, int tt) {
+    if (tt > TC - 1) tt = TC - 1;                             // past the chunk: not used
+#pragma unroll
+    for (int i = 0; i < R / 4; ++i) {
+      o.k[i] = *reinterpret_cast<const float4*>(&sk[buf][tt][4 * LANES * i + 4 * lane]);
+      o.q[i] = *reinterpret_cast<const float4*>(&sq[buf][tt][4 * LANES * i + 4 * lane]);
+    }
+    o.v = sv[buf][tt][cl];
+    o.g = sg[buf][tt];
+  };
+  auto token = [&](const Token& o) {
+    float r[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < R / 4; ++i) {
+      const float ks[4] = {o.k[i].x, o.k[i].y, o.k[i].z, o.k[i].w};
+      const float qs[4] = {o.q[i].x, o.q[i].y, o.q[i].z, o.q[i].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        S[4 * i + e] = fmaf(o.g, S[4 * i + e], ks[e] * o.v);
+        r[e] = fmaf(S[4 * i + e], qs[e], r[e]);
+      }
+    }
+    return (r[0] + r[1]) + (r[2] + r[3]);
+  };
+  float* out = col < dv ? o_out + (size_t)h * dv + col : den_out + h;
+  const size_t ostep = col < dv ? (size_t)H * dv : (size_t)H;
+  {
+    Chunk f;
+    fetch(f, start);
+    stash(f, start, 0);
+  }
+  __syncthreads();
+  int buf = 0;
+  for (int t0 = start; t0 < end; t0 += TC, buf ^= 1) {
+    const int n = end - t0 < TC ? end - t0 : TC;
+    Chunk f;
+    fetch(f, t0 + TC);                  // behind the last chunk: its last token again, for nothing
+    float kept = 0.f;                   // lane l keeps the readout of the chunk's token l
+    Token a, c;
+    // the next token's operands are asked for in front of this token's arithmetic, and stay there
+    __builtin_amdgcn_sched_barrier(0);
+    take(a, buf, 0);
+    auto pair = [&](int tt) {
+      take(c, buf, tt + 1);
+      __builtin_amdgcn_sched_barrier(0);
+      float r0 = token(a);
+      __builtin_amdgcn_sched_barrier(0);
+      take(a, buf, tt + 2);
+      __builtin_amdgcn_sched_barrier(0);
+      float r1 = token(c);
+      ta_sums2<LANES>(r0, r1);
+      kept = lane == tt ? r0 : lane == tt + 1 ? r1 : kept;
+    };
+    if (n == TC) {
+#pragma unroll
+      for (int tt = 0; tt < TC; tt += 2) pair(tt);
+    } else {
+      for (int tt = 0; tt < n; tt += 2) pair(tt);             // (an odd end is filled up with a token that writes nothing)
+    }
+    if (lane < n && mine) out[(size_t)(t0 + lane) * ostep] = kept;
+    // the other buffer's readers are behind the barrier at the end of the turn before
+    stash(f, t0 + TC, buf ^ 1);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int row = 4 * LANES * (i / 4) + 4 * lane + i % 4;
+    if (mine && row < dk) st[row * sstep] = S[i];
+  }
+}
+
+#define MM_FEW_COLUMNS 4096     // columns (sequences x heads x values) up to which 32 lanes share one
+#define MM_MAX_KEY_DIM 1024
+
+// proj: [nt] rows, stride apart, with q and k (H*dk each) and v (H*dv) at columns qoff, koff, voff; q is taken times
+// qscale. keep, write [nt, H] (ta_memory_gates); state [slots, H, dk, dv], n_state [slots, H, dk] float32, moved on.
+// o_out [nt, H, dv] = S_t^T q_t, den_out [nt, H] = n_t . q_t, float32. lanes that share a column (0: chosen by the
+// shape; 16 or 32, where the key width leaves the choice).
+extern "C" int ta_memory_recurrent(hipStream_t stream, int dtype, const void* proj, int stride, int qoff, int koff,
+                                   int voff, float qscale, const float* keep, const float* write, float* state,
+                                   float* n_state, const int* cu_q, const int* slots, int batch, int nt, int H, int dk,
+                                   int dv, int lanes, float* o_out, float* den_out) {
+  TA_REQUIRE(batch > 0 && batch <= 65535 && nt >= batch && H >= 1, "ta_memory_recurrent: batch %d, %d tokens, %d heads", batch, nt, H);
+  TA_REQUIRE(dk >= 1 && dk <= MM_MAX_KEY_DIM && dv >= 1, "ta_memory_recurrent: heads of %d x %d", dk, dv);
+  TA_REQUIRE(qoff >= 0 && koff >= 0 && voff >= 0 && stride >= qoff + H * dk && stride >= koff + H * dk &&
+             stride >= voff + H * dv, "ta_memory_recurrent: rows of %d are too short", stride);
+  TA_REQUIRE(lanes == 0 || lanes == 16 || lanes == 32, "ta_memory_recurrent: %d lanes", lanes);
+  TA_REQUIRE(dtype == TA_F32 || dtype == TA_BF16, "ta_memory_recurrent: unknown dtype %d", dtype);
+  if (lanes == 0) lanes = (long long)batch * H * dv > MM_FEW_COLUMNS ? 16 : 32;
+  if (dk <= 64) lanes = 16;
+  if (dk > 256) lanes = 32;
+  if (dk > 512) lanes = 64;
+  const int cols = 256 / lanes, tiles = (dv + 1 + cols - 1) / cols;
+  TA_REQUIRE(tiles <= 65535, "ta_memory_recurrent: values of %d", dv);
+  dim3 g(H, tiles, batch);
+  const int item = dtype == TA_F32 ? 4 : 2;
+  const bool vec = dk % 4 == 0 && qoff % 4 == 0 && koff % 4 == 0 && stride % 4 == 0 && (uintptr_t)proj % (4 * item) == 0;
+#define MR_RUN(T, L, RR, VE)                                                                                             \
+  memory_recurrent_kernel<T, L, RR, VE><<<g, 256, 0, stream>>>((const T*)proj, stride, qoff, koff, voff, qscale, keep,   \
+                                                               write, state, n_state, cu_q, slots, H, dk, dv, o_out, den_out)
+#define MR_BY_VEC(T, L, RR) \
+  if (vec) MR_RUN(T, L, RR, true); else MR_RUN(T, L, RR, false)
+#define MR_BY_WIDTH(T)                                                      \
+  if (dk <= 64) { MR_BY_VEC(T, 16, 4); }                                    \
+  else if (dk <= 128) {                                                     \
+    if (lanes == 32) { MR_BY_VEC(T, 32, 4); } else { MR_BY_VEC(T, 16, 8); }   \
+  } else if (dk <= 256) {                                                   \
+    if (lanes == 32) { MR_BY_VEC(T, 32, 8); } else { MR_BY_VEC(T, 16, 16); }  \
+  } else if (dk <= 512) { MR_BY_VEC(T, 32, 16); }                           \
+  else { MR_BY_VEC(T, 64, 16); }
+  if (dtype == TA_F32) { MR_BY_WIDTH(float) } else { MR_BY_WIDTH(bf16_t) }
+#undef MR_BY_WIDTH
+#undef MR_BY_VEC
+#undef MR_RUN
+  return ta_check_launch("ta_memory_recurrent");
 }
 
 // ------------------------------------------------------------------ steps of single tokens

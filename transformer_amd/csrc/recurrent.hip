@@ -19,10 +19,6 @@
 //   `ssm_steps` forms step sizes and decays, the recurrence is `gla_recurrent` with q = C, k = B, v = x
 //   (the heads of a group read the same B and C), `gated_group_norm` adds D x, gates and norms.
 //
-// Matrix memory (matrix_memory.hip): the same recurrence with one decay and one key factor per (token,
-//   head) and a normaliser n_t, which decays and is written as S is and whose product with q is the
-//   readout's denominator: it is one more value column whose value is always 1.
-//
 // Short causal convolution (`causal_conv`): per channel over a sequence's tokens, with the last
 //   inputs of every sequence kept between steps; used in front of the state space and by the
 //   attention variant that convolves its q, k and v.
@@ -575,19 +571,16 @@ struct GlaOperands {  // what one thread brings in for a chunk
   float q[GLA_TC * GLA_RT / 256], k[GLA_TC * GLA_RT / 256], a[GLA_TC * GLA_RT / 256], v[GLA_TC * GLA_CT / 256];
 };
 
-// NORM: column dv stands for the normaliser: its value is 1, its state is n_state [slots, H, dk], and its
-// readout goes to the planes of den_out [nt, H].
 // BONUS: the readout comes BEFORE the update and gives the current token a weight of its own,
 // o_t = (S_{t-1} + diag(bonus) k_t v_t^T)^T q_t, then S_t = diag(alpha_t) S_{t-1} + k_t v_t^T.
-template <typename T, int GLA_TC, bool BONUS, bool NORM = false>
+template <typename T, int GLA_TC, bool BONUS>
 __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     const T* __restrict__ proj, int stride, int qoff, int koff, int voff, const float* __restrict__ alpha,
     float qscale, float* __restrict__ state, const int* __restrict__ cu_q, const int* __restrict__ slots,
     int H, int dk, int dv, int col_tiles, size_t plane, float* __restrict__ o_out,
     const float* __restrict__ bonus, const float* __restrict__ head_decay,
     int qk_share = 1, const float* __restrict__ tok_decay = nullptr,
-    const float* __restrict__ tok_kscale = nullptr, float* __restrict__ n_state = nullptr,
-    float* __restrict__ den_out = nullptr) {
+    const float* __restrict__ tok_kscale = nullptr) {
   __shared__ float sq[GLA_TC][GLA_RT], sk[GLA_TC][GLA_RT], sa[GLA_TC][GLA_RT];
   __shared__ float sv[GLA_TC][GLA_CT];
   __shared__ float part[GLA_TC][4][GLA_CT];
@@ -607,7 +600,6 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     for (int c = 0; c < 2; ++c) {
       const int i = row0 + rg * 4 + r, j = col0 + cg * 2 + c;
       S[r][c] = (i < dk && j < dv) ? st[(size_t)i * dv + j] : 0.f;
-      if (NORM && i < dk && j == dv) S[r][c] = n_state[(slot * H + h) * dk + i];
     }
   float bu[4] = {0.f, 0.f, 0.f, 0.f};
   if (BONUS) {
@@ -645,7 +637,7 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
       const int idx = tid + 256 * e, tt = idx / GLA_CT, j = col0 + idx % GLA_CT;
       const bool ok = t0 + tt < end && j < dv;
       const float vv = to_f32(proj[(size_t)(ok ? t0 + tt : start) * stride + voff + h * dv + (ok ? j : 0)]);
-      o.v[e] = ok ? vv : (NORM && j == dv) ? 1.f : 0.f;
+      o.v[e] = ok ? vv : 0.f;
     }
   };
   auto turn = [&](GlaOperands<GLA_TC>& o, int t0) {
@@ -713,9 +705,6 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
       if (col0 + c < dv)
         o_out[rpart * plane + ((size_t)(t0 + tt) * H + h) * dv + col0 + c] =
             (part[tt][0][c] + part[tt][1][c]) + (part[tt][2][c] + part[tt][3][c]);
-      if (NORM && col0 + c == dv)
-        den_out[rpart * (plane / dv) + (size_t)(t0 + tt) * H + h] =
-            (part[tt][0][c] + part[tt][1][c]) + (part[tt][2][c] + part[tt][3][c]);
     }
     // The next turn's stores into sq/sk/sa/sv follow the barrier above, which every thread
     // passes only after its last read of them; `part` is read here and written again only
@@ -734,7 +723,6 @@ __global__ __launch_bounds__(256) void gla_recurrent_kernel(
     for (int c = 0; c < 2; ++c) {
       const int i = row0 + rg * 4 + r, j = col0 + cg * 2 + c;
       if (i < dk && j < dv) st[(size_t)i * dv + j] = S[r][c];
-      if (NORM && i < dk && j == dv) n_state[(slot * H + h) * dk + i] = S[r][c];
     }
 }
 
@@ -750,14 +738,13 @@ static int gla_recurrent_launch(hipStream_t stream, int dtype, int wdtype, const
                                 float* state, const int* cu_q, const int* slots, int batch, int nt, int H, int dk,
                                 int dv, float* o_out, int mode, const float* bonus,
                                 const float* head_decay = nullptr, int qk_share = 1,
-                                const float* tok_decay = nullptr, const float* tok_kscale = nullptr,
-                                float* n_state = nullptr, float* den_out = nullptr) {
+                                const float* tok_decay = nullptr, const float* tok_kscale = nullptr) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && H > 0 && H <= 65535 && nt >= batch,
              "ta_gla_recurrent: bad batch %d / heads %d / tokens %d", batch, H, nt);
   TA_REQUIRE(qk_share >= 1 && H % qk_share == 0, "ta_gla_recurrent: %d heads do not form groups of %d", H, qk_share);
   TA_REQUIRE(dk >= 1 && dv >= 1 && (head_decay || tok_decay || (rank >= 1 && rank <= 8192)),
              "ta_gla_recurrent: bad widths %d / %d / %d", dk, dv, rank);
-  const int parts = (dk + GLA_RT - 1) / GLA_RT, tiles = (dv + (n_state ? 1 : 0) + GLA_CT - 1) / GLA_CT;
+  const int parts = (dk + GLA_RT - 1) / GLA_RT, tiles = (dv + GLA_CT - 1) / GLA_CT;
   TA_REQUIRE(parts * tiles <= 65535, "ta_gla_recurrent: heads of %d x %d are too large", dk, dv);
   const int n = H * dk;
   dim3 gd(nt, (n + 255) / 256 < 64 ? (n + 255) / 256 : 64);
@@ -774,17 +761,11 @@ static int gla_recurrent_launch(hipStream_t stream, int dtype, int wdtype, const
   dim3 g(batch, H, parts * tiles);
   const size_t plane = (size_t)nt * H * dv;
   const bool few = nt <= 8 * batch;         // at most 8 tokens a sequence on average: short chunks
-#define GLA_RUN(T, TC, ...)                                                                                 \
-  gla_recurrent_kernel<T, TC, __VA_ARGS__><<<g, 256, 0, stream>>>((const T*)proj, stride, qoff, koff, voff, alpha, qscale, \
+#define GLA_RUN(T, TC, B)                                                                                   \
+  gla_recurrent_kernel<T, TC, B><<<g, 256, 0, stream>>>((const T*)proj, stride, qoff, koff, voff, alpha, qscale, \
                                                         state, cu_q, slots, H, dk, dv, tiles, plane, o_out, bonus, \
-                                                        head_decay, qk_share, tok_decay, tok_kscale, n_state, den_out)
-  if (n_state) {
-    if (dtype == TA_F32) {
-      if (few) GLA_RUN(float, 8, false, true); else GLA_RUN(float, 32, false, true);
-    } else {
-      if (few) GLA_RUN(bf16_t, 8, false, true); else GLA_RUN(bf16_t, 32, false, true);
-    }
-  } else if (bonus) {
+                                                        head_decay, qk_share, tok_decay, tok_kscale)
+  if (bonus) {
     if (dtype == TA_F32) {
       if (few) GLA_RUN(float, 8, true); else GLA_RUN(float, 32, true);
     } else {
@@ -833,21 +814,6 @@ extern "C" int ta_decay_recurrent(hipStream_t stream, int dtype, const void* pro
   return gla_recurrent_launch(stream, dtype, dtype, proj, stride, qoff, koff, voff, nullptr, 0, 0, 0, nullptr,
                               nullptr, 1.0f, qscale, nullptr, state, cu_q, slots, batch, nt, H, dk, dv, o_out, 0,
                               nullptr, head_decay);
-}
-
-// The recurrence of the matrix memory: keep and write [nt, H] float32 (ta_memory_gates), q, k, v at column
-// offsets of the rows of ``proj``, the query times qscale; n_state [slots, H, dk] float32. o_out
-// [ta_gla_row_parts(dk), nt, H, dv] and den_out [ta_gla_row_parts(dk), nt, H]: planes that add up to S_t^T q
-// and n_t . q.
-extern "C" int ta_memory_recurrent(hipStream_t stream, int dtype, const void* proj, int stride, int qoff, int koff,
-                                   int voff, float qscale, const float* keep, const float* write, float* state,
-                                   float* n_state, const int* cu_q, const int* slots, int batch, int nt, int H, int dk,
-                                   int dv, float* o_out, float* den_out) {
-  TA_REQUIRE(keep != nullptr && write != nullptr && n_state != nullptr && den_out != nullptr,
-             "ta_memory_recurrent: weights, normaliser and denominators are required");
-  return gla_recurrent_launch(stream, dtype, dtype, proj, stride, qoff, koff, voff, nullptr, 0, 0, 0, nullptr, nullptr,
-                              1.0f, qscale, nullptr, state, cu_q, slots, batch, nt, H, dk, dv, o_out, 0, nullptr,
-                              nullptr, 1, keep, write, n_state, den_out);
 }
 
 // ------------------------------------------------------------------ gla: head norm and output gate

@@ -2238,6 +2238,9 @@ def delta_step(qkv: torch.Tensor, proj: torch.Tensor, a_off: int, g_off: int, b_
 
 
 # ------------------------------------------------------------------ matrix memory
+MEMORY_MAX_KEY_DIM = 1024
+
+
 def _memory_columns(what, proj, offs, H, dk, dv):
     """Checks that q, k, v, gate, i, f (or the first of them) lie inside the rows of ``proj``."""
     for off, n in zip(offs, (H * dk, H * dk, H * dv, H * dv, H, H)):
@@ -2270,27 +2273,28 @@ def memory_gates(proj: torch.Tensor, i_off: int, f_off: int, i_bias, f_bias, cap
 
 def memory_recurrent(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_scale: float, keep: torch.Tensor,
                      write: torch.Tensor, state: torch.Tensor, n_state: torch.Tensor, cu_q, slots, o_out: torch.Tensor,
-                     den_out: torch.Tensor) -> torch.Tensor:
+                     den_out: torch.Tensor, lanes: int = 0) -> torch.Tensor:
     """The matrix memory along every sequence: S <- keep S + write k v^T, n <- keep n + write k, o = S^T (q_scale q),
-    den = n . (q_scale q). ``state`` [slots, H, dk, dv], ``n_state`` [slots, H, dk] float32; o_out
-    [gla_row_parts(dk), nt, H, dv] and den_out [gla_row_parts(dk), nt, H] float32 planes that add up."""
+    den = n . (q_scale q). ``state`` [slots, H, dk, dv], ``n_state`` [slots, H, dk] float32; o_out [nt,
+    H, dv] and den_out [nt, H] float32. lanes that share a column: 16 or 32 (0: chosen by the shape)."""
     _dev(proj, "proj", contiguous=False); _dev(state, "state", torch.float32)
     nt, stride = _rows2d(proj, "proj")
     batch = _step_tables(cu_q, slots, nt, "memory_recurrent")
     if state.dim() != 4:
         raise KernelError(f"memory_recurrent: state is {tuple(state.shape)}")
     S, H, dk, dv = state.shape
-    parts = gla_row_parts(dk)
     for t, n, shape in ((keep, "keep", (nt, H)), (write, "write", (nt, H)), (n_state, "n_state", (S, H, dk)),
-                        (o_out, "o_out", (parts, nt, H, dv)), (den_out, "den_out", (parts, nt, H))):
+                        (o_out, "o_out", (nt, H, dv)), (den_out, "den_out", (nt, H))):
         _dev(t, n, torch.float32)
         if tuple(t.shape) != shape:
             raise KernelError(f"memory_recurrent: {n} is {tuple(t.shape)}, expected {shape}")
+    if dk > MEMORY_MAX_KEY_DIM:
+        raise KernelError(f"memory_recurrent: key widths up to {MEMORY_MAX_KEY_DIM}, not {dk}")
     _memory_columns("memory_recurrent", proj, (q_off, k_off, v_off), H, dk, dv)
     _check(library().ta_memory_recurrent(
         _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), c_int(q_off), c_int(k_off), c_int(v_off),
         c_float(q_scale), _ptr(keep), _ptr(write), _ptr(state), _ptr(n_state), _ptr(cu_q), _ptr(slots), c_int(batch),
-        c_int(nt), c_int(H), c_int(dk), c_int(dv), _ptr(o_out), _ptr(den_out)))
+        c_int(nt), c_int(H), c_int(dk), c_int(dv), c_int(lanes), _ptr(o_out), _ptr(den_out)))
     return o_out
 
 

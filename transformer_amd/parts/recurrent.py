@@ -425,6 +425,8 @@ class MatrixMemory(Part):
         s = spec
         if min(s.num_heads, s.key_dim, s.value_dim) < 1 or not s.gate_cap > 0:
             raise PartError(f"matrix memory: {s.num_heads} heads of {s.key_dim} / {s.value_dim}, gates capped at {s.gate_cap}")
+        if s.key_dim > kernels.MEMORY_MAX_KEY_DIM:
+            raise PartError(f"matrix memory: key widths up to {kernels.MEMORY_MAX_KEY_DIM}, not {s.key_dim}")
         self.spec, self.dtype = s, dtype
         self.nk, self.nv = s.num_heads * s.key_dim, s.num_heads * s.value_dim
         i_off = 2 * self.nk + 2 * self.nv
@@ -470,11 +472,10 @@ class MatrixMemory(Part):
         keep, write, floor = (take(f"memory.{n}", (nt, H), f32) for n in ("keep", "write", "floor"))
         kernels.memory_gates(proj, i_off, f_off, *biases, float(s.gate_cap), m_state, ctx.cu_q, ctx.slots,
                              ctx.max_qlen, keep, write, floor)
-        parts = kernels.gla_row_parts(dk)
-        o, den = take("memory.o", (parts, nt, H, dv), f32), take("memory.den", (parts, nt, H), f32)
+        o, den = take("memory.o", (nt, H, dv), f32), take("memory.den", (nt, H), f32)
         kernels.memory_recurrent(proj, q_off, k_off, v_off, q_scale, keep, write, state, n_state, ctx.cu_q, ctx.slots, o, den)
-        kernels.head_norm_gate(o, proj[:, g_off:g_off + self.nv], H, dv, self.w["norm.weight"], float(s.eps), y, "sigmoid",
-                               den=den, floor=floor)
+        kernels.head_norm_gate(o.unsqueeze(0), proj[:, g_off:g_off + self.nv], H, dv, self.w["norm.weight"], float(s.eps),
+                               y, "sigmoid", den=den.unsqueeze(0), floor=floor)
         return finish(y, self.w["out.weight"], ctx.ws, "memory.delta", fold, into)
 
 
