@@ -255,7 +255,7 @@ def _memory_part(w, m, dtype):
 
 CUTS = [(37, 1, 18), (1, 1, 1), (2, 2, 2), (2, 2, 2), (1, 1, 1), (18, 1, 16)]
 MEMORY_GEOMS = [(2, 32, 64, 10.0), (3, 20, 12, 4.0), (1, 1, 1, 5.0), (5, 33, 7, 15.0), (2, 6, 66, 2.0), (4, 128, 128, 12.0), (1, 64, 200, 8.0),
-                (2, 256, 512, 15.0), (3, 16, 100, 7.0), (1, 300, 40, 9.0), (2, 40, 127, 3.0)]
+                (2, 256, 512, 15.0), (3, 16, 100, 7.0), (1, 300, 40, 9.0), (2, 40, 127, 3.0), (1, 100, 1202, 6.0), (1, 1000, 1111, 5.0)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)

@@ -11,7 +11,9 @@
 //   memory_recurrent : walks a sequence's tokens in order with S in registers; the normaliser is one more value
 //                  column whose value is always 1
 //   memory_step  : a step of single tokens in one kernel: gates, the state's update, the readout with its
-//                  denominator, the head's norm and the output gate
+//                  denominator, the head's norm and the output gate; heads too large for one workgroup take
+//                  two kernels, the second of which moves normaliser and maximum on and does what needs the whole
+//                  readout
 //
 // keep is formed as exp(f - (m_t - m_(t-1))): where m_t is the rounded f + m_(t-1), the difference of the
 // two maxima is exact and keep makes up for that rounding.
@@ -322,26 +324,44 @@ extern "C" int ta_memory_recurrent(hipStream_t stream, int dtype, const void* pr
 // ------------------------------------------------------------------ steps of single tokens
 // One workgroup of MS_NT threads per (head, sequence). A thread keeps VW neighbouring value columns of every
 // RG-th key channel; the whole state is asked for before anything else is done.
+// SPLIT: a workgroup owns dvt of the head's columns, leaves their readout in o_out [batch, H, dv] as it is, and
+// changes neither n nor m, which the other workgroups of the head read as well.
 #define MS_NT 512
 
-template <typename T, int VW, int ROWS>
+struct MemoryGates {
+  float keep, write, m;
+};
+// of one token, from what stood in m_state before it
+template <typename T>
+__device__ __forceinline__ MemoryGates mm_gates(const T* __restrict__ row, int ioff, int foff, int h,
+                                                const float* __restrict__ ibias, const float* __restrict__ fbias,
+                                                float cap, float before) {
+  const float i = mm_cap(to_f32(row[ioff + h]) + ibias[h], cap);
+  const float f = mm_log_sigmoid(mm_cap(to_f32(row[foff + h]) + fbias[h], cap));
+  const float m = fmaxf(f + before, i);
+  return MemoryGates{expf(f - (m - before)), expf(i - m), m};
+}
+
+template <typename T, int VW, int ROWS, bool SPLIT>
 __global__ __launch_bounds__(MS_NT) void memory_step_kernel(
     const T* __restrict__ proj, int stride, int qoff, int koff, int voff, int goff, int ioff, int foff,
     const float* __restrict__ ibias, const float* __restrict__ fbias, float cap, float* __restrict__ state,
     float* __restrict__ n_state, float* __restrict__ m_state, const int* __restrict__ slots, int H, int dk, int dv,
-    float qscale, const float* __restrict__ norm_w, float eps, T* __restrict__ out) {
+    float qscale, const float* __restrict__ norm_w, float eps, T* __restrict__ out, int dvt, float* __restrict__ o_out) {
   extern __shared__ float lds[];
-  const int CV = dv / VW, RG = MS_NT / CV;           // column groups; row groups
+  const int CV = dvt / VW, RG = MS_NT / CV;          // column groups; row groups
+  const int cb = SPLIT ? blockIdx.z * dvt : 0;       // this workgroup's first column and their number
+  const int dvc = SPLIT && dv - cb < dvt ? dv - cb : dvt;
   float* qs = lds;                                   // [dk]
   float* ks = qs + dk;                               // [dk], times the write weight
-  float* pr = ks + dk;                               // [RG][dv]
+  float* pr = ks + dk;                               // [RG][dvt]
   __shared__ float red[MS_NT / TA_WAVE], redn[MS_NT / TA_WAVE];
   const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
   const size_t slot = (size_t)slots[b];
-  float* st = state + (slot * H + h) * dk * (size_t)dv;
+  float* st = state + (slot * H + h) * dk * (size_t)dv + cb;
   float* ns = n_state + (slot * H + h) * dk;
   const int r0 = tid / CV, c0 = (tid % CV) * VW;
-  const bool on = r0 < RG;
+  const bool on = r0 < RG && c0 < dvc;
   float S[ROWS][VW];
 #pragma unroll
   for (int i = 0; i < ROWS; ++i) {
@@ -361,27 +381,28 @@ __global__ __launch_bounds__(MS_NT) void memory_step_kernel(
   const T* row = proj + (size_t)b * stride;
   float v[VW];
 #pragma unroll
-  for (int e = 0; e < VW; ++e) v[e] = on ? to_f32(row[voff + h * dv + c0 + e]) : 0.f;
+  for (int e = 0; e < VW; ++e) v[e] = on ? to_f32(row[voff + h * dv + cb + c0 + e]) : 0.f;
   // the gates, by every thread for itself
-  const float i = mm_cap(to_f32(row[ioff + h]) + ibias[h], cap);
-  const float f = mm_log_sigmoid(mm_cap(to_f32(row[foff + h]) + fbias[h], cap));
-  const float before = m_state[slot * H + h];
-  const float m = fmaxf(f + before, i);
-  const float keep = expf(f - (m - before)), write = expf(i - m);
+  const MemoryGates gt = mm_gates(row, ioff, foff, h, ibias, fbias, cap, m_state[slot * H + h]);
+  const float keep = gt.keep, write = gt.write, m = gt.m;
   // the normaliser and its product with q
   float dot = 0.f;
   for (int c = tid; c < dk; c += MS_NT) {
     const float q = to_f32(row[qoff + h * dk + c]) * qscale, k = to_f32(row[koff + h * dk + c]) * write;
-    const float n = fmaf(keep, ns[c], k);
     qs[c] = q;
     ks[c] = k;
-    ns[c] = n;
-    dot = fmaf(n, q, dot);
+    if (!SPLIT) {
+      const float n = fmaf(keep, ns[c], k);
+      ns[c] = n;
+      dot = fmaf(n, q, dot);
+    }
   }
-  dot = wave_sum(dot);
-  if (tid % TA_WAVE == 0) redn[tid / TA_WAVE] = dot;
+  if (!SPLIT) {
+    dot = wave_sum(dot);
+    if (tid % TA_WAVE == 0) redn[tid / TA_WAVE] = dot;
+  }
   __syncthreads();                                   // (every thread has read m_state before one writes it)
-  if (tid == 0) m_state[slot * H + h] = m;
+  if (!SPLIT && tid == 0) m_state[slot * H + h] = m;
   // ---- the update and the readout
   float r[VW];
 #pragma unroll
@@ -403,9 +424,17 @@ __global__ __launch_bounds__(MS_NT) void memory_step_kernel(
   }
   if (on) {
 #pragma unroll
-    for (int e = 0; e < VW; ++e) pr[r0 * dv + c0 + e] = r[e];
+    for (int e = 0; e < VW; ++e) pr[r0 * dvt + c0 + e] = r[e];
   }
   __syncthreads();
+  if (SPLIT) {
+    for (int j = tid; j < dvc; j += MS_NT) {
+      float o = 0.f;
+      for (int g = 0; g < RG; ++g) o += pr[g * dvt + j];
+      o_out[((size_t)b * H + h) * dv + cb + j] = o;
+    }
+    return;
+  }
   float below = 0.f;
 #pragma unroll
   for (int w = 0; w < MS_NT / TA_WAVE; ++w) below += redn[w];
@@ -431,6 +460,63 @@ __global__ __launch_bounds__(MS_NT) void memory_step_kernel(
   }
 }
 
+// What SPLIT leaves: normaliser, maximum and denominator, then norm and gate of the whole readout.
+#define MF_NT 256
+template <typename T>
+__global__ __launch_bounds__(MF_NT) void memory_step_finish_kernel(
+    const T* __restrict__ proj, int stride, int qoff, int koff, int goff, int ioff, int foff,
+    const float* __restrict__ ibias, const float* __restrict__ fbias, float cap, float* __restrict__ n_state,
+    float* __restrict__ m_state, const int* __restrict__ slots, int H, int dk, int dv, float qscale,
+    const float* __restrict__ norm_w, float eps, const float* __restrict__ o_in, T* __restrict__ out) {
+  constexpr int KEEP = 4;                            // columns a thread holds in registers; more are read twice
+  __shared__ float red[MF_NT / TA_WAVE], redn[MF_NT / TA_WAVE];
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const size_t at = (size_t)slots[b] * H + h;
+  const T* row = proj + (size_t)b * stride;
+  const float* src = o_in + ((size_t)b * H + h) * dv;
+  float o[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i) {
+    const int j = tid + MF_NT * i;
+    o[i] = j < dv ? src[j] : 0.f;
+    ss = fmaf(o[i], o[i], ss);
+  }
+  for (int j = tid + MF_NT * KEEP; j < dv; j += MF_NT) ss = fmaf(src[j], src[j], ss);
+  const MemoryGates gt = mm_gates(row, ioff, foff, h, ibias, fbias, cap, m_state[at]);
+  float dot = 0.f;
+  float* ns = n_state + at * dk;
+  for (int c = tid; c < dk; c += MF_NT) {
+    const float n = fmaf(gt.keep, ns[c], to_f32(row[koff + h * dk + c]) * gt.write);
+    ns[c] = n;
+    dot = fmaf(n, to_f32(row[qoff + h * dk + c]) * qscale, dot);
+  }
+  ss = wave_sum(ss);
+  dot = wave_sum(dot);
+  if (tid % TA_WAVE == 0) {
+    red[tid / TA_WAVE] = ss;
+    redn[tid / TA_WAVE] = dot;
+  }
+  __syncthreads();                                   // (every thread has read m_state before one writes it)
+  if (tid == 0) m_state[at] = gt.m;
+  float tot = 0.f, den = 0.f;
+#pragma unroll
+  for (int w = 0; w < MF_NT / TA_WAVE; ++w) {
+    tot += red[w];
+    den += redn[w];
+  }
+  const float below = 1.0f / (fmaxf(fabsf(den), expf(-gt.m)) + MM_FLOOR_EPS);
+  const float fac = below * rsqrtf(tot * below * below / (float)dv + eps);
+  auto put = [&](int j, float v) {
+    const float g = to_f32(row[goff + h * dv + j]);
+    out[(size_t)b * H * dv + (size_t)h * dv + j] = from_f32<T>(v * fac * norm_w[h * dv + j] / (1.0f + expf(-g)));
+  };
+#pragma unroll
+  for (int i = 0; i < KEEP; ++i)
+    if (tid + MF_NT * i < dv) put(tid + MF_NT * i, o[i]);
+  for (int j = tid + MF_NT * KEEP; j < dv; j += MF_NT) put(j, src[j]);
+}
+
 static int memory_step_rows(int dk, int dv) {         // key channels a thread keeps; 0: not taken
   const int cv = dv % 4 == 0 ? dv / 4 : dv;
   if (cv < 1 || cv > MS_NT) return 0;
@@ -443,19 +529,32 @@ static size_t memory_step_lds(int dk, int dv) {
   return ((size_t)2 * dk + (size_t)(MS_NT / cv) * dv) * sizeof(float);
 }
 
-// Whether ta_memory_step takes heads of dk x dv.
+static bool memory_step_whole(int dk, int dv) { return memory_step_rows(dk, dv) > 0 && memory_step_lds(dk, dv) <= 60000; }
+static int memory_step_tile(int dk, int dv) {         // columns of a workgroup where the head is cut; 0: not taken
+  const int widest = dv % 4 == 0 ? 128 : 64;
+  for (int t = widest; t >= 32; t /= 2)
+    if (memory_step_rows(dk, dv % 4 == 0 ? t : t + 1) > 0 && memory_step_lds(dk, dv % 4 == 0 ? t : t + 1) <= 60000)
+      return dv % 4 == 0 ? t : t + 1;                 // (an odd width: one column a thread, as where 4 does not divide dv)
+  return 0;
+}
+
+// How ta_memory_step takes heads of dk x dv: 1 in one kernel, 2 in two (with scratch for the readout), 0 not at all.
 extern "C" int ta_memory_step_fits(int dk, int dv) {
-  return dk >= 1 && dv >= 1 && memory_step_rows(dk, dv) > 0 && memory_step_lds(dk, dv) <= 60000;
+  if (dk < 1 || dv < 1) return 0;
+  if (memory_step_whole(dk, dv)) return 1;
+  const int t = memory_step_tile(dk, dv);
+  return t > 0 && (dv + t - 1) / t <= 65535 ? 2 : 0;
 }
 
 // proj: [batch] rows, stride apart, with q and k (H*dk each), v and the output gate (H*dv each), the input and
 // the forget gates' numbers (H each) at columns qoff, koff, voff, goff, ioff, foff. state [slots, H, dk, dv],
 // n_state [slots, H, dk], m_state [slots, H] float32; norm_w [H*dv]; out [batch, H*dv] = the readout over its
-// root mean square per head, times norm_w, times sigmoid(gate).
+// root mean square per head, times norm_w, times sigmoid(gate). scratch: [batch, H, dv] float32 where
+// ta_memory_step_fits says 2 (else null).
 extern "C" int ta_memory_step(hipStream_t stream, int dtype, const void* proj, int stride, int qoff, int koff, int voff,
                               int goff, int ioff, int foff, const float* ibias, const float* fbias, float cap,
                               float* state, float* n_state, float* m_state, const int* slots, int batch, int H, int dk,
-                              int dv, float qscale, const float* norm_w, float eps, void* out) {
+                              int dv, float qscale, const float* norm_w, float eps, float* scratch, void* out) {
   TA_REQUIRE(batch > 0 && batch <= 65535 && H >= 1 && H <= 65535, "ta_memory_step: batch %d, %d heads", batch, H);
   TA_REQUIRE(ta_memory_step_fits(dk, dv), "ta_memory_step: heads of %d x %d", dk, dv);
   TA_REQUIRE(qoff >= 0 && koff >= 0 && voff >= 0 && goff >= 0 && ioff >= 0 && foff >= 0 && stride >= qoff + H * dk &&
@@ -463,13 +562,19 @@ extern "C" int ta_memory_step(hipStream_t stream, int dtype, const void* proj, i
              stride >= foff + H, "ta_memory_step: rows of %d are too short", stride);
   TA_REQUIRE(cap > 0.f, "ta_memory_step: the cap must be positive, got %g", (double)cap);
   TA_REQUIRE(dv % 4 != 0 || (uintptr_t)state % 16 == 0, "ta_memory_step: the state must be 16-byte aligned");
-  const int rows = memory_step_rows(dk, dv);
-  const size_t lds = memory_step_lds(dk, dv);
-  dim3 g(H, batch);
-#define MS_RUN(T, VWV, RW)                                                                                             \
-  memory_step_kernel<T, VWV, RW><<<g, MS_NT, lds, stream>>>((const T*)proj, stride, qoff, koff, voff, goff, ioff, foff, \
-                                                            ibias, fbias, cap, state, n_state, m_state, slots, H, dk,  \
-                                                            dv, qscale, norm_w, eps, (T*)out)
+  const bool split = !memory_step_whole(dk, dv);
+  TA_REQUIRE(!split || scratch != nullptr, "ta_memory_step: heads of %d x %d need scratch memory", dk, dv);
+  TA_REQUIRE(dtype == TA_F32 || dtype == TA_BF16, "ta_memory_step: unknown dtype %d", dtype);
+  const int dvt = split ? memory_step_tile(dk, dv) : dv;
+  const int rows = memory_step_rows(dk, dvt);
+  const size_t lds = memory_step_lds(dk, dvt);
+  dim3 g(H, batch, split ? (dv + dvt - 1) / dvt : 1);
+#define MS_KERNEL(T, VWV, RW, SP)                                                                                   \
+  memory_step_kernel<T, VWV, RW, SP><<<g, MS_NT, lds, stream>>>(                                                    \
+      (const T*)proj, stride, qoff, koff, voff, goff, ioff, foff, ibias, fbias, cap, state, n_state, m_state, slots, \
+      H, dk, dv, qscale, norm_w, eps, (T*)out, dvt, scratch)
+#define MS_RUN(T, VWV, RW) \
+  if (split) MS_KERNEL(T, VWV, RW, true); else MS_KERNEL(T, VWV, RW, false)
 #define MS_BY_ROWS(T, VWV)                 \
   switch (rows) {                          \
     case 4: MS_RUN(T, VWV, 4); break;      \
@@ -479,11 +584,18 @@ extern "C" int ta_memory_step(hipStream_t stream, int dtype, const void* proj, i
   }
 #define MS_BY_COLS(T) \
   if (dv % 4 == 0) { MS_BY_ROWS(T, 4) } else { MS_BY_ROWS(T, 1) }
-  if (dtype == TA_F32) { MS_BY_COLS(float) }
-  else if (dtype == TA_BF16) { MS_BY_COLS(bf16_t) }
-  else return ta_fail("ta_memory_step: unknown dtype %d", dtype);
+  if (dtype == TA_F32) { MS_BY_COLS(float) } else { MS_BY_COLS(bf16_t) }
 #undef MS_BY_COLS
 #undef MS_BY_ROWS
 #undef MS_RUN
+#undef MS_KERNEL
+  const int rc = ta_check_launch("ta_memory_step");
+  if (rc != 0 || !split) return rc;
+#define MF_RUN(T)                                                                                                   \
+  memory_step_finish_kernel<T><<<dim3(H, batch), MF_NT, 0, stream>>>((const T*)proj, stride, qoff, koff, goff, ioff, \
+                                                                     foff, ibias, fbias, cap, n_state, m_state, slots, \
+                                                                     H, dk, dv, qscale, norm_w, eps, scratch, (T*)out)
+  if (dtype == TA_F32) MF_RUN(float); else MF_RUN(bf16_t);
+#undef MF_RUN
   return ta_check_launch("ta_memory_step");
 }

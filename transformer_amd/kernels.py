@@ -2298,17 +2298,18 @@ def memory_recurrent(proj: torch.Tensor, q_off: int, k_off: int, v_off: int, q_s
     return o_out
 
 
-def memory_step_fits(key_dim: int, value_dim: int) -> bool:
-    """Whether ``memory_step`` takes heads of this size."""
-    return bool(library().ta_memory_step_fits(c_int(key_dim), c_int(value_dim)))
+def memory_step_fits(key_dim: int, value_dim: int) -> int:
+    """How ``memory_step`` takes heads of this size: 1 in one kernel, 2 in two (with scratch memory), 0 not at all."""
+    return int(library().ta_memory_step_fits(c_int(key_dim), c_int(value_dim)))
 
 
 def memory_step(proj: torch.Tensor, offsets: Sequence[int], i_bias, f_bias, cap: float, state: torch.Tensor,
                 n_state: torch.Tensor, m_state: torch.Tensor, slots, q_scale: float, norm_w, eps: float,
-                out: torch.Tensor) -> torch.Tensor:
-    """A step of single tokens of the matrix memory in one kernel (row b belongs to sequence b). offsets: columns
+                out: torch.Tensor, scratch: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A step of single tokens of the matrix memory in one kernel, or two (``memory_step_fits``) (row b belongs to sequence b). offsets: columns
     of q, k, v, the output gate, the input and the forget gates in the rows of ``proj``. out [batch, H*dv] = o /
-    rms(o per head) * norm_w * sigmoid(gate), o = S^T q / (max(|n . q|, exp(-m)) + 1e-6)."""
+    rms(o per head) * norm_w * sigmoid(gate), o = S^T q / (max(|n . q|, exp(-m)) + 1e-6). scratch [batch, H, dv]
+    float32 where the heads take two kernels."""
     _dev(proj, "proj", contiguous=False); _dev(state, "state", torch.float32); _dev(out, "out", proj.dtype)
     B, stride = _rows2d(proj, "proj")
     _dev(slots, "slots", torch.int32)
@@ -2323,8 +2324,16 @@ def memory_step(proj: torch.Tensor, offsets: Sequence[int], i_bias, f_bias, cap:
     if slots.numel() != B or out.shape != (B, H * dv):
         raise KernelError(f"memory_step: {slots.numel()} slots, out {tuple(out.shape)} for {B} rows of {H} heads of {dv}")
     _memory_columns("memory_step", proj, offsets, H, dk, dv)
+    if memory_step_fits(dk, dv) == 2:
+        if scratch is None:
+            raise KernelError(f"memory_step: heads of {dk} x {dv} need scratch memory")
+        _dev(scratch, "scratch", torch.float32)
+        if scratch.shape != (B, H, dv):
+            raise KernelError(f"memory_step: scratch is {tuple(scratch.shape)}, expected {(B, H, dv)}")
+    else:
+        scratch = None
     _check(library().ta_memory_step(
         _stream(), c_int(_code(proj.dtype)), _ptr(proj), c_int(stride), *[c_int(int(o)) for o in offsets], _ptr(i_bias),
         _ptr(f_bias), c_float(cap), _ptr(state), _ptr(n_state), _ptr(m_state), _ptr(slots), c_int(B), c_int(H), c_int(dk),
-        c_int(dv), c_float(q_scale), _ptr(norm_w), c_float(eps), _ptr(out)))
+        c_int(dv), c_float(q_scale), _ptr(norm_w), c_float(eps), _ptr(scratch), _ptr(out)))
     return out

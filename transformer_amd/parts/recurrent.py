@@ -415,8 +415,8 @@ class MatrixMemory(Part):
     """The matrix memory with exponential gates, a running maximum and a normaliser (``MatrixMemorySpec``).
 
     One product gives [q | k | v | output gate | input gates | forget gates]. A step of single tokens then takes
-    ONE kernel to the normed and gated readout (``kernels.memory_step``). Longer steps, and heads too large for
-    it: ``kernels.memory_gates`` forms the weights of all tokens by a scan over the running maximum,
+    ONE kernel to the normed and gated readout (``kernels.memory_step``; large heads two). Longer steps, and heads too
+    large for that: ``kernels.memory_gates`` forms the weights of all tokens by a scan over the running maximum,
     ``kernels.memory_recurrent`` walks the tokens with the normaliser as one more value column, and the head norm
     divides by the denominator first. State, normaliser, maximum, gates and readout stay float32."""
     graph_safe = True
@@ -465,9 +465,11 @@ class MatrixMemory(Part):
         y = take("memory.y", (nt, self.nv), self.dtype)
         q_off, k_off, v_off, g_off, i_off, f_off = self.offsets
         q_scale, biases = float(dk) ** -0.5, (self.w["i.bias"], self.w["f.bias"])
-        if ctx.all_single and kernels.memory_step_fits(dk, dv):
+        fits = kernels.memory_step_fits(dk, dv) if ctx.all_single else 0
+        if fits:
+            scratch = take("memory.step", (nt, H, dv), f32) if fits == 2 else None
             kernels.memory_step(proj, self.offsets, *biases, float(s.gate_cap), state, n_state, m_state, ctx.slots, q_scale,
-                                self.w["norm.weight"], float(s.eps), y)
+                                self.w["norm.weight"], float(s.eps), y, scratch)
             return finish(y, self.w["out.weight"], ctx.ws, "memory.delta", fold, into)
         keep, write, floor = (take(f"memory.{n}", (nt, H), f32) for n in ("keep", "write", "floor"))
         kernels.memory_gates(proj, i_off, f_off, *biases, float(s.gate_cap), m_state, ctx.cu_q, ctx.slots,
