@@ -461,7 +461,7 @@ def test_delta_rule_with_one_of_its_inputs_low_rank(ranks):
 
 
 MOE_GEOMS = [(6, 2, 20, 40, 3, 1.7), (5, 5, 17, 33, 0, 1.0), (3, 5, 24, 64, 2, 0.6), (1, 1, 30, 48, 0, 2.0), (1, 2, 8, 72, 4, 1.1),
-             (12, 3, 96, 256, 4, 2.0), (64, 6, 48, 128, 8, 1.5)]
+             (12, 3, 80, 264, 4, 2.0), (64, 6, 48, 128, 8, 1.5)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
